@@ -169,37 +169,20 @@ int create_impl(mmi_duplex* d) {
         return mmi_fail(MMI_ERR_SHAPE, "the codec produces fewer codebooks than the LM expects from the user stream");   // lm.py:683-686
     if (lc.dep_q < 1 || lc.dep_q > mc.q_n_q) return mmi_fail(MMI_ERR_SHAPE, "the LM must generate between 1 and n_q codebooks for the codec");
     if (mc.q_bins != lc.card) return mmi_fail(MMI_ERR_SHAPE, "codec cardinality != LM card");
-    // Stream priorities.  Streams of one priority share a pool of GPU_MAX_HW_QUEUES (4) hardware queues with everything else the
-    // process created at that priority, and two streams that land on one queue do not overlap (profiles/r03_logs: the encoder
-    // and the LM shared queue 4 without priorities).  The LM and the codec are therefore given DIFFERENT priorities (distinct queue
-    // pools); which of the two is the high one matters little (below).
+    // All three streams have the default priority (streams of different priorities in one process have hung on this stack); created
+    // back to back, they land on different hardware queues of the pool of GPU_MAX_HW_QUEUES (4).
     MMI_HIP_CHECK(hipMalloc((void**)&d->flags, (size_t)F_COUNT * 16 * sizeof(long)));
     MMI_HIP_CHECK(hipMemset(d->flags, 0, (size_t)F_COUNT * 16 * sizeof(long)));
-    int lo = 0, hi = 0;
     // MMI_DUPLEX_CODEC_CUS=n (experiment, round 6): the codec streams confined to n of the CUs (a CU mask of n bits, which the driver
     // deals out over the XCDs), so that the depth transformer's launches - 96..176 workgroups that need a whole CU's wave slots each -
-    // find free CUs while the codec of the neighbouring frames runs beside them; such streams have the default priority
+    // find free CUs while the codec of the neighbouring frames runs beside them
     const int codec_cus = getenv("MMI_DUPLEX_CODEC_CUS") ? atoi(getenv("MMI_DUPLEX_CODEC_CUS")) : 0;
     if (codec_cus > 0 && codec_cus < 256) {
         unsigned mask[8] = {0, 0, 0, 0, 0, 0, 0, 0};
         for (int i = 0; i < codec_cus; ++i) mask[i >> 5] |= 1u << (i & 31);
-        int plo = 0, phi = 0;
-        if (hipDeviceGetStreamPriorityRange(&plo, &phi) == hipSuccess && plo != phi) MMI_HIP_CHECK(hipStreamCreateWithPriority(&d->sL, hipStreamNonBlocking, plo));
-        else MMI_HIP_CHECK(hipStreamCreateWithFlags(&d->sL, hipStreamNonBlocking));
+        MMI_HIP_CHECK(hipStreamCreateWithFlags(&d->sL, hipStreamNonBlocking));
         MMI_HIP_CHECK(hipExtStreamCreateWithCUMask(&d->sE, 8, mask));
         MMI_HIP_CHECK(hipExtStreamCreateWithCUMask(&d->sD, 8, mask));
-    } else
-    if (hipDeviceGetStreamPriorityRange(&lo, &hi) == hipSuccess && lo != hi) {
-        // The LM's stream in the high-priority pool, the codec's two in the low one: the step's critical path is the LM's launch
-        // chain, the codec only has to be done by the time the next step wants its codes.  Same-box pairs (round 6,
-        // profiles/r06_logs/ab_stream_priorities.txt): -0.02 ms per 32-session step on average against the reverse (rounds 3-5),
-        // -0.06 ms at 64 sessions; equal priorities: +0.5 ms.  MMI_DUPLEX_PRIO = codec / none select those for an A/B.
-        const char* pe = getenv("MMI_DUPLEX_PRIO");
-        const int mid = (lo + hi) / 2;
-        const int pl = pe && pe[0] == 'c' ? lo : (pe && pe[0] == 'n' ? mid : hi), pc = pe && pe[0] == 'c' ? hi : (pe && pe[0] == 'n' ? mid : lo);
-        MMI_HIP_CHECK(hipStreamCreateWithPriority(&d->sL, hipStreamNonBlocking, pl));
-        MMI_HIP_CHECK(hipStreamCreateWithPriority(&d->sE, hipStreamNonBlocking, pc));
-        MMI_HIP_CHECK(hipStreamCreateWithPriority(&d->sD, hipStreamNonBlocking, pc));
     } else {
         MMI_HIP_CHECK(hipStreamCreateWithFlags(&d->sL, hipStreamNonBlocking));
         MMI_HIP_CHECK(hipStreamCreateWithFlags(&d->sE, hipStreamNonBlocking));

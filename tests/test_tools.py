@@ -85,8 +85,7 @@ def test_built_library_has_no_in_place_cross_swizzled_packed_fp32_instruction():
     """The instruction form that stood in k_gemm_xp's RoPE epilogue when its output was not reproducible (round 4's driver failure;
     HISTORY.md round 5 10a: `v_pk_mul_f32 v[14:15], v[30:31], v[14:15] op_sel:[0,1] op_sel_hi:[1,0]`) must not come back through a
     compiler update or a new epilogue: the gfx950 code objects of the library `build()` produced are disassembled and scanned
-    (scripts/isa_scan_packed_swizzle.py; the sequence alone is exact on the chip - scripts/pk_hazard_repro.hip, 6.6e8 wave executions -
-    so this is a tripwire around a context-dependent failure that was never explained, not a proven erratum)."""
+    (scripts/isa_scan_packed_swizzle.py).  The build also switches packed fp32 math off altogether (moshi_amd/build.py)."""
     import subprocess
     import sys
     from pathlib import Path
