@@ -15,13 +15,14 @@ import torch
 
 _PKG = Path(__file__).resolve().parent
 DEFAULT_LIB = _PKG / "libmoshi_mi.so"
+TLM_LIB = _PKG / "libmoshi_tlm.so"
 
 MMI_OK, MMI_ERR_INVALID, MMI_ERR_SHAPE, MMI_ERR_STATE, MMI_ERR_HIP, MMI_ERR_MISSING_WEIGHT, MMI_ERR_UNSUPPORTED, MMI_ERR_BUSY, \
     MMI_ERR_NO_CHANNEL = 0, -1, -2, -3, -4, -5, -6, -7, -8
-MMI_F32, MMI_BF16, MMI_I64, MMI_F16, MMI_I8, MMI_F8E4M3 = 0, 1, 2, 3, 4, 5
+MMI_F32, MMI_BF16, MMI_I64, MMI_F16, MMI_I8, MMI_F8E4M3, MMI_I32 = 0, 1, 2, 3, 4, 5, 6
 
 _DTYPES = {torch.float32: MMI_F32, torch.bfloat16: MMI_BF16, torch.int64: MMI_I64, torch.float16: MMI_F16,
-           torch.int8: MMI_I8, torch.float8_e4m3fn: MMI_F8E4M3}
+           torch.int8: MMI_I8, torch.float8_e4m3fn: MMI_F8E4M3, torch.int32: MMI_I32}
 
 
 class TensorDesc(C.Structure):
@@ -77,6 +78,26 @@ class BatcherStats(C.Structure):
     _fields_ = [("steps", C.c_int64), ("frames", C.c_int64), ("dropped_frames", C.c_int64), ("used_slots", C.c_int32),
                 ("total_slots", C.c_int32), ("last_step_ms", C.c_float)]
 
+
+class TLMLayer(C.Structure):
+    _fields_ = [("mixer", C.c_int32), ("width", C.c_int32), ("heads", C.c_int32), ("dim", C.c_int32), ("vdim", C.c_int32),
+                ("rot_dim", C.c_int32), ("q_rank", C.c_int32), ("kv_rank", C.c_int32), ("window", C.c_int32), ("scale", C.c_float),
+                ("rot_base", C.c_double), ("mlp", C.c_int32), ("experts", C.c_int32), ("top", C.c_int32), ("ff", C.c_int32),
+                ("act", C.c_int32), ("router", C.c_int32)]
+
+
+class TLMCfg(C.Structure):
+    _fields_ = [("vocab", C.c_int32), ("width", C.c_int32), ("n_layers", C.c_int32), ("layers", C.POINTER(TLMLayer)),
+                ("loop_start", C.c_int32), ("loop_stop", C.c_int32), ("loop_times", C.c_int32), ("norm_groups", C.c_int32),
+                ("norm_eps", C.c_float), ("logit_scale", C.c_float), ("dtype", C.c_int32)]
+
+
+# include/moshi_tlm.h
+TLM_MIX_LATENT_ATTENTION, TLM_MIX_MINGRU = 1, 2
+TLM_MLP_NONE, TLM_MLP_MOE = 0, 1
+TLM_ACT_RELU2, TLM_ROUTE_TOKEN_TABLE = 1, 1
+(TLM_PAGE_TOKENS, TLM_TOTAL_PAGES, TLM_FREE_PAGES, TLM_FREE_SLOTS, TLM_POSITION, TLM_HELD_PAGES, TLM_WEIGHT_BYTES, TLM_LAYER_RUNS,
+ TLM_GRAPHS) = range(9)
 
 # name -> (restype, argtypes); every symbol include/moshi_mi.h declares
 _P = C.c_void_p
@@ -154,14 +175,30 @@ SIGNATURES = {
                                      C.POINTER(C.c_char_p)]),
 }
 
+# include/moshi_tlm.h (libmoshi_tlm.so; the error plumbing is linked into both libraries)
+TLM_SIGNATURES = {
+    "mmi_version": (C.c_int, []),
+    "mmi_last_error": (C.c_char_p, []),
+    "mmi_tlm_create": (C.c_int, [C.POINTER(TLMCfg), C.POINTER(TensorDesc), C.c_int32, C.c_int32, C.c_int64, C.c_int32, C.POINTER(_P)]),
+    "mmi_tlm_destroy": (None, [_P]),
+    "mmi_tlm_open": (C.c_int, [_P, C.POINTER(C.c_int32)]),
+    "mmi_tlm_close": (C.c_int, [_P, C.c_int32]),
+    "mmi_tlm_step": (C.c_int, [_P, C.c_int32, _P, _P, _P, C.c_int32, _P, _P, _P]),
+    "mmi_tlm_sample": (C.c_int, [_P, C.c_int32, _P, _P, _P, _P, C.c_uint64, _P, _P]),
+    "mmi_tlm_info": (C.c_int64, [_P, C.c_int32, C.c_int32]),
+    "mmi_tlm_pages_needed": (C.c_int64, [_P, C.c_int32, C.c_int64]),
+    "mmi_tlm_set_taps": (C.c_int, [_P, _P]),
+    "mmi_tlm_launch_list": (C.c_int64, [_P, _P, C.c_int64]),
+}
+
 
 class Lib:
     """A loaded engine library with typed entry points and the reference's error conventions."""
 
-    def __init__(self, path: Path):
+    def __init__(self, path: Path, signatures=None):
         self.path = Path(path)
         self.cdll = C.CDLL(str(self.path))
-        for name, (res, args) in SIGNATURES.items():
+        for name, (res, args) in (SIGNATURES if signatures is None else signatures).items():
             fn = getattr(self.cdll, name)  # AttributeError if the library does not export the ABI
             fn.restype = res
             fn.argtypes = args
@@ -212,6 +249,23 @@ def load(path: Optional[Path] = None) -> Lib:
                 "moshi_amd has no CPU/PyTorch fallback for this path.")
         _default = Lib(DEFAULT_LIB)
     return _default
+
+
+_default_tlm: Optional[Lib] = None
+
+
+def load_tlm(path: Optional[Path] = None) -> Lib:
+    """Load the token-LM library: the in-tree gfx950 build, or a loud failure."""
+    global _default_tlm
+    if path is not None:
+        return Lib(Path(path), TLM_SIGNATURES)
+    if _default_tlm is None:
+        if not TLM_LIB.exists():
+            raise RuntimeError(
+                f"{TLM_LIB} is missing: build the HIP extension first (python -m moshi_amd.build). "
+                "moshi_amd has no CPU/PyTorch fallback for this path.")
+        _default_tlm = Lib(TLM_LIB, TLM_SIGNATURES)
+    return _default_tlm
 
 
 def tensor_descs(state: Dict[str, torch.Tensor]):

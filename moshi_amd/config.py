@@ -8,7 +8,7 @@ architecture are used by the tests (oracle-sized).
 from __future__ import annotations
 
 from dataclasses import dataclass, field
-from typing import List
+from typing import List, Optional
 
 
 @dataclass
@@ -172,3 +172,118 @@ def tiny_lm_config() -> LMConfig:
     return LMConfig(dim=128, num_heads=4, num_layers=2, hidden_scale=4.125, context=12, n_q=16, dep_q=8, card=64,
                     text_card=96, depformer_dim=64, depformer_dim_feedforward=int(4.125 * 64),
                     depformer_num_heads=2, depformer_num_layers=2)
+
+
+# --------------------------------------------------------------------------------------------------------------------
+# token language models (libmoshi_tlm.so)
+# --------------------------------------------------------------------------------------------------------------------
+@dataclass
+class LatentAttentionConfig:
+    """Attention whose keys and values are projections of one cached latent, plus one rotated key part shared by the heads."""
+    heads: int
+    dim: int
+    vdim: int
+    rot_dim: int
+    q_rank: int
+    kv_rank: int
+    scale: float
+    rot_base: float = 10000.0
+    window: int = 0                     # keys seen, the position itself included; 0 = every earlier one
+
+
+@dataclass
+class MinGRUConfig:
+    """Minimal GRU: an element-wise recurrence gated by projections of its input alone (nothing multiplies the state by a matrix)."""
+    width: int
+
+
+@dataclass
+class MoEConfig:
+    """Experts chosen by a table over token ids."""
+    experts: int
+    top: int
+    ff: int
+    activation: str = "relu2"
+    router: str = "token_table"
+
+
+@dataclass
+class TokenLayerConfig:
+    mixer: object                       # LatentAttentionConfig | MinGRUConfig
+    mlp: Optional[MoEConfig] = None
+
+
+@dataclass
+class TokenLMConfig:
+    """A decoder-only network over token ids: parallel sublayers behind one grouped RMS norm, layer scales, and optionally a weight-tied
+    repetition of layers [loop_start, loop_stop), whose second and later passes re-inject the embedding."""
+    architecture: str
+    vocab: int
+    width: int
+    layers: List[TokenLayerConfig]
+    norm_groups: int = 1
+    norm_eps: float = 1e-6
+    logit_scale: float = 1.0
+    loop_start: int = 0
+    loop_stop: int = 0                  # start == stop: nothing is repeated
+    loop_times: int = 1
+
+    @property
+    def layer_runs(self) -> List[int]:
+        """Layer index of every execution, in order."""
+        n = list(range(len(self.layers)))
+        if self.loop_stop <= self.loop_start:
+            return n
+        return n[:self.loop_start] + n[self.loop_start:self.loop_stop] * self.loop_times + n[self.loop_stop:]
+
+
+def _known(d: dict, keys, what: str) -> dict:
+    extra = sorted(set(d) - set(keys))
+    if extra:
+        raise ValueError(f"{what}: unknown entries {extra}")
+    return d
+
+
+def kesirax_config(raw: dict) -> TokenLMConfig:
+    """config.json of a Kesirax model -> TokenLMConfig.  Sizes and constants come from the file; the structure (latent attention and
+    minGRU mixers beside token-table experts with squared-ReLU activations) is the design's."""
+    def mlp(m):
+        if m is None:
+            return None
+        _known(m, ("kind", "expert", "router"), "mlp")
+        if m.get("kind", "moe") != "moe":
+            raise ValueError(f"mlp kind {m['kind']!r} is not part of this design")
+        return MoEConfig(experts=int(m["router"]["experts"]), top=int(m["router"]["top"]), ff=int(m["expert"]["ff"]))
+
+    def mixer(kind, m):
+        if kind == "mingru":
+            return MinGRUConfig(width=int(m["width"]))
+        if kind == "latent_attention":
+            rot = m.get("rot") or {}
+            if rot and int(rot["dims"]) != int(m["rot_dim"]):
+                raise ValueError("latent attention rotates its whole rotated part: rot.dims must equal rot_dim")
+            return LatentAttentionConfig(
+                heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]), rot_dim=int(m["rot_dim"]), q_rank=int(m["q_rank"]),
+                kv_rank=int(m["kv_rank"]), scale=float(m["scale"]), rot_base=float(rot.get("base", 10000.0)),
+                window=int((m.get("mask") or {}).get("size", 0)))
+        raise ValueError(f"mixer type {kind!r} is not part of this design")
+
+    layers = [TokenLayerConfig(mixer(l["type"], l["mixer"]), mlp(l.get("mlp"))) for l in raw["layers"]]
+    norm, loop = raw["norm"], raw.get("loop") or {}
+    return TokenLMConfig(
+        architecture=raw["architecture"], vocab=int(raw["vocab"]), width=int(raw["width"]), layers=layers, norm_groups=int(norm.get("groups", 1)),
+        norm_eps=float(norm["eps"]), logit_scale=float(raw.get("logit_scale", 1.0)), loop_start=int(loop.get("start", 0)),
+        loop_stop=int(loop.get("stop", 0)), loop_times=int(loop.get("times", 1)))
+
+
+# config.json `architecture` -> parser; the registry `loaders.get_token_lm` and the command lines choose a model class by
+TOKEN_LM_ARCHITECTURES = {"Kesirax": kesirax_config}
+
+
+def tiny_token_lm_config() -> TokenLMConfig:
+    """A Kesirax network at oracle size, with sizes that are no multiples of the kernels' tiles."""
+    att = LatentAttentionConfig(heads=3, dim=24, vdim=20, rot_dim=12, q_rank=40, kv_rank=36, scale=0.17, rot_base=5000.0, window=37)
+    moe = MoEConfig(experts=5, top=2, ff=44)
+    return TokenLMConfig("Kesirax", vocab=101, width=96, norm_groups=3, norm_eps=1e-5, logit_scale=0.7, loop_start=1, loop_stop=3, loop_times=2,
+                         layers=[TokenLayerConfig(MinGRUConfig(72), moe), TokenLayerConfig(att, moe), TokenLayerConfig(MinGRUConfig(72), None),
+                                 TokenLayerConfig(att, MoEConfig(experts=4, top=1, ff=52))])

@@ -1,0 +1,1322 @@
+// Token language models behind the C ABI of include/moshi_tlm.h: decoder-only networks whose layers are described by mmi_tlm_cfg,
+// stepped over mixed batches (prompt portions beside single tokens) from a paged latent cache and recurrent state slots.
+//
+//   step   = prepare (tokens, block tables, rotation tables) -> routing -> per layer run:
+//              residual + norm | mixer projections, expert up | mixer core | mixer output, expert down
+//            -> residual + norm of the wanted rows -> head
+//   The sublayers of a layer read one norm, so the mixer's input projection and the experts' up projection are one launch, and so
+//   are the mixer's output projection and the experts' down projection (TlmJobs).
+// Steps that only bring single tokens are captured into a hipGraph per shape (batch, wanted rows, attention split): everything that
+// varies between two such steps is device memory uploaded in one copy.
+#include "mmi_common.h"
+#include "mmi_graph.h"
+#include "../../include/moshi_tlm.h"
+#include "lm_kernels.h"
+#include "tlm_kernels.h"
+
+#include <math.h>
+#include <algorithm>
+#include <map>
+#include <memory>
+#include <tuple>
+
+int64_t mmi_copy_launch_log(const std::vector<std::string>& log, char* buf, int64_t cap);
+
+namespace {
+
+int round_up(int v, int m) { return (v + m - 1) / m * m; }
+
+struct Mat {                       // one packed matrix, or `groups` of equal shape
+    u32x4* wp = nullptr;
+    int NT = 0, KS = 0;
+    long gs = 0;                   // fragments x 64 per group
+    long bytes() const { return gs * 16; }
+};
+
+struct Layer {
+    mmi_tlm_layer c;
+    float *norm = nullptr, *ls1 = nullptr, *ls2 = nullptr;
+    // minGRU
+    Mat zcg, out;
+    float* bias = nullptr;
+    int wp = 0;
+    // latent attention
+    Mat in, uqn, uqr, uk, uv;
+    float *qw = nullptr, *cw = nullptr;
+    int qp = 0, kvp = 0, rp = 0, hp = 0, dim_p = 0, vdim_p = 0, lat_ks = 0, k_ks = 0, nd = 0, q_ks = 0;
+    int rope = -1, geo = -1;
+    // experts
+    Mat up, down;
+    int route = -1;
+};
+
+struct Run {                       // one execution of a layer: repeated layers share weights, not state
+    int layer = 0;
+    bool add_emb = false;
+    void *kc = nullptr, *vc = nullptr;
+    float* state = nullptr;
+};
+
+struct Slot {
+    bool live = false;
+    int64_t pos = 0;
+    int par = 0;                   // which copy of the recurrent state is current
+    int64_t first_page = 0;        // pages before it have left every window
+    std::vector<int> pages;        // pages[i] holds positions 64 (first_page + i) ..
+};
+
+struct Staging {
+    int* host = nullptr;
+    hipEvent_t ev = nullptr;
+    bool used = false;
+};
+
+// where the parts of a step's metadata sit in the uploaded block (ints)
+struct Meta {
+    int htok, pos, rslot, crow, want, erow0, elen, epos0, eslot, tile0, seg, upd, total;
+};
+
+struct Shape {                     // what a launch list depends on
+    int T = 0, n_want = 0, n_entries = 0, n_seg = 0, nsplit = 1;
+    bool pairs = false;            // some sequence spans several scan segments
+    std::vector<int> tiles;        // attention column tiles per head count
+    Meta m;
+    float* logits = nullptr;
+    float* taps = nullptr;
+};
+
+}  // namespace
+
+struct mmi_tlm {
+    mmi_tlm_cfg cfg;
+    std::vector<Layer> layers;
+    std::vector<Run> runs;
+    int device = 0;
+    bool f32 = false;
+    int kstep = 32, V = 8, esize = 2;
+    int ld = 0, h_ks = 0;
+    int max_slots = 0, max_pages = 0, max_T = 0;
+    bool has_attn = false, has_gru = false;
+    int64_t max_window = 0;        // 0: some layer sees every earlier position
+    MmiArena wts, st, scratch;
+    uint16_t* embed = nullptr;
+    float* final_norm = nullptr;
+    Mat head;
+    std::vector<int> geo;          // distinct head counts
+    std::vector<std::pair<double, int>> ropes;      // distinct (base, dims)
+    std::vector<TlmRope> rope_host;
+    TlmRope* rope_dev = nullptr;
+    std::vector<TlmRouteLayer> route_host;
+    TlmRouteLayer* route_dev = nullptr;
+    int max_experts = 0, max_top = 0;
+    long tile_ld = 0, list_ld = 0;
+    // scratch
+    float *x = nullptr, *mix = nullptr, *dn = nullptr, *zcg = nullptr, *lat = nullptr, *gate = nullptr, *pair = nullptr, *po = nullptr, *pml = nullptr;
+    void *h = nullptr, *y = nullptr, *cq = nullptr, *qn = nullptr, *q = nullptr, *ao = nullptr, *o = nullptr, *hid = nullptr;
+    int *list = nullptr, *tiles = nullptr, *n_tiles = nullptr, *tok = nullptr, *meta = nullptr, *last_tok = nullptr, *block_table = nullptr;
+    float* logits = nullptr;       // [max_slots][vocab] for captured steps
+    uint16_t* samp_rows = nullptr; int samp_ld = 0;
+    int* samp_map = nullptr; unsigned long long* samp_rng = nullptr; int* samp_zero = nullptr;
+    uint64_t samp_count = 0;
+    long split_elems = 0;          // partial-sum capacity of mix / dn / lat in rows
+    // host state
+    std::vector<Slot> slots;
+    std::vector<int> free_pages;
+    Staging staging[4];
+    int stage_at = 0;
+    size_t meta_cap = 0;
+    float* taps = nullptr;
+    bool graphs = true;
+    hipStream_t cap_stream = nullptr;
+    std::map<std::tuple<int, int, int>, std::unique_ptr<MmiProgram>> progs;
+    std::vector<std::string> last_log;
+    long weight_bytes = 0;
+};
+
+namespace {
+
+constexpr int MAX_SPLIT = 8;
+constexpr int ROWS_MAX = 64;       // up to here a step takes the weight-streaming kernel
+constexpr int MAX_PARTIALS = 512;  // (column tile, split) pairs of the attention
+
+// ------------------------------------------------------------------------------------------------
+// weights
+// ------------------------------------------------------------------------------------------------
+struct Loader {
+    mmi_tlm* m;
+    MmiWeights W;
+    int* map = nullptr;            // device scratch for a row and a column map
+    size_t map_cap = 0;
+    ~Loader() { if (map) hipFree(map); }
+
+    int find(const std::string& name, int dtype, std::initializer_list<int64_t> shape, const mmi_tensor_desc** out) {
+        const mmi_tensor_desc* d = W.find(name);
+        if (!d) return mmi_fail(MMI_ERR_MISSING_WEIGHT, "missing weight: " + name);
+        if (d->dtype != dtype) return mmi_fail(MMI_ERR_UNSUPPORTED, "unexpected dtype of " + name);
+        if (d->ndim != (int)shape.size()) return mmi_fail(MMI_ERR_SHAPE, "unexpected rank of " + name);
+        int i = 0;
+        for (int64_t s : shape) {
+            if (d->shape[i] != s)
+                return mmi_fail(MMI_ERR_SHAPE, "shape mismatch for " + name + ": dimension " + std::to_string(i) + " is " + std::to_string(d->shape[i]) +
+                                                   ", expected " + std::to_string(s));
+            ++i;
+        }
+        *out = d;
+        return MMI_OK;
+    }
+    int upload(const std::vector<int>& a, const std::vector<int>& b) {
+        const size_t n = a.size() + b.size();
+        if (n > map_cap) {
+            if (map) hipFree(map);
+            map = nullptr;
+            MMI_HIP_CHECK(hipMalloc((void**)&map, n * sizeof(int)));
+            map_cap = n;
+        }
+        MMI_HIP_CHECK(hipDeviceSynchronize());
+        MMI_HIP_CHECK(hipMemcpy(map, a.data(), a.size() * sizeof(int), hipMemcpyHostToDevice));
+        if (!b.empty()) MMI_HIP_CHECK(hipMemcpy(map + a.size(), b.data(), b.size() * sizeof(int), hipMemcpyHostToDevice));
+        return MMI_OK;
+    }
+    int alloc(Mat* mat, int groups, int NT, int KS) {
+        mat->NT = NT;
+        mat->KS = KS;
+        mat->gs = (long)NT * KS * 64;
+        MMI_HIP_CHECK(m->wts.alloc(&mat->wp, (size_t)groups * mat->gs));
+        m->weight_bytes += groups * mat->bytes();
+        return MMI_OK;
+    }
+    // tiles 0 .. rows/16 of the source (through the maps) become tiles t * tmul + toff of `dst`; the maps stay on the device until the
+    // next upload, so packing many matrices of one shape uploads them once
+    int pack(const mmi_tensor_desc* d, u32x4* dst, int rows, int cols, long sr, long sc, int tmul = 1, int toff = 0, long src_off = 0) {
+        const int NT = rows / 16, KS = cols / m->kstep;
+        const long n = (long)NT * KS * 64 * m->V;
+        const int blocks = (int)mmi_cdiv64(n, 256);
+        const uint16_t* src = (const uint16_t*)d->data + src_off;
+        if (m->f32) MMI_LAUNCH((k_tlm_pack<TlmF32>), blocks, 256, 0, (hipStream_t)0, src, sr, sc, map, map + rows, (float*)dst, NT, KS, tmul, toff);
+        else MMI_LAUNCH((k_tlm_pack<TlmBf16>), blocks, 256, 0, (hipStream_t)0, src, sr, sc, map, map + rows, (uint16_t*)dst, NT, KS, tmul, toff);
+        MMI_CHECK_LAUNCH();
+        return MMI_OK;
+    }
+    int ident(int n, int padded_rows, int k, int padded_cols) {
+        std::vector<int> a(padded_rows, -1), b(padded_cols, -1);
+        for (int i = 0; i < n; ++i) a[i] = i;
+        for (int i = 0; i < k; ++i) b[i] = i;
+        return upload(a, b);
+    }
+    // plain [N][K] linear
+    int linear(const std::string& name, int N, int K, Mat* mat) {
+        const mmi_tensor_desc* d;
+        int rc;
+        const int rows = round_up(N, 16), cols = round_up(K, m->kstep);
+        if ((rc = find(name, MMI_BF16, {N, K}, &d)) || (rc = alloc(mat, 1, rows / 16, cols / m->kstep)) || (rc = ident(N, rows, K, cols))) return rc;
+        return pack(d, mat->wp, rows, cols, K, 1);
+    }
+    int vec(const std::string& name, int n, int padded, float** out) {
+        const mmi_tensor_desc* d;
+        int rc = find(name, MMI_BF16, {n}, &d);
+        if (rc) return rc;
+        MMI_HIP_CHECK(m->wts.alloc(out, padded));
+        return vec_into(d, n, padded, *out);
+    }
+    int vec_into(const mmi_tensor_desc* d, int n, int padded, float* out) {
+        std::vector<int> a(padded, -1);
+        for (int i = 0; i < n; ++i) a[i] = i;
+        int rc = upload(a, {});
+        if (rc) return rc;
+        MMI_LAUNCH(k_tlm_vec, mmi_cdiv(padded, 256), 256, 0, (hipStream_t)0, (const uint16_t*)d->data, map, out, padded);
+        MMI_CHECK_LAUNCH();
+        return MMI_OK;
+    }
+};
+
+int load_mingru(Loader& ld, Layer& L, const std::string& p) {
+    mmi_tlm* m = ld.m;
+    const int w = L.c.width, D = m->cfg.width;
+    L.wp = round_up(w, 16);
+    const int cols = round_up(D, m->kstep);
+    int rc;
+    if ((rc = ld.alloc(&L.zcg, 1, 3 * L.wp / 16, cols / m->kstep)) || (rc = ld.ident(w, L.wp, D, cols))) return rc;
+    const char* parts[3] = {"z", "x", "g"};
+    const mmi_tensor_desc* d;
+    for (int k = 0; k < 3; ++k) {
+        if ((rc = ld.find(p + ".mix." + parts[k], MMI_BF16, {w, D}, &d))) return rc;
+        if ((rc = ld.pack(d, L.zcg.wp, L.wp, cols, D, 1, 3, k))) return rc;
+    }
+    MMI_HIP_CHECK(m->wts.alloc(&L.bias, (size_t)2 * L.wp));
+    for (int k = 0; k < 2; ++k) {
+        if ((rc = ld.find(p + ".mix." + parts[k] + ".b", MMI_BF16, {w}, &d)) || (rc = ld.vec_into(d, w, L.wp, L.bias + (size_t)k * L.wp))) return rc;
+    }
+    return ld.linear(p + ".mix.o", D, w, &L.out);
+}
+
+int load_latent_attention(Loader& ld, Layer& L, const std::string& p) {
+    mmi_tlm* m = ld.m;
+    const mmi_tlm_layer& c = L.c;
+    const int D = m->cfg.width, H = c.heads, ks = m->kstep, hd = c.dim + c.rot_dim;
+    L.qp = round_up(c.q_rank, 16);
+    L.kvp = round_up(c.kv_rank, 16);
+    L.rp = round_up(c.rot_dim, 16);
+    L.hp = round_up(H, 16);
+    L.dim_p = round_up(c.dim, ks);
+    L.vdim_p = round_up(c.vdim, 16);
+    L.lat_ks = round_up(c.kv_rank, ks) / ks;
+    L.k_ks = L.lat_ks + round_up(c.rot_dim, ks) / ks;
+    L.nd = L.kvp / 16;
+    L.q_ks = round_up(c.q_rank, ks) / ks;
+    auto turn = [&](int j) { return j / 2 + (j & 1) * (c.rot_dim / 2); };     // rotation partners side by side
+    const mmi_tensor_desc* d;
+    int rc;
+    const std::string mx = p + ".mix.";
+    // [query latent | latent | rotated key part | gates] of one input projection
+    const int cols = round_up(D, ks);
+    std::vector<int> cm(cols, -1);
+    for (int i = 0; i < D; ++i) cm[i] = i;
+    if ((rc = ld.alloc(&L.in, 1, (L.qp + L.kvp + L.rp + L.hp) / 16, cols / ks))) return rc;
+    if ((rc = ld.find(mx + "dq", MMI_BF16, {c.q_rank, D}, &d)) || (rc = ld.ident(c.q_rank, L.qp, D, cols)) || (rc = ld.pack(d, L.in.wp, L.qp, cols, D, 1))) return rc;
+    if ((rc = ld.find(mx + "dkv", MMI_BF16, {c.kv_rank + c.rot_dim, D}, &d)) || (rc = ld.ident(c.kv_rank, L.kvp, D, cols)) ||
+        (rc = ld.pack(d, L.in.wp, L.kvp, cols, D, 1, 1, L.qp / 16)))
+        return rc;
+    if (L.rp) {
+        std::vector<int> rm(L.rp, -1);
+        for (int j = 0; j < c.rot_dim; ++j) rm[j] = c.kv_rank + turn(j);
+        if ((rc = ld.upload(rm, cm)) || (rc = ld.pack(d, L.in.wp, L.rp, cols, D, 1, 1, (L.qp + L.kvp) / 16))) return rc;
+    }
+    if ((rc = ld.find(mx + "g", MMI_BF16, {H, D}, &d)) || (rc = ld.ident(H, L.hp, D, cols)) ||
+        (rc = ld.pack(d, L.in.wp, L.hp, cols, D, 1, 1, (L.qp + L.kvp + L.rp) / 16)))
+        return rc;
+    if ((rc = ld.vec(mx + "dq.norm", c.q_rank, L.qp, &L.qw)) || (rc = ld.vec(mx + "dkv.norm", c.kv_rank, L.kvp, &L.cw))) return rc;
+    // queries: un-rotated parts head by head, then rotated parts (one group per head)
+    if ((rc = ld.find(mx + "uq", MMI_BF16, {(int64_t)H * hd, c.q_rank}, &d))) return rc;
+    {
+        const int qc = L.q_ks * ks;
+        std::vector<int> rm((size_t)H * L.dim_p, -1), qm(qc, -1);
+        for (int i = 0; i < c.q_rank; ++i) qm[i] = i;
+        for (int h = 0; h < H; ++h)
+            for (int j = 0; j < c.dim; ++j) rm[(size_t)h * L.dim_p + j] = h * hd + j;
+        if ((rc = ld.alloc(&L.uqn, 1, (int)rm.size() / 16, L.q_ks)) || (rc = ld.upload(rm, qm)) || (rc = ld.pack(d, L.uqn.wp, (int)rm.size(), qc, c.q_rank, 1))) return rc;
+        if (L.rp) {
+            std::vector<int> rr((size_t)H * L.rp, -1);
+            for (int h = 0; h < H; ++h)
+                for (int j = 0; j < c.rot_dim; ++j) rr[(size_t)h * L.rp + j] = h * hd + c.dim + turn(j);
+            if ((rc = ld.alloc(&L.uqr, H, L.rp / 16, L.q_ks)) || (rc = ld.upload(rr, qm)) || (rc = ld.pack(d, L.uqr.wp, (int)rr.size(), qc, c.q_rank, 1))) return rc;
+        }
+    }
+    // key projection, transposed per head (it is applied to the query), and value projection per head
+    if ((rc = ld.find(mx + "uk", MMI_BF16, {(int64_t)H * c.dim, c.kv_rank}, &d)) || (rc = ld.alloc(&L.uk, H, L.kvp / 16, L.dim_p / ks)) ||
+        (rc = ld.ident(c.kv_rank, L.kvp, c.dim, L.dim_p)))
+        return rc;
+    for (int h = 0; h < H; ++h)
+        if ((rc = ld.pack(d, L.uk.wp + h * L.uk.gs, L.kvp, L.dim_p, 1, c.kv_rank, 1, 0, (long)h * c.dim * c.kv_rank))) return rc;
+    if ((rc = ld.find(mx + "uv", MMI_BF16, {(int64_t)H * c.vdim, c.kv_rank}, &d)) || (rc = ld.alloc(&L.uv, H, L.vdim_p / 16, L.lat_ks)) ||
+        (rc = ld.ident(c.vdim, L.vdim_p, c.kv_rank, L.lat_ks * ks)))
+        return rc;
+    for (int h = 0; h < H; ++h)
+        if ((rc = ld.pack(d, L.uv.wp + h * L.uv.gs, L.vdim_p, L.lat_ks * ks, c.kv_rank, 1, 1, 0, (long)h * c.vdim * c.kv_rank))) return rc;
+    // output projection over the padded heads
+    const int ok = round_up(H * L.vdim_p, ks), rows = round_up(D, 16);
+    std::vector<int> rm(rows, -1), om(ok, -1);
+    for (int i = 0; i < D; ++i) rm[i] = i;
+    for (int h = 0; h < H; ++h)
+        for (int j = 0; j < c.vdim; ++j) om[h * L.vdim_p + j] = h * c.vdim + j;
+    if ((rc = ld.find(mx + "o", MMI_BF16, {D, (int64_t)H * c.vdim}, &d)) || (rc = ld.alloc(&L.out, 1, rows / 16, ok / ks)) || (rc = ld.upload(rm, om))) return rc;
+    return ld.pack(d, L.out.wp, rows, ok, (long)H * c.vdim, 1);
+}
+
+int load_moe(Loader& ld, Layer& L, const std::string& p) {
+    mmi_tlm* m = ld.m;
+    const mmi_tlm_layer& c = L.c;
+    const int D = m->cfg.width, E = c.experts, rows_u = round_up(c.ff, 16), cols_u = round_up(D, m->kstep), rows_d = round_up(D, 16), cols_d = round_up(c.ff, m->kstep);
+    const mmi_tensor_desc* d;
+    int rc;
+    if ((rc = ld.alloc(&L.up, E, rows_u / 16, cols_u / m->kstep)) || (rc = ld.alloc(&L.down, E, rows_d / 16, cols_d / m->kstep))) return rc;
+    if ((rc = ld.ident(c.ff, rows_u, D, cols_u))) return rc;
+    for (int e = 0; e < E; ++e)
+        if ((rc = ld.find(p + ".mlp.e" + std::to_string(e) + ".up", MMI_BF16, {c.ff, D}, &d)) || (rc = ld.pack(d, L.up.wp + e * L.up.gs, rows_u, cols_u, D, 1))) return rc;
+    if ((rc = ld.ident(D, rows_d, c.ff, cols_d))) return rc;
+    for (int e = 0; e < E; ++e)
+        if ((rc = ld.find(p + ".mlp.e" + std::to_string(e) + ".down", MMI_BF16, {D, c.ff}, &d)) || (rc = ld.pack(d, L.down.wp + e * L.down.gs, rows_d, cols_d, c.ff, 1))) return rc;
+    if ((rc = ld.find(p + ".mlp.table", MMI_I32, {m->cfg.vocab, c.top}, &d))) return rc;
+    const size_t n = (size_t)m->cfg.vocab * c.top;
+    std::vector<int> t(n);
+    MMI_HIP_CHECK(hipMemcpy(t.data(), d->data, n * sizeof(int), hipMemcpyDeviceToHost));
+    for (size_t i = 0; i < n; ++i)
+        if (t[i] < 0 || t[i] >= E) return mmi_fail(MMI_ERR_INVALID, p + ".mlp.table names an expert that does not exist");
+    int* dev = nullptr;
+    MMI_HIP_CHECK(m->wts.alloc(&dev, n));
+    MMI_HIP_CHECK(hipMemcpy(dev, d->data, n * sizeof(int), hipMemcpyDeviceToDevice));
+    L.route = (int)m->route_host.size();
+    m->route_host.push_back(TlmRouteLayer{dev, E, c.top});
+    m->max_experts = std::max(m->max_experts, E);
+    m->max_top = std::max(m->max_top, c.top);
+    return MMI_OK;
+}
+
+int check_cfg(const mmi_tlm_cfg& c) {
+    if (c.vocab < 1 || c.width < 1 || c.n_layers < 1 || !c.layers) return mmi_fail(MMI_ERR_INVALID, "token LM: empty configuration");
+    if (c.dtype != MMI_BF16 && c.dtype != MMI_F32) return mmi_fail(MMI_ERR_UNSUPPORTED, "token LM: dtype must be bf16 or fp32");
+    if (c.norm_groups < 1 || c.width % c.norm_groups) return mmi_fail(MMI_ERR_INVALID, "token LM: width must be a multiple of the norm groups");
+    if (c.width > 8192) return mmi_fail(MMI_ERR_UNSUPPORTED, "token LM: width above 8192");
+    if (c.loop_start < 0 || c.loop_stop < c.loop_start || c.loop_stop > c.n_layers || (c.loop_stop > c.loop_start && c.loop_times < 1))
+        return mmi_fail(MMI_ERR_INVALID, "token LM: bad layer repetition");
+    for (int i = 0; i < c.n_layers; ++i) {
+        const mmi_tlm_layer& l = c.layers[i];
+        const std::string at = "token LM, layer " + std::to_string(i) + ": ";
+        if (l.mixer == MMI_TLM_MIX_MINGRU) {
+            if (l.width < 1) return mmi_fail(MMI_ERR_INVALID, at + "minGRU width");
+        } else if (l.mixer == MMI_TLM_MIX_LATENT_ATTENTION) {
+            if (l.heads < 1 || l.dim < 1 || l.vdim < 1 || l.q_rank < 1 || l.kv_rank < 1 || l.rot_dim < 0 || l.rot_dim % 2 || l.window < 0)
+                return mmi_fail(MMI_ERR_INVALID, at + "latent attention sizes");
+            if (l.kv_rank > 512) return mmi_fail(MMI_ERR_UNSUPPORTED, at + "kv_rank above 512");
+            if (l.rot_dim > 128) return mmi_fail(MMI_ERR_UNSUPPORTED, at + "rot_dim above 128");
+            if (round_up(l.q_rank, 16) + round_up(l.kv_rank, 16) + round_up(l.rot_dim, 16) + round_up(l.heads, 16) > 8192)
+                return mmi_fail(MMI_ERR_UNSUPPORTED, at + "query latent above the kernel's row buffer");
+        } else {
+            return mmi_fail(MMI_ERR_UNSUPPORTED, at + "unknown mixer");
+        }
+        if (l.mlp == MMI_TLM_MLP_MOE) {
+            if (l.experts < 1 || l.top < 1 || l.top > l.experts || l.ff < 1) return mmi_fail(MMI_ERR_INVALID, at + "expert sizes");
+            if (l.experts > 4096) return mmi_fail(MMI_ERR_UNSUPPORTED, at + "more than 4096 experts");
+            if (l.act != MMI_TLM_ACT_RELU2 || l.router != MMI_TLM_ROUTE_TOKEN_TABLE) return mmi_fail(MMI_ERR_UNSUPPORTED, at + "unknown expert activation or router");
+        } else if (l.mlp != MMI_TLM_MLP_NONE) {
+            return mmi_fail(MMI_ERR_UNSUPPORTED, at + "unknown feed-forward");
+        }
+    }
+    return MMI_OK;
+}
+
+// ------------------------------------------------------------------------------------------------
+// buffers
+// ------------------------------------------------------------------------------------------------
+int alloc_packed(mmi_tlm* m, void** p, long rows, int ks) {
+    const size_t n = (size_t)((rows + 15) / 16) * ks * 64;
+    u32x4* q = nullptr;
+    MMI_HIP_CHECK(m->scratch.alloc(&q, n));
+    MMI_HIP_CHECK(hipMemset(q, 0, n * 16));              // padding columns are read (times zero weights): keep them finite
+    *p = q;
+    return MMI_OK;
+}
+int alloc_f32(mmi_tlm* m, float** p, size_t n) {
+    MMI_HIP_CHECK(m->scratch.alloc(p, n));
+    MMI_HIP_CHECK(hipMemset(*p, 0, std::max<size_t>(n, 1) * sizeof(float)));
+    return MMI_OK;
+}
+
+int alloc_buffers(mmi_tlm* m) {
+    const mmi_tlm_cfg& c = m->cfg;
+    const int T = m->max_T, ks = m->kstep;
+    int rc;
+    m->split_elems = std::max((long)T, (long)MAX_SPLIT * ROWS_MAX);
+    int gru_w = 0, y_ks = 0, lat_ld = 0, cq_ks = 0, qn_ks = 0, o_ks = 0, hid_ks = 0, gate_ld = 0, nd = 0;
+    long q_elems = 0, ao_elems = 0;
+    for (const Layer& L : m->layers) {
+        if (L.c.mixer == MMI_TLM_MIX_MINGRU) {
+            gru_w = std::max(gru_w, L.wp);
+            y_ks = std::max(y_ks, L.out.KS);
+        } else {
+            lat_ld = std::max(lat_ld, L.qp + L.kvp + L.rp + L.hp);
+            cq_ks = std::max(cq_ks, L.q_ks);
+            qn_ks = std::max(qn_ks, L.c.heads * L.dim_p / ks);
+            q_elems = std::max(q_elems, (long)((T * (long)L.c.heads + 15) / 16) * L.k_ks);
+            ao_elems = std::max(ao_elems, (long)((T * (long)L.c.heads + 15) / 16) * L.lat_ks);
+            o_ks = std::max(o_ks, L.out.KS);
+            gate_ld = std::max(gate_ld, L.c.heads);
+            nd = std::max(nd, L.nd);
+        }
+        if (L.c.mlp == MMI_TLM_MLP_MOE) hid_ks = std::max(hid_ks, L.down.KS);
+    }
+    if ((rc = alloc_f32(m, &m->x, (size_t)T * m->ld)) || (rc = alloc_packed(m, &m->h, std::max(T, m->max_slots), m->h_ks)) ||
+        (rc = alloc_f32(m, &m->mix, (size_t)m->split_elems * m->ld)))
+        return rc;
+    if (m->has_gru) {
+        const int n_seg = T / TLM_SEG + m->max_slots + 1;
+        if ((rc = alloc_f32(m, &m->zcg, (size_t)T * 3 * gru_w)) || (rc = alloc_packed(m, &m->y, T, y_ks)) || (rc = alloc_f32(m, &m->pair, (size_t)n_seg * 2 * gru_w))) return rc;
+    }
+    if (m->has_attn) {
+        if ((rc = alloc_f32(m, &m->lat, (size_t)m->split_elems * lat_ld)) || (rc = alloc_packed(m, &m->cq, T, cq_ks)) || (rc = alloc_packed(m, &m->qn, T, qn_ks)) ||
+            (rc = alloc_packed(m, &m->q, q_elems * 16, 1)) || (rc = alloc_packed(m, &m->ao, ao_elems * 16, 1)) || (rc = alloc_packed(m, &m->o, T, o_ks)) ||
+            (rc = alloc_f32(m, &m->gate, (size_t)T * gate_ld)) || (rc = alloc_f32(m, &m->po, (size_t)MAX_PARTIALS * nd * 256)) ||
+            (rc = alloc_f32(m, &m->pml, (size_t)MAX_PARTIALS * 32)))
+            return rc;
+        for (TlmRope& r : m->rope_host)
+            if ((rc = alloc_f32(m, &r.out, (size_t)T * r.ld * 2))) return rc;
+    }
+    if (!m->route_host.empty()) {
+        const size_t nl = m->route_host.size();
+        m->list_ld = (long)T * m->max_top;
+        m->tile_ld = (long)T * m->max_top / 16 + m->max_experts + 1;
+        if ((rc = alloc_packed(m, &m->hid, (long)T * m->max_top, hid_ks)) ||
+            (rc = alloc_f32(m, &m->dn, (size_t)std::max((long)T, (long)MAX_SPLIT * ROWS_MAX) * m->max_top * m->ld)))
+            return rc;
+        MMI_HIP_CHECK(m->scratch.alloc(&m->list, nl * m->list_ld));
+        MMI_HIP_CHECK(m->scratch.alloc(&m->tiles, nl * m->tile_ld * 3));
+        MMI_HIP_CHECK(m->scratch.alloc(&m->n_tiles, nl));
+        MMI_HIP_CHECK(m->scratch.alloc(&m->route_dev, nl));
+        MMI_HIP_CHECK(hipMemcpy(m->route_dev, m->route_host.data(), nl * sizeof(TlmRouteLayer), hipMemcpyHostToDevice));
+    }
+    MMI_HIP_CHECK(m->scratch.alloc(&m->rope_dev, std::max<size_t>(1, m->rope_host.size())));
+    if (!m->rope_host.empty()) MMI_HIP_CHECK(hipMemcpy(m->rope_dev, m->rope_host.data(), m->rope_host.size() * sizeof(TlmRope), hipMemcpyHostToDevice));
+    MMI_HIP_CHECK(m->scratch.alloc(&m->tok, T));
+    MMI_HIP_CHECK(hipMemset(m->tok, 0, (size_t)T * sizeof(int)));
+    MMI_HIP_CHECK(m->scratch.alloc(&m->last_tok, m->max_slots));
+    MMI_HIP_CHECK(hipMemset(m->last_tok, 0, (size_t)m->max_slots * sizeof(int)));
+    MMI_HIP_CHECK(m->scratch.alloc(&m->block_table, (size_t)m->max_slots * std::max(1, m->max_pages) + 1));
+    MMI_HIP_CHECK(hipMemset(m->block_table, 0, ((size_t)m->max_slots * std::max(1, m->max_pages) + 1) * sizeof(int)));
+    if ((rc = alloc_f32(m, &m->logits, (size_t)m->max_slots * c.vocab))) return rc;
+    m->samp_ld = round_up(c.vocab, 8);
+    MMI_HIP_CHECK(m->scratch.alloc(&m->samp_rows, (size_t)m->max_slots * m->samp_ld));
+    MMI_HIP_CHECK(m->scratch.alloc(&m->samp_map, 4 * (size_t)m->max_slots));
+    MMI_HIP_CHECK(m->scratch.alloc(&m->samp_rng, 8));
+    MMI_HIP_CHECK(m->scratch.alloc(&m->samp_zero, 1));
+    MMI_HIP_CHECK(hipMemset(m->samp_zero, 0, sizeof(int)));
+    // metadata: 4 ints per token + wanted rows, per-entry arrays, tile prefixes, segments, block-table updates
+    m->meta_cap = 64 + (size_t)5 * T + 4 * (size_t)m->max_slots + m->geo.size() * ((size_t)m->max_slots + 1) + 8 * ((size_t)T / TLM_SEG + m->max_slots + 1) +
+                  2 * ((size_t)T / TLM_PAGE + 2 * (size_t)m->max_slots + 2);
+    MMI_HIP_CHECK(m->scratch.alloc(&m->meta, m->meta_cap));
+    for (Staging& s : m->staging) {
+        MMI_HIP_CHECK(hipHostMalloc((void**)&s.host, m->meta_cap * sizeof(int), 0));
+        MMI_HIP_CHECK(hipEventCreateWithFlags(&s.ev, hipEventDisableTiming));
+    }
+    return MMI_OK;
+}
+
+int alloc_state(mmi_tlm* m) {
+    for (Run& r : m->runs) {
+        const Layer& L = m->layers[r.layer];
+        if (L.c.mixer == MMI_TLM_MIX_MINGRU) {
+            const size_t n = (size_t)m->max_slots * 2 * L.wp;
+            MMI_HIP_CHECK(m->st.alloc(&r.state, n));
+            MMI_HIP_CHECK(hipMemset(r.state, 0, n * sizeof(float)));
+        } else {
+            const size_t nk = (size_t)m->max_pages * 4 * L.k_ks * 64, nv = (size_t)m->max_pages * L.nd * 16 * TLM_PAGE * m->esize / 16;
+            u32x4 *k = nullptr, *v = nullptr;
+            MMI_HIP_CHECK(m->st.alloc(&k, nk));
+            MMI_HIP_CHECK(m->st.alloc(&v, nv));
+            MMI_HIP_CHECK(hipMemset(k, 0, nk * 16));      // masked keys of a block are multiplied by zero weights: never-written rows must be finite
+            MMI_HIP_CHECK(hipMemset(v, 0, nv * 16));
+            r.kc = k;
+            r.vc = v;
+        }
+    }
+    return MMI_OK;
+}
+
+// ------------------------------------------------------------------------------------------------
+// launch list
+// ------------------------------------------------------------------------------------------------
+struct Plan { bool rows; int mt, fm; };      // weight-streaming kernel with mt row tiles, or the tiled kernel with 32 fm rows per block
+Plan plan_rows(int T) {
+    Plan p{T <= ROWS_MAX, 1, 2};
+    p.mt = T <= 16 ? 1 : (T <= 32 ? 2 : 4);
+    p.fm = T >= 1024 ? 4 : 2;
+    return p;
+}
+int plan_tile(const Plan& p) { return p.rows ? 16 * p.mt : 32 * p.fm; }
+
+TlmJob base_job(const Mat& w, const void* x, int xks) {
+    TlmJob j;
+    memset(&j, 0, sizeof(j));
+    j.wp = w.wp;
+    j.wgs = w.gs;
+    j.xp = (const u32x4*)x;
+    j.xks = xks;
+    j.KS = w.KS;
+    j.NT = w.NT;
+    j.groups = 1;
+    j.ksplit = 1;
+    j.in_mul = 1;
+    j.out_mul = 1;
+    j.scale = 1.f;
+    return j;
+}
+TlmJob dense_job(const Mat& w, const void* x, int xks, int rows) {
+    TlmJob j = base_job(w, x, xks);
+    j.rows = rows;
+    return j;
+}
+TlmJob routed_job(mmi_tlm* m, const Layer& L, const Mat& w, const void* x, int xks, int in_div, int T, const Plan& p) {
+    TlmJob j = base_job(w, x, xks);
+    j.list = m->list + (long)L.route * m->list_ld;
+    j.tiles = m->tiles + (long)L.route * m->tile_ld * 3;
+    j.n_tiles = m->n_tiles + L.route;
+    j.in_div = in_div;
+    const int pairs = T * L.c.top;
+    j.rblocks = std::min(pairs, std::min(L.c.experts, pairs) + pairs / plan_tile(p));      // every expert's run ends in at most one partial tile
+    return j;
+}
+// K split so that a product with few n-tiles still covers the chip; the consumer sums the fp32 partials
+int split_for(const Plan& p, const Mat& w, int blocks) {
+    if (!p.rows) return 1;
+    int s = 1;
+    while (s < MAX_SPLIT && blocks * s < 384 && w.KS / (2 * s) >= 8) s *= 2;
+    return s;
+}
+
+template <class Tr>
+int launch_jobs_t(hipStream_t s, const Plan& p, TlmJobs& J) {
+    long total = 0;
+    for (int i = 0; i < J.n; ++i) {
+        TlmJob& j = J.j[i];
+        if (!j.list) j.rblocks = mmi_cdiv(j.rows, plan_tile(p));
+        j.blocks = (p.rows ? j.NT : mmi_cdiv(j.NT, 2 * p.fm)) * (j.list ? 1 : j.groups) * j.ksplit * j.rblocks;
+        total += j.blocks;
+    }
+    const int grid = (int)total;
+    if (p.rows) {
+        if (p.mt == 1) MMI_LAUNCH((k_tlm_gemm_rows<Tr, 1, 8, 4>), grid, 512, 0, s, J);
+        else if (p.mt == 2) MMI_LAUNCH((k_tlm_gemm_rows<Tr, 2, 8, 2>), grid, 512, 0, s, J);
+        else MMI_LAUNCH((k_tlm_gemm_rows<Tr, 4, 8, 2>), grid, 512, 0, s, J);
+    } else {
+        if (p.fm == 4) MMI_LAUNCH((k_tlm_gemm_tile<Tr, 4, 4>), grid, 256, 0, s, J);
+        else MMI_LAUNCH((k_tlm_gemm_tile<Tr, 2, 2>), grid, 256, 0, s, J);
+    }
+    MMI_CHECK_LAUNCH();
+    return MMI_OK;
+}
+int launch_jobs(mmi_tlm* m, hipStream_t s, const Plan& p, TlmJobs J) {
+    return m->f32 ? launch_jobs_t<TlmF32>(s, p, J) : launch_jobs_t<TlmBf16>(s, p, J);
+}
+
+template <class Tr, int WK>
+int launch_attn_w(hipStream_t s, dim3 grid, const TlmAttnArgs& a) {
+    if (a.nd <= 4) MMI_LAUNCH((k_tlm_attn<Tr, 4, WK>), grid, 256, 0, s, a);
+    else if (a.nd <= 8) MMI_LAUNCH((k_tlm_attn<Tr, 8, WK>), grid, 256, 0, s, a);
+    else if (a.nd <= 16) MMI_LAUNCH((k_tlm_attn<Tr, 16, WK>), grid, 256, 0, s, a);
+    else MMI_LAUNCH((k_tlm_attn<Tr, 32, WK>), grid, 256, 0, s, a);
+    MMI_CHECK_LAUNCH();
+    return MMI_OK;
+}
+template <class Tr>
+int launch_attn_t(hipStream_t s, const TlmAttnArgs& a) {
+    int rc;
+    if (a.n_tiles >= 1024) {
+        if ((rc = launch_attn_w<Tr, 1>(s, dim3(mmi_cdiv(a.n_tiles, 4), 1), a))) return rc;
+    } else {
+        if ((rc = launch_attn_w<Tr, 4>(s, dim3(a.n_tiles, a.nsplit), a))) return rc;
+    }
+    if (a.nsplit > 1) {
+        MMI_LAUNCH((k_tlm_attn_combine<Tr>), a.n_tiles, 256, 0, s, a);
+        MMI_CHECK_LAUNCH();
+    }
+    return MMI_OK;
+}
+
+struct Carry {                    // what the next residual launch has to add
+    const float* mix = nullptr; int mix_p = 1; const float* ls1 = nullptr;
+    const float* dn = nullptr; int dn_p = 1, top = 1; const float* ls2 = nullptr;
+};
+
+void add_resid(mmi_tlm* m, MmiProgram& P, const Shape& sh, const Carry& c, int emb_mode, float* tap, const float* w, void* out, const int* rows, int n) {
+    TlmResidArgs a;
+    memset(&a, 0, sizeof(a));
+    a.x = m->x;
+    a.width = m->cfg.width;
+    a.ld = m->ld;
+    a.mix = c.mix;
+    a.mix_p = c.mix_p;
+    a.mix_ps = (long)sh.T * m->ld;
+    a.ls1 = c.ls1;
+    a.dn = c.dn;
+    a.dn_p = c.dn_p;
+    a.top = c.top;
+    a.dn_ps = (long)sh.T * c.top * m->ld;
+    a.ls2 = c.ls2;
+    a.emb = m->embed;
+    a.tok = m->tok;
+    a.emb_mode = emb_mode;
+    a.tap = tap;
+    a.w = w;
+    a.groups = m->cfg.norm_groups;
+    a.eps = m->cfg.norm_eps;
+    a.out = out;
+    a.KS = m->h_ks;
+    a.rows = rows;
+    const size_t smem = ((size_t)m->ld + 5 * (size_t)m->cfg.norm_groups + 8) * sizeof(float);
+    const bool f32 = m->f32;
+    P.add([=](hipStream_t s) {
+        if (f32) MMI_LAUNCH((k_tlm_resid_norm<TlmF32>), n, 256, smem, s, a);
+        else MMI_LAUNCH((k_tlm_resid_norm<TlmBf16>), n, 256, smem, s, a);
+        MMI_CHECK_LAUNCH();
+        return (int)MMI_OK;
+    });
+}
+void add_jobs(mmi_tlm* m, MmiProgram& P, const Plan& p, const TlmJobs& J, long bytes) {
+    P.add([=](hipStream_t s) { return launch_jobs(m, s, p, J); }, bytes);
+}
+
+// mixer cores: fill `first` with the product(s) that read the norm, queue everything up to the output projection's operand, and
+// return the output projection
+struct MixerOut { const Mat* w; const void* x; int xks; };
+
+MixerOut build_mingru(mmi_tlm* m, MmiProgram& P, const Shape& sh, const Layer& L, const Run& r, TlmJobs first, const Plan& p, const std::string& site) {
+    const int T = sh.T;
+    TlmJob j = dense_job(L.zcg, m->h, m->h_ks, T);
+    j.epi = TLM_EPI_GRU;
+    j.out = m->zcg;
+    j.out_ld = L.wp;
+    j.bias = L.bias;
+    first.j[first.n++] = j;
+    P.site(site + "in");
+    add_jobs(m, P, p, first, L.zcg.bytes());
+    TlmScanArgs a;
+    memset(&a, 0, sizeof(a));
+    a.zcg = m->zcg;
+    a.width = L.wp;
+    a.seg = (const TlmSeg*)(m->meta + sh.m.seg);
+    a.state = r.state;
+    a.pair = m->pair;
+    a.out = m->y;
+    a.out_ks = L.out.KS;
+    const bool f32 = m->f32, pairs = sh.pairs;
+    const int n_seg = sh.n_seg, block = L.wp >= 256 ? 256 : 64;
+    P.site(site + "scan");
+    P.add([=](hipStream_t s) {
+        const dim3 grid(mmi_cdiv(a.width, block), n_seg);
+        if (pairs) MMI_LAUNCH(k_tlm_scan_pairs, grid, block, 0, s, a);
+        if (f32) MMI_LAUNCH((k_tlm_scan<TlmF32>), grid, block, 0, s, a);
+        else MMI_LAUNCH((k_tlm_scan<TlmBf16>), grid, block, 0, s, a);
+        MMI_CHECK_LAUNCH();
+        return (int)MMI_OK;
+    });
+    return MixerOut{&L.out, m->y, L.out.KS};
+}
+
+MixerOut build_latent_attention(mmi_tlm* m, MmiProgram& P, const Shape& sh, const Layer& L, const Run& r, TlmJobs first, const Plan& p, const std::string& site) {
+    const int T = sh.T, H = L.c.heads;
+    const bool f32 = m->f32;
+    const int ld = L.qp + L.kvp + L.rp + L.hp;
+    TlmJob j = dense_job(L.in, m->h, m->h_ks, T);
+    j.epi = TLM_EPI_F32;
+    j.out = m->lat;
+    j.out_ld = ld;
+    j.out_ps = (long)T * ld;
+    j.ksplit = split_for(p, L.in, L.in.NT);
+    const int in_p = j.ksplit;
+    first.j[first.n++] = j;
+    P.site(site + "in");
+    add_jobs(m, P, p, first, L.in.bytes());
+
+    TlmLatentArgs a;
+    memset(&a, 0, sizeof(a));
+    a.in = m->lat;
+    a.in_p = in_p;
+    a.in_ps = (long)T * ld;
+    a.ld = ld;
+    a.q_rank = L.c.q_rank;
+    a.kv_rank = L.c.kv_rank;
+    a.rot = L.c.rot_dim;
+    a.heads = H;
+    a.qp = L.qp;
+    a.kvp = L.kvp;
+    a.rp = L.rp;
+    a.qw = L.qw;
+    a.cw = L.cw;
+    a.eps = m->cfg.norm_eps;
+    const float* rope = L.rope >= 0 ? m->rope_host[L.rope].out : nullptr;
+    const int rope_ld = L.rope >= 0 ? m->rope_host[L.rope].ld : 0;
+    a.rope = rope;
+    a.rope_ld = rope_ld;
+    a.crow = m->meta + sh.m.crow;
+    a.q = m->cq;
+    a.q_ks = L.q_ks;
+    a.kc = r.kc;
+    a.k_ks = L.k_ks;
+    a.rot_k0 = L.lat_ks * m->kstep;
+    a.vc = r.vc;
+    a.nd = L.nd;
+    a.gate = m->gate;
+    a.gate_ld = H;
+    P.site(site + "latent");
+    P.add([=](hipStream_t s) {
+        if (f32) MMI_LAUNCH((k_tlm_latent<TlmF32>), T, 256, (size_t)ld * sizeof(float), s, a);
+        else MMI_LAUNCH((k_tlm_latent<TlmBf16>), T, 256, (size_t)ld * sizeof(float), s, a);
+        MMI_CHECK_LAUNCH();
+        return (int)MMI_OK;
+    });
+
+    TlmJobs Q;
+    memset(&Q, 0, sizeof(Q));
+    TlmJob& jn = Q.j[Q.n++];
+    jn = dense_job(L.uqn, m->cq, L.q_ks, T);
+    jn.epi = TLM_EPI_PACK;
+    jn.out = m->qn;
+    const int qn_ks = H * L.dim_p / m->kstep;
+    jn.out_ld = qn_ks;
+    if (L.rp) {
+        TlmJob& jr = Q.j[Q.n++];
+        jr = dense_job(L.uqr, m->cq, L.q_ks, T);
+        jr.groups = H;
+        jr.epi = TLM_EPI_ROPE;
+        jr.out = m->q;
+        jr.out_ld = L.k_ks;
+        jr.out_mul = H;
+        jr.out_gadd = 1;
+        jr.out_k0 = L.lat_ks * m->kstep;
+        jr.rope = rope;
+        jr.rope_ld = rope_ld;
+    }
+    P.site(site + "q");
+    add_jobs(m, P, p, Q, L.uqn.bytes() + H * L.uqr.bytes());
+
+    memset(&Q, 0, sizeof(Q));
+    TlmJob& jk = Q.j[Q.n++];
+    jk = dense_job(L.uk, m->qn, qn_ks, T);
+    jk.groups = H;
+    jk.xkg = L.dim_p / m->kstep;
+    jk.epi = TLM_EPI_PACK;
+    jk.out = m->q;
+    jk.out_ld = L.k_ks;
+    jk.out_mul = H;
+    jk.out_gadd = 1;
+    P.site(site + "absorb");
+    add_jobs(m, P, p, Q, H * L.uk.bytes());
+
+    TlmAttnArgs t;
+    memset(&t, 0, sizeof(t));
+    t.q = m->q;
+    t.kc = r.kc;
+    t.vc = r.vc;
+    t.out = m->ao;
+    t.heads = H;
+    t.q_ks = L.k_ks;
+    t.nd = L.nd;
+    t.out_ks = L.lat_ks;
+    t.window = L.c.window;
+    t.scale = L.c.scale * 1.44269504088896340736f;
+    t.n_entries = sh.n_entries;
+    t.n_tiles = sh.tiles[L.geo];
+    t.nsplit = t.n_tiles >= 1024 ? 1 : std::max(1, std::min(sh.nsplit, MAX_PARTIALS / std::max(1, t.n_tiles)));
+    t.tile0 = m->meta + sh.m.tile0 + L.geo * (sh.n_entries + 1);
+    t.erow0 = m->meta + sh.m.erow0;
+    t.elen = m->meta + sh.m.elen;
+    t.epos0 = m->meta + sh.m.epos0;
+    t.eslot = m->meta + sh.m.eslot;
+    t.block_table = m->block_table;
+    t.bt_ld = std::max(1, m->max_pages);
+    t.po = m->po;
+    t.pml = m->pml;
+    P.site(site + "attn");
+    P.add([=](hipStream_t s) { return f32 ? launch_attn_t<TlmF32>(s, t) : launch_attn_t<TlmBf16>(s, t); });
+
+    memset(&Q, 0, sizeof(Q));
+    TlmJob& jv = Q.j[Q.n++];
+    jv = dense_job(L.uv, m->ao, L.lat_ks, T);
+    jv.groups = H;
+    jv.in_mul = H;
+    jv.in_gadd = 1;
+    jv.epi = TLM_EPI_PACK;
+    jv.out = m->o;
+    jv.out_ld = L.out.KS;
+    jv.out_kg = L.vdim_p;
+    jv.gate = m->gate;
+    jv.gate_ld = H;
+    P.site(site + "value");
+    add_jobs(m, P, p, Q, H * L.uv.bytes());
+    return MixerOut{&L.out, m->o, L.out.KS};
+}
+
+void build_program(mmi_tlm* m, MmiProgram& P, const Shape& sh) {
+    const int T = sh.T;
+    const Plan p = plan_rows(T);
+    TlmPrepArgs a;
+    memset(&a, 0, sizeof(a));
+    a.T = T;
+    a.n_ropes = (int)m->rope_host.size();
+    a.n_updates = m->meta;
+    a.htok = m->meta + sh.m.htok;
+    a.pos = m->meta + sh.m.pos;
+    a.rslot = m->meta + sh.m.rslot;
+    a.last_tok = m->last_tok;
+    a.tok = m->tok;
+    a.updates = m->meta + sh.m.upd;
+    a.block_table = m->block_table;
+    a.rope = m->rope_dev;
+    P.site("prepare");
+    P.add([=](hipStream_t s) {
+        MMI_LAUNCH(k_tlm_prepare, std::min(512, mmi_cdiv(T * 16, 256) + 1), 256, 0, s, a);
+        MMI_CHECK_LAUNCH();
+        return (int)MMI_OK;
+    });
+    if (!m->route_host.empty()) {
+        TlmRouteArgs ra;
+        memset(&ra, 0, sizeof(ra));
+        ra.layers = m->route_dev;
+        ra.tok = m->tok;
+        ra.T = T;
+        ra.tile = plan_tile(p);
+        ra.list = m->list;
+        ra.list_ld = m->list_ld;
+        ra.tiles = m->tiles;
+        ra.tile_ld = m->tile_ld;
+        ra.n_tiles = m->n_tiles;
+        const int nl = (int)m->route_host.size(), block = T * m->max_top <= 256 ? 256 : 1024;
+        const size_t smem = (size_t)2 * m->max_experts * sizeof(unsigned);
+        P.site("route");
+        P.add([=](hipStream_t s) {
+            MMI_LAUNCH(k_tlm_route, nl, block, smem, s, ra);
+            MMI_CHECK_LAUNCH();
+            return (int)MMI_OK;
+        });
+    }
+    Carry c;
+    const size_t tap_ld = (size_t)T * m->ld;
+    for (size_t i = 0; i < m->runs.size(); ++i) {
+        const Run& r = m->runs[i];
+        const Layer& L = m->layers[r.layer];
+        const std::string site = (L.c.mixer == MMI_TLM_MIX_MINGRU ? "gru." : "mla.");
+        P.site(site + "norm");
+        add_resid(m, P, sh, c, i == 0 ? TLM_EMB_SET : (r.add_emb ? TLM_EMB_ADD : TLM_EMB_NONE), sh.taps && i ? sh.taps + (i - 1) * tap_ld : nullptr, L.norm, m->h,
+                  nullptr, T);
+        const bool moe = L.c.mlp == MMI_TLM_MLP_MOE;
+        TlmJobs first;
+        memset(&first, 0, sizeof(first));
+        if (moe) {
+            TlmJob& j = first.j[first.n++];
+            j = routed_job(m, L, L.up, m->h, m->h_ks, L.c.top, T, p);
+            j.epi = TLM_EPI_PACK;
+            j.act = TLM_ACT_RELU2;
+            j.out = m->hid;
+            j.out_ld = L.down.KS;
+        }
+        const MixerOut mo = L.c.mixer == MMI_TLM_MIX_MINGRU ? build_mingru(m, P, sh, L, r, first, p, site) : build_latent_attention(m, P, sh, L, r, first, p, site);
+        TlmJobs J;
+        memset(&J, 0, sizeof(J));
+        c = Carry();
+        if (moe) {
+            TlmJob& j = J.j[J.n++];
+            j = routed_job(m, L, L.down, m->hid, L.down.KS, 1, T, p);
+            j.ksplit = split_for(p, L.down, j.NT * j.rblocks);
+            j.epi = TLM_EPI_F32;
+            j.out = m->dn;
+            j.out_ld = m->ld;
+            j.out_ps = (long)T * L.c.top * m->ld;
+            c.dn = m->dn;
+            c.dn_p = j.ksplit;
+            c.top = L.c.top;
+            c.ls2 = L.ls2;
+        }
+        TlmJob& j = J.j[J.n++];
+        j = dense_job(*mo.w, mo.x, mo.xks, T);
+        j.ksplit = split_for(p, *mo.w, j.NT);
+        j.epi = TLM_EPI_F32;
+        j.out = m->mix;
+        j.out_ld = m->ld;
+        j.out_ps = (long)T * m->ld;
+        c.mix = m->mix;
+        c.mix_p = j.ksplit;
+        c.ls1 = L.ls1;
+        P.site(site + "out");
+        add_jobs(m, P, p, J, mo.w->bytes());
+    }
+    if (sh.taps) {
+        P.site("taps");
+        add_resid(m, P, sh, c, TLM_EMB_NONE, sh.taps + (m->runs.size() - 1) * tap_ld, nullptr, nullptr, nullptr, T);
+        c = Carry();                                                     // (the residual has been written back)
+    }
+    if (sh.n_want > 0) {
+        P.site("final_norm");
+        add_resid(m, P, sh, c, TLM_EMB_NONE, nullptr, m->final_norm, m->h, m->meta + sh.m.want, sh.n_want);
+        const Plan hp = plan_rows(sh.n_want);
+        TlmJobs J;
+        memset(&J, 0, sizeof(J));
+        TlmJob& j = J.j[J.n++];
+        j = dense_job(m->head, m->h, m->h_ks, sh.n_want);
+        j.epi = TLM_EPI_LOGITS;
+        j.out = sh.logits;
+        j.out_ld = m->cfg.vocab;
+        j.n_valid = m->cfg.vocab;
+        j.scale = m->cfg.logit_scale;
+        P.site("head");
+        add_jobs(m, P, hp, J, m->head.bytes());
+    }
+}
+
+// ------------------------------------------------------------------------------------------------
+// cache manager
+// ------------------------------------------------------------------------------------------------
+int64_t pages_for(const mmi_tlm* m, const Slot* s, int64_t n) {
+    if (!m->has_attn) return 0;
+    const int64_t pos = s ? s->pos : 0;
+    const int64_t have = s ? s->first_page + (int64_t)s->pages.size() : 0;
+    return std::max<int64_t>(0, (pos + n + TLM_PAGE - 1) / TLM_PAGE - have);
+}
+void release_behind_window(mmi_tlm* m, Slot& s) {
+    if (!m->has_attn || m->max_window <= 0) return;
+    const int64_t first_seen = s.pos - m->max_window + 1;               // the oldest position the next token can see
+    while (!s.pages.empty() && (s.first_page + 1) * TLM_PAGE <= first_seen) {
+        m->free_pages.push_back(s.pages.front());
+        s.pages.erase(s.pages.begin());
+        ++s.first_page;
+    }
+}
+void release_slot(mmi_tlm* m, Slot& s) {
+    for (int p : s.pages) m->free_pages.push_back(p);
+    s = Slot();
+}
+
+void destroy(mmi_tlm* m) {
+    hipDeviceSynchronize();
+    for (auto& p : m->progs) p.second->clear();
+    for (Staging& s : m->staging) {
+        if (s.host) hipHostFree(s.host);
+        if (s.ev) hipEventDestroy(s.ev);
+    }
+    if (m->cap_stream) hipStreamDestroy(m->cap_stream);
+    m->wts.release();
+    m->st.release();
+    m->scratch.release();
+    delete m;
+}
+
+int create_impl(mmi_tlm* m, const mmi_tensor_desc* weights, int n_weights) {
+    const mmi_tlm_cfg& c = m->cfg;
+    MMI_HIP_CHECK(hipGetDevice(&m->device));
+    m->f32 = c.dtype == MMI_F32;
+    m->kstep = m->f32 ? TlmF32::KSTEP : TlmBf16::KSTEP;
+    m->V = m->f32 ? TlmF32::V : TlmBf16::V;
+    m->esize = m->f32 ? 4 : 2;
+    m->ld = round_up(c.width, 16);
+    m->h_ks = round_up(c.width, m->kstep) / m->kstep;
+    Loader ld;
+    ld.m = m;
+    ld.W = MmiWeights{weights, n_weights};
+    const mmi_tensor_desc* d;
+    int rc;
+    if ((rc = ld.find("embed", MMI_BF16, {c.vocab, c.width}, &d))) return rc;
+    MMI_HIP_CHECK(m->wts.alloc(&m->embed, (size_t)c.vocab * c.width));
+    MMI_HIP_CHECK(hipMemcpy(m->embed, d->data, (size_t)c.vocab * c.width * 2, hipMemcpyDeviceToDevice));
+    if ((rc = ld.vec("final.norm", c.width, m->ld, &m->final_norm)) || (rc = ld.linear("head", c.vocab, c.width, &m->head))) return rc;
+    bool unlimited = false;
+    for (int i = 0; i < c.n_layers; ++i) {
+        m->layers.emplace_back();
+        Layer& L = m->layers.back();
+        L.c = c.layers[i];
+        const std::string p = "l" + std::to_string(i);
+        if ((rc = ld.vec(p + ".norm1", c.width, m->ld, &L.norm)) || (rc = ld.vec(p + ".ls1", c.width, m->ld, &L.ls1))) return rc;
+        if (L.c.mixer == MMI_TLM_MIX_MINGRU) {
+            m->has_gru = true;
+            if ((rc = load_mingru(ld, L, p))) return rc;
+        } else {
+            m->has_attn = true;
+            if (L.c.window <= 0) unlimited = true;
+            m->max_window = std::max<int64_t>(m->max_window, L.c.window);
+            if ((rc = load_latent_attention(ld, L, p))) return rc;
+            L.geo = (int)(std::find(m->geo.begin(), m->geo.end(), L.c.heads) - m->geo.begin());
+            if (L.geo == (int)m->geo.size()) m->geo.push_back(L.c.heads);
+            if (L.c.rot_dim > 0) {
+                const std::pair<double, int> key(L.c.rot_base, L.c.rot_dim);
+                L.rope = (int)(std::find(m->ropes.begin(), m->ropes.end(), key) - m->ropes.begin());
+                if (L.rope == (int)m->ropes.size()) {
+                    m->ropes.push_back(key);
+                    const int half = L.c.rot_dim / 2;
+                    std::vector<float> f(half);
+                    for (int k = 0; k < half; ++k) f[k] = (float)pow(L.c.rot_base, -2.0 * k / L.c.rot_dim);
+                    float* dev = nullptr;
+                    MMI_HIP_CHECK(m->wts.alloc(&dev, half));
+                    MMI_HIP_CHECK(hipMemcpy(dev, f.data(), half * sizeof(float), hipMemcpyHostToDevice));
+                    m->rope_host.push_back(TlmRope{dev, half, L.rp / 2, nullptr});
+                }
+            }
+        }
+        if (L.c.mlp == MMI_TLM_MLP_MOE) {
+            if ((rc = ld.vec(p + ".ls2", c.width, m->ld, &L.ls2)) || (rc = load_moe(ld, L, p))) return rc;
+        }
+    }
+    if (unlimited) m->max_window = 0;
+    const int times = c.loop_stop > c.loop_start ? c.loop_times : 1;
+    const int start = c.loop_stop > c.loop_start ? c.loop_start : c.n_layers, stop = c.loop_stop > c.loop_start ? c.loop_stop : c.n_layers;
+    auto run = [&](int layer, bool add) {
+        Run r;
+        r.layer = layer;
+        r.add_emb = add;
+        m->runs.push_back(r);
+    };
+    for (int i = 0; i < start; ++i) run(i, false);
+    for (int t = 0; t < times; ++t)
+        for (int i = start; i < stop; ++i) run(i, t > 0 && i == start);
+    for (int i = stop; i < c.n_layers; ++i) run(i, false);
+    m->slots.resize(m->max_slots);
+    for (int i = m->max_pages - 1; i >= 0; --i) m->free_pages.push_back(i);
+    if ((rc = alloc_state(m)) || (rc = alloc_buffers(m))) return rc;
+    m->graphs = mmi_graphs_enabled();
+    if (m->graphs) MMI_HIP_CHECK(hipStreamCreateWithFlags(&m->cap_stream, hipStreamNonBlocking));
+    MMI_HIP_CHECK(hipDeviceSynchronize());
+    return MMI_OK;
+}
+
+}  // namespace
+
+extern "C" int mmi_tlm_create(const mmi_tlm_cfg* cfg, const mmi_tensor_desc* weights, int32_t n_weights, int32_t max_slots, int64_t max_tokens,
+                              int32_t max_step_tokens, mmi_tlm** out) {
+    if (!cfg || !weights || !out || max_slots < 1 || max_slots > 4096 || max_tokens < 1 || max_step_tokens < 1)
+        return mmi_fail(MMI_ERR_INVALID, "mmi_tlm_create: bad arguments");
+    int rc = check_cfg(*cfg);
+    if (rc) return rc;
+    mmi_tlm* m = new mmi_tlm();
+    m->cfg = *cfg;
+    m->max_slots = max_slots;
+    m->max_pages = (int)mmi_cdiv64(max_tokens, TLM_PAGE);
+    m->max_T = max_step_tokens;
+    rc = create_impl(m, weights, n_weights);
+    m->cfg.layers = nullptr;                         // the caller's array; the engine keeps its own copies
+    if (rc) {
+        destroy(m);
+        return rc;
+    }
+    *out = m;
+    return MMI_OK;
+}
+
+extern "C" void mmi_tlm_destroy(mmi_tlm* m) {
+    if (!m) return;
+    MmiDeviceGuard g(m->device);
+    destroy(m);
+}
+
+extern "C" int mmi_tlm_open(mmi_tlm* m, int32_t* slot) {
+    if (!m || !slot) return mmi_fail(MMI_ERR_INVALID, "mmi_tlm_open: null argument");
+    for (size_t i = 0; i < m->slots.size(); ++i)
+        if (!m->slots[i].live) {
+            m->slots[i] = Slot();
+            m->slots[i].live = true;
+            *slot = (int32_t)i;
+            return MMI_OK;
+        }
+    return mmi_fail(MMI_ERR_BUSY, "every sequence slot is taken");
+}
+
+extern "C" int mmi_tlm_close(mmi_tlm* m, int32_t slot) {
+    if (!m || slot < 0 || slot >= m->max_slots || !m->slots[slot].live) return mmi_fail(MMI_ERR_NO_CHANNEL, "no open sequence in this slot");
+    release_slot(m, m->slots[slot]);
+    return MMI_OK;
+}
+
+extern "C" int64_t mmi_tlm_pages_needed(const mmi_tlm* m, int32_t slot, int64_t n) {
+    if (!m || slot >= m->max_slots) return -1;
+    return pages_for(m, slot < 0 ? nullptr : &m->slots[slot], n);
+}
+
+extern "C" int64_t mmi_tlm_info(const mmi_tlm* m, int32_t which, int32_t slot) {
+    if (!m) return -1;
+    const bool ok = slot >= 0 && slot < m->max_slots && m->slots[slot].live;
+    switch (which) {
+        case MMI_TLM_PAGE_TOKENS: return TLM_PAGE;
+        case MMI_TLM_TOTAL_PAGES: return m->max_pages;
+        case MMI_TLM_FREE_PAGES: return (int64_t)m->free_pages.size();
+        case MMI_TLM_FREE_SLOTS: {
+            int64_t n = 0;
+            for (const Slot& s : m->slots) n += !s.live;
+            return n;
+        }
+        case MMI_TLM_POSITION: return ok ? m->slots[slot].pos : -1;
+        case MMI_TLM_HELD_PAGES: return ok ? (int64_t)m->slots[slot].pages.size() : -1;
+        case MMI_TLM_WEIGHT_BYTES: return m->weight_bytes;
+        case MMI_TLM_LAYER_RUNS: return (int64_t)m->runs.size();
+        case MMI_TLM_GRAPHS: return (int64_t)m->progs.size();
+    }
+    return -1;
+}
+
+extern "C" int mmi_tlm_set_taps(mmi_tlm* m, float* taps) {
+    if (!m) return mmi_fail(MMI_ERR_INVALID, "mmi_tlm_set_taps: null handle");
+    if (taps && m->cfg.width != m->ld) return mmi_fail(MMI_ERR_UNSUPPORTED, "taps need a width that is a multiple of 16");
+    m->taps = taps;
+    return MMI_OK;
+}
+
+extern "C" int64_t mmi_tlm_launch_list(const mmi_tlm* m, char* buf, int64_t cap) { return m ? mmi_copy_launch_log(m->last_log, buf, cap) : -1; }
+
+extern "C" int mmi_tlm_step(mmi_tlm* m, int32_t n_entries, const int32_t* slots, const int32_t* counts, const int32_t* tokens, int32_t n_want,
+                            const int32_t* want, float* logits, mmi_stream stream) {
+    if (!m || n_entries < 0 || n_want < 0 || (n_entries && (!slots || !counts || !tokens)) || (n_want && (!want || !logits)))
+        return mmi_fail(MMI_ERR_INVALID, "mmi_tlm_step: bad arguments");
+    if (n_entries == 0) return MMI_OK;
+    MmiDeviceGuard guard(m->device);
+    hipStream_t s = (hipStream_t)stream;
+    // ---- validate, nothing changed yet
+    if (n_entries > m->max_slots) return mmi_fail(MMI_ERR_SHAPE, "more entries than slots");
+    std::vector<char> seen(m->max_slots, 0);
+    int64_t T64 = 0, need = 0;
+    for (int e = 0; e < n_entries; ++e) {
+        if (slots[e] < 0 || slots[e] >= m->max_slots || !m->slots[slots[e]].live) return mmi_fail(MMI_ERR_NO_CHANNEL, "no open sequence in this slot");
+        if (seen[slots[e]]++) return mmi_fail(MMI_ERR_INVALID, "a slot appears twice in one step");
+        if (counts[e] < 1) return mmi_fail(MMI_ERR_INVALID, "an entry brings no token");
+        T64 += counts[e];
+        if (m->slots[slots[e]].pos + counts[e] > (int64_t)1 << 24) return mmi_fail(MMI_ERR_SHAPE, "position above 2^24");
+        need += pages_for(m, &m->slots[slots[e]], counts[e]);
+    }
+    if (T64 > m->max_T) return mmi_fail(MMI_ERR_SHAPE, "the step brings more tokens than max_step_tokens");
+    const int T = (int)T64;
+    for (int i = 0; i < T; ++i)
+        if (tokens[i] < -1 || tokens[i] >= m->cfg.vocab) return mmi_fail(MMI_ERR_INVALID, "token outside the vocabulary");
+    for (int i = 0; i < n_want; ++i)
+        if (want[i] < 0 || want[i] >= T || (i && want[i] <= want[i - 1])) return mmi_fail(MMI_ERR_INVALID, "wanted rows must ascend within the step");
+    if (need > (int64_t)m->free_pages.size()) return mmi_fail(MMI_ERR_BUSY, "the cache pool has too few free pages");
+
+    // ---- metadata block
+    Shape sh;
+    sh.T = T;
+    sh.n_want = n_want;
+    sh.n_entries = n_entries;
+    for (int e = 0; e < n_entries; ++e) {
+        const int n = mmi_cdiv(counts[e], TLM_SEG);
+        sh.n_seg += n;
+        sh.pairs |= n > 1;
+    }
+    Meta& M = sh.m;
+    int at = 16;
+    auto take = [&](int n) {
+        const int o = at;
+        at += round_up(n, 4);
+        return o;
+    };
+    M.htok = take(T);
+    M.pos = take(T);
+    M.rslot = take(T);
+    M.crow = take(T);
+    M.want = take(n_want);
+    M.erow0 = take(n_entries);
+    M.elen = take(n_entries);
+    M.epos0 = take(n_entries);
+    M.eslot = take(n_entries);
+    M.tile0 = take((int)m->geo.size() * (n_entries + 1));
+    M.seg = take(8 * sh.n_seg);
+    M.upd = at;
+    M.total = at + 2 * (int)need;
+    if ((size_t)M.total > m->meta_cap) return mmi_fail(MMI_ERR_SHAPE, "step metadata above its buffer");
+    Staging& st = m->staging[m->stage_at];
+    m->stage_at = (m->stage_at + 1) & 3;
+    if (st.used) MMI_HIP_CHECK(hipEventSynchronize(st.ev));
+    int* b = st.host;
+    memset(b, 0, 16 * sizeof(int));
+    int upd = 0, row = 0, seg = 0;
+    int64_t blocks = 0;
+    TlmSeg* sg = (TlmSeg*)(b + M.seg);
+    sh.tiles.assign(m->geo.size(), 0);
+    for (int e = 0; e < n_entries; ++e) {
+        Slot& S = m->slots[slots[e]];
+        for (int64_t n = pages_for(m, &S, counts[e]); n > 0; --n) {
+            const int page = m->free_pages.back();
+            m->free_pages.pop_back();
+            const int64_t idx = (int64_t)slots[e] * m->max_pages + (S.first_page + (int64_t)S.pages.size()) % m->max_pages;
+            S.pages.push_back(page);
+            b[M.upd + 2 * upd] = (int)idx;
+            b[M.upd + 2 * upd + 1] = page;
+            ++upd;
+        }
+        b[M.erow0 + e] = row;
+        b[M.elen + e] = counts[e];
+        b[M.epos0 + e] = (int)S.pos;
+        b[M.eslot + e] = slots[e];
+        for (size_t g = 0; g < m->geo.size(); ++g) {
+            b[M.tile0 + (int)g * (n_entries + 1) + e] = sh.tiles[g];
+            sh.tiles[g] += mmi_cdiv(counts[e] * m->geo[g], 16);
+        }
+        for (int o = 0, k = 0; o < counts[e]; o += TLM_SEG, ++k) {
+            const int n = std::min(TLM_SEG, counts[e] - o);
+            sg[seg++] = TlmSeg{row + o, n, slots[e], S.par, k, o + n == counts[e] ? 1 : 0, S.pos == 0 ? 1 : 0, 0};
+        }
+        for (int i = 0; i < counts[e]; ++i, ++row) {
+            const int64_t pos = S.pos + i;
+            b[M.htok + row] = tokens[row];
+            b[M.pos + row] = (int)pos;
+            b[M.rslot + row] = slots[e];
+            b[M.crow + row] = m->has_attn ? S.pages[pos / TLM_PAGE - S.first_page] * TLM_PAGE + (int)(pos % TLM_PAGE) : 0;
+        }
+        int64_t span = S.pos + counts[e];
+        if (m->max_window > 0) span = std::min<int64_t>(span, m->max_window + counts[e]);
+        blocks = std::max(blocks, span / 32 + 1);
+        S.pos += counts[e];
+        S.par ^= 1;
+    }
+    for (size_t g = 0; g < m->geo.size(); ++g) b[M.tile0 + (int)g * (n_entries + 1) + n_entries] = sh.tiles[g];
+    for (int i = 0; i < n_want; ++i) b[M.want + i] = want[i];
+    b[0] = upd;
+    // few column tiles and long contexts: split the keys over workgroups, at least 8 blocks of 32 keys each
+    int tiles_max = 1;
+    for (int t : sh.tiles) tiles_max = std::max(tiles_max, t);
+    while (sh.nsplit < 64 && tiles_max * sh.nsplit * 2 <= MAX_PARTIALS && blocks / (sh.nsplit * 2) >= 8) sh.nsplit *= 2;
+    MMI_HIP_CHECK(hipMemcpyAsync(m->meta, b, (size_t)M.total * sizeof(int), hipMemcpyHostToDevice, s));
+    MMI_HIP_CHECK(hipEventRecord(st.ev, s));
+    st.used = true;
+
+    // ---- launches
+    int rc = MMI_OK;
+    sh.taps = m->taps;
+    const bool decode = T == n_entries && T <= ROWS_MAX && !m->taps;
+    if (decode) {
+        sh.logits = m->logits;
+        auto& prog = m->progs[std::make_tuple(T, n_want, sh.nsplit)];
+        if (!prog) {
+            prog.reset(new MmiProgram());
+            build_program(m, *prog, sh);
+        }
+        rc = prog->run(s, m->graphs, m->cap_stream);
+        m->last_log = prog->launch_log();
+        if (!rc && n_want && logits != m->logits)
+            MMI_HIP_CHECK(hipMemcpyAsync(logits, m->logits, (size_t)n_want * m->cfg.vocab * sizeof(float), hipMemcpyDeviceToDevice, s));
+    } else {
+        sh.logits = logits;
+        MmiProgram P;
+        build_program(m, P, sh);
+        rc = P.run_eager(s);
+        m->last_log = P.launch_log();
+    }
+    for (int e = 0; e < n_entries; ++e) release_behind_window(m, m->slots[slots[e]]);
+    return rc;
+}
+
+extern "C" int mmi_tlm_sample(mmi_tlm* m, int32_t n, const float* logits, const int32_t* slots, const float* temp, const int32_t* top_k, uint64_t seed,
+                              int32_t* out, mmi_stream stream) {
+    if (!m || n < 1 || n > m->max_slots || !logits || !slots || !temp || !top_k || !out) return mmi_fail(MMI_ERR_INVALID, "mmi_tlm_sample: bad arguments");
+    MmiDeviceGuard guard(m->device);
+    hipStream_t s = (hipStream_t)stream;
+    const int V = m->cfg.vocab;
+    for (int i = 0; i < n; ++i) {
+        if (slots[i] < 0 || slots[i] >= m->max_slots) return mmi_fail(MMI_ERR_INVALID, "slot out of range");
+        if (temp[i] > 0.f && m->samp_ld > 32768) return mmi_fail(MMI_ERR_UNSUPPORTED, "sampling needs a vocabulary of at most 32768 entries (greedy does not)");
+    }
+    Staging& st = m->staging[m->stage_at];
+    m->stage_at = (m->stage_at + 1) & 3;
+    if (st.used) MMI_HIP_CHECK(hipEventSynchronize(st.ev));
+    memcpy(st.host, slots, (size_t)n * sizeof(int));
+    unsigned long long rng[2] = {seed, m->samp_count++};
+    memcpy(st.host + round_up(n, 2), rng, sizeof(rng));
+    MMI_HIP_CHECK(hipMemcpyAsync(m->samp_map, st.host, (size_t)n * sizeof(int), hipMemcpyHostToDevice, s));
+    MMI_HIP_CHECK(hipMemcpyAsync(m->samp_rng, st.host + round_up(n, 2), sizeof(rng), hipMemcpyHostToDevice, s));
+    MMI_HIP_CHECK(hipEventRecord(st.ev, s));
+    st.used = true;
+    for (int i = 0; i < n;) {                        // runs of rows with the same parameters
+        int k = i + 1;
+        while (k < n && (temp[i] <= 0.f ? temp[k] <= 0.f : (temp[k] == temp[i] && top_k[k] == top_k[i]))) ++k;
+        const int rows = k - i;
+        if (temp[i] <= 0.f) {
+            MMI_LAUNCH(k_tlm_argmax, rows, 256, 0, s, logits + (size_t)i * V, V, m->samp_map + i, out + i, m->last_tok);
+        } else {
+            const int ld = m->samp_ld;
+            uint16_t* r = m->samp_rows + (size_t)i * ld;
+            MMI_LAUNCH(k_tlm_sample_rows, (int)mmi_cdiv64((int64_t)rows * ld, 256), 256, 0, s, logits + (size_t)i * V, V, r, ld, rows);
+            SampleArgs a;
+            memset(&a, 0, sizeof(a));
+            a.logits = r;
+            a.ld = ld;
+            a.V = ld;
+            a.k = top_k[i] >= V || top_k[i] < 0 ? 0 : top_k[i];
+            a.temp = temp[i];
+            a.use_sampling = 1;
+            a.use_noise = m->samp_zero;
+            a.rng = m->samp_rng;
+            a.site = i;
+            a.out = out + i;
+            a.out_stride = 1;
+            a.B = rows;
+            a.use_forced = m->samp_zero;
+            if (ld <= 2048) MMI_LAUNCH((k_sample<256, 8, true>), rows, 256, 0, s, a);
+            else if (ld <= 8192) MMI_LAUNCH((k_sample<1024, 8, true>), rows, 1024, 0, s, a);
+            else MMI_LAUNCH((k_sample<1024, 32, true>), rows, 1024, 0, s, a);
+            MMI_LAUNCH(k_tlm_last_tok, mmi_cdiv(rows, 64), 64, 0, s, out + i, m->samp_map + i, m->last_tok, rows);
+        }
+        MMI_CHECK_LAUNCH();
+        i = k;
+    }
+    return MMI_OK;
+}

@@ -1,0 +1,894 @@
+// Kernels of the token language models (tlm_engine.hip): decoder-only networks over token ids whose layers are described by data
+// (mmi_tlm_cfg), served from a paged cache and per-sequence recurrent state, any mixture of prompt portions and single tokens per step.
+//
+// Every kernel is written once for two number formats: TlmBf16 (bf16 operands on v_mfma_f32_16x16x32_bf16, fp32 accumulation) and
+// TlmF32 (fp32 operands on v_mfma_f32_16x16x4_f32, an exact fma chain).  Positions, angles, attention scores and weights, norms, the
+// residual stream, gates and recurrent state are fp32 in both.
+//
+// Data layout in HBM
+//   fragment     64 lanes x 16 bytes: 16 rows x KSTEP reduction indices (bf16: 32, fp32: 16); lane (i, kq) = 16 kq + i holds row i,
+//                k = V kq .. V kq + V - 1 (V = 8 bf16 / 4 fp32).  It is the A operand (row = output feature), the B operand (row = token)
+//                and, at fp32, four 16x16x4 steps at once: element e of every lane is one step (any k order serves, both operands use it).
+//   weights      Wp[n-tile][k-step][lane][V]            (16-row tiles, zero padded; the layout of the Moshi LM's 16-row tile)
+//   activations  Xp[row / 16][k-step][lane][V]          (tlm_index; written by the producing epilogue)
+//   key cache    the same matrix with row = 64 page + offset: k = latent, then the rotated key part
+//   value cache  Vp[page][latent / 16][key group][lane][V]: the transposed operand.  Lane (d, kq), element e of a group of 4 V keys is
+//                key 16 (e / 4) + 4 kq + e % 4 - exactly the keys whose scores the same lane holds after S = K Q^T, so the softmax
+//                weights go from accumulator to operand without leaving the lane.
+//   residual     x[token][ld] fp32
+#pragma once
+#include "mmi_common.h"
+
+struct TlmBf16 {
+    typedef uint16_t elem;
+    static constexpr int V = 8, KSTEP = 32;
+    static __device__ __forceinline__ f32x4 mfma(u32x4 a, u32x4 b, f32x4 c) { return mmi_mfma_bf16_16x16x32(a, b, c); }
+    static __device__ __forceinline__ uint16_t cvt(float v) { return mmi_f32_to_bf16(v); }
+    static __device__ __forceinline__ void store4(uint16_t* p, f32x4 v) {
+        u32x2 o = {mmi_pack_bf16x2(v[0], v[1]), mmi_pack_bf16x2(v[2], v[3])};
+        *reinterpret_cast<u32x2*>(p) = o;
+    }
+};
+struct TlmF32 {
+    typedef float elem;
+    static constexpr int V = 4, KSTEP = 16;
+    static __device__ __forceinline__ f32x4 mfma(u32x4 a, u32x4 b, f32x4 c) {
+        const f32x4 fa = __builtin_bit_cast(f32x4, a), fb = __builtin_bit_cast(f32x4, b);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) c = mmi_mfma_f32_16x16x4(fa[e], fb[e], c);
+        return c;
+    }
+    static __device__ __forceinline__ float cvt(float v) { return v; }
+    static __device__ __forceinline__ void store4(float* p, f32x4 v) { *reinterpret_cast<f32x4*>(p) = v; }
+};
+
+// element (row, k) of a fragment-packed matrix with `ks` k-steps per row tile
+template <class Tr>
+MMI_HD long tlm_index(long row, int k, int ks) {
+    return (((row >> 4) * ks + k / Tr::KSTEP) * 64 + ((k % Tr::KSTEP) / Tr::V) * 16 + (row & 15)) * Tr::V + k % Tr::V;
+}
+
+constexpr int TLM_PAGE = 64;         // tokens per cache page
+
+// element of the value cache: latent dimension d of the token at `off` of a page (nd = 16-wide blocks of the latent)
+template <class Tr>
+MMI_HD long tlm_vindex(long page, int off, int d, int nd) {
+    constexpr int GK = 4 * Tr::V;                       // keys of one fragment
+    const int w = off % GK;
+    return (((page * nd + (d >> 4)) * (TLM_PAGE / GK) + off / GK) * 64 + ((w & 15) >> 2) * 16 + (d & 15)) * Tr::V + (w >> 4) * 4 + (w & 3);
+}
+
+__device__ __forceinline__ float tlm_sigmoid(float x) { return 1.0f / (1.0f + expf(-x)); }
+__device__ __forceinline__ float tlm_wave_sum(float x) {
+    x = mmi_group_sum<16>(x);
+    x += mmi_shfl_xor(x, 16);
+    x += mmi_shfl_xor(x, 32);
+    return x;
+}
+
+// ------------------------------------------------------------------------------------------------
+// weight import: bf16 checkpoint tensor -> fragments, through a row and a column map (-1 = zero padding).  Source element
+// (row r, column c) is src[r * sr + c * sc], so a transposed operand is the same call with the strides exchanged.
+// ------------------------------------------------------------------------------------------------
+template <class Tr>
+__global__ void k_tlm_pack(const uint16_t* __restrict__ src, long sr, long sc, const int* __restrict__ rowmap, const int* __restrict__ colmap,
+                           typename Tr::elem* __restrict__ dst, int NT, int KS, int tmul, int toff) {
+    const long idx = (long)blockIdx.x * blockDim.x + threadIdx.x;
+    if (idx >= (long)NT * KS * 64 * Tr::V) return;
+    const int e = (int)(idx % Tr::V);
+    const long f = idx / Tr::V;
+    const int lane = (int)(f & 63);
+    const int ks = (int)((f >> 6) % KS), nt = (int)((f >> 6) / KS);
+    const int r = rowmap[nt * 16 + (lane & 15)], c = colmap[ks * Tr::KSTEP + (lane >> 4) * Tr::V + e];
+    const uint16_t h = (r < 0 || c < 0) ? (uint16_t)0 : src[(long)r * sr + (long)c * sc];
+    const long at = (((long)nt * tmul + toff) * KS + ks) * 64 * Tr::V + (long)lane * Tr::V + e;      // tile nt of this call is tile nt * tmul + toff of the matrix
+    if constexpr (Tr::V == 8) dst[at] = h;
+    else dst[at] = mmi_bf16_to_f32(h);
+}
+// bf16 vector -> fp32, gathered through a map, zero where the map is negative
+__global__ void k_tlm_vec(const uint16_t* __restrict__ src, const int* __restrict__ map, float* __restrict__ dst, int n) {
+    const int i = (int)(blockIdx.x * blockDim.x + threadIdx.x);
+    if (i < n) dst[i] = map[i] < 0 ? 0.f : mmi_bf16_to_f32(src[map[i]]);
+}
+
+// ------------------------------------------------------------------------------------------------
+// step preparation
+// ------------------------------------------------------------------------------------------------
+struct TlmRope { const float* freq; int half, ld; float* out; };      // out [row][ld][2]: (cos, sin), (1, 0) past `half`
+struct TlmPrepArgs {
+    int T, n_ropes;
+    const int* n_updates;
+    const int* htok;          // token per row; negative: the token last sampled for the row's slot
+    const int* pos;
+    const int* rslot;
+    const int* last_tok;      // [slots]
+    int* tok;
+    const int* updates;       // (block-table index, page) pairs
+    int* block_table;
+    const TlmRope* rope;
+};
+__global__ void k_tlm_prepare(TlmPrepArgs a) {
+    const int i0 = (int)(blockIdx.x * blockDim.x + threadIdx.x), n = (int)(gridDim.x * blockDim.x);
+    for (int i = i0; i < *a.n_updates; i += n) a.block_table[a.updates[2 * i]] = a.updates[2 * i + 1];
+    for (int i = i0; i < a.T; i += n) {
+        const int t = a.htok[i];
+        a.tok[i] = t >= 0 ? t : a.last_tok[a.rslot[i]];
+    }
+    for (int r = 0; r < a.n_ropes; ++r) {
+        const TlmRope q = a.rope[r];
+        for (long i = i0; i < (long)a.T * q.ld; i += n) {
+            const int row = (int)(i / q.ld), j = (int)(i % q.ld);
+            float c = 1.f, s = 0.f;
+            if (j < q.half) {
+                const float ang = (float)a.pos[row] * q.freq[j];
+                c = cosf(ang);
+                s = sinf(ang);
+            }
+            q.out[2 * i] = c;
+            q.out[2 * i + 1] = s;
+        }
+    }
+}
+
+// Token-table routing: the experts of a row are table[token][0 .. top).  One workgroup per routed layer sorts the step's
+// (row, choice) pairs by expert - the order inside an expert is irrelevant, every pair is computed and stored on its own - and cuts
+// each expert's run into tiles of `tile` pairs.
+struct TlmRouteLayer { const int* table; int experts, top; };
+struct TlmRouteArgs {
+    const TlmRouteLayer* layers;
+    const int* tok;
+    int T, tile;
+    int* list;                // [layer][list_ld] pair ids row * top + choice, by expert
+    long list_ld;
+    int* tiles;               // [layer][tile_ld][3]: expert, first pair, pairs
+    long tile_ld;
+    int* n_tiles;             // [layer]
+};
+__global__ __launch_bounds__(1024) void k_tlm_route(TlmRouteArgs a) {
+    MMI_DYN_SHARED(unsigned, cnt);                       // [experts] pair counts, then [experts] insertion points
+    const TlmRouteLayer L = a.layers[blockIdx.x];
+    const int E = L.experts, top = L.top, tid = (int)threadIdx.x, nthr = (int)blockDim.x;
+    unsigned* at = cnt + E;
+    for (int e = tid; e < E; e += nthr) cnt[e] = 0u;
+    __syncthreads();
+    const int n = a.T * top;
+    for (int i = tid; i < n; i += nthr) mmi_atomic_add(&cnt[L.table[(long)a.tok[i / top] * top + i % top]], 1u);
+    __syncthreads();
+    if (tid == 0) {
+        unsigned s = 0;
+        int nt = 0;
+        int* tl = a.tiles + (long)blockIdx.x * a.tile_ld * 3;
+        for (int e = 0; e < E; ++e) {
+            const int c = (int)cnt[e];
+            at[e] = s;
+            for (int o = 0; o < c; o += a.tile) {
+                tl[3 * nt] = e;
+                tl[3 * nt + 1] = (int)s + o;
+                tl[3 * nt + 2] = c - o < a.tile ? c - o : a.tile;
+                ++nt;
+            }
+            s += (unsigned)c;
+        }
+        a.n_tiles[blockIdx.x] = nt;
+    }
+    __syncthreads();
+    int* list = a.list + (long)blockIdx.x * a.list_ld;
+    for (int i = tid; i < n; i += nthr) list[mmi_atomic_add(&at[L.table[(long)a.tok[i / top] * top + i % top]], 1u)] = i;
+}
+
+// ------------------------------------------------------------------------------------------------
+// residual update + grouped RMS norm: one workgroup per row
+//   x <- x + ls1 * sum_p mix[p] + ls2 * (1 / top) * sum_choice sum_p dn[p]   (the split-K partials of the two sublayers' last products)
+//   x <- emb[token] (first layer) or x + emb[token] (start of a repeated pass), then h = norm(x) * w -> packed operand
+// ------------------------------------------------------------------------------------------------
+enum { TLM_EMB_NONE = 0, TLM_EMB_SET = 1, TLM_EMB_ADD = 2 };
+struct TlmResidArgs {
+    float* x;
+    int width, ld;                       // ld: row stride of x, mix, dn (width rounded up to 16)
+    const float* mix; int mix_p; long mix_ps; const float* ls1;
+    const float* dn; int dn_p; long dn_ps; int top; const float* ls2;
+    const uint16_t* emb; const int* tok; int emb_mode;
+    float* tap;                          // copy of the residual stream before the embedding is added again, or null
+    const float* w; int groups; float eps;
+    void* out; int KS;                   // packed; null: no norm
+    const int* rows;                     // row list (the residual is then not written back), or null
+};
+template <class Tr>
+__global__ __launch_bounds__(256) void k_tlm_resid_norm(TlmResidArgs a) {
+    MMI_DYN_SHARED(float, row);          // [ld] the row, then [groups * parts] partial sums, then [groups] 1 / rms
+    const int tid = (int)threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int r = a.rows ? a.rows[blockIdx.x] : (int)blockIdx.x;
+    float* x = a.x + (long)r * a.ld;
+    for (int k = 4 * tid; k < a.ld; k += 1024) {
+        f32x4 v = {0.f, 0.f, 0.f, 0.f}, ev = v;
+        if (a.emb_mode != TLM_EMB_NONE) {
+            const uint16_t* e = a.emb + (long)a.tok[r] * a.width + k;
+#pragma unroll
+            for (int q = 0; q < 4; ++q)
+                if (k + q < a.width) ev[q] = mmi_bf16_to_f32(e[q]);
+        }
+        if (a.emb_mode == TLM_EMB_SET) {
+            v = ev;
+        } else {
+            v = *reinterpret_cast<const f32x4*>(x + k);
+            f32x4 d = {0.f, 0.f, 0.f, 0.f};
+            if (a.mix) {
+                for (int p = 0; p < a.mix_p; ++p) d += *reinterpret_cast<const f32x4*>(a.mix + p * a.mix_ps + (long)r * a.ld + k);
+                d *= *reinterpret_cast<const f32x4*>(a.ls1 + k);
+            }
+            if (a.dn) {
+                f32x4 f = {0.f, 0.f, 0.f, 0.f};
+                for (int c = 0; c < a.top; ++c)
+                    for (int p = 0; p < a.dn_p; ++p) f += *reinterpret_cast<const f32x4*>(a.dn + p * a.dn_ps + ((long)r * a.top + c) * a.ld + k);
+                d += f * (1.0f / (float)a.top) * *reinterpret_cast<const f32x4*>(a.ls2 + k);
+            }
+            v += d;
+            if (a.tap) *reinterpret_cast<f32x4*>(a.tap + (long)r * a.ld + k) = v;
+            if (a.emb_mode == TLM_EMB_ADD) v += ev;
+        }
+        if (!a.rows) *reinterpret_cast<f32x4*>(x + k) = v;
+        *reinterpret_cast<f32x4*>(row + k) = v;
+    }
+    if (!a.out) return;                                       // uniform over the grid
+    const int gs = a.width / a.groups;
+    const int parts = a.groups < 4 ? 4 / a.groups : 1;        // waves per group
+    float* part = row + a.ld;
+    float* inv = part + a.groups * parts;
+    __syncthreads();
+    const int per = (gs + parts - 1) / parts;
+    for (int t = wave; t < a.groups * parts; t += 4) {
+        const int g = t / parts, p = t - g * parts;
+        const int lo = p * per, hi = lo + per < gs ? lo + per : gs;
+        float s = 0.f;
+        for (int k = lo + lane; k < hi; k += 64) s = mmi_fma(row[g * gs + k], row[g * gs + k], s);
+        s = tlm_wave_sum(s);
+        if (lane == 0) part[t] = s;
+    }
+    __syncthreads();
+    for (int g = tid; g < a.groups; g += 256) {
+        float s = 0.f;
+        for (int p = 0; p < parts; ++p) s += part[g * parts + p];
+        inv[g] = 1.0f / sqrtf(s / (float)gs + a.eps);
+    }
+    __syncthreads();
+    typename Tr::elem* out = (typename Tr::elem*)a.out;
+    for (int k = 4 * tid; k < a.ld; k += 1024) {
+        f32x4 v = *reinterpret_cast<const f32x4*>(row + k);
+        const f32x4 w = *reinterpret_cast<const f32x4*>(a.w + k);
+#pragma unroll
+        for (int q = 0; q < 4; ++q) v[q] = k + q < a.width ? v[q] * inv[(k + q) / gs] * w[q] : 0.f;
+        Tr::store4(out + tlm_index<Tr>(blockIdx.x, k, a.KS), v);
+    }
+}
+
+// ------------------------------------------------------------------------------------------------
+// matrix products: up to three of them per launch, each dense, grouped (per head) or routed (per expert)
+// ------------------------------------------------------------------------------------------------
+enum { TLM_EPI_F32 = 0, TLM_EPI_PACK = 1, TLM_EPI_ROPE = 2, TLM_EPI_GRU = 3, TLM_EPI_LOGITS = 4 };
+enum { TLM_ACT_NONE = 0, TLM_ACT_RELU2 = 1 };
+struct TlmJob {
+    const u32x4* wp; long wgs;           // packed weights; fragments x 64 per group
+    const u32x4* xp; int xks, xkg;       // packed activations, their k-steps per row tile; k-step offset per group
+    int KS, NT, groups, ksplit;
+    int rows, rblocks;                   // dense rows; row blocks (routed: the bound on the number of tiles)
+    int in_mul, in_gadd;                 // activation row of row r in group g: r * in_mul + g * in_gadd
+    const int* list;                     // routed: pair list, tiles (expert, first, pairs), their number; activation row = pair / in_div
+    const int* tiles;
+    const int* n_tiles;
+    int in_div;
+    int epi, act;
+    void* out; int out_ld; long out_ps;  // fp32: row stride, stride per K split; packed: k-steps per row tile
+    int out_mul, out_gadd, out_k0, out_kg;
+    const float* bias;                   // GRU: [2][width]
+    const float* gate; int gate_ld;      // PACK: factor per (row, group), or null
+    const float* rope; int rope_ld;      // ROPE: (cos, sin) per row
+    int n_valid;                         // LOGITS: columns
+    float scale;
+    int blocks;
+};
+struct TlmJobs {
+    TlmJob j[3];
+    int n;
+};
+
+template <class Tr>
+__device__ __forceinline__ void tlm_epilogue(const TlmJob& j, int g, int split, int id, int nt, int quad, f32x4 v) {
+    const int n0 = nt * 16 + 4 * quad;
+    const long orow = (long)id * j.out_mul + (long)g * j.out_gadd;
+    if (j.epi == TLM_EPI_F32) {
+        *reinterpret_cast<f32x4*>((float*)j.out + split * j.out_ps + orow * j.out_ld + n0) = v;
+    } else if (j.epi == TLM_EPI_PACK) {
+        if (j.act == TLM_ACT_RELU2) {
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const float r = v[e] > 0.f ? v[e] : 0.f;
+                v[e] = r * r;
+            }
+        }
+        if (j.gate) v *= j.gate[(long)id * j.gate_ld + g];
+        Tr::store4((typename Tr::elem*)j.out + tlm_index<Tr>(orow, j.out_k0 + g * j.out_kg + n0, j.out_ld), v);
+    } else if (j.epi == TLM_EPI_ROPE) {
+        // rotation pairs are adjacent (the weight rows are interleaved at load)
+        const f32x4 cs = *reinterpret_cast<const f32x4*>(j.rope + ((long)id * j.rope_ld + n0 / 2) * 2);
+        const f32x4 o = {v[0] * cs[0] - v[1] * cs[1], v[1] * cs[0] + v[0] * cs[1], v[2] * cs[2] - v[3] * cs[3], v[3] * cs[2] + v[2] * cs[3]};
+        Tr::store4((typename Tr::elem*)j.out + tlm_index<Tr>(orow, j.out_k0 + g * j.out_kg + n0, j.out_ld), o);
+    } else if (j.epi == TLM_EPI_GRU) {
+        // n-tiles alternate gate, candidate, output gate of the same 16 channels
+        const int kind = nt % 3, c = (nt / 3) * 16 + 4 * quad;
+        const int w = j.out_ld;
+        f32x4 o;
+        if (kind == 2) {
+#pragma unroll
+            for (int e = 0; e < 4; ++e) o[e] = v[e] * tlm_sigmoid(v[e]);
+        } else {
+            v += *reinterpret_cast<const f32x4*>(j.bias + kind * w + c);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) o[e] = (kind == 1 && v[e] >= 0.f) ? v[e] + 0.5f : tlm_sigmoid(v[e]);
+        }
+        *reinterpret_cast<f32x4*>((float*)j.out + (orow * 3 + kind) * w + c) = o;
+    } else {
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+            if (n0 + e < j.n_valid) ((float*)j.out)[orow * j.out_ld + n0 + e] = v[e] * j.scale;
+    }
+}
+
+// Few rows (<= 16 MT per block): the weights are an HBM stream.  A workgroup owns one n-tile; its waves split K, each with U weight
+// fragments in flight per register buffer; partial tiles are summed through LDS in a fixed order.
+template <class Tr, int MT, int WAVES, int U>
+__global__ __launch_bounds__(WAVES * 64) void k_tlm_gemm_rows(TlmJobs jobs) {
+    int b = (int)blockIdx.x, ji = 0;
+    while (ji + 1 < jobs.n && b >= jobs.j[ji].blocks) b -= jobs.j[ji++].blocks;
+    const TlmJob& j = jobs.j[ji];
+    const int lane = (int)threadIdx.x & 63, wave = (int)threadIdx.x >> 6, bl = lane & 15;
+    const int nt = b % j.NT;
+    b /= j.NT;
+    const int split = b % j.ksplit;
+    b /= j.ksplit;
+    int g = b % j.groups, rb = b / j.groups, r0 = rb * 16 * MT, n;
+    if (j.list) {
+        if (rb >= *j.n_tiles) return;
+        g = j.tiles[3 * rb];
+        r0 = j.tiles[3 * rb + 1];
+        n = j.tiles[3 * rb + 2];
+    } else {
+        n = j.rows - r0 < 16 * MT ? j.rows - r0 : 16 * MT;
+    }
+    const int nm = (n + 15) >> 4;
+    int id[MT];
+    const u32x4* xq[MT];
+#pragma unroll
+    for (int m = 0; m < MT; ++m) {
+        const int i = m * 16 + bl < n ? m * 16 + bl : n - 1;
+        id[m] = j.list ? j.list[r0 + i] : r0 + i;
+        const long in = j.list ? id[m] / j.in_div : (long)id[m] * j.in_mul + (long)g * j.in_gadd;
+        xq[m] = j.xp + ((in >> 4) * j.xks + (long)g * j.xkg) * 64 + (in & 15) + (lane >> 4) * 16;
+    }
+    // K range of this split, then of this wave
+    const int sper = (j.KS + j.ksplit - 1) / j.ksplit;
+    const int s0 = min(j.KS, split * sper), s1 = min(j.KS, s0 + sper);
+    const int wper = (s1 - s0 + WAVES - 1) / WAVES;
+    const int k0 = min(s1, s0 + wave * wper), nk = min(s1, k0 + wper) - k0;
+    const u32x4* wq = j.wp + (long)g * j.wgs + ((long)nt * j.KS + k0) * 64 + lane;
+    f32x4 acc[MT];
+#pragma unroll
+    for (int m = 0; m < MT; ++m) acc[m] = f32x4{0.f, 0.f, 0.f, 0.f};
+    u32x4 wA[U], wB[U], xA[MT][U], xB[MT][U];
+#define TLM_LOAD(W_, X_, base)                                                                              \
+    _Pragma("unroll") for (int u = 0; u < U; ++u) {                                                         \
+        const int k_ = (base) + u < nk ? (base) + u : nk - 1;                                               \
+        W_[u] = mmi_load_nt(wq + (long)k_ * 64);                                                            \
+        _Pragma("unroll") for (int m = 0; m < MT; ++m) if (m < nm) X_[m][u] = xq[m][(long)(k0 + k_) * 64];  \
+    }
+#define TLM_MMA(W_, X_, base)                                                                               \
+    _Pragma("unroll") for (int u = 0; u < U; ++u)                                                           \
+        if ((base) + u < nk) {                                                                              \
+            _Pragma("unroll") for (int m = 0; m < MT; ++m) if (m < nm) acc[m] = Tr::mfma(W_[u], X_[m][u], acc[m]); \
+        }
+    if (nk > 0) {
+        TLM_LOAD(wA, xA, 0);
+        for (int k = 0;;) {
+            if (k + U < nk) { TLM_LOAD(wB, xB, k + U); }
+            TLM_MMA(wA, xA, k);
+            k += U;
+            if (k >= nk) break;
+            if (k + U < nk) { TLM_LOAD(wA, xA, k + U); }
+            TLM_MMA(wB, xB, k);
+            k += U;
+            if (k >= nk) break;
+        }
+    }
+#undef TLM_LOAD
+#undef TLM_MMA
+    MMI_SHARED __attribute__((aligned(16))) f32x4 red[WAVES * MT * 64];
+#pragma unroll
+    for (int m = 0; m < MT; ++m) red[(wave * MT + m) * 64 + lane] = acc[m];
+    __syncthreads();
+#pragma unroll
+    for (int m = 0; m < MT; ++m) {
+        if (m % WAVES != wave || m * 16 + bl >= n) continue;
+        f32x4 v = red[m * 64 + lane];
+#pragma unroll
+        for (int w = 1; w < WAVES; ++w) v += red[(w * MT + m) * 64 + lane];
+        tlm_epilogue<Tr>(j, g, split, id[m], nt, lane >> 4, v);
+    }
+}
+
+// Many rows: 2 x 2 waves over a tile of 32 FN features x 32 FM rows, two k-steps per stage, double-buffered in LDS.  Operands arrive
+// as whole fragments (one 16-byte vector per lane), so staging and operand reads are conflict-free without a swizzle.
+template <class Tr, int FN, int FM>
+__global__ __launch_bounds__(256) void k_tlm_gemm_tile(TlmJobs jobs) {
+    constexpr int NF = 2 * FN + 2 * FM, NI = NF / 4;          // fragments per k-step; per wave
+    MMI_SHARED __attribute__((aligned(16))) u32x4 lds[2 * 2 * NF * 64];
+    // consecutive workgroups go round the 8 XCDs: give each XCD a contiguous run of tiles so that its L2 sees the shared operand
+    const int nb = (int)gridDim.x, xper = nb >> 3, xrem = nb & 7, xcd = (int)blockIdx.x & 7;
+    int b = xcd * xper + (xcd < xrem ? xcd : xrem) + ((int)blockIdx.x >> 3), ji = 0;
+    while (ji + 1 < jobs.n && b >= jobs.j[ji].blocks) b -= jobs.j[ji++].blocks;
+    const TlmJob& j = jobs.j[ji];
+    const int lane = (int)threadIdx.x & 63, wave = (int)threadIdx.x >> 6, bl = lane & 15;
+    const int ntb = (j.NT + 2 * FN - 1) / (2 * FN);
+    int g, rb, nb0, n, r0;
+    if (j.list) {
+        nb0 = b % ntb;
+        rb = b / ntb;
+        if (rb >= *j.n_tiles) return;
+        g = j.tiles[3 * rb];
+        r0 = j.tiles[3 * rb + 1];
+        n = j.tiles[3 * rb + 2];
+    } else {
+        rb = b % j.rblocks;
+        b /= j.rblocks;
+        nb0 = b % ntb;
+        g = b / ntb;
+        r0 = rb * 32 * FM;
+        n = j.rows - r0 < 32 * FM ? j.rows - r0 : 32 * FM;
+    }
+    const int nt0 = nb0 * 2 * FN;
+    const u32x4* src[NI];
+#pragma unroll
+    for (int i = 0; i < NI; ++i) {
+        const int f = wave + 4 * i;
+        if (f < 2 * FN) {
+            const int nt = nt0 + f < j.NT ? nt0 + f : j.NT - 1;
+            src[i] = j.wp + (long)g * j.wgs + (long)nt * j.KS * 64 + lane;
+        } else {
+            const int m = (f - 2 * FN) * 16 + bl, ii = m < n ? m : n - 1;
+            const int id = j.list ? j.list[r0 + ii] : r0 + ii;
+            const long in = j.list ? id / j.in_div : (long)id * j.in_mul + (long)g * j.in_gadd;
+            src[i] = j.xp + ((in >> 4) * j.xks + (long)g * j.xkg) * 64 + (in & 15) + (lane >> 4) * 16;
+        }
+    }
+    const int wn = wave & 1, wm = wave >> 1;
+    f32x4 acc[FN][FM];
+#pragma unroll
+    for (int x = 0; x < FN; ++x)
+#pragma unroll
+        for (int y = 0; y < FM; ++y) acc[x][y] = f32x4{0.f, 0.f, 0.f, 0.f};
+    u32x4 st[2][NI];
+#define TLM_FETCH(k)                                                                       \
+    _Pragma("unroll") for (int kk = 0; kk < 2; ++kk) {                                     \
+        const int k_ = (k) + kk < j.KS ? (k) + kk : j.KS - 1;                              \
+        _Pragma("unroll") for (int i = 0; i < NI; ++i) st[kk][i] = src[i][(long)k_ * 64];  \
+    }
+#define TLM_STAGE(buf)                                                                     \
+    _Pragma("unroll") for (int kk = 0; kk < 2; ++kk)                                       \
+        _Pragma("unroll") for (int i = 0; i < NI; ++i) lds[(((buf) * 2 + kk) * NF + wave + 4 * i) * 64 + lane] = st[kk][i];
+    TLM_FETCH(0);
+    TLM_STAGE(0);
+    __syncthreads();
+    int cur = 0;
+    for (int k = 0; k < j.KS; k += 2) {
+        const bool more = k + 2 < j.KS;
+        if (more) { TLM_FETCH(k + 2); }
+#pragma unroll
+        for (int kk = 0; kk < 2; ++kk) {
+            if (k + kk < j.KS) {
+                const u32x4* base = lds + ((cur * 2 + kk) * NF) * 64 + lane;
+                u32x4 av[FN], bv[FM];
+#pragma unroll
+                for (int x = 0; x < FN; ++x) av[x] = base[(wn * FN + x) * 64];
+#pragma unroll
+                for (int y = 0; y < FM; ++y) bv[y] = base[(2 * FN + wm * FM + y) * 64];
+#pragma unroll
+                for (int x = 0; x < FN; ++x)
+#pragma unroll
+                    for (int y = 0; y < FM; ++y) acc[x][y] = Tr::mfma(av[x], bv[y], acc[x][y]);
+            }
+        }
+        if (more) { TLM_STAGE(cur ^ 1); }
+        __syncthreads();
+        cur ^= 1;
+    }
+#undef TLM_FETCH
+#undef TLM_STAGE
+#pragma unroll
+    for (int y = 0; y < FM; ++y) {
+        const int m = (wm * FM + y) * 16 + bl;
+        if (m >= n) continue;
+        const int id = j.list ? j.list[r0 + m] : r0 + m;
+#pragma unroll
+        for (int x = 0; x < FN; ++x) {
+            const int nt = nt0 + wn * FN + x;
+            if (nt < j.NT) tlm_epilogue<Tr>(j, g, 0, id, nt, lane >> 4, acc[x][y]);
+        }
+    }
+}
+
+// ------------------------------------------------------------------------------------------------
+// latent attention
+// ------------------------------------------------------------------------------------------------
+// One workgroup per token, on the columns [query latent | latent | rotated key part | head gates] of the input projection (fp32
+// split-K partials): the two RMS norms, the rotation of the key part, the cache write and the sigmoid of the gates.
+struct TlmLatentArgs {
+    const float* in; int in_p; long in_ps; int ld;       // ld: columns per row (every section rounded up to 16)
+    int q_rank, kv_rank, rot, heads;
+    int qp, kvp, rp;                                     // section widths
+    const float* qw; const float* cw; float eps;
+    const float* rope; int rope_ld;
+    const int* crow;                                     // cache row of the token: 64 page + offset
+    void* q; int q_ks;
+    void* kc; int k_ks, rot_k0;
+    void* vc; int nd;
+    float* gate; int gate_ld;
+};
+template <class Tr>
+__global__ __launch_bounds__(256) void k_tlm_latent(TlmLatentArgs a) {
+    typedef typename Tr::elem elem;
+    MMI_DYN_SHARED(float, row);                          // [ld]
+    MMI_SHARED float part[2][4];
+    const int t = (int)blockIdx.x, tid = (int)threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    float sq = 0.f, sc = 0.f;
+    for (int k = 4 * tid; k < a.ld; k += 1024) {
+        f32x4 v = *reinterpret_cast<const f32x4*>(a.in + (long)t * a.ld + k);
+        for (int p = 1; p < a.in_p; ++p) v += *reinterpret_cast<const f32x4*>(a.in + p * a.in_ps + (long)t * a.ld + k);
+        *reinterpret_cast<f32x4*>(row + k) = v;
+        const float s = v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];     // the padding columns are zero
+        if (k < a.qp) sq += s;
+        else if (k < a.qp + a.kvp) sc += s;
+    }
+    sq = tlm_wave_sum(sq);
+    sc = tlm_wave_sum(sc);
+    if (lane == 0) {
+        part[0][wave] = sq;
+        part[1][wave] = sc;
+    }
+    __syncthreads();
+    const float iq = 1.0f / sqrtf((part[0][0] + part[0][1] + part[0][2] + part[0][3]) / (float)a.q_rank + a.eps);
+    const float ic = 1.0f / sqrtf((part[1][0] + part[1][1] + part[1][2] + part[1][3]) / (float)a.kv_rank + a.eps);
+    const long cr = a.crow[t];
+    const long page = cr / TLM_PAGE;
+    const int off = (int)(cr % TLM_PAGE);
+    for (int k = 4 * tid; k < a.ld; k += 1024) {
+        f32x4 v = *reinterpret_cast<const f32x4*>(row + k);
+        if (k < a.qp) {
+            v *= iq * *reinterpret_cast<const f32x4*>(a.qw + k);
+            Tr::store4((elem*)a.q + tlm_index<Tr>(t, k, a.q_ks), v);
+        } else if (k < a.qp + a.kvp) {
+            const int d = k - a.qp;
+            v *= ic * *reinterpret_cast<const f32x4*>(a.cw + d);
+            Tr::store4((elem*)a.kc + tlm_index<Tr>(cr, d, a.k_ks), v);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) ((elem*)a.vc)[tlm_vindex<Tr>(page, off, d + e, a.nd)] = Tr::cvt(v[e]);
+        } else if (k < a.qp + a.kvp + a.rp) {
+            const int d = k - a.qp - a.kvp;
+            const f32x4 cs = *reinterpret_cast<const f32x4*>(a.rope + ((long)t * a.rope_ld + d / 2) * 2);
+            const f32x4 o = {v[0] * cs[0] - v[1] * cs[1], v[1] * cs[0] + v[0] * cs[1], v[2] * cs[2] - v[3] * cs[3], v[3] * cs[2] + v[2] * cs[3]};
+            Tr::store4((elem*)a.kc + tlm_index<Tr>(cr, a.rot_k0 + d, a.k_ks), o);
+        } else {
+            const int h = k - a.qp - a.kvp - a.rp;
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+                if (h + e < a.heads) a.gate[(long)t * a.gate_ld + h + e] = tlm_sigmoid(v[e]);
+        }
+    }
+}
+
+// Attention over the latent cache.  All heads share one key per position - (latent, rotated part) against the queries absorbed
+// through the key projection - and the value is the latent itself, so (token, head) pairs are the columns of one product and a key
+// fragment serves 16 of them.  A column tile never mixes sequences.  Keys are walked in blocks of 32; a column sees key j of its
+// token at position i when 0 <= i - j < window.
+struct TlmAttnArgs {
+    const void* q;                       // packed rows token * heads + head
+    const void* kc;
+    const void* vc;
+    void* out;                           // packed rows token * heads + head, latent columns
+    int heads, q_ks, nd, out_ks;
+    int window;                          // 0: every earlier position
+    float scale;                         // times log2(e)
+    int n_entries, n_tiles, nsplit;
+    const int* tile0;                    // [entries + 1] first column tile of each entry
+    const int* erow0; const int* elen; const int* epos0; const int* eslot;
+    const int* block_table; int bt_ld;   // [slot][bt_ld]: page of positions 64 i .. at i % bt_ld
+    float* po;                           // nsplit > 1: [tile][split][nd][64] f32x4 un-normalised sums
+    float* pml;                          // [tile][split][2][16]: running maximum, sum of weights
+};
+struct TlmCols { int entry, c0, ncol; };
+__device__ __forceinline__ TlmCols tlm_find_tile(const TlmAttnArgs& a, int tile) {
+    int lo = 0, hi = a.n_entries - 1;
+    while (lo < hi) {                                   // last entry whose first tile is <= tile
+        const int mid = (lo + hi + 1) >> 1;
+        if (a.tile0[mid] <= tile) lo = mid;
+        else hi = mid - 1;
+    }
+    TlmCols c;
+    c.entry = lo;
+    c.c0 = (tile - a.tile0[lo]) * 16;
+    c.ncol = a.elen[lo] * a.heads;
+    return c;
+}
+
+template <class Tr>
+__device__ __forceinline__ void tlm_attn_store(const TlmAttnArgs& a, const TlmCols& c, int bl, int kq, int db, f32x4 v) {
+    const int col = c.c0 + bl;
+    if (col >= c.ncol) return;
+    const long orow = (long)a.erow0[c.entry] * a.heads + col;
+    Tr::store4((typename Tr::elem*)a.out + tlm_index<Tr>(orow, db * 16 + 4 * kq, a.out_ks), v);
+}
+
+// ND: bound on the 16-wide latent blocks.  WK waves of a workgroup share one column tile (each takes every WK-th key block; their
+// sums meet in LDS), the other 4 / WK groups take further tiles.
+template <class Tr, int ND, int WK>
+__global__ __launch_bounds__(256) void k_tlm_attn(TlmAttnArgs a) {
+    constexpr int NQ = ND * 16 / Tr::KSTEP + 128 / Tr::KSTEP;      // query fragments: latent + at most 128 rotated dimensions
+    constexpr int NB = 32 / (4 * Tr::V);                           // value fragments per 32 keys
+    MMI_SHARED float ml[2][4][16];
+    MMI_SHARED __attribute__((aligned(16))) f32x4 ob[WK > 1 ? 4 * 8 * 64 : 1];
+    const int lane = (int)threadIdx.x & 63, wave = (int)threadIdx.x >> 6, bl = lane & 15, kq = lane >> 4;
+    const int tile = (int)blockIdx.x * (4 / WK) + wave / WK, wk = wave % WK, split = (int)blockIdx.y;
+    if (tile >= a.n_tiles) return;                                 // WK == 4: the whole workgroup; WK == 1: no barrier follows
+    const TlmCols c = tlm_find_tile(a, tile);
+    const int col = c.c0 + bl < c.ncol ? c.c0 + bl : c.ncol - 1;
+    const int pos0 = a.epos0[c.entry];
+    const int pc = pos0 + col / a.heads;                           // position of this lane's column
+    const int plo = pos0 + c.c0 / a.heads, phi = pos0 + (min(c.c0 + 15, c.ncol - 1)) / a.heads;
+    const int klo = a.window > 0 && plo - a.window + 1 > 0 ? plo - a.window + 1 : 0;
+    int b0 = klo / 32, b1 = phi / 32 + 1;
+    if (a.nsplit > 1) {
+        const int per = (b1 - b0 + a.nsplit - 1) / a.nsplit;
+        b0 = min(b1, b0 + split * per);
+        b1 = min(b1, b0 + per);
+    }
+    const int* bt = a.block_table + (long)a.eslot[c.entry] * a.bt_ld;
+    const u32x4* kc = (const u32x4*)a.kc;
+    const u32x4* vc = (const u32x4*)a.vc;
+    u32x4 qf[NQ];
+    {
+        const long qrow = (long)a.erow0[c.entry] * a.heads + col;
+        const u32x4* qp = (const u32x4*)a.q + (qrow >> 4) * a.q_ks * 64 + kq * 16 + (qrow & 15);
+#pragma unroll
+        for (int s = 0; s < NQ; ++s)
+            if (s < a.q_ks) qf[s] = qp[s * 64];
+    }
+    f32x4 acc[ND];
+#pragma unroll
+    for (int d = 0; d < ND; ++d) acc[d] = f32x4{0.f, 0.f, 0.f, 0.f};
+    float m = -1e30f, l = 0.f;
+    for (int kb = b0 + wk; kb < b1; kb += WK) {
+        const long page = bt[(kb >> 1) % a.bt_ld];
+        const u32x4* kp = kc + (page * 4 + (kb & 1) * 2) * a.q_ks * 64 + lane;
+        f32x4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = s0;
+#pragma unroll
+        for (int s = 0; s < NQ; ++s)
+            if (s < a.q_ks) {
+                s0 = Tr::mfma(kp[s * 64], qf[s], s0);
+                s1 = Tr::mfma(kp[(a.q_ks + s) * 64], qf[s], s1);
+            }
+        float mx = m;
+        const int d0 = pc - (kb * 32 + 4 * kq);                    // position minus the key of register 0
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int e0 = d0 - r, e1 = d0 - r - 16;
+            s0[r] = e0 >= 0 && (a.window <= 0 || e0 < a.window) ? s0[r] * a.scale : -INFINITY;
+            s1[r] = e1 >= 0 && (a.window <= 0 || e1 < a.window) ? s1[r] * a.scale : -INFINITY;
+            mx = fmaxf(mx, fmaxf(s0[r], s1[r]));
+        }
+        mx = fmaxf(mx, mmi_shfl_xor(mx, 16));
+        mx = fmaxf(mx, mmi_shfl_xor(mx, 32));
+        const float al = exp2f(m - mx);
+        m = mx;
+        l *= al;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            s0[r] = exp2f(s0[r] - mx);
+            s1[r] = exp2f(s1[r] - mx);
+            l += s0[r] + s1[r];
+        }
+        u32x4 pf[NB];
+        if constexpr (NB == 1) {
+            pf[0] = u32x4{mmi_pack_bf16x2(s0[0], s0[1]), mmi_pack_bf16x2(s0[2], s0[3]), mmi_pack_bf16x2(s1[0], s1[1]), mmi_pack_bf16x2(s1[2], s1[3])};
+        } else {
+            pf[0] = __builtin_bit_cast(u32x4, s0);
+            pf[NB - 1] = __builtin_bit_cast(u32x4, s1);
+        }
+        const u32x4* vp = vc + (page * a.nd * (2 * NB) + (kb & 1) * NB) * 64 + lane;
+#pragma unroll
+        for (int d = 0; d < ND; ++d)
+            if (d < a.nd) {
+                acc[d] *= al;
+#pragma unroll
+                for (int q = 0; q < NB; ++q) acc[d] = Tr::mfma(vp[(d * 2 * NB + q) * 64], pf[q], acc[d]);
+            }
+    }
+    l += mmi_shfl_xor(l, 16);
+    l += mmi_shfl_xor(l, 32);
+    if constexpr (WK > 1) {
+        if (kq == 0) {
+            ml[0][wave][bl] = m;
+            ml[1][wave][bl] = l;
+        }
+        __syncthreads();
+        float M = -1e30f, L = 0.f;
+#pragma unroll
+        for (int w = 0; w < WK; ++w) M = fmaxf(M, ml[0][w][bl]);
+#pragma unroll
+        for (int w = 0; w < WK; ++w) L += ml[1][w][bl] * exp2f(ml[0][w][bl] - M);
+        const float f = exp2f(m - M);
+        m = M;
+        l = L;
+        const float inv = a.nsplit > 1 ? 1.f : 1.0f / l;
+#pragma unroll
+        for (int d0 = 0; d0 < ND; d0 += 8) {
+            if (d0 >= a.nd) break;
+            if (d0) __syncthreads();
+#pragma unroll
+            for (int d = 0; d < 8; ++d)
+                if (d0 + d < ND) ob[(wave * 8 + d) * 64 + lane] = acc[d0 + d < ND ? d0 + d : 0] * f;
+            __syncthreads();
+#pragma unroll
+            for (int d = wave; d < 8; d += WK) {
+                if (d0 + d >= a.nd) break;
+                f32x4 v = ob[d * 64 + lane];
+#pragma unroll
+                for (int w = 1; w < WK; ++w) v += ob[(w * 8 + d) * 64 + lane];
+                if (a.nsplit > 1) *reinterpret_cast<f32x4*>(a.po + ((((long)tile * a.nsplit + split) * a.nd + d0 + d) * 64 + lane) * 4) = v;
+                else tlm_attn_store<Tr>(a, c, bl, kq, d0 + d, v * inv);
+            }
+        }
+    } else {
+        const float inv = a.nsplit > 1 ? 1.f : 1.0f / l;
+#pragma unroll
+        for (int d = 0; d < ND; ++d)
+            if (d < a.nd) {
+                if (a.nsplit > 1) *reinterpret_cast<f32x4*>(a.po + ((((long)tile * a.nsplit + split) * a.nd + d) * 64 + lane) * 4) = acc[d];
+                else tlm_attn_store<Tr>(a, c, bl, kq, d, acc[d] * inv);
+            }
+    }
+    if (a.nsplit > 1 && wk == 0 && kq == 0) {
+        float* q = a.pml + ((long)tile * a.nsplit + split) * 32;
+        q[bl] = m;
+        q[16 + bl] = l;
+    }
+}
+
+// the splits of one column tile -> output; one workgroup per tile, waves over the latent blocks
+template <class Tr>
+__global__ __launch_bounds__(256) void k_tlm_attn_combine(TlmAttnArgs a) {
+    const int lane = (int)threadIdx.x & 63, wave = (int)threadIdx.x >> 6, bl = lane & 15, kq = lane >> 4, tile = (int)blockIdx.x;
+    const TlmCols c = tlm_find_tile(a, tile);
+    const float* q = a.pml + (long)tile * a.nsplit * 32;
+    float M = -1e30f, L = 0.f;
+    for (int s = 0; s < a.nsplit; ++s) M = fmaxf(M, q[s * 32 + bl]);
+    for (int s = 0; s < a.nsplit; ++s) L += q[s * 32 + 16 + bl] * exp2f(q[s * 32 + bl] - M);
+    const float inv = 1.0f / L;
+    for (int d = wave; d < a.nd; d += 4) {
+        f32x4 v = {0.f, 0.f, 0.f, 0.f};
+        for (int s = 0; s < a.nsplit; ++s)
+            v += *reinterpret_cast<const f32x4*>(a.po + ((((long)tile * a.nsplit + s) * a.nd + d) * 64 + lane) * 4) * exp2f(q[s * 32 + bl] - M);
+        tlm_attn_store<Tr>(a, c, bl, kq, d, v * inv);
+    }
+}
+
+// ------------------------------------------------------------------------------------------------
+// minimal gated recurrence: S_t = (1 - z_t) S_(t-1) + z_t c_t, output S_t * g_t, from the fp32 gates the projection's epilogue stored.
+// A step's sequences are cut into segments of at most TLM_SEG tokens.  The recurrence is linear in S, so a segment is the pair
+// (A, B) with S_end = A S_begin + B: the first launch computes the pairs (only when some sequence has more than one segment), the
+// second starts every segment from its predecessors' pairs.  State is [slot][2][width]: read one copy, write the other, so that a
+// segment's write cannot be seen by another segment of the same sequence.
+// ------------------------------------------------------------------------------------------------
+constexpr int TLM_SEG = 32;
+struct TlmSeg { int row0, n, slot, par, index, last, fresh, pad; };      // index: number of the segment in its sequence; fresh: position 0
+struct TlmScanArgs {
+    const float* zcg;             // [row][3][width]
+    int width;                    // padded to 16
+    const TlmSeg* seg;
+    float* state;
+    float* pair;                  // [segment][2][width]
+    void* out; int out_ks;
+};
+__global__ __launch_bounds__(256) void k_tlm_scan_pairs(TlmScanArgs a) {
+    const int c = (int)(blockIdx.x * blockDim.x + threadIdx.x);
+    const TlmSeg s = a.seg[blockIdx.y];
+    if (c >= a.width || s.last) return;
+    const float* p = a.zcg + (long)s.row0 * 3 * a.width + c;
+    float A = 1.f, B = 0.f;
+    for (int i0 = 0; i0 < s.n; i0 += 8) {
+        float z[8], u[8];
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+            const long o = (long)(i0 + i < s.n ? i0 + i : s.n - 1) * 3 * a.width;
+            z[i] = p[o];
+            u[i] = p[o + a.width];
+        }
+#pragma unroll
+        for (int i = 0; i < 8; ++i)
+            if (i0 + i < s.n) {
+                A *= 1.0f - z[i];
+                B = mmi_fma(1.0f - z[i], B, z[i] * u[i]);
+            }
+    }
+    a.pair[(long)blockIdx.y * 2 * a.width + c] = A;
+    a.pair[((long)blockIdx.y * 2 + 1) * a.width + c] = B;
+}
+template <class Tr>
+__global__ __launch_bounds__(256) void k_tlm_scan(TlmScanArgs a) {
+    const int c = (int)(blockIdx.x * blockDim.x + threadIdx.x);
+    const TlmSeg s = a.seg[blockIdx.y];
+    if (c >= a.width) return;
+    const float* p = a.zcg + (long)s.row0 * 3 * a.width + c;
+    typename Tr::elem* out = (typename Tr::elem*)a.out;
+    float S = s.fresh ? 0.f : a.state[((long)s.slot * 2 + s.par) * a.width + c];
+    const float* q = a.pair + (long)((int)blockIdx.y - s.index) * 2 * a.width + c;
+    for (int i = 0; i < s.index; ++i) S = mmi_fma(q[(long)i * 2 * a.width], S, q[((long)i * 2 + 1) * a.width]);
+    for (int i0 = 0; i0 < s.n; i0 += 8) {
+        float z[8], u[8], g[8];
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+            const long o = (long)(i0 + i < s.n ? i0 + i : s.n - 1) * 3 * a.width;
+            z[i] = p[o];
+            u[i] = p[o + a.width];
+            g[i] = p[o + 2 * a.width];
+        }
+#pragma unroll
+        for (int i = 0; i < 8; ++i)
+            if (i0 + i < s.n) {
+                S = mmi_fma(1.0f - z[i], S, z[i] * u[i]);
+                out[tlm_index<Tr>(s.row0 + i0 + i, c, a.out_ks)] = Tr::cvt(S * g[i]);
+            }
+    }
+    if (s.last) a.state[((long)s.slot * 2 + (s.par ^ 1)) * a.width + c] = S;
+}
+
+// ------------------------------------------------------------------------------------------------
+// sampling helpers
+// ------------------------------------------------------------------------------------------------
+// greedy: index of the largest logit, the lowest index on ties; out[map[row]] (map: row -> slot)
+__global__ __launch_bounds__(256) void k_tlm_argmax(const float* __restrict__ logits, int V, const int* __restrict__ map, int* __restrict__ out,
+                                                    int* __restrict__ last_tok) {
+    MMI_SHARED float bv[256];
+    MMI_SHARED int bi[256];
+    const int tid = (int)threadIdx.x;
+    const float* p = logits + (long)blockIdx.x * V;
+    float best = -INFINITY;
+    int at = 0;
+    for (int i = tid; i < V; i += 256)
+        if (p[i] > best) { best = p[i]; at = i; }
+    bv[tid] = best;
+    bi[tid] = at;
+    __syncthreads();
+    for (int s = 128; s > 0; s >>= 1) {
+        if (tid < s && (bv[tid + s] > bv[tid] || (bv[tid + s] == bv[tid] && bi[tid + s] < bi[tid]))) {
+            bv[tid] = bv[tid + s];
+            bi[tid] = bi[tid + s];
+        }
+        __syncthreads();
+    }
+    if (tid == 0) {
+        out[blockIdx.x] = bi[0];
+        last_tok[map[blockIdx.x]] = bi[0];
+    }
+}
+// fp32 logits -> the sampler's bf16 rows of ld columns (padding: -inf, never drawn)
+__global__ void k_tlm_sample_rows(const float* __restrict__ logits, int V, uint16_t* __restrict__ dst, int ld, int n) {
+    const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i >= (long)n * ld) return;
+    const int c = (int)(i % ld);
+    dst[i] = c < V ? mmi_f32_to_bf16(logits[(i / ld) * V + c]) : (uint16_t)0xff80u;
+}
+__global__ void k_tlm_last_tok(const int* __restrict__ out, const int* __restrict__ map, int* __restrict__ last_tok, int n) {
+    const int i = (int)(blockIdx.x * blockDim.x + threadIdx.x);
+    if (i < n) last_tok[map[i]] = out[i];
+}
+__global__ void k_tlm_fill(float* __restrict__ p, float v, long n) {
+    const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i < n) p[i] = v;
+}

@@ -21,9 +21,10 @@ from typing import Any, Dict, Optional
 
 import torch
 
-from .config import LMConfig, MimiConfig
+from .config import TOKEN_LM_ARCHITECTURES, LMConfig, MimiConfig, TokenLMConfig
 from .lm import ConditionFuser, LMModel
 from .mimi import MimiModel
+from .tlm import TokenLM
 
 
 # Names the reference's callers import from this module (server.py / run_inference.py argparse defaults, scripts): the released
@@ -183,6 +184,34 @@ def get_moshi_lm(filename: str | Path | None, lm_kwargs: Optional[Dict[str, Any]
         state_patch(state)
     already = any(v.dtype in (torch.int8, torch.float8_e4m3fn) for v in state.values())
     return LMModel(state, cfg, device=device, max_batch=max_batch, lib=lib, quantize=False if already else quantize, fuser=fuser)
+
+
+def is_token_lm(path: str | Path) -> bool:
+    """True when `path` (a directory with config.json, or the file) describes a token language model: its `architecture` is in the
+    registry (config.TOKEN_LM_ARCHITECTURES).  Moshi checkpoints have no such key."""
+    path = Path(path)
+    cfg = path / "config.json" if path.is_dir() else path
+    return cfg.exists() and json.loads(cfg.read_text()).get("architecture") in TOKEN_LM_ARCHITECTURES
+
+
+def token_lm_config_from_dict(raw: dict) -> TokenLMConfig:
+    name = raw.get("architecture")
+    if name not in TOKEN_LM_ARCHITECTURES:
+        raise ValueError(f"unknown architecture {name!r} (known: {sorted(TOKEN_LM_ARCHITECTURES)})")
+    return TOKEN_LM_ARCHITECTURES[name](raw)
+
+
+def get_token_lm(path: str | Path, device: torch.device | str = "cuda", dtype: torch.dtype = torch.bfloat16, max_slots: int = 32,
+                 max_tokens: int = 65536, max_step_tokens: Optional[int] = None, load_weight: bool = True, lib=None) -> TokenLM:
+    """A token language model from a directory holding config.json and model.safetensors (load_weight=False: seeded random weights)."""
+    path = Path(path)
+    cfg = token_lm_config_from_dict(json.loads((path / "config.json").read_text()))
+    if load_weight:
+        state = _load_state(path / MOSHI_NAME)
+    else:
+        from .weights import random_token_lm_state_dict
+        state = random_token_lm_state_dict(cfg, seed=0)
+    return TokenLM(state, cfg, device=device, dtype=dtype, max_slots=max_slots, max_tokens=max_tokens, max_step_tokens=max_step_tokens, lib=lib)
 
 
 def export_quantized(src: str | Path, dst: str | Path, fmt: str = "int8", lm_kwargs: Optional[dict] = None) -> Dict[str, int]:

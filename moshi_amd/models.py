@@ -3,7 +3,8 @@
 `moshi.models` to `moshi_amd.models`."""
 from . import loaders  # noqa: F401
 from .lm import LMGen, LMModel  # noqa: F401
-from .loaders import get_mimi, get_moshi_lm  # noqa: F401
+from .loaders import get_mimi, get_moshi_lm, get_token_lm  # noqa: F401
 from .mimi import MimiModel  # noqa: F401
+from .tlm import TokenLM  # noqa: F401
 
-__all__ = ["MimiModel", "LMModel", "LMGen", "get_mimi", "get_moshi_lm", "loaders"]
+__all__ = ["MimiModel", "LMModel", "LMGen", "get_mimi", "get_moshi_lm", "loaders", "TokenLM", "get_token_lm"]

@@ -14,7 +14,7 @@ from typing import Dict, List, Tuple
 
 import torch
 
-from .config import LMConfig, MimiConfig
+from .config import LatentAttentionConfig, LMConfig, MimiConfig, TokenLMConfig
 
 Spec = List[Tuple[str, Tuple[int, ...], str]]  # (name, shape, kind)
 
@@ -134,10 +134,38 @@ def lm_state_spec(cfg: LMConfig) -> Spec:
     return spec
 
 
+def token_lm_state_spec(cfg: TokenLMConfig) -> Spec:
+    """Names and shapes of a token LM's tensors (model.safetensors: bf16, tables int32).  Linear weights are [out, in]."""
+    d = cfg.width
+    spec: Spec = [("embed", (cfg.vocab, d), "emb:1")]
+    for i, layer in enumerate(cfg.layers):
+        p, m = f"l{i}", layer.mixer
+        spec.append((f"{p}.norm1", (d,), "alpha"))
+        if isinstance(m, LatentAttentionConfig):
+            spec += [(f"{p}.mix.dq", (m.q_rank, d), f"fan:{d}"), (f"{p}.mix.dq.norm", (m.q_rank,), "alpha"),
+                     (f"{p}.mix.uq", (m.heads * (m.dim + m.rot_dim), m.q_rank), f"fan:{m.q_rank}"),
+                     (f"{p}.mix.dkv", (m.kv_rank + m.rot_dim, d), f"fan:{d}"), (f"{p}.mix.dkv.norm", (m.kv_rank,), "alpha"),
+                     (f"{p}.mix.uk", (m.heads * m.dim, m.kv_rank), f"fan:{m.kv_rank}"), (f"{p}.mix.uv", (m.heads * m.vdim, m.kv_rank), f"fan:{m.kv_rank}"),
+                     (f"{p}.mix.g", (m.heads, d), f"fan:{d}"), (f"{p}.mix.o", (d, m.heads * m.vdim), f"fan:{m.heads * m.vdim}")]
+        else:
+            spec += [(f"{p}.mix.z", (m.width, d), f"fan:{d}"), (f"{p}.mix.z.b", (m.width,), "norm_b"), (f"{p}.mix.x", (m.width, d), f"fan:{d}"),
+                     (f"{p}.mix.x.b", (m.width,), "norm_b"), (f"{p}.mix.g", (m.width, d), f"fan:{d}"), (f"{p}.mix.o", (d, m.width), f"fan:{m.width}")]
+        spec.append((f"{p}.ls1", (d,), "layer_scale"))
+        if layer.mlp is not None:
+            for e in range(layer.mlp.experts):
+                spec += [(f"{p}.mlp.e{e}.up", (layer.mlp.ff, d), f"fan:{d}"), (f"{p}.mlp.e{e}.down", (d, layer.mlp.ff), f"fan:{layer.mlp.ff}")]
+            spec += [(f"{p}.mlp.table", (cfg.vocab, layer.mlp.top), f"table:{layer.mlp.experts}"), (f"{p}.ls2", (d,), "layer_scale")]
+    spec += [("final.norm", (d,), "alpha"), ("head", (cfg.vocab, d), f"fan:{d}")]
+    return spec
+
+
 def _draw(shape, kind: str, gen: torch.Generator, device, dtype) -> torch.Tensor:
     """One synthetic tensor.  Drawn on `device` when it is a GPU (fast for the 7B benchmark model)."""
     def rnd(fn, *a):
         return fn(*a, generator=gen, device=device, dtype=torch.float32)
+    if kind.startswith("table:"):                      # [rows, top] distinct choices out of n
+        n = int(kind[6:])
+        return torch.rand((shape[0], n), generator=gen, device=device).argsort(dim=1)[:, :shape[1]].to(torch.int32).contiguous()
     if kind.startswith("fan:"):
         fan = int(kind[4:])
         t = (rnd(torch.rand, shape) * 2 - 1) * math.sqrt(3.0 / fan)   # unit-gain uniform
@@ -173,6 +201,10 @@ def random_mimi_state_dict(cfg: MimiConfig, seed: int = 1234, device="cpu") -> D
 
 def random_lm_state_dict(cfg: LMConfig, seed: int = 4242, device="cpu", dtype=torch.bfloat16) -> Dict[str, torch.Tensor]:
     return random_state_dict(lm_state_spec(cfg), seed, device, dtype)
+
+
+def random_token_lm_state_dict(cfg: TokenLMConfig, seed: int = 77, device="cpu", dtype=torch.bfloat16) -> Dict[str, torch.Tensor]:
+    return random_state_dict(token_lm_state_spec(cfg), seed, device, dtype)
 
 
 # --------------------------------------------------------------------------------------------------------------------

@@ -13,7 +13,9 @@ HERE = Path(__file__).resolve().parent
 ROOT = HERE.parent.parent
 CSRC = ROOT / "moshi_amd" / "csrc"
 LIB = HERE / "libmoshi_sim.so"
+TLM_LIB = HERE / "libmoshi_tlm_sim.so"
 SOURCES = ["api_common.hip", "mimi_engine.hip", "lm_engine.hip", "batcher.hip", "duplex.hip"]
+TLM_SOURCES = ["api_common.hip", "tlm_engine.hip"]
 
 
 def _cxx() -> str:
@@ -23,32 +25,38 @@ def _cxx() -> str:
     raise RuntimeError("clang++ not found")
 
 
-def needs_build() -> bool:
-    if not LIB.exists():
+def needs_build(lib: Path = LIB) -> bool:
+    if not lib.exists():
         return True
-    t = LIB.stat().st_mtime
-    deps = list(CSRC.glob("*")) + list(HERE.glob("*.h")) + list(HERE.glob("*.cpp")) + [ROOT / "include" / "moshi_mi.h"]
+    t = lib.stat().st_mtime
+    deps = (list(CSRC.glob("*.h")) + list(CSRC.glob("*.hip")) + list(HERE.glob("*.h")) + list(HERE.glob("*.cpp")) +
+            list((ROOT / "include").glob("*.h")))
     return any(p.stat().st_mtime > t for p in deps)
 
 
-def build(force: bool = False, verbose: bool = False) -> Path:
+def build_tlm(force: bool = False, verbose: bool = False) -> Path:
+    """The token-LM library (libmoshi_tlm.so's sources) on the simulator."""
+    return build(force, verbose, TLM_LIB, TLM_SOURCES)
+
+
+def build(force: bool = False, verbose: bool = False, lib: Path = LIB, sources=None) -> Path:
     """Several test workers may call this at once: the compile runs under a file lock."""
     import fcntl
     with open(HERE / ".build.lock", "w") as lock:
         fcntl.flock(lock, fcntl.LOCK_EX)
         try:
-            return _build_locked(force, verbose)
+            return _build_locked(force, verbose, lib, SOURCES if sources is None else sources)
         finally:
             fcntl.flock(lock, fcntl.LOCK_UN)
 
 
-def _build_locked(force: bool, verbose: bool) -> Path:
-    if not force and not needs_build():
-        return LIB
+def _build_locked(force: bool, verbose: bool, lib: Path, sources) -> Path:
+    if not force and not needs_build(lib):
+        return lib
     objs, jobs = [], []
     common = [_cxx(), "-O2", "-g", "-std=c++17", "-fPIC", "-ffp-contract=off", "-pthread", "-Wno-unused-value",
               f"-I{HERE}", f"-I{CSRC}"]
-    for name in SOURCES:
+    for name in sources:
         src = CSRC / name
         if not src.exists():
             continue
@@ -65,9 +73,9 @@ def _build_locked(force: bool, verbose: bool) -> Path:
     for p, cmd in jobs:
         if p.wait() != 0:
             raise RuntimeError("sim build failed: " + " ".join(cmd))
-    cmd = [_cxx(), "-shared", "-fPIC", "-pthread", "-o", str(LIB)] + [str(o) for o in objs]
+    cmd = [_cxx(), "-shared", "-fPIC", "-pthread", "-o", str(lib)] + [str(o) for o in objs]
     subprocess.check_call(cmd)
-    return LIB
+    return lib
 
 
 def build_asan(out_dir: Path) -> Path:
