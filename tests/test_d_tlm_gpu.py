@@ -1,0 +1,56 @@
+"""Token language models on a real MI355X: the cases of tests/tlm_cases.py through libmoshi_tlm.so (hipGraph replay in decode steps)."""
+import pytest
+
+from tests import tlm_cases as tc
+
+pytestmark = pytest.mark.gpu
+DEV = "cuda"
+
+
+@pytest.fixture(scope="session")
+def lib():
+    import torch
+    assert torch.cuda.is_available(), "-m gpu tests need a GPU"
+    from moshi_amd import _capi
+    return _capi.load_tlm()
+
+
+@pytest.mark.parametrize("dtype", [tc.F32, tc.BF16], ids=["fp32", "bf16"])
+@pytest.mark.parametrize("name", sorted(tc.MECHANISMS))
+def test_mechanism(lib, name, dtype):
+    tc.check_mechanism(name, DEV, lib, dtype)
+
+
+def test_activation_branches(lib):
+    tc.check_activation_branches(DEV, lib)
+
+
+@pytest.mark.parametrize("dtype", [tc.F32, tc.BF16], ids=["fp32", "bf16"])
+@pytest.mark.parametrize("case", ["portions", "prompt_then_decode", "unequal_batch", "batched_decode", "reuse", "long_decode", "long_prompt", "first_tokens"])
+def test_feeding(lib, case, dtype):
+    getattr(tc, f"check_{case}")(DEV, lib, dtype)
+
+
+@pytest.mark.parametrize("window", [70, 64, 0])
+def test_single_keys(lib, window):
+    tc.check_single_keys(DEV, lib, window)
+
+
+def test_state_reaches_far_back(lib):
+    tc.check_far_state(DEV, lib)
+
+
+def test_greedy_generation_through_the_scheduler(lib):
+    tc.check_generation(DEV, lib)
+
+
+def test_sampling(lib):
+    tc.check_sampling(DEV, lib)
+
+
+def test_limits_and_errors(lib):
+    tc.check_limits(DEV, lib)
+
+
+def test_trace_replay(lib, tmp_path):
+    tc.check_replay(DEV, lib, tmp_path)
