@@ -36,8 +36,8 @@ def parse():
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=60)
     ap.add_argument("--warmup", type=int, default=12)
-    ap.add_argument("--workload", default="auto", choices=["auto", "duplex", "mimi", "lm", "served", "launchcheck"],
-                    help="served: the duplex step driven through the session batcher with HOST PCM in / PCM + tokens out "
+    ap.add_argument("--workload", default="auto", choices=["auto", "duplex", "mimi", "lm", "served", "launchcheck", "tlm"],
+                    help="tlm: token language models (bench_tlm.py, one GPU); served: the duplex step driven through the session batcher with HOST PCM in / PCM + tokens out "
                          "(pinned staging, H2D + D2H and one synchronisation per step included): the PCIe-inclusive rate")
     ap.add_argument("--batch", type=int, default=32, help="sessions per GPU (BASELINE.json configs[3]: 32)")
     ap.add_argument("--no-cpu-baseline", action="store_true")
@@ -60,6 +60,8 @@ def parse():
                     help="debug / tuning: move every session to this ring depth instead (overrides --kv-depth; not a named configuration)")
     ap.add_argument("--no-extras", action="store_true",
                     help="skip the extra figures of the default line: `full_context` (every session 3000 positions deep), `c3` (one session), `c5` (64 sessions, int8 x int8) and `c2` (the codec alone, 8 streams)")
+    ap.add_argument("--tlm-size", default="", help="tlm workload: only these sizes (comma separated widths)")
+    ap.add_argument("--tlm-batches", default="1,16,64", help="tlm workload: decode batches")
     ap.add_argument("--no-pin", action="store_true", help="do not pin the rank's host thread to its own block of cores")
     return ap.parse_args()
 
@@ -328,6 +330,11 @@ def main():
     rank, local, world, dist = dist_setup(args.gpus)
     dev = torch.device("cuda", local)
     cores = None if args.no_pin else pin_host_thread(rank, world)
+    if args.workload == "tlm":
+        if world != 1:
+            raise SystemExit("bench.py: --workload tlm runs on one GPU")
+        import bench_tlm
+        return bench_tlm.main(args, dev)
     from moshi_amd import MimiConfig, MimiModel
     from moshi_amd.weights import random_mimi_state_dict
 

@@ -195,6 +195,15 @@ __device__ __forceinline__ void mmi_store_relaxed_agent(unsigned* p, unsigned v)
     __hip_atomic_store(p, v, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
 }
 
+// The instruction scheduler moves nothing across this point: keeps a batch of loads issued ahead of the products that consume the batch
+// before it (left alone it sinks each load to its use when registers are short, and the loads then wait for one another)
+__device__ __forceinline__ void mmi_sched_barrier() { __builtin_amdgcn_sched_barrier(0); }
+// a value that is the same in every lane (a wave index, what was loaded through one), told to the compiler: it stays in scalar registers,
+// and loads addressed by it are scalar loads - they do not queue behind the vector loads in flight
+__device__ __forceinline__ int mmi_uniform(int v) { return __builtin_amdgcn_readfirstlane(v); }
+// true in every lane when any lane's flag is set
+__device__ __forceinline__ bool mmi_any(bool v) { return __any(v) != 0; }
+
 // streamed-once weights: non-temporal so they do not evict the activations / KV the other kernels reuse
 __device__ __forceinline__ u32x4 mmi_load_nt(const u32x4* p) { return __builtin_nontemporal_load(p); }
 __device__ __forceinline__ f32x4 mmi_load_nt(const f32x4* p) { return __builtin_nontemporal_load(p); }

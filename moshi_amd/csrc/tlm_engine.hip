@@ -16,9 +16,11 @@
 
 #include <math.h>
 #include <algorithm>
+#include <array>
 #include <map>
 #include <memory>
 #include <tuple>
+#include <type_traits>
 
 int64_t mmi_copy_launch_log(const std::vector<std::string>& log, char* buf, int64_t cap);
 
@@ -43,7 +45,7 @@ struct Layer {
     // latent attention
     Mat in, uqn, uqr, uk, uv;
     float *qw = nullptr, *cw = nullptr;
-    int qp = 0, kvp = 0, rp = 0, hp = 0, dim_p = 0, vdim_p = 0, lat_ks = 0, k_ks = 0, nd = 0, q_ks = 0;
+    int qp = 0, kvp = 0, rp = 0, hp = 0, dim_p = 0, vdim_p = 0, lat_ks = 0, k_ks = 0, nd = 0, q_ks = 0, qn_ks = 0;
     int rope = -1, geo = -1;
     // experts
     Mat up, down;
@@ -53,7 +55,7 @@ struct Layer {
 struct Run {                       // one execution of a layer: repeated layers share weights, not state
     int layer = 0;
     bool add_emb = false;
-    void *kc = nullptr, *vc = nullptr;
+    void* kc = nullptr;
     float* state = nullptr;
 };
 
@@ -80,6 +82,7 @@ struct Shape {                     // what a launch list depends on
     int T = 0, n_want = 0, n_entries = 0, n_seg = 0, nsplit = 1;
     bool pairs = false;            // some sequence spans several scan segments
     std::vector<int> tiles;        // attention column tiles per head count
+    std::vector<std::array<int, 2>> groups;        // column groups of 4 and of 8 tiles per head count
     Meta m;
     float* logits = nullptr;
     float* taps = nullptr;
@@ -137,6 +140,7 @@ namespace {
 
 constexpr int MAX_SPLIT = 8;
 constexpr int ROWS_MAX = 64;       // up to here a step takes the weight-streaming kernel
+constexpr int ATTN_TILE_GROUPS = 128;     // from this many column groups the attention stages keys through LDS
 constexpr int MAX_PARTIALS = 512;  // (column tile, split) pairs of the attention
 
 // ------------------------------------------------------------------------------------------------
@@ -263,6 +267,7 @@ int load_latent_attention(Loader& ld, Layer& L, const std::string& p) {
     L.k_ks = L.lat_ks + round_up(c.rot_dim, ks) / ks;
     L.nd = L.kvp / 16;
     L.q_ks = round_up(c.q_rank, ks) / ks;
+    L.qn_ks = H * L.dim_p / ks;
     auto turn = [&](int j) { return j / 2 + (j & 1) * (c.rot_dim / 2); };     // rotation partners side by side
     const mmi_tensor_desc* d;
     int rc;
@@ -403,7 +408,7 @@ int alloc_f32(mmi_tlm* m, float** p, size_t n) {
 
 int alloc_buffers(mmi_tlm* m) {
     const mmi_tlm_cfg& c = m->cfg;
-    const int T = m->max_T, ks = m->kstep;
+    const int T = m->max_T;
     int rc;
     m->split_elems = std::max((long)T, (long)MAX_SPLIT * ROWS_MAX);
     int gru_w = 0, y_ks = 0, lat_ld = 0, cq_ks = 0, qn_ks = 0, o_ks = 0, hid_ks = 0, gate_ld = 0, nd = 0;
@@ -415,7 +420,7 @@ int alloc_buffers(mmi_tlm* m) {
         } else {
             lat_ld = std::max(lat_ld, L.qp + L.kvp + L.rp + L.hp);
             cq_ks = std::max(cq_ks, L.q_ks);
-            qn_ks = std::max(qn_ks, L.c.heads * L.dim_p / ks);
+            qn_ks = std::max(qn_ks, L.qn_ks);
             q_elems = std::max(q_elems, (long)((T * (long)L.c.heads + 15) / 16) * L.k_ks);
             ao_elems = std::max(ao_elems, (long)((T * (long)L.c.heads + 15) / 16) * L.lat_ks);
             o_ks = std::max(o_ks, L.out.KS);
@@ -469,7 +474,7 @@ int alloc_buffers(mmi_tlm* m) {
     MMI_HIP_CHECK(m->scratch.alloc(&m->samp_zero, 1));
     MMI_HIP_CHECK(hipMemset(m->samp_zero, 0, sizeof(int)));
     // metadata: 4 ints per token + wanted rows, per-entry arrays, tile prefixes, segments, block-table updates
-    m->meta_cap = 64 + (size_t)5 * T + 4 * (size_t)m->max_slots + m->geo.size() * ((size_t)m->max_slots + 1) + 8 * ((size_t)T / TLM_SEG + m->max_slots + 1) +
+    m->meta_cap = 64 + (size_t)5 * T + 4 * (size_t)m->max_slots + 3 * m->geo.size() * ((size_t)m->max_slots + 1) + 8 * ((size_t)T / TLM_SEG + m->max_slots + 1) +
                   2 * ((size_t)T / TLM_PAGE + 2 * (size_t)m->max_slots + 2);
     MMI_HIP_CHECK(m->scratch.alloc(&m->meta, m->meta_cap));
     for (Staging& s : m->staging) {
@@ -487,14 +492,11 @@ int alloc_state(mmi_tlm* m) {
             MMI_HIP_CHECK(m->st.alloc(&r.state, n));
             MMI_HIP_CHECK(hipMemset(r.state, 0, n * sizeof(float)));
         } else {
-            const size_t nk = (size_t)m->max_pages * 4 * L.k_ks * 64, nv = (size_t)m->max_pages * L.nd * 16 * TLM_PAGE * m->esize / 16;
-            u32x4 *k = nullptr, *v = nullptr;
+            const size_t nk = (size_t)m->max_pages * 4 * L.k_ks * 64;
+            u32x4* k = nullptr;
             MMI_HIP_CHECK(m->st.alloc(&k, nk));
-            MMI_HIP_CHECK(m->st.alloc(&v, nv));
             MMI_HIP_CHECK(hipMemset(k, 0, nk * 16));      // masked keys of a block are multiplied by zero weights: never-written rows must be finite
-            MMI_HIP_CHECK(hipMemset(v, 0, nv * 16));
             r.kc = k;
-            r.vc = v;
         }
     }
     return MMI_OK;
@@ -543,31 +545,46 @@ TlmJob routed_job(mmi_tlm* m, const Layer& L, const Mat& w, const void* x, int x
     j.rblocks = std::min(pairs, std::min(L.c.experts, pairs) + pairs / plan_tile(p));      // every expert's run ends in at most one partial tile
     return j;
 }
+int rows_ntw(const Plan& p);
 // K split so that a product with few n-tiles still covers the chip; the consumer sums the fp32 partials
 int split_for(const Plan& p, const Mat& w, int blocks) {
     if (!p.rows) return 1;
     int s = 1;
-    while (s < MAX_SPLIT && blocks * s < 384 && w.KS / (2 * s) >= 8) s *= 2;
+    while (s < MAX_SPLIT && blocks * s < 384 * rows_ntw(p) && w.KS / (2 * s) >= 8) s *= 2;
     return s;
 }
 
+int rows_ntw(const Plan& p) { return p.mt; }                // n-tiles per workgroup of the weight-streaming kernel
 template <class Tr>
 int launch_jobs_t(hipStream_t s, const Plan& p, TlmJobs& J) {
-    long total = 0;
-    for (int i = 0; i < J.n; ++i) {
-        TlmJob& j = J.j[i];
-        if (!j.list) j.rblocks = mmi_cdiv(j.rows, plan_tile(p));
-        j.blocks = (p.rows ? j.NT : mmi_cdiv(j.NT, 2 * p.fm)) * (j.list ? 1 : j.groups) * j.ksplit * j.rblocks;
-        total += j.blocks;
-    }
-    const int grid = (int)total;
-    if (p.rows) {
-        if (p.mt == 1) MMI_LAUNCH((k_tlm_gemm_rows<Tr, 1, 8, 4>), grid, 512, 0, s, J);
-        else if (p.mt == 2) MMI_LAUNCH((k_tlm_gemm_rows<Tr, 2, 8, 2>), grid, 512, 0, s, J);
-        else MMI_LAUNCH((k_tlm_gemm_rows<Tr, 4, 8, 2>), grid, 512, 0, s, J);
-    } else {
-        if (p.fm == 4) MMI_LAUNCH((k_tlm_gemm_tile<Tr, 4, 4>), grid, 256, 0, s, J);
-        else MMI_LAUNCH((k_tlm_gemm_tile<Tr, 2, 2>), grid, 256, 0, s, J);
+    // the tiled kernel takes 256 features at a time where that still covers the chip
+    int fn = p.fm;
+    for (int pass = 0; pass < 2; ++pass) {
+        long total = 0;
+        if (!p.rows && p.fm == 4 && pass == 0) fn = 8;
+        for (int i = 0; i < J.n; ++i) {
+            TlmJob& j = J.j[i];
+            if (!j.list) j.rblocks = mmi_cdiv(j.rows, plan_tile(p));
+            j.blocks = (p.rows ? mmi_cdiv(j.NT, rows_ntw(p)) : mmi_cdiv(j.NT, 2 * fn)) * (j.list ? 1 : j.groups) * j.ksplit * j.rblocks;
+            total += j.blocks;
+        }
+        if (fn == 8 && total < 256) {
+            fn = 4;
+            continue;
+        }
+        const int grid = (int)total;
+        if (p.rows) {
+            if (p.mt == 1) MMI_LAUNCH((k_tlm_gemm_rows<Tr, 1, 1, 8, 4>), grid, 512, 0, s, J);
+            else if (p.mt == 2) MMI_LAUNCH((k_tlm_gemm_rows<Tr, 2, 2, 8, 2>), grid, 512, 0, s, J);
+            else MMI_LAUNCH((k_tlm_gemm_rows<Tr, 4, 4, 4, 2>), grid, 256, 0, s, J);
+        } else if (fn == 8) {
+            MMI_LAUNCH((k_tlm_gemm_tile<Tr, 8, 4, 1>), grid, 256, 0, s, J);
+        } else if (p.fm == 4) {
+            MMI_LAUNCH((k_tlm_gemm_tile<Tr, 4, 4, 2>), grid, 256, 0, s, J);
+        } else {
+            MMI_LAUNCH((k_tlm_gemm_tile<Tr, 2, 2, 2>), grid, 256, 0, s, J);
+        }
+        break;
     }
     MMI_CHECK_LAUNCH();
     return MMI_OK;
@@ -576,28 +593,43 @@ int launch_jobs(mmi_tlm* m, hipStream_t s, const Plan& p, TlmJobs J) {
     return m->f32 ? launch_jobs_t<TlmF32>(s, p, J) : launch_jobs_t<TlmBf16>(s, p, J);
 }
 
-template <class Tr, int WK>
-int launch_attn_w(hipStream_t s, dim3 grid, const TlmAttnArgs& a) {
-    if (a.nd <= 4) MMI_LAUNCH((k_tlm_attn<Tr, 4, WK>), grid, 256, 0, s, a);
-    else if (a.nd <= 8) MMI_LAUNCH((k_tlm_attn<Tr, 8, WK>), grid, 256, 0, s, a);
-    else if (a.nd <= 16) MMI_LAUNCH((k_tlm_attn<Tr, 16, WK>), grid, 256, 0, s, a);
-    else MMI_LAUNCH((k_tlm_attn<Tr, 32, WK>), grid, 256, 0, s, a);
-    MMI_CHECK_LAUNCH();
-    return MMI_OK;
+// the instantiation for a layer's latent blocks and rotated k-steps
+template <class Tr, class F>
+int attn_dispatch(int nd, int rk, F f) {
+    constexpr int R1 = 32 / Tr::KSTEP, R2 = 64 / Tr::KSTEP, R4 = 128 / Tr::KSTEP;
+#define TLM_ND(ND_)                                                                                                  \
+    if (nd <= ND_) {                                                                                                 \
+        if (rk <= R1) return f(std::integral_constant<int, ND_>(), std::integral_constant<int, R1>());               \
+        if (rk <= R2) return f(std::integral_constant<int, ND_>(), std::integral_constant<int, R2>());               \
+        return f(std::integral_constant<int, ND_>(), std::integral_constant<int, R4>());                             \
+    }
+    TLM_ND(4) TLM_ND(8) TLM_ND(16) TLM_ND(32)
+#undef TLM_ND
+    return mmi_fail(MMI_ERR_UNSUPPORTED, "latent too wide");
 }
+int attn_group_tiles(int nd, bool f32) { return nd <= (f32 ? 8 : 16) ? 8 : 4; }      // column tiles a workgroup of k_tlm_attn_tile takes (TlmAttnTile::QT)
+
 template <class Tr>
-int launch_attn_t(hipStream_t s, const TlmAttnArgs& a) {
-    int rc;
-    if (a.n_tiles >= 1024) {
-        if ((rc = launch_attn_w<Tr, 1>(s, dim3(mmi_cdiv(a.n_tiles, 4), 1), a))) return rc;
-    } else {
-        if ((rc = launch_attn_w<Tr, 4>(s, dim3(a.n_tiles, a.nsplit), a))) return rc;
-    }
-    if (a.nsplit > 1) {
-        MMI_LAUNCH((k_tlm_attn_combine<Tr>), a.n_tiles, 256, 0, s, a);
+int launch_attn_t(hipStream_t s, const TlmAttnArgs& a, bool tiled) {
+    const int rk = a.q_ks - a.out_ks;
+    return attn_dispatch<Tr>(a.nd, rk, [&](auto nd, auto rks) {
+        constexpr int ND = decltype(nd)::value, RK = decltype(rks)::value;
+        if constexpr (Tr::V == 8 || ND <= 16) if (tiled) {
+            constexpr size_t smem = TlmAttnTile<Tr, ND, RK>::smem();
+            static_assert(smem <= 160 * 1024, "LDS of a CU");
+            if (smem > 64 * 1024) {
+                static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(&k_tlm_attn_tile<Tr, ND, RK>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
+                MMI_HIP_CHECK(attr);
+            }
+            MMI_LAUNCH((k_tlm_attn_tile<Tr, ND, RK>), a.n_tiles, 256, smem, s, a);
+            MMI_CHECK_LAUNCH();
+            return (int)MMI_OK;
+        }
+        MMI_LAUNCH((k_tlm_attn<Tr, ND, RK>), dim3(round_up(a.n_tiles, 8), a.nsplit), 256, 0, s, a);
+        if (a.nsplit > 1) MMI_LAUNCH((k_tlm_attn_combine<Tr>), dim3(a.n_tiles, mmi_cdiv(a.nd, 8)), 256, 0, s, a);
         MMI_CHECK_LAUNCH();
-    }
-    return MMI_OK;
+        return (int)MMI_OK;
+    });
 }
 
 struct Carry {                    // what the next residual launch has to add
@@ -630,11 +662,12 @@ void add_resid(mmi_tlm* m, MmiProgram& P, const Shape& sh, const Carry& c, int e
     a.out = out;
     a.KS = m->h_ks;
     a.rows = rows;
-    const size_t smem = ((size_t)m->ld + 5 * (size_t)m->cfg.norm_groups + 8) * sizeof(float);
+    const int block = n <= 256 ? std::min(1024, std::max(256, round_up(m->ld / 4, 64))) : 256;     // few rows: one vector per thread
+    const size_t smem = ((size_t)m->ld + 2 * (size_t)m->cfg.norm_groups + block / 64 + 8) * sizeof(float);
     const bool f32 = m->f32;
     P.add([=](hipStream_t s) {
-        if (f32) MMI_LAUNCH((k_tlm_resid_norm<TlmF32>), n, 256, smem, s, a);
-        else MMI_LAUNCH((k_tlm_resid_norm<TlmBf16>), n, 256, smem, s, a);
+        if (f32) MMI_LAUNCH((k_tlm_resid_norm<TlmF32>), n, block, smem, s, a);
+        else MMI_LAUNCH((k_tlm_resid_norm<TlmBf16>), n, block, smem, s, a);
         MMI_CHECK_LAUNCH();
         return (int)MMI_OK;
     });
@@ -721,8 +754,6 @@ MixerOut build_latent_attention(mmi_tlm* m, MmiProgram& P, const Shape& sh, cons
     a.kc = r.kc;
     a.k_ks = L.k_ks;
     a.rot_k0 = L.lat_ks * m->kstep;
-    a.vc = r.vc;
-    a.nd = L.nd;
     a.gate = m->gate;
     a.gate_ld = H;
     P.site(site + "latent");
@@ -739,8 +770,7 @@ MixerOut build_latent_attention(mmi_tlm* m, MmiProgram& P, const Shape& sh, cons
     jn = dense_job(L.uqn, m->cq, L.q_ks, T);
     jn.epi = TLM_EPI_PACK;
     jn.out = m->qn;
-    const int qn_ks = H * L.dim_p / m->kstep;
-    jn.out_ld = qn_ks;
+    jn.out_ld = L.qn_ks;
     if (L.rp) {
         TlmJob& jr = Q.j[Q.n++];
         jr = dense_job(L.uqr, m->cq, L.q_ks, T);
@@ -759,7 +789,7 @@ MixerOut build_latent_attention(mmi_tlm* m, MmiProgram& P, const Shape& sh, cons
 
     memset(&Q, 0, sizeof(Q));
     TlmJob& jk = Q.j[Q.n++];
-    jk = dense_job(L.uk, m->qn, qn_ks, T);
+    jk = dense_job(L.uk, m->qn, L.qn_ks, T);
     jk.groups = H;
     jk.xkg = L.dim_p / m->kstep;
     jk.epi = TLM_EPI_PACK;
@@ -774,7 +804,6 @@ MixerOut build_latent_attention(mmi_tlm* m, MmiProgram& P, const Shape& sh, cons
     memset(&t, 0, sizeof(t));
     t.q = m->q;
     t.kc = r.kc;
-    t.vc = r.vc;
     t.out = m->ao;
     t.heads = H;
     t.q_ks = L.k_ks;
@@ -783,9 +812,12 @@ MixerOut build_latent_attention(mmi_tlm* m, MmiProgram& P, const Shape& sh, cons
     t.window = L.c.window;
     t.scale = L.c.scale * 1.44269504088896340736f;
     t.n_entries = sh.n_entries;
-    t.n_tiles = sh.tiles[L.geo];
-    t.nsplit = t.n_tiles >= 1024 ? 1 : std::max(1, std::min(sh.nsplit, MAX_PARTIALS / std::max(1, t.n_tiles)));
-    t.tile0 = m->meta + sh.m.tile0 + L.geo * (sh.n_entries + 1);
+    const bool wide = attn_group_tiles(L.nd, f32) == 8;
+    const bool tiled = sh.groups[L.geo][wide] >= ATTN_TILE_GROUPS && !(f32 && L.nd > 16);     // fp32 with a wide latent: the operands do not fit the registers
+    const int kind = tiled ? (wide ? 2 : 1) : 0;       // which of the three prefix arrays
+    t.n_tiles = tiled ? sh.groups[L.geo][kind - 1] : sh.tiles[L.geo];
+    t.nsplit = tiled ? 1 : std::max(1, std::min(sh.nsplit, (L.nd > 16 ? 256 : MAX_PARTIALS) / std::max(1, t.n_tiles)));     // (a wide latent: one workgroup per CU)
+    t.tile0 = m->meta + sh.m.tile0 + (3 * L.geo + kind) * (sh.n_entries + 1);
     t.erow0 = m->meta + sh.m.erow0;
     t.elen = m->meta + sh.m.elen;
     t.epos0 = m->meta + sh.m.epos0;
@@ -795,7 +827,7 @@ MixerOut build_latent_attention(mmi_tlm* m, MmiProgram& P, const Shape& sh, cons
     t.po = m->po;
     t.pml = m->pml;
     P.site(site + "attn");
-    P.add([=](hipStream_t s) { return f32 ? launch_attn_t<TlmF32>(s, t) : launch_attn_t<TlmBf16>(s, t); });
+    P.add([=](hipStream_t s) { return f32 ? launch_attn_t<TlmF32>(s, t, tiled) : launch_attn_t<TlmBf16>(s, t, tiled); });
 
     memset(&Q, 0, sizeof(Q));
     TlmJob& jv = Q.j[Q.n++];
@@ -1178,7 +1210,7 @@ extern "C" int mmi_tlm_step(mmi_tlm* m, int32_t n_entries, const int32_t* slots,
     M.elen = take(n_entries);
     M.epos0 = take(n_entries);
     M.eslot = take(n_entries);
-    M.tile0 = take((int)m->geo.size() * (n_entries + 1));
+    M.tile0 = take(3 * (int)m->geo.size() * (n_entries + 1));
     M.seg = take(8 * sh.n_seg);
     M.upd = at;
     M.total = at + 2 * (int)need;
@@ -1192,6 +1224,7 @@ extern "C" int mmi_tlm_step(mmi_tlm* m, int32_t n_entries, const int32_t* slots,
     int64_t blocks = 0;
     TlmSeg* sg = (TlmSeg*)(b + M.seg);
     sh.tiles.assign(m->geo.size(), 0);
+    sh.groups.assign(m->geo.size(), {0, 0});
     for (int e = 0; e < n_entries; ++e) {
         Slot& S = m->slots[slots[e]];
         for (int64_t n = pages_for(m, &S, counts[e]); n > 0; --n) {
@@ -1208,8 +1241,14 @@ extern "C" int mmi_tlm_step(mmi_tlm* m, int32_t n_entries, const int32_t* slots,
         b[M.epos0 + e] = (int)S.pos;
         b[M.eslot + e] = slots[e];
         for (size_t g = 0; g < m->geo.size(); ++g) {
-            b[M.tile0 + (int)g * (n_entries + 1) + e] = sh.tiles[g];
-            sh.tiles[g] += mmi_cdiv(counts[e] * m->geo[g], 16);
+            int* t = b + M.tile0 + 3 * (int)g * (n_entries + 1) + e;
+            const int n = mmi_cdiv(counts[e] * m->geo[g], 16);
+            t[0] = sh.tiles[g];
+            t[n_entries + 1] = sh.groups[g][0];
+            t[2 * (n_entries + 1)] = sh.groups[g][1];
+            sh.tiles[g] += n;
+            sh.groups[g][0] += mmi_cdiv(n, 4);
+            sh.groups[g][1] += mmi_cdiv(n, 8);
         }
         for (int o = 0, k = 0; o < counts[e]; o += TLM_SEG, ++k) {
             const int n = std::min(TLM_SEG, counts[e] - o);
@@ -1228,13 +1267,12 @@ extern "C" int mmi_tlm_step(mmi_tlm* m, int32_t n_entries, const int32_t* slots,
         S.pos += counts[e];
         S.par ^= 1;
     }
-    for (size_t g = 0; g < m->geo.size(); ++g) b[M.tile0 + (int)g * (n_entries + 1) + n_entries] = sh.tiles[g];
     for (int i = 0; i < n_want; ++i) b[M.want + i] = want[i];
     b[0] = upd;
-    // few column tiles and long contexts: split the keys over workgroups, at least 8 blocks of 32 keys each
+    // few column tiles and long contexts: split the keys over workgroups, at least 4 blocks of 32 keys each
     int tiles_max = 1;
     for (int t : sh.tiles) tiles_max = std::max(tiles_max, t);
-    while (sh.nsplit < 64 && tiles_max * sh.nsplit * 2 <= MAX_PARTIALS && blocks / (sh.nsplit * 2) >= 8) sh.nsplit *= 2;
+    while (sh.nsplit < 16 && tiles_max * sh.nsplit * 2 <= MAX_PARTIALS && blocks / (sh.nsplit * 2) >= 4) sh.nsplit *= 2;
     MMI_HIP_CHECK(hipMemcpyAsync(m->meta, b, (size_t)M.total * sizeof(int), hipMemcpyHostToDevice, s));
     MMI_HIP_CHECK(hipEventRecord(st.ev, s));
     st.used = true;

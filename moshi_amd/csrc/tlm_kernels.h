@@ -12,9 +12,9 @@
 //   weights      Wp[n-tile][k-step][lane][V]            (16-row tiles, zero padded; the layout of the Moshi LM's 16-row tile)
 //   activations  Xp[row / 16][k-step][lane][V]          (tlm_index; written by the producing epilogue)
 //   key cache    the same matrix with row = 64 page + offset: k = latent, then the rotated key part
-//   value cache  Vp[page][latent / 16][key group][lane][V]: the transposed operand.  Lane (d, kq), element e of a group of 4 V keys is
-//                key 16 (e / 4) + 4 kq + e % 4 - exactly the keys whose scores the same lane holds after S = K Q^T, so the softmax
-//                weights go from accumulator to operand without leaving the lane.
+//                There is no second copy for the values (the value IS the latent): the transposed operand of the value product comes out
+//                of the matrix core, K x identity (TlmFlip) - lane (d, kq) of its accumulators holds keys 4 kq .. 4 kq + 3, exactly the
+//                keys whose scores the same lane holds after S = K Q^T, so the softmax weights become an operand without leaving the lane.
 //   residual     x[token][ld] fp32
 #pragma once
 #include "mmi_common.h"
@@ -49,14 +49,6 @@ MMI_HD long tlm_index(long row, int k, int ks) {
 }
 
 constexpr int TLM_PAGE = 64;         // tokens per cache page
-
-// element of the value cache: latent dimension d of the token at `off` of a page (nd = 16-wide blocks of the latent)
-template <class Tr>
-MMI_HD long tlm_vindex(long page, int off, int d, int nd) {
-    constexpr int GK = 4 * Tr::V;                       // keys of one fragment
-    const int w = off % GK;
-    return (((page * nd + (d >> 4)) * (TLM_PAGE / GK) + off / GK) * 64 + ((w & 15) >> 2) * 16 + (d & 15)) * Tr::V + (w >> 4) * 4 + (w & 3);
-}
 
 __device__ __forceinline__ float tlm_sigmoid(float x) { return 1.0f / (1.0f + expf(-x)); }
 __device__ __forceinline__ float tlm_wave_sum(float x) {
@@ -194,12 +186,12 @@ struct TlmResidArgs {
     const int* rows;                     // row list (the residual is then not written back), or null
 };
 template <class Tr>
-__global__ __launch_bounds__(256) void k_tlm_resid_norm(TlmResidArgs a) {
+__global__ __launch_bounds__(1024) void k_tlm_resid_norm(TlmResidArgs a) {
     MMI_DYN_SHARED(float, row);          // [ld] the row, then [groups * parts] partial sums, then [groups] 1 / rms
-    const int tid = (int)threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int tid = (int)threadIdx.x, lane = tid & 63, wave = tid >> 6, nthr = (int)blockDim.x, nw = nthr >> 6;
     const int r = a.rows ? a.rows[blockIdx.x] : (int)blockIdx.x;
     float* x = a.x + (long)r * a.ld;
-    for (int k = 4 * tid; k < a.ld; k += 1024) {
+    for (int k = 4 * tid; k < a.ld; k += 4 * nthr) {
         f32x4 v = {0.f, 0.f, 0.f, 0.f}, ev = v;
         if (a.emb_mode != TLM_EMB_NONE) {
             const uint16_t* e = a.emb + (long)a.tok[r] * a.width + k;
@@ -213,12 +205,14 @@ __global__ __launch_bounds__(256) void k_tlm_resid_norm(TlmResidArgs a) {
             v = *reinterpret_cast<const f32x4*>(x + k);
             f32x4 d = {0.f, 0.f, 0.f, 0.f};
             if (a.mix) {
+#pragma unroll 8
                 for (int p = 0; p < a.mix_p; ++p) d += *reinterpret_cast<const f32x4*>(a.mix + p * a.mix_ps + (long)r * a.ld + k);
                 d *= *reinterpret_cast<const f32x4*>(a.ls1 + k);
             }
             if (a.dn) {
                 f32x4 f = {0.f, 0.f, 0.f, 0.f};
                 for (int c = 0; c < a.top; ++c)
+#pragma unroll 8
                     for (int p = 0; p < a.dn_p; ++p) f += *reinterpret_cast<const f32x4*>(a.dn + p * a.dn_ps + ((long)r * a.top + c) * a.ld + k);
                 d += f * (1.0f / (float)a.top) * *reinterpret_cast<const f32x4*>(a.ls2 + k);
             }
@@ -231,12 +225,12 @@ __global__ __launch_bounds__(256) void k_tlm_resid_norm(TlmResidArgs a) {
     }
     if (!a.out) return;                                       // uniform over the grid
     const int gs = a.width / a.groups;
-    const int parts = a.groups < 4 ? 4 / a.groups : 1;        // waves per group
+    const int parts = a.groups < nw ? nw / a.groups : 1;        // waves per group
     float* part = row + a.ld;
     float* inv = part + a.groups * parts;
     __syncthreads();
     const int per = (gs + parts - 1) / parts;
-    for (int t = wave; t < a.groups * parts; t += 4) {
+    for (int t = wave; t < a.groups * parts; t += nw) {
         const int g = t / parts, p = t - g * parts;
         const int lo = p * per, hi = lo + per < gs ? lo + per : gs;
         float s = 0.f;
@@ -245,14 +239,14 @@ __global__ __launch_bounds__(256) void k_tlm_resid_norm(TlmResidArgs a) {
         if (lane == 0) part[t] = s;
     }
     __syncthreads();
-    for (int g = tid; g < a.groups; g += 256) {
+    for (int g = tid; g < a.groups; g += nthr) {
         float s = 0.f;
         for (int p = 0; p < parts; ++p) s += part[g * parts + p];
         inv[g] = 1.0f / sqrtf(s / (float)gs + a.eps);
     }
     __syncthreads();
     typename Tr::elem* out = (typename Tr::elem*)a.out;
-    for (int k = 4 * tid; k < a.ld; k += 1024) {
+    for (int k = 4 * tid; k < a.ld; k += 4 * nthr) {
         f32x4 v = *reinterpret_cast<const f32x4*>(row + k);
         const f32x4 w = *reinterpret_cast<const f32x4*>(a.w + k);
 #pragma unroll
@@ -291,13 +285,13 @@ struct TlmJobs {
     int n;
 };
 
-template <class Tr>
+template <class Tr, int EPI>
 __device__ __forceinline__ void tlm_epilogue(const TlmJob& j, int g, int split, int id, int nt, int quad, f32x4 v) {
     const int n0 = nt * 16 + 4 * quad;
     const long orow = (long)id * j.out_mul + (long)g * j.out_gadd;
-    if (j.epi == TLM_EPI_F32) {
+    if constexpr (EPI == TLM_EPI_F32) {
         *reinterpret_cast<f32x4*>((float*)j.out + split * j.out_ps + orow * j.out_ld + n0) = v;
-    } else if (j.epi == TLM_EPI_PACK) {
+    } else if constexpr (EPI == TLM_EPI_PACK) {
         if (j.act == TLM_ACT_RELU2) {
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
@@ -307,12 +301,12 @@ __device__ __forceinline__ void tlm_epilogue(const TlmJob& j, int g, int split, 
         }
         if (j.gate) v *= j.gate[(long)id * j.gate_ld + g];
         Tr::store4((typename Tr::elem*)j.out + tlm_index<Tr>(orow, j.out_k0 + g * j.out_kg + n0, j.out_ld), v);
-    } else if (j.epi == TLM_EPI_ROPE) {
+    } else if constexpr (EPI == TLM_EPI_ROPE) {
         // rotation pairs are adjacent (the weight rows are interleaved at load)
         const f32x4 cs = *reinterpret_cast<const f32x4*>(j.rope + ((long)id * j.rope_ld + n0 / 2) * 2);
         const f32x4 o = {v[0] * cs[0] - v[1] * cs[1], v[1] * cs[0] + v[0] * cs[1], v[2] * cs[2] - v[3] * cs[3], v[3] * cs[2] + v[2] * cs[3]};
         Tr::store4((typename Tr::elem*)j.out + tlm_index<Tr>(orow, j.out_k0 + g * j.out_kg + n0, j.out_ld), o);
-    } else if (j.epi == TLM_EPI_GRU) {
+    } else if constexpr (EPI == TLM_EPI_GRU) {
         // n-tiles alternate gate, candidate, output gate of the same 16 channels
         const int kind = nt % 3, c = (nt / 3) * 16 + 4 * quad;
         const int w = j.out_ld;
@@ -333,16 +327,29 @@ __device__ __forceinline__ void tlm_epilogue(const TlmJob& j, int g, int split, 
     }
 }
 
-// Few rows (<= 16 MT per block): the weights are an HBM stream.  A workgroup owns one n-tile; its waves split K, each with U weight
-// fragments in flight per register buffer; partial tiles are summed through LDS in a fixed order.
-template <class Tr, int MT, int WAVES, int U>
-__global__ __launch_bounds__(WAVES * 64) void k_tlm_gemm_rows(TlmJobs jobs) {
+template <int E>
+struct TlmEpi { static constexpr int value = E; };
+// f(TlmEpi<kind>()) once per workgroup: the kinds' code is laid out one after the other, not interleaved per tile
+template <class F>
+__device__ __forceinline__ void tlm_with_epilogue(int epi, F f) {
+    if (epi == TLM_EPI_F32) f(TlmEpi<TLM_EPI_F32>());
+    else if (epi == TLM_EPI_PACK) f(TlmEpi<TLM_EPI_PACK>());
+    else if (epi == TLM_EPI_ROPE) f(TlmEpi<TLM_EPI_ROPE>());
+    else if (epi == TLM_EPI_GRU) f(TlmEpi<TLM_EPI_GRU>());
+    else f(TlmEpi<TLM_EPI_LOGITS>());
+}
+
+// Few rows (<= 16 MT per block): the weights are an HBM stream.  A workgroup owns NTW n-tiles; its waves split K, each with U k-steps
+// of weight fragments in flight per register buffer; partial tiles are summed through LDS in a fixed order.  Every activation fragment
+// (an L2 read) meets NTW weight fragments, so that with many rows the activations do not cost more than the weights.
+template <class Tr, int MT, int NTW, int WAVES, int U>
+__global__ __launch_bounds__(WAVES * 64, WAVES == 4 ? 2 : 1) void k_tlm_gemm_rows(TlmJobs jobs) {
     int b = (int)blockIdx.x, ji = 0;
     while (ji + 1 < jobs.n && b >= jobs.j[ji].blocks) b -= jobs.j[ji++].blocks;
-    const TlmJob& j = jobs.j[ji];
-    const int lane = (int)threadIdx.x & 63, wave = (int)threadIdx.x >> 6, bl = lane & 15;
-    const int nt = b % j.NT;
-    b /= j.NT;
+    const TlmJob j = jobs.j[ji];             // (a copy: its fields live in scalar registers)
+    const int lane = (int)threadIdx.x & 63, wave = mmi_uniform((int)threadIdx.x >> 6), bl = lane & 15;
+    const int ntb = (j.NT + NTW - 1) / NTW, nt0 = (b % ntb) * NTW;
+    b /= ntb;
     const int split = b % j.ksplit;
     b /= j.ksplit;
     int g = b % j.groups, rb = b / j.groups, r0 = rb * 16 * MT, n;
@@ -354,8 +361,7 @@ __global__ __launch_bounds__(WAVES * 64) void k_tlm_gemm_rows(TlmJobs jobs) {
     } else {
         n = j.rows - r0 < 16 * MT ? j.rows - r0 : 16 * MT;
     }
-    const int nm = (n + 15) >> 4;
-    int id[MT];
+    int id[MT];                                               // rows past n repeat the last one, and are dropped at the end
     const u32x4* xq[MT];
 #pragma unroll
     for (int m = 0; m < MT; ++m) {
@@ -369,63 +375,96 @@ __global__ __launch_bounds__(WAVES * 64) void k_tlm_gemm_rows(TlmJobs jobs) {
     const int s0 = min(j.KS, split * sper), s1 = min(j.KS, s0 + sper);
     const int wper = (s1 - s0 + WAVES - 1) / WAVES;
     const int k0 = min(s1, s0 + wave * wper), nk = min(s1, k0 + wper) - k0;
-    const u32x4* wq = j.wp + (long)g * j.wgs + ((long)nt * j.KS + k0) * 64 + lane;
-    f32x4 acc[MT];
+    const u32x4* wq[NTW];
 #pragma unroll
-    for (int m = 0; m < MT; ++m) acc[m] = f32x4{0.f, 0.f, 0.f, 0.f};
-    u32x4 wA[U], wB[U], xA[MT][U], xB[MT][U];
+    for (int t = 0; t < NTW; ++t) wq[t] = j.wp + (long)g * j.wgs + ((long)min(nt0 + t, j.NT - 1) * j.KS + k0) * 64 + lane;
+    f32x4 acc[NTW][MT];
+#pragma unroll
+    for (int t = 0; t < NTW; ++t)
+#pragma unroll
+        for (int m = 0; m < MT; ++m) acc[t][m] = f32x4{0.f, 0.f, 0.f, 0.f};
+    u32x4 wA[U][NTW], wB[U][NTW], xA[U][MT], xB[U][MT];
 #define TLM_LOAD(W_, X_, base)                                                                              \
     _Pragma("unroll") for (int u = 0; u < U; ++u) {                                                         \
-        const int k_ = (base) + u < nk ? (base) + u : nk - 1;                                               \
-        W_[u] = mmi_load_nt(wq + (long)k_ * 64);                                                            \
-        _Pragma("unroll") for (int m = 0; m < MT; ++m) if (m < nm) X_[m][u] = xq[m][(long)(k0 + k_) * 64];  \
+        _Pragma("unroll") for (int t = 0; t < NTW; ++t) W_[u][t] = mmi_load_nt(wq[t] + (long)((base) + u) * 64); \
+        _Pragma("unroll") for (int m = 0; m < MT; ++m) X_[u][m] = xq[m][(long)(k0 + (base) + u) * 64];      \
     }
-#define TLM_MMA(W_, X_, base)                                                                               \
-    _Pragma("unroll") for (int u = 0; u < U; ++u)                                                           \
-        if ((base) + u < nk) {                                                                              \
-            _Pragma("unroll") for (int m = 0; m < MT; ++m) if (m < nm) acc[m] = Tr::mfma(W_[u], X_[m][u], acc[m]); \
-        }
-    if (nk > 0) {
+#define TLM_MMA1(W_, X_, u)                                                                                 \
+        _Pragma("unroll") for (int m = 0; m < MT; ++m)                                                      \
+            _Pragma("unroll") for (int t = 0; t < NTW; ++t) acc[t][m] = Tr::mfma(W_[u][t], X_[u][m], acc[t][m]);
+#define TLM_MMA(W_, X_)                                                                                     \
+    _Pragma("unroll") for (int u = 0; u < U; ++u) { TLM_MMA1(W_, X_, u) }
+    // no load of the steady state is conditional, so that the wait before a product only covers the older buffer
+    const int nfull = nk / U, rem = nk - nfull * U;
+    if (nfull > 0) {
         TLM_LOAD(wA, xA, 0);
-        for (int k = 0;;) {
-            if (k + U < nk) { TLM_LOAD(wB, xB, k + U); }
-            TLM_MMA(wA, xA, k);
-            k += U;
-            if (k >= nk) break;
-            if (k + U < nk) { TLM_LOAD(wA, xA, k + U); }
-            TLM_MMA(wB, xB, k);
-            k += U;
-            if (k >= nk) break;
+        int i = 0;
+        for (; i + 2 < nfull; i += 2) {
+            TLM_LOAD(wB, xB, (i + 1) * U);
+            mmi_sched_barrier();
+            TLM_MMA(wA, xA);
+            TLM_LOAD(wA, xA, (i + 2) * U);
+            mmi_sched_barrier();
+            TLM_MMA(wB, xB);
+        }
+        if (nfull - i == 2) {
+            TLM_LOAD(wB, xB, (i + 1) * U);
+            mmi_sched_barrier();
+            TLM_MMA(wA, xA);
+            TLM_MMA(wB, xB);
+        } else {
+            TLM_MMA(wA, xA);
         }
     }
+    if (rem > 0) {                                            // fewer than U k-steps: requested together, from valid addresses
+#pragma unroll
+        for (int u = 0; u < U - 1; ++u) {
+            const int k = nfull * U + min(u, rem - 1);
+#pragma unroll
+            for (int t = 0; t < NTW; ++t) wA[u][t] = mmi_load_nt(wq[t] + (long)k * 64);
+#pragma unroll
+            for (int m = 0; m < MT; ++m) xA[u][m] = xq[m][(long)(k0 + k) * 64];
+        }
+#pragma unroll
+        for (int u = 0; u < U - 1; ++u)
+            if (u < rem) { TLM_MMA1(wA, xA, u) }
+    }
+#undef TLM_MMA1
 #undef TLM_LOAD
 #undef TLM_MMA
-    MMI_SHARED __attribute__((aligned(16))) f32x4 red[WAVES * MT * 64];
+    MMI_SHARED __attribute__((aligned(16))) f32x4 red[WAVES * NTW * MT * 64];
 #pragma unroll
-    for (int m = 0; m < MT; ++m) red[(wave * MT + m) * 64 + lane] = acc[m];
+    for (int t = 0; t < NTW; ++t)
+#pragma unroll
+        for (int m = 0; m < MT; ++m) red[((wave * NTW + t) * MT + m) * 64 + lane] = acc[t][m];
     __syncthreads();
+    tlm_with_epilogue(j.epi, [&](auto epi) __attribute__((always_inline)) {
 #pragma unroll
-    for (int m = 0; m < MT; ++m) {
-        if (m % WAVES != wave || m * 16 + bl >= n) continue;
-        f32x4 v = red[m * 64 + lane];
+        for (int t = 0; t < NTW; ++t)
 #pragma unroll
-        for (int w = 1; w < WAVES; ++w) v += red[(w * MT + m) * 64 + lane];
-        tlm_epilogue<Tr>(j, g, split, id[m], nt, lane >> 4, v);
-    }
+            for (int m = 0; m < MT; ++m) {
+                if ((t * MT + m) % WAVES != wave || m * 16 + bl >= n || nt0 + t >= j.NT) continue;
+                f32x4 v = red[(t * MT + m) * 64 + lane];
+#pragma unroll
+                for (int w = 1; w < WAVES; ++w) v += red[((w * NTW + t) * MT + m) * 64 + lane];
+                tlm_epilogue<Tr, decltype(epi)::value>(j, g, split, id[m], nt0 + t, lane >> 4, v);
+            }
+    });
 }
 
-// Many rows: 2 x 2 waves over a tile of 32 FN features x 32 FM rows, two k-steps per stage, double-buffered in LDS.  Operands arrive
-// as whole fragments (one 16-byte vector per lane), so staging and operand reads are conflict-free without a swizzle.
-template <class Tr, int FN, int FM>
-__global__ __launch_bounds__(256) void k_tlm_gemm_tile(TlmJobs jobs) {
+// Many rows: 2 x 2 waves over a tile of 32 FN features x 32 FM rows, SK k-steps per stage, double-buffered in LDS, with the loads of the
+// two stages after the current one in flight in registers.  Operands arrive as whole fragments (one 16-byte vector per lane), so
+// staging and operand reads are conflict-free without a swizzle.
+template <class Tr, int FN, int FM, int SK>
+__global__ __launch_bounds__(256, 2) void k_tlm_gemm_tile(TlmJobs jobs) {
     constexpr int NF = 2 * FN + 2 * FM, NI = NF / 4;          // fragments per k-step; per wave
-    MMI_SHARED __attribute__((aligned(16))) u32x4 lds[2 * 2 * NF * 64];
+    MMI_SHARED __attribute__((aligned(16))) u32x4 lds[2 * SK * NF * 64];
     // consecutive workgroups go round the 8 XCDs: give each XCD a contiguous run of tiles so that its L2 sees the shared operand
     const int nb = (int)gridDim.x, xper = nb >> 3, xrem = nb & 7, xcd = (int)blockIdx.x & 7;
     int b = xcd * xper + (xcd < xrem ? xcd : xrem) + ((int)blockIdx.x >> 3), ji = 0;
     while (ji + 1 < jobs.n && b >= jobs.j[ji].blocks) b -= jobs.j[ji++].blocks;
-    const TlmJob& j = jobs.j[ji];
-    const int lane = (int)threadIdx.x & 63, wave = (int)threadIdx.x >> 6, bl = lane & 15;
+    const TlmJob j = jobs.j[ji];             // (a copy: its fields live in scalar registers)
+    const int lane = (int)threadIdx.x & 63, wave = mmi_uniform((int)threadIdx.x >> 6), bl = lane & 15;
     const int ntb = (j.NT + 2 * FN - 1) / (2 * FN);
     int g, rb, nb0, n, r0;
     if (j.list) {
@@ -444,18 +483,19 @@ __global__ __launch_bounds__(256) void k_tlm_gemm_tile(TlmJobs jobs) {
         n = j.rows - r0 < 32 * FM ? j.rows - r0 : 32 * FM;
     }
     const int nt0 = nb0 * 2 * FN;
-    const u32x4* src[NI];
+    const u32x4* wbase = j.wp + (long)g * j.wgs;
+    int off[NI];                                              // fragment i of this wave, lane: 16-byte vectors from its operand's base
 #pragma unroll
     for (int i = 0; i < NI; ++i) {
         const int f = wave + 4 * i;
-        if (f < 2 * FN) {
+        if (4 * i < 2 * FN) {
             const int nt = nt0 + f < j.NT ? nt0 + f : j.NT - 1;
-            src[i] = j.wp + (long)g * j.wgs + (long)nt * j.KS * 64 + lane;
+            off[i] = nt * j.KS * 64 + lane;
         } else {
             const int m = (f - 2 * FN) * 16 + bl, ii = m < n ? m : n - 1;
             const int id = j.list ? j.list[r0 + ii] : r0 + ii;
             const long in = j.list ? id / j.in_div : (long)id * j.in_mul + (long)g * j.in_gadd;
-            src[i] = j.xp + ((in >> 4) * j.xks + (long)g * j.xkg) * 64 + (in & 15) + (lane >> 4) * 16;
+            off[i] = (int)((in >> 4) * j.xks + (long)g * j.xkg) * 64 + (int)(in & 15) + (lane >> 4) * 16;
         }
     }
     const int wn = wave & 1, wm = wave >> 1;
@@ -464,54 +504,60 @@ __global__ __launch_bounds__(256) void k_tlm_gemm_tile(TlmJobs jobs) {
     for (int x = 0; x < FN; ++x)
 #pragma unroll
         for (int y = 0; y < FM; ++y) acc[x][y] = f32x4{0.f, 0.f, 0.f, 0.f};
-    u32x4 st[2][NI];
-#define TLM_FETCH(k)                                                                       \
-    _Pragma("unroll") for (int kk = 0; kk < 2; ++kk) {                                     \
-        const int k_ = (k) + kk < j.KS ? (k) + kk : j.KS - 1;                              \
-        _Pragma("unroll") for (int i = 0; i < NI; ++i) st[kk][i] = src[i][(long)k_ * 64];  \
+    u32x4 st[2][SK][NI];
+#define TLM_FETCH(set, stage)                                                                   \
+    _Pragma("unroll") for (int kk = 0; kk < SK; ++kk) {                                         \
+        const int k_ = (stage) * SK + kk < j.KS ? (stage) * SK + kk : j.KS - 1;                 \
+        _Pragma("unroll") for (int i = 0; i < NI; ++i) st[set][kk][i] = (4 * i < 2 * FN ? wbase : j.xp)[(unsigned)(off[i] + k_ * 64)];  \
     }
-#define TLM_STAGE(buf)                                                                     \
-    _Pragma("unroll") for (int kk = 0; kk < 2; ++kk)                                       \
-        _Pragma("unroll") for (int i = 0; i < NI; ++i) lds[(((buf) * 2 + kk) * NF + wave + 4 * i) * 64 + lane] = st[kk][i];
-    TLM_FETCH(0);
-    TLM_STAGE(0);
-    __syncthreads();
-    int cur = 0;
-    for (int k = 0; k < j.KS; k += 2) {
-        const bool more = k + 2 < j.KS;
-        if (more) { TLM_FETCH(k + 2); }
-#pragma unroll
-        for (int kk = 0; kk < 2; ++kk) {
-            if (k + kk < j.KS) {
-                const u32x4* base = lds + ((cur * 2 + kk) * NF) * 64 + lane;
-                u32x4 av[FN], bv[FM];
-#pragma unroll
-                for (int x = 0; x < FN; ++x) av[x] = base[(wn * FN + x) * 64];
-#pragma unroll
-                for (int y = 0; y < FM; ++y) bv[y] = base[(2 * FN + wm * FM + y) * 64];
-#pragma unroll
-                for (int x = 0; x < FN; ++x)
-#pragma unroll
-                    for (int y = 0; y < FM; ++y) acc[x][y] = Tr::mfma(av[x], bv[y], acc[x][y]);
-            }
+#define TLM_STAGE(set, buf)                                                                     \
+    _Pragma("unroll") for (int kk = 0; kk < SK; ++kk)                                           \
+        _Pragma("unroll") for (int i = 0; i < NI; ++i) lds[(((buf) * SK + kk) * NF + wave + 4 * i) * 64 + lane] = st[set][kk][i];
+#define TLM_COMPUTE(buf, stage)                                                                 \
+    _Pragma("unroll") for (int kk = 0; kk < SK; ++kk)                                           \
+        if ((stage) * SK + kk < j.KS) {                                                         \
+            const u32x4* base = lds + (((buf) * SK + kk) * NF) * 64 + lane;                     \
+            u32x4 bv[FM];                                                                       \
+            _Pragma("unroll") for (int y = 0; y < FM; ++y) bv[y] = base[(2 * FN + wm * FM + y) * 64]; \
+            _Pragma("unroll") for (int x = 0; x < FN; ++x) {                                    \
+                const u32x4 av = base[(wn * FN + x) * 64];                                      \
+                _Pragma("unroll") for (int y = 0; y < FM; ++y) acc[x][y] = Tr::mfma(av, bv[y], acc[x][y]); \
+            }                                                                                   \
         }
-        if (more) { TLM_STAGE(cur ^ 1); }
+    // (fetches past the end repeat the last k-step: an unconditional load keeps the wait in front of a stage to the older set)
+    const int ns = (j.KS + SK - 1) / SK;
+    TLM_FETCH(0, 0);
+    TLM_FETCH(1, 1);
+    TLM_STAGE(0, 0);
+    __syncthreads();
+    for (int s = 0; s < ns; s += 2) {                         // stage s in buffer 0 and register set 0, stage s + 1 in 1 and 1
+        TLM_FETCH(0, s + 2);
+        mmi_sched_barrier();
+        TLM_COMPUTE(0, s);
+        TLM_STAGE(1, 1);
         __syncthreads();
-        cur ^= 1;
+        TLM_FETCH(1, s + 3);
+        mmi_sched_barrier();
+        TLM_COMPUTE(1, s + 1);
+        TLM_STAGE(0, 0);
+        __syncthreads();
     }
+#undef TLM_COMPUTE
 #undef TLM_FETCH
 #undef TLM_STAGE
+    tlm_with_epilogue(j.epi, [&](auto epi) __attribute__((always_inline)) {
 #pragma unroll
-    for (int y = 0; y < FM; ++y) {
-        const int m = (wm * FM + y) * 16 + bl;
-        if (m >= n) continue;
-        const int id = j.list ? j.list[r0 + m] : r0 + m;
+        for (int y = 0; y < FM; ++y) {
+            const int m = (wm * FM + y) * 16 + bl;
+            if (m >= n) continue;
+            const int id = j.list ? j.list[r0 + m] : r0 + m;
 #pragma unroll
-        for (int x = 0; x < FN; ++x) {
-            const int nt = nt0 + wn * FN + x;
-            if (nt < j.NT) tlm_epilogue<Tr>(j, g, 0, id, nt, lane >> 4, acc[x][y]);
+            for (int x = 0; x < FN; ++x) {
+                const int nt = nt0 + wn * FN + x;
+                if (nt < j.NT) tlm_epilogue<Tr, decltype(epi)::value>(j, g, 0, id, nt, lane >> 4, acc[x][y]);
+            }
         }
-    }
+    });
 }
 
 // ------------------------------------------------------------------------------------------------
@@ -528,7 +574,6 @@ struct TlmLatentArgs {
     const int* crow;                                     // cache row of the token: 64 page + offset
     void* q; int q_ks;
     void* kc; int k_ks, rot_k0;
-    void* vc; int nd;
     float* gate; int gate_ld;
 };
 template <class Tr>
@@ -540,6 +585,7 @@ __global__ __launch_bounds__(256) void k_tlm_latent(TlmLatentArgs a) {
     float sq = 0.f, sc = 0.f;
     for (int k = 4 * tid; k < a.ld; k += 1024) {
         f32x4 v = *reinterpret_cast<const f32x4*>(a.in + (long)t * a.ld + k);
+#pragma unroll 4
         for (int p = 1; p < a.in_p; ++p) v += *reinterpret_cast<const f32x4*>(a.in + p * a.in_ps + (long)t * a.ld + k);
         *reinterpret_cast<f32x4*>(row + k) = v;
         const float s = v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];     // the padding columns are zero
@@ -556,8 +602,6 @@ __global__ __launch_bounds__(256) void k_tlm_latent(TlmLatentArgs a) {
     const float iq = 1.0f / sqrtf((part[0][0] + part[0][1] + part[0][2] + part[0][3]) / (float)a.q_rank + a.eps);
     const float ic = 1.0f / sqrtf((part[1][0] + part[1][1] + part[1][2] + part[1][3]) / (float)a.kv_rank + a.eps);
     const long cr = a.crow[t];
-    const long page = cr / TLM_PAGE;
-    const int off = (int)(cr % TLM_PAGE);
     for (int k = 4 * tid; k < a.ld; k += 1024) {
         f32x4 v = *reinterpret_cast<const f32x4*>(row + k);
         if (k < a.qp) {
@@ -567,8 +611,6 @@ __global__ __launch_bounds__(256) void k_tlm_latent(TlmLatentArgs a) {
             const int d = k - a.qp;
             v *= ic * *reinterpret_cast<const f32x4*>(a.cw + d);
             Tr::store4((elem*)a.kc + tlm_index<Tr>(cr, d, a.k_ks), v);
-#pragma unroll
-            for (int e = 0; e < 4; ++e) ((elem*)a.vc)[tlm_vindex<Tr>(page, off, d + e, a.nd)] = Tr::cvt(v[e]);
         } else if (k < a.qp + a.kvp + a.rp) {
             const int d = k - a.qp - a.kvp;
             const f32x4 cs = *reinterpret_cast<const f32x4*>(a.rope + ((long)t * a.rope_ld + d / 2) * 2);
@@ -590,13 +632,12 @@ __global__ __launch_bounds__(256) void k_tlm_latent(TlmLatentArgs a) {
 struct TlmAttnArgs {
     const void* q;                       // packed rows token * heads + head
     const void* kc;
-    const void* vc;
     void* out;                           // packed rows token * heads + head, latent columns
     int heads, q_ks, nd, out_ks;
     int window;                          // 0: every earlier position
     float scale;                         // times log2(e)
     int n_entries, n_tiles, nsplit;
-    const int* tile0;                    // [entries + 1] first column tile of each entry
+    const int* tile0;                    // [entries + 1] first column tile (k_tlm_attn_tile: column group) of each entry
     const int* erow0; const int* elen; const int* epos0; const int* eslot;
     const int* block_table; int bt_ld;   // [slot][bt_ld]: page of positions 64 i .. at i % bt_ld
     float* po;                           // nsplit > 1: [tile][split][nd][64] f32x4 un-normalised sums
@@ -604,12 +645,10 @@ struct TlmAttnArgs {
 };
 struct TlmCols { int entry, c0, ncol; };
 __device__ __forceinline__ TlmCols tlm_find_tile(const TlmAttnArgs& a, int tile) {
-    int lo = 0, hi = a.n_entries - 1;
-    while (lo < hi) {                                   // last entry whose first tile is <= tile
-        const int mid = (lo + hi + 1) >> 1;
-        if (a.tile0[mid] <= tile) lo = mid;
-        else hi = mid - 1;
-    }
+    // the last entry whose first tile is <= tile: all prefixes compared at once (a binary search would be a chain of dependent loads)
+    unsigned below = 0;
+    for (int e = mmi_lane(); e < a.n_entries; e += 64) below += a.tile0[e] <= tile ? 1u : 0u;
+    const int lo = mmi_uniform((int)mmi_wave_sum_u32(below) - 1);
     TlmCols c;
     c.entry = lo;
     c.c0 = (tile - a.tile0[lo]) * 16;
@@ -625,17 +664,167 @@ __device__ __forceinline__ void tlm_attn_store(const TlmAttnArgs& a, const TlmCo
     Tr::store4((typename Tr::elem*)a.out + tlm_index<Tr>(orow, db * 16 + 4 * kq, a.out_ks), v);
 }
 
-// ND: bound on the 16-wide latent blocks.  WK waves of a workgroup share one column tile (each takes every WK-th key block; their
-// sums meet in LDS), the other 4 / WK groups take further tiles.
-template <class Tr, int ND, int WK>
+// Shapes are template bounds - ND 16-wide latent blocks, RK k-steps of the rotated part - and the loops run over the bounds without a
+// branch, so that a block's loads are all in flight together: fragments past the model's own sizes repeat a valid address against zero
+// query fragments, value blocks past them are dropped at the end.
+template <class Tr, int ND, int RK>
+struct TlmQuery {
+    static constexpr int LK = ND * 16 / Tr::KSTEP, NK = LK + RK;
+    static constexpr int NB = 32 / (4 * Tr::V);                    // value fragments per 32 keys and latent block
+    u32x4 f[NK];
+    static __device__ __forceinline__ u32x4 fragment(const TlmAttnArgs& a, const u32x4* qp, int s) {
+        const int o = s < LK ? s : a.out_ks + s - LK;
+        const u32x4 zero = {0u, 0u, 0u, 0u};
+        return (s < LK ? s < a.out_ks : o < a.q_ks) ? qp[o * 64] : zero;
+    }
+    __device__ __forceinline__ void load(const TlmAttnArgs& a, long qrow, int kq) {
+        const u32x4* qp = (const u32x4*)a.q + (qrow >> 4) * a.q_ks * 64 + kq * 16 + (qrow & 15);
+#pragma unroll
+        for (int s = 0; s < NK; ++s) f[s] = fragment(a, qp, s);
+    }
+};
+// 32 (16 at fp32) keys x KSTEP latent dimensions -> the transposed operand, through the matrix core: K x identity is exact
+template <class Tr>
+struct TlmFlip {
+    static constexpr int H = Tr::KSTEP / 16;                       // 16-wide latent blocks per k-step
+    u32x4 id[H];
+    __device__ __forceinline__ void init(int bl, int kq) {
+#pragma unroll
+        for (int h = 0; h < H; ++h) {
+            if constexpr (Tr::V == 8) {
+                const int e = 16 * h + bl - 8 * kq;                // k = 8 kq + e meets column bl where k = 16 h + bl
+#pragma unroll
+                for (int i = 0; i < 4; ++i) id[h][i] = e == 2 * i ? 0x00003f80u : (e == 2 * i + 1 ? 0x3f800000u : 0u);
+            } else {
+#pragma unroll
+                for (int i = 0; i < 4; ++i) id[h][i] = 4 * kq + i == bl ? 0x3f800000u : 0u;
+            }
+        }
+    }
+    // bf16: latent block h of the two 16-key fragments of a k-step; fp32: of one
+    __device__ __forceinline__ u32x4 turn(u32x4 k0, u32x4 k1, int h) const {
+        const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+        const f32x4 a = Tr::mfma(k0, id[h], zero);
+        if constexpr (Tr::V == 8) {
+            const f32x4 b = Tr::mfma(k1, id[h], zero);
+            return u32x4{mmi_pack_bf16x2(a[0], a[1]), mmi_pack_bf16x2(a[2], a[3]), mmi_pack_bf16x2(b[0], b[1]), mmi_pack_bf16x2(b[2], b[3])};
+        } else {
+            return __builtin_bit_cast(u32x4, a);
+        }
+    }
+};
+// k-step of the cache that fragment s of the bound stands for
+template <int LK>
+__device__ __forceinline__ int tlm_kstep_of(const TlmAttnArgs& a, int s) {
+    return s < LK ? min(s, a.out_ks - 1) : min(a.out_ks + s - LK, a.q_ks - 1);
+}
+// scores of 32 keys -> softmax weights as operand fragments, the running maximum and sum moved on; returns the factor of older sums
+template <class Tr>
+__device__ __forceinline__ float tlm_softmax_block(const TlmAttnArgs& a, f32x4 s0, f32x4 s1, int d0, float& m, float& l, u32x4 (&pf)[32 / (4 * Tr::V)]) {
+    constexpr int NB = 32 / (4 * Tr::V);
+    float mx = m;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+        const int e0 = d0 - r, e1 = d0 - r - 16;
+        s0[r] = e0 >= 0 && (a.window <= 0 || e0 < a.window) ? s0[r] * a.scale : -INFINITY;
+        s1[r] = e1 >= 0 && (a.window <= 0 || e1 < a.window) ? s1[r] * a.scale : -INFINITY;
+        mx = fmaxf(mx, fmaxf(s0[r], s1[r]));
+    }
+    mx = fmaxf(mx, mmi_shfl_xor(mx, 16));
+    mx = fmaxf(mx, mmi_shfl_xor(mx, 32));
+    const float al = exp2f(m - mx);
+    m = mx;
+    l *= al;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+        s0[r] = exp2f(s0[r] - mx);
+        s1[r] = exp2f(s1[r] - mx);
+        l += s0[r] + s1[r];
+    }
+    if constexpr (NB == 1) {
+        pf[0] = u32x4{mmi_pack_bf16x2(s0[0], s0[1]), mmi_pack_bf16x2(s0[2], s0[3]), mmi_pack_bf16x2(s1[0], s1[1]), mmi_pack_bf16x2(s1[2], s1[3])};
+    } else {
+        pf[0] = __builtin_bit_cast(u32x4, s0);
+        pf[NB - 1] = __builtin_bit_cast(u32x4, s1);
+    }
+    return al;
+}
+
+// One block of 32 keys as a stream of fragments out of LDS - keys 0-15 and 16-31 of every k-step, then the turned values - consumed in
+// groups of G, the next group read while one is used.
+template <class Tr, int ND, int RK, int QT, int G>
+struct TlmAttnStream {
+    typedef TlmQuery<Tr, ND, RK> Q;
+    static constexpr int NB = Q::NB, NK = Q::NK, F = 2 * NK + ND * NB, NG = ((F + G - 1) / G + 1) / 2 * 2;      // an even number of groups: group g always meets buffer g & 1
+    u32x4 fr[2][G];
+    f32x4 s[QT][2];
+    u32x4 pf[QT][NB];
+    float m[QT], l[QT];
+    f32x4 acc[QT][ND];
+    __device__ __forceinline__ void clear() {
+#pragma unroll
+        for (int t = 0; t < QT; ++t) {
+            m[t] = -1e30f;
+            l[t] = 0.f;
+#pragma unroll
+            for (int d = 0; d < ND; ++d) acc[t][d] = f32x4{0.f, 0.f, 0.f, 0.f};
+        }
+    }
+    // at(f): address of fragment f for this lane
+    template <class At>
+    __device__ __forceinline__ void load(int buf, int g, At at) {
+#pragma unroll
+        for (int i = 0; i < G; ++i)
+            if (g * G + i < F) fr[buf][i] = *at(g * G + i);
+    }
+    // q(t, k): query fragment k of column tile t
+    template <class Qf>
+    __device__ __forceinline__ void use(const TlmAttnArgs& a, Qf q, int buf, int g, const int (&d0)[QT]) {
+#pragma unroll
+        for (int i = 0; i < G; ++i) {
+            const int f = g * G + i;
+            if (f >= F) continue;
+            if (f < 2 * NK) {
+#pragma unroll
+                for (int t = 0; t < QT; ++t) s[t][f & 1] = Tr::mfma(fr[buf][i], q(t, f >> 1), f < 2 ? f32x4{0.f, 0.f, 0.f, 0.f} : s[t][f & 1]);
+                if (f == 2 * NK - 1) soften(a, d0);
+            } else {
+                const int d = (f - 2 * NK) / NB;
+#pragma unroll
+                for (int t = 0; t < QT; ++t) acc[t][d] = Tr::mfma(fr[buf][i], pf[t][(f - 2 * NK) % NB], acc[t][d]);
+            }
+        }
+    }
+    // scores -> softmax weights; the sums so far are rescaled when some column's maximum has moved
+    __device__ __forceinline__ void soften(const TlmAttnArgs& a, const int (&d0)[QT]) {
+        float al[QT];
+        bool moved = false;
+#pragma unroll
+        for (int t = 0; t < QT; ++t) {
+            al[t] = tlm_softmax_block<Tr>(a, s[t][0], s[t][1], d0[t], m[t], l[t], pf[t]);
+            moved = moved || al[t] != 1.f;
+        }
+        if (mmi_any(moved)) {
+#pragma unroll
+            for (int t = 0; t < QT; ++t)
+#pragma unroll
+                for (int d = 0; d < ND; ++d) acc[t][d] *= al[t];
+        }
+    }
+};
+
+// Few column tiles (decoding): the four waves of a workgroup share one column tile, each takes every 4th key block straight from the
+// cache, and their sums meet in LDS.  gridDim.y > 1: the keys are also split over workgroups (k_tlm_attn_combine).
+template <class Tr, int ND, int RK>
 __global__ __launch_bounds__(256) void k_tlm_attn(TlmAttnArgs a) {
-    constexpr int NQ = ND * 16 / Tr::KSTEP + 128 / Tr::KSTEP;      // query fragments: latent + at most 128 rotated dimensions
-    constexpr int NB = 32 / (4 * Tr::V);                           // value fragments per 32 keys
+    typedef TlmQuery<Tr, ND, RK> Q;
+    constexpr int NB = Q::NB, WK = 4;
     MMI_SHARED float ml[2][4][16];
-    MMI_SHARED __attribute__((aligned(16))) f32x4 ob[WK > 1 ? 4 * 8 * 64 : 1];
-    const int lane = (int)threadIdx.x & 63, wave = (int)threadIdx.x >> 6, bl = lane & 15, kq = lane >> 4;
-    const int tile = (int)blockIdx.x * (4 / WK) + wave / WK, wk = wave % WK, split = (int)blockIdx.y;
-    if (tile >= a.n_tiles) return;                                 // WK == 4: the whole workgroup; WK == 1: no barrier follows
+    MMI_SHARED __attribute__((aligned(16))) f32x4 ob[4 * 8 * 64];
+    const int lane = (int)threadIdx.x & 63, wave = mmi_uniform((int)threadIdx.x >> 6), bl = lane & 15, kq = lane >> 4, split = (int)blockIdx.y;
+    // consecutive workgroups go round the 8 XCDs: neighbouring tiles (heads of one sequence read the same keys) to one XCD's L2
+    const int tile = ((int)blockIdx.x & 7) * ((int)gridDim.x >> 3) + ((int)blockIdx.x >> 3);
+    if (tile >= a.n_tiles) return;
     const TlmCols c = tlm_find_tile(a, tile);
     const int col = c.c0 + bl < c.ncol ? c.c0 + bl : c.ncol - 1;
     const int pos0 = a.epos0[c.entry];
@@ -649,129 +838,240 @@ __global__ __launch_bounds__(256) void k_tlm_attn(TlmAttnArgs a) {
         b1 = min(b1, b0 + per);
     }
     const int* bt = a.block_table + (long)a.eslot[c.entry] * a.bt_ld;
-    const u32x4* kc = (const u32x4*)a.kc;
-    const u32x4* vc = (const u32x4*)a.vc;
-    u32x4 qf[NQ];
-    {
-        const long qrow = (long)a.erow0[c.entry] * a.heads + col;
-        const u32x4* qp = (const u32x4*)a.q + (qrow >> 4) * a.q_ks * 64 + kq * 16 + (qrow & 15);
-#pragma unroll
-        for (int s = 0; s < NQ; ++s)
-            if (s < a.q_ks) qf[s] = qp[s * 64];
-    }
     f32x4 acc[ND];
 #pragma unroll
     for (int d = 0; d < ND; ++d) acc[d] = f32x4{0.f, 0.f, 0.f, 0.f};
     float m = -1e30f, l = 0.f;
-    for (int kb = b0 + wk; kb < b1; kb += WK) {
-        const long page = bt[(kb >> 1) % a.bt_ld];
-        const u32x4* kp = kc + (page * 4 + (kb & 1) * 2) * a.q_ks * 64 + lane;
+    TlmFlip<Tr> flip;
+    flip.init(bl, kq);
+    // the waves share the column tile: its query fragments stay in LDS, the registers are for keys in flight
+    MMI_SHARED __attribute__((aligned(16))) u32x4 ql[Q::NK * 64];
+    {
+        const long qrow = (long)a.erow0[c.entry] * a.heads + col;
+        const u32x4* qp = (const u32x4*)a.q + (qrow >> 4) * a.q_ks * 64 + kq * 16 + (qrow & 15);
+        for (int s = wave; s < Q::NK; s += WK) ql[s * 64 + lane] = Q::fragment(a, qp, s);
+        __syncthreads();
+    }
+    // A block's key fragments stay in registers from the scores to the values (turned there), and each one's register asks for the next
+    // block's fragment as soon as it has been used: a block is read once, and nearly a whole block is always in flight.
+    constexpr int NK = Q::NK, LK = Q::LK, FH = TlmFlip<Tr>::H, GK = 4;
+    u32x4 fr[NK][2];
+    const u32x4* kp = (const u32x4*)a.kc;
+    auto block = [&](int kb) __attribute__((always_inline)) {
+        const long page = bt[(min(kb, b1 - 1) >> 1) % a.bt_ld];    // (past the end: the last block again)
+        kp = (const u32x4*)a.kc + (page * 4 + (kb & 1) * 2) * a.q_ks * 64 + lane;
+    };
+    auto load = [&](int k) __attribute__((always_inline)) {
+        const int o = tlm_kstep_of<LK>(a, k);
+        fr[k][0] = kp[o * 64];
+        fr[k][1] = kp[(a.q_ks + o) * 64];
+    };
+    if (b0 + wave < b1) {
+        block(b0 + wave);
+#pragma unroll
+        for (int k = 0; k < NK; ++k) load(k);
+    }
+    for (int kb = b0 + wave; kb < b1; kb += WK) {
+        block(kb + WK);
         f32x4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = s0;
 #pragma unroll
-        for (int s = 0; s < NQ; ++s)
-            if (s < a.q_ks) {
-                s0 = Tr::mfma(kp[s * 64], qf[s], s0);
-                s1 = Tr::mfma(kp[(a.q_ks + s) * 64], qf[s], s1);
-            }
-        float mx = m;
-        const int d0 = pc - (kb * 32 + 4 * kq);                    // position minus the key of register 0
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-            const int e0 = d0 - r, e1 = d0 - r - 16;
-            s0[r] = e0 >= 0 && (a.window <= 0 || e0 < a.window) ? s0[r] * a.scale : -INFINITY;
-            s1[r] = e1 >= 0 && (a.window <= 0 || e1 < a.window) ? s1[r] * a.scale : -INFINITY;
-            mx = fmaxf(mx, fmaxf(s0[r], s1[r]));
+        for (int k = 0; k < NK; ++k) {
+            const u32x4 qv = ql[k * 64 + lane];
+            s0 = Tr::mfma(fr[k][0], qv, s0);
+            s1 = Tr::mfma(fr[k][1], qv, s1);
         }
-        mx = fmaxf(mx, mmi_shfl_xor(mx, 16));
-        mx = fmaxf(mx, mmi_shfl_xor(mx, 32));
-        const float al = exp2f(m - mx);
-        m = mx;
-        l *= al;
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-            s0[r] = exp2f(s0[r] - mx);
-            s1[r] = exp2f(s1[r] - mx);
-            l += s0[r] + s1[r];
-        }
+        for (int k = LK; k < NK; ++k) load(k);
+        mmi_sched_barrier();
         u32x4 pf[NB];
-        if constexpr (NB == 1) {
-            pf[0] = u32x4{mmi_pack_bf16x2(s0[0], s0[1]), mmi_pack_bf16x2(s0[2], s0[3]), mmi_pack_bf16x2(s1[0], s1[1]), mmi_pack_bf16x2(s1[2], s1[3])};
-        } else {
-            pf[0] = __builtin_bit_cast(u32x4, s0);
-            pf[NB - 1] = __builtin_bit_cast(u32x4, s1);
+        const float al = tlm_softmax_block<Tr>(a, s0, s1, pc - (kb * 32 + 4 * kq), m, l, pf);
+        if (mmi_any(al != 1.f)) {
+#pragma unroll
+            for (int d = 0; d < ND; ++d) acc[d] *= al;
         }
-        const u32x4* vp = vc + (page * a.nd * (2 * NB) + (kb & 1) * NB) * 64 + lane;
 #pragma unroll
-        for (int d = 0; d < ND; ++d)
-            if (d < a.nd) {
-                acc[d] *= al;
+        for (int k0 = 0; k0 < LK; k0 += GK) {
 #pragma unroll
-                for (int q = 0; q < NB; ++q) acc[d] = Tr::mfma(vp[(d * 2 * NB + q) * 64], pf[q], acc[d]);
-            }
+            for (int k = k0; k < k0 + GK && k < LK; ++k)
+#pragma unroll
+                for (int h = 0; h < FH; ++h) {
+                    acc[k * FH + h] = Tr::mfma(flip.turn(fr[k][0], fr[k][1], h), pf[0], acc[k * FH + h]);
+                    if constexpr (NB == 2) acc[k * FH + h] = Tr::mfma(flip.turn(fr[k][1], fr[k][1], h), pf[NB - 1], acc[k * FH + h]);
+                }
+#pragma unroll
+            for (int k = k0; k < k0 + GK && k < LK; ++k) load(k);
+            mmi_sched_barrier();
+        }
     }
     l += mmi_shfl_xor(l, 16);
     l += mmi_shfl_xor(l, 32);
-    if constexpr (WK > 1) {
-        if (kq == 0) {
-            ml[0][wave][bl] = m;
-            ml[1][wave][bl] = l;
-        }
+    if (kq == 0) {
+        ml[0][wave][bl] = m;
+        ml[1][wave][bl] = l;
+    }
+    __syncthreads();
+    float M = -1e30f, L = 0.f;
+#pragma unroll
+    for (int w = 0; w < WK; ++w) M = fmaxf(M, ml[0][w][bl]);
+#pragma unroll
+    for (int w = 0; w < WK; ++w) L += ml[1][w][bl] * exp2f(ml[0][w][bl] - M);
+    const float f = exp2f(m - M);
+    const float inv = a.nsplit > 1 ? 1.f : 1.0f / L;
+#pragma unroll
+    for (int d0 = 0; d0 < ND; d0 += 8) {
+        if (d0 >= a.nd) break;
+        if (d0) __syncthreads();
+#pragma unroll
+        for (int d = 0; d < 8; ++d)
+            if (d0 + d < ND) ob[(wave * 8 + d) * 64 + lane] = acc[d0 + d < ND ? d0 + d : 0] * f;
         __syncthreads();
-        float M = -1e30f, L = 0.f;
 #pragma unroll
-        for (int w = 0; w < WK; ++w) M = fmaxf(M, ml[0][w][bl]);
+        for (int d = wave; d < 8; d += WK) {
+            if (d0 + d >= a.nd) break;
+            f32x4 v = ob[d * 64 + lane];
 #pragma unroll
-        for (int w = 0; w < WK; ++w) L += ml[1][w][bl] * exp2f(ml[0][w][bl] - M);
-        const float f = exp2f(m - M);
-        m = M;
-        l = L;
-        const float inv = a.nsplit > 1 ? 1.f : 1.0f / l;
+            for (int w = 1; w < WK; ++w) v += ob[(w * 8 + d) * 64 + lane];
+            if (a.nsplit > 1) *reinterpret_cast<f32x4*>(a.po + ((((long)tile * a.nsplit + split) * a.nd + d0 + d) * 64 + lane) * 4) = v;
+            else tlm_attn_store<Tr>(a, c, bl, kq, d0 + d, v * inv);
+        }
+    }
+    if (a.nsplit > 1 && wave == 0 && kq == 0) {
+        float* p = a.pml + ((long)tile * a.nsplit + split) * 32;
+        p[bl] = M;
+        p[16 + bl] = L;
+    }
+}
+
+// Many columns (prompts): four waves x QT column tiles of one sequence walk the same keys; a block's fragments are staged through LDS
+// once for all of them (NBUF buffers, the next block in flight in registers while this one is used).
+template <class Tr, int ND, int RK>
+struct TlmAttnTile {
+    static constexpr int QT = ND <= (Tr::V == 8 ? 16 : 8) ? 2 : 1;
+    static constexpr int NF = 2 * TlmQuery<Tr, ND, RK>::NK + ND * TlmQuery<Tr, ND, RK>::NB;      // fragments per 32 keys
+    static constexpr int NBUF = 2 * NF <= 152 ? 2 : 1;
+    static constexpr size_t smem() { return (size_t)NBUF * NF * 1024; }
+};
+template <class Tr, int ND, int RK>
+__global__ __launch_bounds__(256) void k_tlm_attn_tile(TlmAttnArgs a) {
+    typedef TlmQuery<Tr, ND, RK> Q;
+    typedef TlmAttnTile<Tr, ND, RK> P;
+    constexpr int NB = Q::NB, NK = Q::NK, QT = P::QT, NF = P::NF, NBUF = P::NBUF, NI = (NK + 3) / 4, FH = TlmFlip<Tr>::H;
+    MMI_DYN_SHARED(u32x4, lds);
+    const int lane = (int)threadIdx.x & 63, wave = mmi_uniform((int)threadIdx.x >> 6), bl = lane & 15, kq = lane >> 4;
+    int g = (int)blockIdx.x;
+    TlmCols c;                                                     // (tile0 counts groups of 64 QT columns here)
+    {
+        c = tlm_find_tile(a, g);
+        c.c0 *= 4 * QT;
+    }
+    const int pos0 = a.epos0[c.entry];
+    const int plo = pos0 + c.c0 / a.heads, phi = pos0 + min(c.c0 + 64 * QT - 1, c.ncol - 1) / a.heads;
+    const int klo = a.window > 0 && plo - a.window + 1 > 0 ? plo - a.window + 1 : 0;
+    const int b0 = klo / 32, b1 = phi / 32 + 1;
+    const int* bt = a.block_table + (long)a.eslot[c.entry] * a.bt_ld;
+    typedef TlmAttnStream<Tr, ND, RK, QT, (ND >= 16 ? 4 : 8)> S;
+    Q q[QT];
+    S sm;
+    sm.clear();
+    TlmFlip<Tr> flip;
+    flip.init(bl, kq);
+    int pc[QT], c0[QT];
 #pragma unroll
-        for (int d0 = 0; d0 < ND; d0 += 8) {
-            if (d0 >= a.nd) break;
-            if (d0) __syncthreads();
+    for (int t = 0; t < QT; ++t) {
+        c0[t] = c.c0 + (wave * QT + t) * 16;
+        const int col = c0[t] + bl < c.ncol ? c0[t] + bl : c.ncol - 1;
+        pc[t] = pos0 + col / a.heads;
+        q[t].load(a, (long)a.erow0[c.entry] * a.heads + col, kq);
+    }
+    // fragments of a block in LDS: keys 0-15 and 16-31 of each k-step, then the turned values; wave w brings k-steps w, w + 4, ..
+    u32x4 st[NI][2];
+    auto page_of = [&](int kb) __attribute__((always_inline)) { return bt[(min(kb, b1 - 1) >> 1) % a.bt_ld]; };
+    long page = page_of(b0);                                       // of the block fetched next
+    auto fetch = [&](int kb) __attribute__((always_inline)) {
+        const u32x4* kp = (const u32x4*)a.kc + (page * 4 + (kb & 1) * 2) * a.q_ks * 64 + lane;
 #pragma unroll
-            for (int d = 0; d < 8; ++d)
-                if (d0 + d < ND) ob[(wave * 8 + d) * 64 + lane] = acc[d0 + d < ND ? d0 + d : 0] * f;
-            __syncthreads();
+        for (int i = 0; i < NI; ++i) {
+            const int o = tlm_kstep_of<Q::LK>(a, min(wave + 4 * i, NK - 1));
+            st[i][0] = kp[o * 64];
+            st[i][1] = kp[(a.q_ks + o) * 64];
+        }
+        page = page_of(kb + 1);
+    };
+    auto stage = [&](int buf) __attribute__((always_inline)) {
+        u32x4* base = lds + buf * NF * 64 + lane;
 #pragma unroll
-            for (int d = wave; d < 8; d += WK) {
-                if (d0 + d >= a.nd) break;
-                f32x4 v = ob[d * 64 + lane];
+        for (int i = 0; i < NI; ++i) {
+            const int k = wave + 4 * i;
+            if (4 * i + 3 >= NK && k >= NK) continue;
+            base[(2 * k) * 64] = st[i][0];
+            base[(2 * k + 1) * 64] = st[i][1];
+            if (4 * i + 3 >= Q::LK && k >= Q::LK) continue;          // the rotated part has no value
 #pragma unroll
-                for (int w = 1; w < WK; ++w) v += ob[(w * 8 + d) * 64 + lane];
-                if (a.nsplit > 1) *reinterpret_cast<f32x4*>(a.po + ((((long)tile * a.nsplit + split) * a.nd + d0 + d) * 64 + lane) * 4) = v;
-                else tlm_attn_store<Tr>(a, c, bl, kq, d0 + d, v * inv);
+            for (int h = 0; h < FH; ++h) {
+                const int d = k * FH + h;
+                if constexpr (NB == 1) {
+                    base[(2 * NK + d) * 64] = flip.turn(st[i][0], st[i][1], h);
+                } else {
+                    base[(2 * NK + d * NB) * 64] = flip.turn(st[i][0], st[i][0], h);
+                    base[(2 * NK + d * NB + NB - 1) * 64] = flip.turn(st[i][1], st[i][1], h);
+                }
             }
         }
-    } else {
-        const float inv = a.nsplit > 1 ? 1.f : 1.0f / l;
+    };
+    fetch(b0);
+    stage(0);
+    __syncthreads();
+    int cur = 0;
+    for (int kb = b0; kb < b1; ++kb) {
+        fetch(kb + 1);                                             // (past the end: the last block's page again)
+        mmi_sched_barrier();
+        const u32x4* base = lds + cur * NF * 64 + lane;
+        auto at = [&](int f) __attribute__((always_inline)) -> const u32x4* { return base + f * 64; };
+        auto qf = [&](int t, int k) __attribute__((always_inline)) { return q[t].f[k]; };
+        int d0[QT];
+#pragma unroll
+        for (int t = 0; t < QT; ++t) d0[t] = pc[t] - (kb * 32 + 4 * kq);
+        sm.load(0, 0, at);
+#pragma unroll
+        for (int g = 0; g < S::NG; ++g) {
+            if (g + 1 < S::NG) sm.load((g + 1) & 1, g + 1, at);
+            mmi_sched_barrier();
+            sm.use(a, qf, g & 1, g, d0);
+        }
+        if constexpr (NBUF == 1) __syncthreads();
+        else cur ^= 1;
+        stage(cur);
+        __syncthreads();
+    }
+#pragma unroll
+    for (int t = 0; t < QT; ++t) {
+        float l = sm.l[t];
+        l += mmi_shfl_xor(l, 16);
+        l += mmi_shfl_xor(l, 32);
+        const float inv = 1.0f / l;
+        TlmCols o = c;
+        o.c0 = c0[t];
 #pragma unroll
         for (int d = 0; d < ND; ++d)
-            if (d < a.nd) {
-                if (a.nsplit > 1) *reinterpret_cast<f32x4*>(a.po + ((((long)tile * a.nsplit + split) * a.nd + d) * 64 + lane) * 4) = acc[d];
-                else tlm_attn_store<Tr>(a, c, bl, kq, d, acc[d] * inv);
-            }
-    }
-    if (a.nsplit > 1 && wk == 0 && kq == 0) {
-        float* q = a.pml + ((long)tile * a.nsplit + split) * 32;
-        q[bl] = m;
-        q[16 + bl] = l;
+            if (d < a.nd) tlm_attn_store<Tr>(a, o, bl, kq, d, sm.acc[t][d] * inv);
     }
 }
 
 // the splits of one column tile -> output; one workgroup per tile, waves over the latent blocks
 template <class Tr>
 __global__ __launch_bounds__(256) void k_tlm_attn_combine(TlmAttnArgs a) {
-    const int lane = (int)threadIdx.x & 63, wave = (int)threadIdx.x >> 6, bl = lane & 15, kq = lane >> 4, tile = (int)blockIdx.x;
+    const int lane = (int)threadIdx.x & 63, wave = mmi_uniform((int)threadIdx.x >> 6), bl = lane & 15, kq = lane >> 4, tile = (int)blockIdx.x;
     const TlmCols c = tlm_find_tile(a, tile);
     const float* q = a.pml + (long)tile * a.nsplit * 32;
     float M = -1e30f, L = 0.f;
+#pragma unroll 4
     for (int s = 0; s < a.nsplit; ++s) M = fmaxf(M, q[s * 32 + bl]);
+#pragma unroll 4
     for (int s = 0; s < a.nsplit; ++s) L += q[s * 32 + 16 + bl] * exp2f(q[s * 32 + bl] - M);
     const float inv = 1.0f / L;
-    for (int d = wave; d < a.nd; d += 4) {
+    for (int d = wave + 4 * (int)blockIdx.y; d < a.nd; d += 4 * (int)gridDim.y) {
         f32x4 v = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
         for (int s = 0; s < a.nsplit; ++s)
             v += *reinterpret_cast<const f32x4*>(a.po + ((((long)tile * a.nsplit + s) * a.nd + d) * 64 + lane) * 4) * exp2f(q[s * 32 + bl] - M);
         tlm_attn_store<Tr>(a, c, bl, kq, d, v * inv);

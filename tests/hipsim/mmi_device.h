@@ -344,6 +344,9 @@ inline unsigned mmi_arrive_release(unsigned* counter) { return __atomic_fetch_ad
 inline void mmi_acquire_agent() { __atomic_thread_fence(__ATOMIC_ACQUIRE); }
 inline void mmi_store_relaxed_agent(unsigned* p, unsigned v) { __atomic_store_n(p, v, __ATOMIC_RELEASE); }
 
+inline void mmi_sched_barrier() {}
+inline int mmi_uniform(int v) { return v; }
+inline bool mmi_any(bool v) { unsigned x = v ? 1u : 0u; for (int m = 1; m < 64; m <<= 1) { const unsigned o = mmi_shfl_xor(x, m); x = o > x ? o : x; } return x != 0; }
 inline u32x4 mmi_load_nt(const u32x4* p) { return *p; }
 inline f32x4 mmi_load_nt(const f32x4* p) { return *p; }
 inline float mmi_rsqrtf(float x) { return 1.0f / sqrtf(x); }
