@@ -281,6 +281,8 @@ class CheckpointInfo:
         cfg_file = path / "config.json" if path.is_dir() else path
         root = cfg_file.parent
         raw = json.loads(cfg_file.read_text())
+        if raw.get("architecture") in TOKEN_LM_ARCHITECTURES:
+            raise ValueError(f"{cfg_file} describes a token language model ({raw['architecture']}): load it with loaders.get_token_lm")
         lm_config = dict(raw)
         names = {k: lm_config.pop(k, None) for k in ("moshi_name", "mimi_name", "tokenizer_name")}
         model_type = lm_config.pop("model_type", "moshi")

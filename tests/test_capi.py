@@ -100,7 +100,7 @@ def test_struct_layouts_of_the_header_equal_the_ctypes_binding(tmp_path):
         for f in fields:
             lines.append(f'  printf("{s} {f} %zu\\n", offsetof({s}, {f}));')
     for e in ("MMI_OK", "MMI_ERR_INVALID", "MMI_ERR_SHAPE", "MMI_ERR_STATE", "MMI_ERR_HIP", "MMI_ERR_MISSING_WEIGHT", "MMI_ERR_UNSUPPORTED",
-              "MMI_ERR_BUSY", "MMI_ERR_NO_CHANNEL", "MMI_F32", "MMI_BF16", "MMI_I64", "MMI_F16", "MMI_I8", "MMI_F8E4M3"):
+              "MMI_ERR_BUSY", "MMI_ERR_NO_CHANNEL", "MMI_F32", "MMI_BF16", "MMI_I64", "MMI_F16", "MMI_I8", "MMI_F8E4M3", "MMI_I32"):
         lines.append(f'  printf("enum {e} %d\\n", (int){e});')
     lines += ['  return 0;', '}']
     src = tmp_path / "layout.c"
