@@ -31,6 +31,12 @@ def test_feeding(lib, case, dtype):
     getattr(tc, f"check_{case}")(DEV, lib, dtype)
 
 
+@pytest.mark.parametrize("dtype", [tc.F32, tc.BF16], ids=["fp32", "bf16"])
+@pytest.mark.parametrize("name", sorted(tc.WIDE_PROMPTS))
+def test_long_prompt_per_latent_width(lib, name, dtype):
+    tc.check_long_prompt(DEV, lib, dtype, n=700, cfg=tc.WIDE_PROMPTS[name])
+
+
 @pytest.mark.parametrize("window", [70, 64, 0])
 def test_single_keys(lib, window):
     tc.check_single_keys(DEV, lib, window)

@@ -39,6 +39,8 @@ MECHANISMS = {
     "window_one": one_layer(replace(ATT, window=1)),
     "no_window": one_layer(replace(ATT, window=0)),
     "wide_latent": one_layer(replace(ATT, kv_rank=200, q_rank=17, rot_dim=40)),
+    "widest_latent": one_layer(replace(ATT, kv_rank=500, q_rank=33, rot_dim=128, heads=2)),
+    "latent_of_eight_tiles": one_layer(replace(ATT, kv_rank=120, rot_dim=66, heads=5)),
     "latent_of_one_tile": one_layer(replace(ATT, kv_rank=16, dim=32, vdim=32, rot_dim=32)),
     "one_group": one_layer(MinGRUConfig(24), norm_groups=1),
     "six_groups": one_layer(MinGRUConfig(24), norm_groups=6),
@@ -208,6 +210,15 @@ def check_long_decode(dev, lib, dtype=F32, n=330, pool=256):
     assert lm.position(slot) == n and lm.info(5, slot) <= 2          # held pages: a window of 37 spans at most two
     lm.close(slot)
     assert lm.free_pages == lm.total_pages
+
+
+# per bound of the attention kernels' latent, heads enough for their key-staging form
+WIDE_PROMPTS = {
+    "latent_36": one_layer(replace(ATT, heads=26)),
+    "latent_128": one_layer(replace(ATT, heads=26, kv_rank=128, rot_dim=40, window=300)),
+    "latent_200": one_layer(replace(ATT, heads=26, kv_rank=200, rot_dim=80, window=0)),
+    "latent_500": one_layer(replace(ATT, heads=14, kv_rank=500, rot_dim=64, window=129)),
+}
 
 
 def check_long_prompt(dev, lib, dtype=F32, n=1300, cfg=None):
