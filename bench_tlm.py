@@ -117,7 +117,7 @@ def bench_model(cfg, dev, steps, warmup, batches=(1, 16, 64), dtype=torch.bfloat
     return out
 
 
-def bench_moshi(width, layers, dev, steps, warmup, batches):
+def bench_moshi(width, layers, dev, steps, warmup, batches, launch_lists=None):
     """The temporal transformer alone (no depth transformer), same width, layer count, ring depth and batch."""
     from moshi_amd.config import LMConfig
     from moshi_amd.lm import LMGen, LMModel
@@ -133,6 +133,11 @@ def bench_moshi(width, layers, dev, steps, warmup, batches):
             gen.step(codes)
         gen.seek([DEPTH] * B)
         dt = timed(lambda: gen.step(codes), steps, warmup, dev)
+        if launch_lists:
+            from pathlib import Path
+            from moshi_amd import _capi
+            ll = _capi.launch_list(lambda b, n: lm._lib.mmi_lm_launch_list(lm._handle, b, n), with_bytes=True)
+            (Path(launch_lists) / f"launch_list_moshi_{width}_decode{B}.tsv").write_text("".join(f"{s}\t{k}\t{b}\n" for s, k, b in ll))
         h = cfg.ffn_hidden
         nb = 2 * (layers * (4 * width * width + 3 * h * width) + cfg.text_card * width) + B * layers * 2 * 2 * width * DEPTH
         out[str(B)] = {"ms": 1e3 * dt, "tokens_per_s": B / dt, "gb_per_step": nb / 1e9, "gb_per_s": nb / dt / 1e9, "hbm_frac": nb / dt / 1e9 / HBM_PEAK_GBS}
@@ -149,7 +154,7 @@ def main(args, dev):
             continue
         res[name] = bench_model(cfg, dev, args.steps, args.warmup, batches, launch_lists=args.launch_lists, tag=name)
         if not args.no_extras:
-            res[name]["moshi"] = bench_moshi(cfg.width, len(cfg.layer_runs), dev, args.steps, args.warmup, batches)
+            res[name]["moshi"] = bench_moshi(cfg.width, len(cfg.layer_runs), dev, args.steps, args.warmup, batches, args.launch_lists)
     last = list(res)[-1]
     d = res[last]["decode"][str(batches[-1])]
     print(json.dumps({"metric": "decoded tokens/s, token language model", "value": d["tokens_per_s"], "unit": "tokens/s", "n_gpus": 1, "steps": args.steps,

@@ -422,7 +422,7 @@ int alloc_buffers(mmi_tlm* m) {
             cq_ks = std::max(cq_ks, L.q_ks);
             qn_ks = std::max(qn_ks, L.qn_ks);
             q_elems = std::max(q_elems, (long)((T * (long)L.c.heads + 15) / 16) * L.k_ks);
-            ao_elems = std::max(ao_elems, (long)((T * (long)L.c.heads + 15) / 16) * L.lat_ks);
+            ao_elems = std::max(ao_elems, (long)round_up(T, 16) / 16 * L.c.heads * L.lat_ks);
             o_ks = std::max(o_ks, L.out.KS);
             gate_ld = std::max(gate_ld, L.c.heads);
             nd = std::max(nd, L.nd);
@@ -805,6 +805,7 @@ MixerOut build_latent_attention(mmi_tlm* m, MmiProgram& P, const Shape& sh, cons
     t.q = m->q;
     t.kc = r.kc;
     t.out = m->ao;
+    t.out_rows = round_up(T, 16);
     t.heads = H;
     t.q_ks = L.k_ks;
     t.nd = L.nd;
@@ -833,8 +834,7 @@ MixerOut build_latent_attention(mmi_tlm* m, MmiProgram& P, const Shape& sh, cons
     TlmJob& jv = Q.j[Q.n++];
     jv = dense_job(L.uv, m->ao, L.lat_ks, T);
     jv.groups = H;
-    jv.in_mul = H;
-    jv.in_gadd = 1;
+    jv.in_gadd = t.out_rows;
     jv.epi = TLM_EPI_PACK;
     jv.out = m->o;
     jv.out_ld = L.out.KS;

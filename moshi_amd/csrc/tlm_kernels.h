@@ -632,7 +632,7 @@ __global__ __launch_bounds__(256) void k_tlm_latent(TlmLatentArgs a) {
 struct TlmAttnArgs {
     const void* q;                       // packed rows token * heads + head
     const void* kc;
-    void* out;                           // packed rows token * heads + head, latent columns
+    void* out; int out_rows;             // packed rows head * out_rows + token, latent columns (the value projection reads head by head)
     int heads, q_ks, nd, out_ks;
     int window;                          // 0: every earlier position
     float scale;                         // times log2(e)
@@ -660,7 +660,8 @@ template <class Tr>
 __device__ __forceinline__ void tlm_attn_store(const TlmAttnArgs& a, const TlmCols& c, int bl, int kq, int db, f32x4 v) {
     const int col = c.c0 + bl;
     if (col >= c.ncol) return;
-    const long orow = (long)a.erow0[c.entry] * a.heads + col;
+    const int t = col / a.heads;
+    const long orow = (long)(col - t * a.heads) * a.out_rows + a.erow0[c.entry] + t;
     Tr::store4((typename Tr::elem*)a.out + tlm_index<Tr>(orow, db * 16 + 4 * kq, a.out_ks), v);
 }
 
@@ -816,7 +817,7 @@ struct TlmAttnStream {
 // Few column tiles (decoding): the four waves of a workgroup share one column tile, each takes every 4th key block straight from the
 // cache, and their sums meet in LDS.  gridDim.y > 1: the keys are also split over workgroups (k_tlm_attn_combine).
 template <class Tr, int ND, int RK>
-__global__ __launch_bounds__(256) void k_tlm_attn(TlmAttnArgs a) {
+__global__ __launch_bounds__(256, Tr::V == 8 && ND <= 16 ? 2 : 1) void k_tlm_attn(TlmAttnArgs a) {      // two workgroups per CU where the registers allow it
     typedef TlmQuery<Tr, ND, RK> Q;
     constexpr int NB = Q::NB, WK = 4;
     MMI_SHARED float ml[2][4][16];
