@@ -96,7 +96,7 @@ struct mmi_tlm {
     std::vector<Run> runs;
     int device = 0;
     bool f32 = false;
-    int kstep = 32, V = 8, esize = 2;
+    int kstep = 32, V = 8;
     int ld = 0, h_ks = 0;
     int max_slots = 0, max_pages = 0, max_T = 0;
     bool has_attn = false, has_gru = false;
@@ -1005,7 +1005,6 @@ int create_impl(mmi_tlm* m, const mmi_tensor_desc* weights, int n_weights) {
     m->f32 = c.dtype == MMI_F32;
     m->kstep = m->f32 ? TlmF32::KSTEP : TlmBf16::KSTEP;
     m->V = m->f32 ? TlmF32::V : TlmBf16::V;
-    m->esize = m->f32 ? 4 : 2;
     m->ld = round_up(c.width, 16);
     m->h_ks = round_up(c.width, m->kstep) / m->kstep;
     Loader ld;

@@ -1189,7 +1189,3 @@ __global__ void k_tlm_last_tok(const int* __restrict__ out, const int* __restric
     const int i = (int)(blockIdx.x * blockDim.x + threadIdx.x);
     if (i < n) last_tok[map[i]] = out[i];
 }
-__global__ void k_tlm_fill(float* __restrict__ p, float v, long n) {
-    const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
-    if (i < n) p[i] = v;
-}
