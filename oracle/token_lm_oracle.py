@@ -1,5 +1,5 @@
 """Plain numpy restatement of the token language models (moshi_amd/tlm.py), float64, one function per mechanism, whole sequences at
-once: no cache, no state hand-over, no batching.  Checker only - it shares no code with the engine and reads the same state dict.
+once: no cache, no state hand-over, no batching.  For tests only - it shares no code with the engine and reads the same state dict.
 """
 from __future__ import annotations
 
