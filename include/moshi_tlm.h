@@ -10,20 +10,28 @@ extern "C" {
 /* ------------------------------------------------------------------------------------------ */
 /* Token language models: decoder-only networks over token ids (libmoshi_tlm.so)              */
 /* ------------------------------------------------------------------------------------------ */
-/* The layers are data: each has one mixer and one feed-forward reading the same norm (parallel sublayers), layer scales, grouped
- * RMS norms, an optional run of layers repeated with the same weights.  Sequences live in slots; their attention cache is a pool of
- * pages of mmi_tlm_info(MMI_TLM_PAGE_TOKENS) tokens, their recurrent state one entry per slot and recurrent layer run. */
+/* The layers are data: each has one mixer and one feed-forward reading norms of the same input (parallel sublayers), optional layer
+ * scales, grouped RMS norms, an optional run of layers repeated with the same weights.  Sequences live in slots; their attention cache
+ * is a pool of pages of mmi_tlm_info(MMI_TLM_PAGE_TOKENS) tokens, their recurrent state one entry per slot and recurrent layer run. */
 
 /* mixers */
 #define MMI_TLM_MIX_LATENT_ATTENTION 1
 #define MMI_TLM_MIX_MINGRU 2
+#define MMI_TLM_MIX_ATTENTION 3         /* softmax attention, query heads share key/value heads */
+#define MMI_TLM_MIX_CHANNEL_DELTA 4     /* gated delta rule, one decay per key channel */
+#define MMI_TLM_MIX_LIGHTNING 5         /* linear attention, one constant decay per head */
 /* feed-forwards */
 #define MMI_TLM_MLP_NONE 0
 #define MMI_TLM_MLP_MOE 1
-/* expert activations */
+#define MMI_TLM_MLP_DENSE 2             /* gated: gate and up projections, down projection */
+/* feed-forward activations */
 #define MMI_TLM_ACT_RELU2 1
+#define MMI_TLM_ACT_CLAMPED_SWIGLU 2    /* g = min(gate, limit), u = clamp(up, +-limit): g sigmoid(1.702 g) (u + 1) */
 /* routers */
 #define MMI_TLM_ROUTE_TOKEN_TABLE 1
+/* what the passes of the repeated layers start with */
+#define MMI_TLM_LOOP_ADD 0              /* the second and later ones: x + embedding */
+#define MMI_TLM_LOOP_PROJECT 1          /* every one: loop.in [x; embedding] + loop.step[pass] */
 
 typedef struct mmi_tlm_layer {
     int32_t mixer;
@@ -34,6 +42,13 @@ typedef struct mmi_tlm_layer {
     float scale;
     double rot_base;
     int32_t mlp, experts, top, ff, act, router;
+    int32_t kv_heads;                             /* attention, channel delta: key/value (query/key) heads */
+    int32_t keep_first;                           /* attention with a window: first positions that stay visible */
+    int32_t sink;                                 /* attention: one is added to the softmax denominator */
+    int32_t conv;                                 /* channel delta: taps of the short convolutions */
+    int32_t decay_rank, gate_rank;                /* channel delta: ranks of the decay's and the gate's projection */
+    const double* decay;                          /* lightning: [heads], host */
+    float limit;                                  /* clamped SwiGLU */
 } mmi_tlm_layer;
 
 typedef struct mmi_tlm_cfg {
@@ -42,13 +57,19 @@ typedef struct mmi_tlm_cfg {
     int32_t loop_start, loop_stop, loop_times;    /* layers [start, stop) run `times` times; start == stop: no repetition */
     int32_t norm_groups;
     float norm_eps, logit_scale;
+    int32_t loop_inject, norms, layer_scales;     /* norms 2: the feed-forward has a norm of its own; layer_scales: ls1 / ls2 exist */
+    int32_t tied_head;                            /* logits from the (unscaled) embedding table */
+    float embed_scale;
+    int32_t bigram_buckets;                       /* 0: no bigram embedding; row (previous mul_prev + token mul_cur) mod buckets, first token: row `buckets` */
+    int64_t bigram_mul_prev, bigram_mul_cur;
+    int32_t max_positions;                        /* 0: no learned positions; otherwise also the longest sequence */
     int32_t dtype;                                /* MMI_BF16 or MMI_F32: operands of the matrix products, activations and cache */
 } mmi_tlm_cfg;
 
 typedef struct mmi_tlm mmi_tlm;
 
-/* Tensors are bf16 (tables int32), device pointers, copied or repacked: `embed`, `head`, `final.norm`, per layer `l<i>.norm1`, `.ls1`,
- * `.ls2`, `.mix.*`, `.mlp.*`.  max_slots: live sequences; max_tokens: cache pool (rounded up to pages); max_step_tokens: tokens of
+/* Tensors are bf16 (tables int32), device pointers, copied or repacked: `embed`, `bigram`, `pos`, `head`, `final.norm`, `loop.in`,
+ * `loop.step`, per layer `l<i>.norm1`, `.norm2`, `.ls1`, `.ls2`, `.mix.*`, `.mlp.*`.  max_slots: live sequences; max_tokens: cache pool (rounded up to pages); max_step_tokens: tokens of
  * one step. */
 int mmi_tlm_create(const mmi_tlm_cfg* cfg, const mmi_tensor_desc* weights, int32_t n_weights, int32_t max_slots, int64_t max_tokens,
                    int32_t max_step_tokens, mmi_tlm** out);

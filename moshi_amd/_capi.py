@@ -83,19 +83,23 @@ class TLMLayer(C.Structure):
     _fields_ = [("mixer", C.c_int32), ("width", C.c_int32), ("heads", C.c_int32), ("dim", C.c_int32), ("vdim", C.c_int32),
                 ("rot_dim", C.c_int32), ("q_rank", C.c_int32), ("kv_rank", C.c_int32), ("window", C.c_int32), ("scale", C.c_float),
                 ("rot_base", C.c_double), ("mlp", C.c_int32), ("experts", C.c_int32), ("top", C.c_int32), ("ff", C.c_int32),
-                ("act", C.c_int32), ("router", C.c_int32)]
+                ("act", C.c_int32), ("router", C.c_int32), ("kv_heads", C.c_int32), ("keep_first", C.c_int32), ("sink", C.c_int32),
+                ("conv", C.c_int32), ("decay_rank", C.c_int32), ("gate_rank", C.c_int32), ("decay", C.POINTER(C.c_double)), ("limit", C.c_float)]
 
 
 class TLMCfg(C.Structure):
     _fields_ = [("vocab", C.c_int32), ("width", C.c_int32), ("n_layers", C.c_int32), ("layers", C.POINTER(TLMLayer)),
                 ("loop_start", C.c_int32), ("loop_stop", C.c_int32), ("loop_times", C.c_int32), ("norm_groups", C.c_int32),
-                ("norm_eps", C.c_float), ("logit_scale", C.c_float), ("dtype", C.c_int32)]
+                ("norm_eps", C.c_float), ("logit_scale", C.c_float), ("loop_inject", C.c_int32), ("norms", C.c_int32), ("layer_scales", C.c_int32),
+                ("tied_head", C.c_int32), ("embed_scale", C.c_float), ("bigram_buckets", C.c_int32), ("bigram_mul_prev", C.c_int64),
+                ("bigram_mul_cur", C.c_int64), ("max_positions", C.c_int32), ("dtype", C.c_int32)]
 
 
 # include/moshi_tlm.h
-TLM_MIX_LATENT_ATTENTION, TLM_MIX_MINGRU = 1, 2
-TLM_MLP_NONE, TLM_MLP_MOE = 0, 1
-TLM_ACT_RELU2, TLM_ROUTE_TOKEN_TABLE = 1, 1
+TLM_MIX_LATENT_ATTENTION, TLM_MIX_MINGRU, TLM_MIX_ATTENTION, TLM_MIX_CHANNEL_DELTA, TLM_MIX_LIGHTNING = 1, 2, 3, 4, 5
+TLM_MLP_NONE, TLM_MLP_MOE, TLM_MLP_DENSE = 0, 1, 2
+TLM_ACT_RELU2, TLM_ACT_CLAMPED_SWIGLU, TLM_ROUTE_TOKEN_TABLE = 1, 2, 1
+TLM_LOOP_ADD, TLM_LOOP_PROJECT = 0, 1
 (TLM_PAGE_TOKENS, TLM_TOTAL_PAGES, TLM_FREE_PAGES, TLM_FREE_SLOTS, TLM_POSITION, TLM_HELD_PAGES, TLM_WEIGHT_BYTES, TLM_LAYER_RUNS,
  TLM_GRAPHS) = range(9)
 

@@ -198,6 +198,58 @@ class MinGRUConfig:
 
 
 @dataclass
+class GroupedAttentionConfig:
+    """Softmax attention whose query heads share key/value heads (query head h reads key/value head h // (heads / kv_heads)), un-rotated."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    window: int = 0                     # keys seen, the position itself included; 0 = every earlier one
+    keep_first: int = 0                 # with a window: the sequence's first positions that stay visible behind it
+    sink: bool = False                  # one is added to the softmax denominator: a sink of score 0 without a value
+
+
+@dataclass
+class ChannelDeltaConfig:
+    """Gated delta rule with one decay per key channel: short causal convolutions in front of query, key and value, unit queries and keys,
+    low-rank projections of the decay and of the output gate, an RMS norm per head behind it."""
+    heads: int
+    kv_heads: int                       # query/key heads; head h uses h // (heads / kv_heads)
+    dim: int
+    vdim: int
+    conv: int                           # taps, the current token's included
+    decay_rank: int
+    gate_rank: int
+
+
+@dataclass
+class LightningConfig:
+    """Linear attention with one constant decay per head, an RMS norm over all heads and an element-wise gate behind it."""
+    heads: int
+    dim: int
+    vdim: int
+    decay: List[float]                  # per head
+
+
+@dataclass
+class DenseGLUConfig:
+    """Gated feed-forward.  clamped_swiglu: g = min(gate, limit), u = clamp(up, +-limit), g * sigmoid(1.702 g) * (u + 1)."""
+    ff: int
+    limit: float
+    activation: str = "clamped_swiglu"
+
+
+@dataclass
+class BigramConfig:
+    """Embedding of (previous token, token): row (previous * mul_prev + token * mul_cur) mod buckets; a sequence's first token takes row
+    `buckets`."""
+    buckets: int
+    mul_prev: int
+    mul_cur: int
+
+
+@dataclass
 class MoEConfig:
     """Experts chosen by a table over token ids."""
     experts: int
@@ -209,14 +261,14 @@ class MoEConfig:
 
 @dataclass
 class TokenLayerConfig:
-    mixer: object                       # LatentAttentionConfig | MinGRUConfig
-    mlp: Optional[MoEConfig] = None
+    mixer: object                       # LatentAttentionConfig | MinGRUConfig | GroupedAttentionConfig | ChannelDeltaConfig | LightningConfig
+    mlp: object = None                  # MoEConfig | DenseGLUConfig | None
 
 
 @dataclass
 class TokenLMConfig:
-    """A decoder-only network over token ids: parallel sublayers behind one grouped RMS norm, layer scales, and optionally a weight-tied
-    repetition of layers [loop_start, loop_stop), whose second and later passes re-inject the embedding."""
+    """A decoder-only network over token ids: parallel sublayers behind RMS norms of the same input (grouped; one per layer or one per
+    sublayer), optional layer scales, and optionally a weight-tied repetition of layers [loop_start, loop_stop)."""
     architecture: str
     vocab: int
     width: int
@@ -227,6 +279,15 @@ class TokenLMConfig:
     loop_start: int = 0
     loop_stop: int = 0                  # start == stop: nothing is repeated
     loop_times: int = 1
+    # "add": the second and later passes start with x + embedding.  "project": every pass starts with a product of [x; embedding] and
+    # a vector of the pass (tensors loop.in, loop.step)
+    loop_inject: str = "add"
+    norms: int = 1                      # 2: the feed-forward reads a norm of its own (norm2)
+    layer_scales: bool = True           # ls1 / ls2 multiply what the sublayers add
+    embed_scale: float = 1.0
+    bigram: Optional[BigramConfig] = None
+    max_positions: int = 0              # > 0: a learned vector per position (tensor pos) is added to the embedding, and bounds the length
+    tied_head: bool = False             # logits from the (unscaled) embedding table instead of a head of their own
 
     @property
     def layer_runs(self) -> List[int]:
@@ -276,8 +337,58 @@ def kesirax_config(raw: dict) -> TokenLMConfig:
         loop_stop=int(loop.get("stop", 0)), loop_times=int(loop.get("times", 1)))
 
 
-# config.json `architecture` -> parser; the registry `loaders.get_token_lm` and the command lines choose a model class by
-TOKEN_LM_ARCHITECTURES = {"Kesirax": kesirax_config}
+def bibapel_config(raw: dict, shapes: Optional[dict] = None) -> TokenLMConfig:
+    """config.json of a Bibapel model -> TokenLMConfig.  `shapes` (tensor name -> shape) gives the ranks of the low-rank projections, which
+    the file does not name; without it (random weights) they are the sizes of one head."""
+    def rank(i, name, default):
+        return int(shapes[f"l{i}.mix.{name}"][0]) if shapes is not None and f"l{i}.mix.{name}" in shapes else default
+
+    def mlp(m):
+        if m is None:
+            return None
+        _known(m, ("kind", "ff", "limit"), "mlp")
+        if m.get("kind", "dense") != "dense":
+            raise ValueError(f"mlp kind {m['kind']!r} is not part of this design")
+        return DenseGLUConfig(ff=int(m["ff"]), limit=float(m["limit"]))
+
+    def mixer(i, kind, m):
+        heads, dim, vdim = int(m["heads"]), int(m["dim"]), int(m["vdim"])
+        if kind == "attention":
+            _known(m, ("heads", "kv_heads", "dim", "vdim", "scale", "mask"), "attention")
+            mask = m.get("mask") or {}
+            _known(mask, ("size", "keep_first"), "mask")
+            return GroupedAttentionConfig(heads=heads, kv_heads=int(m.get("kv_heads", heads)), dim=dim, vdim=vdim, scale=float(m["scale"]),
+                                          window=int(mask.get("size", 0)), keep_first=int(mask.get("keep_first", 0)), sink=True)
+        if kind == "channel_delta":
+            _known(m, ("heads", "kv_heads", "dim", "vdim", "conv"), "channel_delta")
+            return ChannelDeltaConfig(heads=heads, kv_heads=int(m.get("kv_heads", heads)), dim=dim, vdim=vdim, conv=int(m["conv"]),
+                                      decay_rank=rank(i, "a1", dim), gate_rank=rank(i, "g1", vdim))
+        if kind == "lightning":
+            _known(m, ("heads", "dim", "vdim", "decay"), "lightning")
+            decay = m["decay"] if isinstance(m["decay"], list) else [m["decay"]] * heads
+            if len(decay) != heads:
+                raise ValueError("lightning: one decay per head")
+            return LightningConfig(heads=heads, dim=dim, vdim=vdim, decay=[float(d) for d in decay])
+        raise ValueError(f"mixer type {kind!r} is not part of this design")
+
+    _known(raw, ("architecture", "embedding", "layers", "loop", "max_positions", "norm", "vocab", "width"), "config")
+    emb, loop = raw.get("embedding") or {}, raw.get("loop") or {}
+    _known(emb, ("scale", "bigram"), "embedding")
+    _known(raw["norm"], ("eps",), "norm")
+    _known(loop, ("start", "stop", "times"), "loop")
+    big = emb.get("bigram")
+    return TokenLMConfig(
+        architecture=raw["architecture"], vocab=int(raw["vocab"]), width=int(raw["width"]),
+        layers=[TokenLayerConfig(mixer(i, l["type"], l["mixer"]), mlp(l.get("mlp"))) for i, l in enumerate(raw["layers"])],
+        norm_eps=float(raw["norm"]["eps"]), loop_start=int(loop.get("start", 0)), loop_stop=int(loop.get("stop", 0)),
+        loop_times=int(loop.get("times", 1)), loop_inject="project", norms=2, layer_scales=False, embed_scale=float(emb.get("scale", 1.0)),
+        bigram=BigramConfig(int(big["buckets"]), int(big["mul_prev"]), int(big["mul_cur"])) if big else None,
+        max_positions=int(raw.get("max_positions", 0)), tied_head=True)
+
+
+# config.json `architecture` -> parser (config, tensor shapes); the registry `loaders.get_token_lm` and the command lines choose a model
+# class by
+TOKEN_LM_ARCHITECTURES = {"Kesirax": lambda raw, shapes=None: kesirax_config(raw), "Bibapel": bibapel_config}
 
 
 def tiny_token_lm_config() -> TokenLMConfig:
@@ -287,3 +398,15 @@ def tiny_token_lm_config() -> TokenLMConfig:
     return TokenLMConfig("Kesirax", vocab=101, width=96, norm_groups=3, norm_eps=1e-5, logit_scale=0.7, loop_start=1, loop_stop=3, loop_times=2,
                          layers=[TokenLayerConfig(MinGRUConfig(72), moe), TokenLayerConfig(att, moe), TokenLayerConfig(MinGRUConfig(72), None),
                                  TokenLayerConfig(att, MoEConfig(experts=4, top=1, ff=52))])
+
+
+def tiny_bibapel_config() -> TokenLMConfig:
+    """A Bibapel network at oracle size, with sizes that are no multiples of the kernels' tiles."""
+    delta = ChannelDeltaConfig(heads=4, kv_heads=2, dim=20, vdim=24, conv=3, decay_rank=10, gate_rank=14)
+    att = GroupedAttentionConfig(heads=6, kv_heads=2, dim=24, vdim=20, scale=0.21, window=41, keep_first=5, sink=True)
+    light = LightningConfig(heads=3, dim=18, vdim=28, decay=[0.7, 0.93, 0.995])
+    glu = DenseGLUConfig(ff=72, limit=1.5)
+    return TokenLMConfig("Bibapel", vocab=97, width=80, norm_eps=1e-5, loop_start=1, loop_stop=3, loop_times=2, loop_inject="project", norms=2,
+                         layer_scales=False, embed_scale=0.8, bigram=BigramConfig(buckets=37, mul_prev=11, mul_cur=5), max_positions=1500, tied_head=True,
+                         layers=[TokenLayerConfig(light, glu), TokenLayerConfig(delta, glu), TokenLayerConfig(att, DenseGLUConfig(ff=56, limit=0.9)),
+                                 TokenLayerConfig(delta, None)])

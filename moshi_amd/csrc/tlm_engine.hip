@@ -1,11 +1,11 @@
 // Token language models behind the C ABI of include/moshi_tlm.h: decoder-only networks whose layers are described by mmi_tlm_cfg,
-// stepped over mixed batches (prompt portions beside single tokens) from a paged latent cache and recurrent state slots.
+// stepped over mixed batches (prompt portions beside single tokens) from a paged cache and recurrent state slots.
 //
 //   step   = prepare (tokens, block tables, rotation tables) -> routing -> per layer run:
-//              residual + norm | mixer projections, expert up | mixer core | mixer output, expert down
+//              residual + norm(s) | mixer projections, feed-forward up | mixer core | mixer output, feed-forward down
 //            -> residual + norm of the wanted rows -> head
-//   The sublayers of a layer read one norm, so the mixer's input projection and the experts' up projection are one launch, and so
-//   are the mixer's output projection and the experts' down projection (TlmJobs).
+//   The sublayers of a layer read norms of one input, so the mixer's input projection and the feed-forward's up projection are one
+//   launch, and so are the mixer's output projection and the feed-forward's down projection (TlmJobs).
 // Steps that only bring single tokens are captured into a hipGraph per shape (batch, wanted rows, attention split): everything that
 // varies between two such steps is device memory uploaded in one copy.
 #include "mmi_common.h"
@@ -13,6 +13,8 @@
 #include "../../include/moshi_tlm.h"
 #include "lm_kernels.h"
 #include "tlm_kernels.h"
+#include "tlm_gqa.h"
+#include "tlm_linear.h"
 
 #include <math.h>
 #include <algorithm>
@@ -37,7 +39,7 @@ struct Mat {                       // one packed matrix, or `groups` of equal sh
 
 struct Layer {
     mmi_tlm_layer c;
-    float *norm = nullptr, *ls1 = nullptr, *ls2 = nullptr;
+    float *norm = nullptr, *norm2 = nullptr, *ls1 = nullptr, *ls2 = nullptr;
     // minGRU
     Mat zcg, out;
     float* bias = nullptr;
@@ -47,16 +49,23 @@ struct Layer {
     float *qw = nullptr, *cw = nullptr;
     int qp = 0, kvp = 0, rp = 0, hp = 0, dim_p = 0, vdim_p = 0, lat_ks = 0, k_ks = 0, nd = 0, q_ks = 0, qn_ks = 0;
     int rope = -1, geo = -1;
-    // experts
+    // grouped attention: `in` is [queries | keys | values]; k_ks, nd as above
+    // channel delta: `in` is [q | k | v | beta], `lr` the low-rank halves of decay and gate, `a2` and `g2` the others; lightning: [q | k | v | gate]
+    Mat lr, a2, g2;
+    float *conv_w = nullptr, *decay = nullptr, *nw = nullptr;      // decay: (summand, factor) per column / powers of the constants
+    int in_ld = 0, conv_c = 0, ra = 0, q0 = 0, k0 = 0, v0 = 0, b0 = 0;
+    // feed-forward: experts, or one dense pair (gate and up rows alternate)
     Mat up, down;
     int route = -1;
+    bool linear() const { return c.mixer == MMI_TLM_MIX_CHANNEL_DELTA || c.mixer == MMI_TLM_MIX_LIGHTNING; }
 };
 
 struct Run {                       // one execution of a layer: repeated layers share weights, not state
     int layer = 0;
     bool add_emb = false;
-    void* kc = nullptr;
-    float* state = nullptr;
+    int pass = -1;                 // first layer of a pass that starts with the projection of [x; embedding]
+    void *kc = nullptr, *vc = nullptr;
+    float *state = nullptr, *conv = nullptr;
 };
 
 struct Slot {
@@ -65,6 +74,8 @@ struct Slot {
     int par = 0;                   // which copy of the recurrent state is current
     int64_t first_page = 0;        // pages before it have left every window
     std::vector<int> pages;        // pages[i] holds positions 64 (first_page + i) ..
+    std::vector<int> kept;         // the sequence's first pages, once the windows have passed them but for the positions they keep
+    int page(int64_t i) const { return i < first_page ? kept[(size_t)i] : pages[(size_t)(i - first_page)]; }
 };
 
 struct Staging {
@@ -75,12 +86,13 @@ struct Staging {
 
 // where the parts of a step's metadata sit in the uploaded block (ints)
 struct Meta {
-    int htok, pos, rslot, crow, want, erow0, elen, epos0, eslot, tile0, seg, upd, total;
+    int htok, pos, rslot, crow, prev, next, want, erow0, elen, epos0, eslot, tile0, seg, small, unit, chunk, upd, total;
 };
 
 struct Shape {                     // what a launch list depends on
     int T = 0, n_want = 0, n_entries = 0, n_seg = 0, nsplit = 1;
     bool pairs = false;            // some sequence spans several scan segments
+    int n_small = 0, n_unit = 0, n_chunk = 0;      // sequences stepped token by token, sequences cut into chunks, their chunks
     std::vector<int> tiles;        // attention column tiles per head count
     std::vector<std::array<int, 2>> groups;        // column groups of 4 and of 8 tiles per head count
     Meta m;
@@ -99,10 +111,13 @@ struct mmi_tlm {
     int kstep = 32, V = 8;
     int ld = 0, h_ks = 0;
     int max_slots = 0, max_pages = 0, max_T = 0;
-    bool has_attn = false, has_gru = false;
+    bool has_attn = false, has_latent = false, has_gru = false, has_linear = false;      // has_attn: some layer has a paged cache
     int64_t max_window = 0;        // 0: some layer sees every earlier position
+    int keep_pages = 0;            // with windows: a sequence's first pages that are never released
     MmiArena wts, st, scratch;
-    uint16_t* embed = nullptr;
+    uint16_t *embed = nullptr, *bigram = nullptr, *pos_emb = nullptr;
+    Mat loop_in;
+    float* loop_step = nullptr;    // [times][ld]
     float* final_norm = nullptr;
     Mat head;
     std::vector<int> geo;          // distinct head counts
@@ -115,6 +130,10 @@ struct mmi_tlm {
     long tile_ld = 0, list_ld = 0;
     // scratch
     float *x = nullptr, *mix = nullptr, *dn = nullptr, *zcg = nullptr, *lat = nullptr, *gate = nullptr, *pair = nullptr, *po = nullptr, *pml = nullptr;
+    float *lin = nullptr, *qkv = nullptr, *dec = nullptr, *lgate = nullptr, *lo = nullptr, *cw = nullptr, *cq_g = nullptr, *ckt = nullptr, *cu0 = nullptr, *cp = nullptr,
+          *cgend = nullptr;
+    void *h2 = nullptr, *cat = nullptr, *lr = nullptr;
+    int *brow = nullptr, *prev_tok = nullptr;
     void *h = nullptr, *y = nullptr, *cq = nullptr, *qn = nullptr, *q = nullptr, *ao = nullptr, *o = nullptr, *hid = nullptr;
     int *list = nullptr, *tiles = nullptr, *n_tiles = nullptr, *tok = nullptr, *meta = nullptr, *last_tok = nullptr, *block_table = nullptr;
     float* logits = nullptr;       // [max_slots][vocab] for captured steps
@@ -191,13 +210,13 @@ struct Loader {
     }
     // tiles 0 .. rows/16 of the source (through the maps) become tiles t * tmul + toff of `dst`; the maps stay on the device until the
     // next upload, so packing many matrices of one shape uploads them once
-    int pack(const mmi_tensor_desc* d, u32x4* dst, int rows, int cols, long sr, long sc, int tmul = 1, int toff = 0, long src_off = 0) {
+    int pack(const mmi_tensor_desc* d, u32x4* dst, int rows, int cols, long sr, long sc, int tmul = 1, int toff = 0, long src_off = 0, int keep = 0) {
         const int NT = rows / 16, KS = cols / m->kstep;
         const long n = (long)NT * KS * 64 * m->V;
         const int blocks = (int)mmi_cdiv64(n, 256);
         const uint16_t* src = (const uint16_t*)d->data + src_off;
-        if (m->f32) MMI_LAUNCH((k_tlm_pack<TlmF32>), blocks, 256, 0, (hipStream_t)0, src, sr, sc, map, map + rows, (float*)dst, NT, KS, tmul, toff);
-        else MMI_LAUNCH((k_tlm_pack<TlmBf16>), blocks, 256, 0, (hipStream_t)0, src, sr, sc, map, map + rows, (uint16_t*)dst, NT, KS, tmul, toff);
+        if (m->f32) MMI_LAUNCH((k_tlm_pack<TlmF32>), blocks, 256, 0, (hipStream_t)0, src, sr, sc, map, map + rows, (float*)dst, NT, KS, tmul, toff, keep);
+        else MMI_LAUNCH((k_tlm_pack<TlmBf16>), blocks, 256, 0, (hipStream_t)0, src, sr, sc, map, map + rows, (uint16_t*)dst, NT, KS, tmul, toff, keep);
         MMI_CHECK_LAUNCH();
         return MMI_OK;
     }
@@ -214,6 +233,56 @@ struct Loader {
         const int rows = round_up(N, 16), cols = round_up(K, m->kstep);
         if ((rc = find(name, MMI_BF16, {N, K}, &d)) || (rc = alloc(mat, 1, rows / 16, cols / m->kstep)) || (rc = ident(N, rows, K, cols))) return rc;
         return pack(d, mat->wp, rows, cols, K, 1);
+    }
+    // a bf16 tensor's values on the host (small tensors)
+    int host(const std::string& name, std::initializer_list<int64_t> shape, std::vector<float>* out) {
+        const mmi_tensor_desc* d;
+        int rc = find(name, MMI_BF16, shape, &d);
+        if (rc) return rc;
+        size_t n = 1;
+        for (int64_t s : shape) n *= (size_t)s;
+        std::vector<uint16_t> h(n);
+        MMI_HIP_CHECK(hipMemcpy(h.data(), d->data, n * 2, hipMemcpyDeviceToHost));
+        out->resize(n);
+        for (size_t i = 0; i < n; ++i) (*out)[i] = mmi_bf16_to_f32(h[i]);
+        return MMI_OK;
+    }
+    int to_device(const std::vector<float>& v, float** out) {
+        MMI_HIP_CHECK(m->wts.alloc(out, v.size()));
+        MMI_HIP_CHECK(hipMemcpy(*out, v.data(), v.size() * sizeof(float), hipMemcpyHostToDevice));
+        return MMI_OK;
+    }
+    int table(const std::string& name, int64_t rows, int64_t cols, uint16_t** out) {
+        const mmi_tensor_desc* d;
+        int rc = find(name, MMI_BF16, {rows, cols}, &d);
+        if (rc) return rc;
+        MMI_HIP_CHECK(m->wts.alloc(out, (size_t)(rows * cols)));
+        MMI_HIP_CHECK(hipMemcpy(*out, d->data, (size_t)(rows * cols) * 2, hipMemcpyDeviceToDevice));
+        return MMI_OK;
+    }
+    // head by head linear [heads * n][K] -> tiles toff .. of `mat`, every head padded to np rows
+    int heads(const std::string& name, int heads, int n, int np, int K, Mat* mat, int toff) {
+        const mmi_tensor_desc* d;
+        int rc;
+        const int cols = mat->KS * m->kstep;
+        std::vector<int> a(round_up(heads * np, 16), -1), b(cols, -1);
+        for (int h = 0; h < heads; ++h)
+            for (int i = 0; i < n; ++i) a[(size_t)h * np + i] = h * n + i;
+        for (int i = 0; i < K; ++i) b[i] = i;
+        if ((rc = find(name, MMI_BF16, {(int64_t)heads * n, K}, &d)) || (rc = upload(a, b))) return rc;
+        return pack(d, mat->wp, (int)a.size(), cols, K, 1, 1, toff);
+    }
+    // output projection [N][heads * n] over heads padded to np
+    int over_heads(const std::string& name, int N, int heads, int n, int np, Mat* mat) {
+        const mmi_tensor_desc* d;
+        int rc;
+        const int rows = round_up(N, 16), cols = round_up(heads * np, m->kstep);
+        std::vector<int> a(rows, -1), b(cols, -1);
+        for (int i = 0; i < N; ++i) a[i] = i;
+        for (int h = 0; h < heads; ++h)
+            for (int j = 0; j < n; ++j) b[(size_t)h * np + j] = h * n + j;
+        if ((rc = find(name, MMI_BF16, {N, (int64_t)heads * n}, &d)) || (rc = alloc(mat, 1, rows / 16, cols / m->kstep)) || (rc = upload(a, b))) return rc;
+        return pack(d, mat->wp, rows, cols, (long)heads * n, 1);
     }
     int vec(const std::string& name, int n, int padded, float** out) {
         const mmi_tensor_desc* d;
@@ -327,6 +396,117 @@ int load_latent_attention(Loader& ld, Layer& L, const std::string& p) {
     return ld.pack(d, L.out.wp, rows, ok, (long)H * c.vdim, 1);
 }
 
+int load_attention(Loader& ld, Layer& L, const std::string& p) {
+    mmi_tlm* m = ld.m;
+    const mmi_tlm_layer& c = L.c;
+    const int D = m->cfg.width, H = c.heads, G = c.kv_heads, ks = m->kstep;
+    L.dim_p = round_up(c.dim, ks);
+    L.vdim_p = round_up(c.vdim, 16);
+    L.k_ks = L.dim_p / ks;
+    L.nd = L.vdim_p / 16;
+    const std::string mx = p + ".mix.";
+    int rc;
+    if ((rc = ld.alloc(&L.in, 1, ((H + G) * L.dim_p + G * L.vdim_p) / 16, round_up(D, ks) / ks)) || (rc = ld.heads(mx + "q", H, c.dim, L.dim_p, D, &L.in, 0)) ||
+        (rc = ld.heads(mx + "k", G, c.dim, L.dim_p, D, &L.in, H * L.dim_p / 16)) ||
+        (rc = ld.heads(mx + "v", G, c.vdim, L.vdim_p, D, &L.in, (H + G) * L.dim_p / 16)))
+        return rc;
+    return ld.over_heads(mx + "o", D, H, c.vdim, L.vdim_p, &L.out);
+}
+
+// queries, keys, values of a mixer with a matrix state, and one more section of `extra` heads of `extra_n` columns
+int load_linear_in(Loader& ld, Layer& L, const std::string& mx, int QH, const char* extra, int extra_heads, int extra_n) {
+    mmi_tlm* m = ld.m;
+    const mmi_tlm_layer& c = L.c;
+    const int D = m->cfg.width, H = c.heads;
+    L.dim_p = round_up(c.dim, 16);
+    L.vdim_p = round_up(c.vdim, 16);
+    L.q0 = 0;
+    L.k0 = QH * L.dim_p;
+    L.v0 = 2 * QH * L.dim_p;
+    L.b0 = L.v0 + H * L.vdim_p;
+    const int extra_p = extra_heads > 1 && extra_n > 1 ? round_up(extra_n, 16) : (extra_n > 1 ? L.vdim_p : 1);
+    L.in_ld = L.b0 + round_up(extra_heads * extra_p, 16);
+    int rc;
+    if ((rc = ld.alloc(&L.in, 1, L.in_ld / 16, round_up(D, m->kstep) / m->kstep)) || (rc = ld.heads(mx + "q", QH, c.dim, L.dim_p, D, &L.in, 0)) ||
+        (rc = ld.heads(mx + "k", QH, c.dim, L.dim_p, D, &L.in, L.k0 / 16)) || (rc = ld.heads(mx + "v", H, c.vdim, L.vdim_p, D, &L.in, L.v0 / 16)) ||
+        (rc = ld.heads(mx + extra, extra_heads, extra_n, extra_p, D, &L.in, L.b0 / 16)))
+        return rc;
+    return ld.over_heads(mx + "o", D, H, c.vdim, L.vdim_p, &L.out);
+}
+
+int load_channel_delta(Loader& ld, Layer& L, const std::string& p) {
+    mmi_tlm* m = ld.m;
+    const mmi_tlm_layer& c = L.c;
+    const int D = m->cfg.width, H = c.heads, G = c.kv_heads, ks = m->kstep;
+    const std::string mx = p + ".mix.";
+    int rc;
+    if ((rc = load_linear_in(ld, L, mx, G, "b", H, 1))) return rc;
+    L.conv_c = L.b0;
+    const char* parts[3] = {"q", "k", "v"};
+    std::vector<float> src, w((size_t)c.conv * L.conv_c, 0.f);
+    for (int k = 0; k < 3; ++k) {
+        const int nh = k == 2 ? H : G, n = k == 2 ? c.vdim : c.dim, np = k == 2 ? L.vdim_p : L.dim_p, c0 = k == 0 ? L.q0 : (k == 1 ? L.k0 : L.v0);
+        if ((rc = ld.host(mx + parts[k] + ".conv", {(int64_t)nh * n, c.conv}, &src))) return rc;
+        for (int h = 0; h < nh; ++h)
+            for (int i = 0; i < n; ++i)
+                for (int j = 0; j < c.conv; ++j) w[(size_t)j * L.conv_c + c0 + h * np + i] = src[((size_t)h * n + i) * c.conv + j];
+    }
+    if ((rc = ld.to_device(w, &L.conv_w))) return rc;
+    // decay: exp(-factor softplus(x + summand)), factor = exp(A_log) of the head
+    std::vector<float> alog, bias;
+    if ((rc = ld.host(mx + "A_log", {H}, &alog)) || (rc = ld.host(mx + "dt_bias", {(int64_t)H * c.dim}, &bias))) return rc;
+    const int dcols = H * L.dim_p;
+    std::vector<float> dec((size_t)2 * dcols, 0.f);
+    for (int h = 0; h < H; ++h)
+        for (int i = 0; i < L.dim_p; ++i) {
+            dec[(size_t)h * L.dim_p + i] = i < c.dim ? bias[(size_t)h * c.dim + i] : 0.f;
+            dec[(size_t)dcols + h * L.dim_p + i] = (float)exp((double)alog[h]);
+        }
+    if ((rc = ld.to_device(dec, &L.decay)) || (rc = ld.vec(mx + "norm", c.vdim, L.vdim_p, &L.nw))) return rc;
+    // low-rank halves: both read the layer's norm, so they are one matrix
+    L.ra = round_up(c.decay_rank, ks);
+    const int rg = round_up(c.gate_rank, ks), cols = round_up(D, ks) / ks;
+    if ((rc = ld.alloc(&L.lr, 1, (L.ra + rg) / 16, cols)) || (rc = ld.heads(mx + "a1", 1, c.decay_rank, L.ra, D, &L.lr, 0)) ||
+        (rc = ld.heads(mx + "g1", 1, c.gate_rank, rg, D, &L.lr, L.ra / 16)) || (rc = ld.alloc(&L.a2, 1, dcols / 16, L.ra / ks)) ||
+        (rc = ld.heads(mx + "a2", H, c.dim, L.dim_p, c.decay_rank, &L.a2, 0)) || (rc = ld.alloc(&L.g2, 1, H * L.vdim_p / 16, rg / ks)))
+        return rc;
+    return ld.heads(mx + "g2", H, c.vdim, L.vdim_p, c.gate_rank, &L.g2, 0);
+}
+
+int load_lightning(Loader& ld, Layer& L, const std::string& p) {
+    const mmi_tlm_layer& c = L.c;
+    const int H = c.heads;
+    const std::string mx = p + ".mix.";
+    int rc;
+    if ((rc = load_linear_in(ld, L, mx, H, "g", H, c.vdim))) return rc;
+    std::vector<float> w, wp((size_t)H * L.vdim_p, 0.f), pw((size_t)H * (TLM_CHUNK + 1));
+    if ((rc = ld.host(mx + "norm", {(int64_t)H * c.vdim}, &w))) return rc;
+    for (int h = 0; h < H; ++h) {
+        for (int i = 0; i < c.vdim; ++i) wp[(size_t)h * L.vdim_p + i] = w[(size_t)h * c.vdim + i];
+        for (int i = 0; i <= TLM_CHUNK; ++i) pw[(size_t)h * (TLM_CHUNK + 1) + i] = (float)pow(c.decay[h], i);
+    }
+    if ((rc = ld.to_device(wp, &L.nw))) return rc;
+    return ld.to_device(pw, &L.decay);
+}
+
+int load_dense_glu(Loader& ld, Layer& L, const std::string& p) {
+    mmi_tlm* m = ld.m;
+    const int D = m->cfg.width, F = L.c.ff, rows = round_up(2 * F, 16), cols = round_up(D, m->kstep);
+    const mmi_tensor_desc* d;
+    int rc;
+    if ((rc = ld.alloc(&L.up, 1, rows / 16, cols / m->kstep))) return rc;
+    std::vector<int> cm(cols, -1);
+    for (int i = 0; i < D; ++i) cm[i] = i;
+    for (int k = 0; k < 2; ++k) {                         // gate rows (the others zero), then the up rows between them
+        std::vector<int> rm(rows, -1);
+        for (int i = 0; i < F; ++i) rm[2 * i + k] = i;
+        if ((rc = ld.find(p + (k ? ".mlp.up" : ".mlp.gate"), MMI_BF16, {F, D}, &d)) || (rc = ld.upload(rm, cm)) ||
+            (rc = ld.pack(d, L.up.wp, rows, cols, D, 1, 1, 0, 0, k)))
+            return rc;
+    }
+    return ld.linear(p + ".mlp.down", D, F, &L.down);
+}
+
 int load_moe(Loader& ld, Layer& L, const std::string& p) {
     mmi_tlm* m = ld.m;
     const mmi_tlm_layer& c = L.c;
@@ -363,6 +543,9 @@ int check_cfg(const mmi_tlm_cfg& c) {
     if (c.width > 8192) return mmi_fail(MMI_ERR_UNSUPPORTED, "token LM: width above 8192");
     if (c.loop_start < 0 || c.loop_stop < c.loop_start || c.loop_stop > c.n_layers || (c.loop_stop > c.loop_start && c.loop_times < 1))
         return mmi_fail(MMI_ERR_INVALID, "token LM: bad layer repetition");
+    if (c.loop_inject != MMI_TLM_LOOP_ADD && c.loop_inject != MMI_TLM_LOOP_PROJECT) return mmi_fail(MMI_ERR_UNSUPPORTED, "token LM: unknown start of a pass");
+    if (c.norms < 1 || c.norms > 2) return mmi_fail(MMI_ERR_INVALID, "token LM: one or two norms per layer");
+    if (c.bigram_buckets < 0 || c.max_positions < 0) return mmi_fail(MMI_ERR_INVALID, "token LM: embedding sizes");
     for (int i = 0; i < c.n_layers; ++i) {
         const mmi_tlm_layer& l = c.layers[i];
         const std::string at = "token LM, layer " + std::to_string(i) + ": ";
@@ -375,6 +558,14 @@ int check_cfg(const mmi_tlm_cfg& c) {
             if (l.rot_dim > 128) return mmi_fail(MMI_ERR_UNSUPPORTED, at + "rot_dim above 128");
             if (round_up(l.q_rank, 16) + round_up(l.kv_rank, 16) + round_up(l.rot_dim, 16) + round_up(l.heads, 16) > 8192)
                 return mmi_fail(MMI_ERR_UNSUPPORTED, at + "query latent above the kernel's row buffer");
+        } else if (l.mixer == MMI_TLM_MIX_ATTENTION || l.mixer == MMI_TLM_MIX_CHANNEL_DELTA || l.mixer == MMI_TLM_MIX_LIGHTNING) {
+            const bool shared = l.mixer != MMI_TLM_MIX_LIGHTNING;
+            if (l.heads < 1 || l.dim < 1 || l.vdim < 1 || (shared && (l.kv_heads < 1 || l.heads % l.kv_heads))) return mmi_fail(MMI_ERR_INVALID, at + "head sizes");
+            if (l.dim > 256 || l.vdim > 256) return mmi_fail(MMI_ERR_UNSUPPORTED, at + "heads above 256 dimensions");
+            if (l.heads > 65535) return mmi_fail(MMI_ERR_UNSUPPORTED, at + "more than 65535 heads");
+            if (l.mixer == MMI_TLM_MIX_ATTENTION && (l.window < 0 || l.keep_first < 0)) return mmi_fail(MMI_ERR_INVALID, at + "attention window");
+            if (l.mixer == MMI_TLM_MIX_CHANNEL_DELTA && (l.conv < 1 || l.decay_rank < 1 || l.gate_rank < 1)) return mmi_fail(MMI_ERR_INVALID, at + "delta rule sizes");
+            if (l.mixer == MMI_TLM_MIX_LIGHTNING && !l.decay) return mmi_fail(MMI_ERR_INVALID, at + "no decay");
         } else {
             return mmi_fail(MMI_ERR_UNSUPPORTED, at + "unknown mixer");
         }
@@ -382,6 +573,9 @@ int check_cfg(const mmi_tlm_cfg& c) {
             if (l.experts < 1 || l.top < 1 || l.top > l.experts || l.ff < 1) return mmi_fail(MMI_ERR_INVALID, at + "expert sizes");
             if (l.experts > 4096) return mmi_fail(MMI_ERR_UNSUPPORTED, at + "more than 4096 experts");
             if (l.act != MMI_TLM_ACT_RELU2 || l.router != MMI_TLM_ROUTE_TOKEN_TABLE) return mmi_fail(MMI_ERR_UNSUPPORTED, at + "unknown expert activation or router");
+        } else if (l.mlp == MMI_TLM_MLP_DENSE) {
+            if (l.ff < 1 || !(l.limit > 0.f)) return mmi_fail(MMI_ERR_INVALID, at + "feed-forward sizes");
+            if (l.act != MMI_TLM_ACT_CLAMPED_SWIGLU) return mmi_fail(MMI_ERR_UNSUPPORTED, at + "unknown feed-forward activation");
         } else if (l.mlp != MMI_TLM_MLP_NONE) {
             return mmi_fail(MMI_ERR_UNSUPPORTED, at + "unknown feed-forward");
         }
@@ -406,6 +600,8 @@ int alloc_f32(mmi_tlm* m, float** p, size_t n) {
     return MMI_OK;
 }
 
+int table_ld(const mmi_tlm* m) { return m->keep_pages + std::max(1, m->max_pages); }      // block-table entries per slot
+
 int alloc_buffers(mmi_tlm* m) {
     const mmi_tlm_cfg& c = m->cfg;
     const int T = m->max_T;
@@ -413,10 +609,29 @@ int alloc_buffers(mmi_tlm* m) {
     m->split_elems = std::max((long)T, (long)MAX_SPLIT * ROWS_MAX);
     int gru_w = 0, y_ks = 0, lat_ld = 0, cq_ks = 0, qn_ks = 0, o_ks = 0, hid_ks = 0, gate_ld = 0, nd = 0;
     long q_elems = 0, ao_elems = 0;
+    long lin_ld = 0, conv_c = 0, dec_ld = 0, lgate_ld = 0, lo_ld = 0, heads = 0, hd = 0, hv = 0;
+    int lr_ks = 0;
     for (const Layer& L : m->layers) {
         if (L.c.mixer == MMI_TLM_MIX_MINGRU) {
             gru_w = std::max(gru_w, L.wp);
             y_ks = std::max(y_ks, L.out.KS);
+        } else if (L.c.mixer == MMI_TLM_MIX_ATTENTION) {
+            q_elems = std::max(q_elems, (long)((T * (long)L.c.heads + 15) / 16) * L.k_ks);
+            o_ks = std::max(o_ks, L.out.KS);
+            nd = std::max(nd, L.nd);
+        } else if (L.linear()) {
+            lin_ld = std::max(lin_ld, (long)L.in_ld);
+            conv_c = std::max(conv_c, (long)L.conv_c);
+            heads = std::max(heads, (long)L.c.heads);
+            hd = std::max(hd, (long)L.c.heads * L.dim_p);
+            hv = std::max(hv, (long)L.c.heads * L.vdim_p);
+            o_ks = std::max(o_ks, L.out.KS);
+            if (L.c.mixer == MMI_TLM_MIX_CHANNEL_DELTA) {
+                lr_ks = std::max(lr_ks, L.lr.NT * 16 / m->kstep);
+                dec_ld = std::max(dec_ld, (long)L.c.heads * L.dim_p);
+                lgate_ld = std::max(lgate_ld, (long)L.c.heads * L.vdim_p);
+            }
+            lo_ld = std::max(lo_ld, (long)L.c.heads * L.vdim_p);
         } else {
             lat_ld = std::max(lat_ld, L.qp + L.kvp + L.rp + L.hp);
             cq_ks = std::max(cq_ks, L.q_ks);
@@ -427,7 +642,7 @@ int alloc_buffers(mmi_tlm* m) {
             gate_ld = std::max(gate_ld, L.c.heads);
             nd = std::max(nd, L.nd);
         }
-        if (L.c.mlp == MMI_TLM_MLP_MOE) hid_ks = std::max(hid_ks, L.down.KS);
+        if (L.c.mlp != MMI_TLM_MLP_NONE) hid_ks = std::max(hid_ks, L.down.KS);
     }
     if ((rc = alloc_f32(m, &m->x, (size_t)T * m->ld)) || (rc = alloc_packed(m, &m->h, std::max(T, m->max_slots), m->h_ks)) ||
         (rc = alloc_f32(m, &m->mix, (size_t)m->split_elems * m->ld)))
@@ -436,7 +651,28 @@ int alloc_buffers(mmi_tlm* m) {
         const int n_seg = T / TLM_SEG + m->max_slots + 1;
         if ((rc = alloc_f32(m, &m->zcg, (size_t)T * 3 * gru_w)) || (rc = alloc_packed(m, &m->y, T, y_ks)) || (rc = alloc_f32(m, &m->pair, (size_t)n_seg * 2 * gru_w))) return rc;
     }
-    if (m->has_attn) {
+    if (c.norms == 2 && (rc = alloc_packed(m, &m->h2, std::max(T, m->max_slots), m->h_ks))) return rc;
+    if (m->loop_in.wp && (rc = alloc_packed(m, &m->cat, T, 2 * m->h_ks))) return rc;
+    if (m->has_linear) {
+        const size_t n_chunk = (size_t)T / TLM_CHUNK + std::min(m->max_slots, T / (TLM_SMALL + 1)) + 1;      // only sequences above TLM_SMALL tokens have any
+        if ((rc = alloc_f32(m, &m->lin, (size_t)T * lin_ld)) || (rc = alloc_f32(m, &m->qkv, (size_t)T * conv_c)) || (rc = alloc_f32(m, &m->dec, (size_t)T * dec_ld)) ||
+            (rc = alloc_f32(m, &m->lgate, (size_t)T * lgate_ld)) || (rc = alloc_f32(m, &m->lo, (size_t)T * lo_ld)) || (rc = alloc_packed(m, &m->lr, T, std::max(1, lr_ks))) ||
+            (rc = alloc_f32(m, &m->cw, conv_c ? n_chunk * TLM_CHUNK * hd : 1)) || (rc = alloc_f32(m, &m->cq_g, n_chunk * TLM_CHUNK * hd)) ||
+            (rc = alloc_f32(m, &m->ckt, n_chunk * TLM_CHUNK * hd)) || (rc = alloc_f32(m, &m->cu0, conv_c ? n_chunk * TLM_CHUNK * hv : 1)) ||
+            (rc = alloc_f32(m, &m->cp, n_chunk * TLM_CHUNK * TLM_CHUNK * heads)) || (rc = alloc_f32(m, &m->cgend, n_chunk * hd)))
+            return rc;
+    }
+    if (m->has_attn && !m->has_latent) {
+        if ((rc = alloc_packed(m, &m->q, q_elems * 16, 1)) || (rc = alloc_f32(m, &m->po, (size_t)MAX_PARTIALS * nd * 256)) || (rc = alloc_f32(m, &m->pml, (size_t)MAX_PARTIALS * 32)))
+            return rc;
+    }
+    if (!m->has_latent && (m->has_attn || m->has_linear) && (rc = alloc_packed(m, &m->o, T, o_ks))) return rc;
+    if (c.bigram_buckets > 0) {
+        MMI_HIP_CHECK(m->scratch.alloc(&m->brow, T));
+        MMI_HIP_CHECK(m->scratch.alloc(&m->prev_tok, 2 * (size_t)m->max_slots));
+        MMI_HIP_CHECK(hipMemset(m->prev_tok, 0, 2 * (size_t)m->max_slots * sizeof(int)));
+    }
+    if (m->has_latent) {
         if ((rc = alloc_f32(m, &m->lat, (size_t)m->split_elems * lat_ld)) || (rc = alloc_packed(m, &m->cq, T, cq_ks)) || (rc = alloc_packed(m, &m->qn, T, qn_ks)) ||
             (rc = alloc_packed(m, &m->q, q_elems * 16, 1)) || (rc = alloc_packed(m, &m->ao, ao_elems * 16, 1)) || (rc = alloc_packed(m, &m->o, T, o_ks)) ||
             (rc = alloc_f32(m, &m->gate, (size_t)T * gate_ld)) || (rc = alloc_f32(m, &m->po, (size_t)MAX_PARTIALS * nd * 256)) ||
@@ -444,6 +680,9 @@ int alloc_buffers(mmi_tlm* m) {
             return rc;
         for (TlmRope& r : m->rope_host)
             if ((rc = alloc_f32(m, &r.out, (size_t)T * r.ld * 2))) return rc;
+    }
+    if (m->route_host.empty() && hid_ks) {
+        if ((rc = alloc_packed(m, &m->hid, T, hid_ks)) || (rc = alloc_f32(m, &m->dn, (size_t)std::max((long)T, (long)MAX_SPLIT * ROWS_MAX) * m->ld))) return rc;
     }
     if (!m->route_host.empty()) {
         const size_t nl = m->route_host.size();
@@ -464,8 +703,9 @@ int alloc_buffers(mmi_tlm* m) {
     MMI_HIP_CHECK(hipMemset(m->tok, 0, (size_t)T * sizeof(int)));
     MMI_HIP_CHECK(m->scratch.alloc(&m->last_tok, m->max_slots));
     MMI_HIP_CHECK(hipMemset(m->last_tok, 0, (size_t)m->max_slots * sizeof(int)));
-    MMI_HIP_CHECK(m->scratch.alloc(&m->block_table, (size_t)m->max_slots * std::max(1, m->max_pages) + 1));
-    MMI_HIP_CHECK(hipMemset(m->block_table, 0, ((size_t)m->max_slots * std::max(1, m->max_pages) + 1) * sizeof(int)));
+    const size_t n_table = (size_t)m->max_slots * table_ld(m) + 1;
+    MMI_HIP_CHECK(m->scratch.alloc(&m->block_table, n_table));
+    MMI_HIP_CHECK(hipMemset(m->block_table, 0, n_table * sizeof(int)));
     if ((rc = alloc_f32(m, &m->logits, (size_t)m->max_slots * c.vocab))) return rc;
     m->samp_ld = round_up(c.vocab, 8);
     MMI_HIP_CHECK(m->scratch.alloc(&m->samp_rows, (size_t)m->max_slots * m->samp_ld));
@@ -473,8 +713,8 @@ int alloc_buffers(mmi_tlm* m) {
     MMI_HIP_CHECK(m->scratch.alloc(&m->samp_rng, 8));
     MMI_HIP_CHECK(m->scratch.alloc(&m->samp_zero, 1));
     MMI_HIP_CHECK(hipMemset(m->samp_zero, 0, sizeof(int)));
-    // metadata: 4 ints per token + wanted rows, per-entry arrays, tile prefixes, segments, block-table updates
-    m->meta_cap = 64 + (size_t)5 * T + 4 * (size_t)m->max_slots + 3 * m->geo.size() * ((size_t)m->max_slots + 1) + 8 * ((size_t)T / TLM_SEG + m->max_slots + 1) +
+    // metadata: 6 ints per token + wanted rows, per-entry arrays, tile prefixes, segments, sequences and chunks, block-table updates
+    m->meta_cap = 128 + (size_t)7 * T + 20 * (size_t)m->max_slots + 8 * ((size_t)T / TLM_CHUNK + m->max_slots + 1) + 3 * m->geo.size() * ((size_t)m->max_slots + 1) + 8 * ((size_t)T / TLM_SEG + m->max_slots + 1) +
                   2 * ((size_t)T / TLM_PAGE + 2 * (size_t)m->max_slots + 2);
     MMI_HIP_CHECK(m->scratch.alloc(&m->meta, m->meta_cap));
     for (Staging& s : m->staging) {
@@ -491,6 +731,23 @@ int alloc_state(mmi_tlm* m) {
             const size_t n = (size_t)m->max_slots * 2 * L.wp;
             MMI_HIP_CHECK(m->st.alloc(&r.state, n));
             MMI_HIP_CHECK(hipMemset(r.state, 0, n * sizeof(float)));
+        } else if (L.linear()) {
+            const size_t n = (size_t)m->max_slots * L.c.heads * L.dim_p * L.vdim_p, nc = (size_t)m->max_slots * 2 * std::max(1, L.c.conv - 1) * std::max(1, L.conv_c);
+            MMI_HIP_CHECK(m->st.alloc(&r.state, n));
+            MMI_HIP_CHECK(hipMemset(r.state, 0, n * sizeof(float)));
+            if (L.conv_c) {
+                MMI_HIP_CHECK(m->st.alloc(&r.conv, nc));
+                MMI_HIP_CHECK(hipMemset(r.conv, 0, nc * sizeof(float)));
+            }
+        } else if (L.c.mixer == MMI_TLM_MIX_ATTENTION) {
+            const size_t nk = (size_t)m->max_pages * L.c.kv_heads * 4 * L.k_ks * 64, nv = (size_t)m->max_pages * L.c.kv_heads * (TLM_PAGE / m->kstep) * L.nd * 64;
+            u32x4 *k = nullptr, *v = nullptr;
+            MMI_HIP_CHECK(m->st.alloc(&k, nk));
+            MMI_HIP_CHECK(hipMemset(k, 0, nk * 16));      // (as below)
+            MMI_HIP_CHECK(m->st.alloc(&v, nv));
+            MMI_HIP_CHECK(hipMemset(v, 0, nv * 16));
+            r.kc = k;
+            r.vc = v;
         } else {
             const size_t nk = (size_t)m->max_pages * 4 * L.k_ks * 64;
             u32x4* k = nullptr;
@@ -632,12 +889,46 @@ int launch_attn_t(hipStream_t s, const TlmAttnArgs& a, bool tiled) {
     });
 }
 
+template <class Tr, int D>
+int launch_gqa_d(hipStream_t s, const TlmGqaArgs& a, bool tiled) {
+    if (tiled) {
+        constexpr size_t smem = TlmGqaTile<Tr, D>::smem();
+        static_assert(smem <= 160 * 1024, "LDS of a CU");
+        if (smem > 64 * 1024) {
+            static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(&k_tlm_gqa_tile<Tr, D>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
+            MMI_HIP_CHECK(attr);
+        }
+        MMI_LAUNCH((k_tlm_gqa_tile<Tr, D>), dim3(a.n_tiles, a.kv_heads), 256, smem, s, a);
+    } else {
+        MMI_LAUNCH((k_tlm_gqa<Tr, D>), dim3(a.n_tiles, a.kv_heads, a.nsplit), 256, 0, s, a);
+        if (a.nsplit > 1) MMI_LAUNCH((k_tlm_gqa_combine<Tr>), dim3(a.n_tiles, a.kv_heads), 256, 0, s, a);
+    }
+    MMI_CHECK_LAUNCH();
+    return MMI_OK;
+}
+int gqa_bound(const Layer& L, int kstep) {               // the kernels' bound on both head sizes
+    const int d = std::max(L.k_ks * kstep, L.nd * 16);
+    return d <= 64 ? 64 : (d <= 128 ? 128 : 256);
+}
+template <class Tr>
+int launch_gqa_t(hipStream_t s, const TlmGqaArgs& a, int bound, bool tiled) {
+    if (bound == 64) return launch_gqa_d<Tr, 64>(s, a, tiled);
+    if (bound == 128) return launch_gqa_d<Tr, 128>(s, a, tiled);
+    return launch_gqa_d<Tr, 256>(s, a, tiled);
+}
+
 struct Carry {                    // what the next residual launch has to add
     const float* mix = nullptr; int mix_p = 1; const float* ls1 = nullptr;
     const float* dn = nullptr; int dn_p = 1, top = 1; const float* ls2 = nullptr;
+    const float* vec = nullptr; bool replace = false;      // (mix is the whole new residual, plus vec)
+};
+struct Norms {                    // what it leaves behind: one or two normalised operands, or (raw) the residual itself as an operand
+    const float* w = nullptr; void* out = nullptr;
+    const float* w2 = nullptr; void* out2 = nullptr;
+    void* raw = nullptr;
 };
 
-void add_resid(mmi_tlm* m, MmiProgram& P, const Shape& sh, const Carry& c, int emb_mode, float* tap, const float* w, void* out, const int* rows, int n) {
+void add_resid(mmi_tlm* m, MmiProgram& P, const Shape& sh, const Carry& c, int emb_mode, float* tap, const Norms& o, const int* rows, int n) {
     TlmResidArgs a;
     memset(&a, 0, sizeof(a));
     a.x = m->x;
@@ -652,14 +943,27 @@ void add_resid(mmi_tlm* m, MmiProgram& P, const Shape& sh, const Carry& c, int e
     a.top = c.top;
     a.dn_ps = (long)sh.T * c.top * m->ld;
     a.ls2 = c.ls2;
-    a.emb = m->embed;
-    a.tok = m->tok;
+    a.replace = c.replace;
+    a.vec = c.vec;
+    a.emb.table = m->embed;
+    a.emb.tok = m->tok;
+    a.emb.scale = m->cfg.embed_scale;
+    a.emb.bigram = m->bigram;
+    a.emb.brow = m->brow;
+    a.emb.pos = m->pos_emb;
+    a.emb.at = m->meta + sh.m.pos;
     a.emb_mode = emb_mode;
     a.tap = tap;
-    a.w = w;
+    a.w = o.w;
+    a.w2 = o.w2;
+    a.out2 = o.out2;
+    a.raw = o.raw;
+    a.raw_ks = 2 * m->h_ks;
+    if (emb_mode == TLM_EMB_SET) a.emb_out = m->cat;
+    a.emb_k0 = m->h_ks * m->kstep;
     a.groups = m->cfg.norm_groups;
     a.eps = m->cfg.norm_eps;
-    a.out = out;
+    a.out = o.out;
     a.KS = m->h_ks;
     a.rows = rows;
     const int block = n <= 256 ? std::min(1024, std::max(256, round_up(m->ld / 4, 64))) : 256;     // few rows: one vector per thread
@@ -810,8 +1114,7 @@ MixerOut build_latent_attention(mmi_tlm* m, MmiProgram& P, const Shape& sh, cons
     t.q_ks = L.k_ks;
     t.nd = L.nd;
     t.out_ks = L.lat_ks;
-    t.window = L.c.window;
-    t.scale = L.c.scale * 1.44269504088896340736f;
+    t.mask = TlmMask{L.c.window, 0, L.c.scale * 1.44269504088896340736f};
     t.n_entries = sh.n_entries;
     const bool wide = attn_group_tiles(L.nd, f32) == 8;
     const bool tiled = sh.groups[L.geo][wide] >= ATTN_TILE_GROUPS && !(f32 && L.nd > 16);     // fp32 with a wide latent: the operands do not fit the registers
@@ -823,8 +1126,7 @@ MixerOut build_latent_attention(mmi_tlm* m, MmiProgram& P, const Shape& sh, cons
     t.elen = m->meta + sh.m.elen;
     t.epos0 = m->meta + sh.m.epos0;
     t.eslot = m->meta + sh.m.eslot;
-    t.block_table = m->block_table;
-    t.bt_ld = std::max(1, m->max_pages);
+    t.pages = TlmPages{m->block_table, table_ld(m), m->keep_pages};
     t.po = m->po;
     t.pml = m->pml;
     P.site(site + "attn");
@@ -846,6 +1148,215 @@ MixerOut build_latent_attention(mmi_tlm* m, MmiProgram& P, const Shape& sh, cons
     return MixerOut{&L.out, m->o, L.out.KS};
 }
 
+MixerOut build_attention(mmi_tlm* m, MmiProgram& P, const Shape& sh, const Layer& L, const Run& r, TlmJobs first, const Plan& p, const std::string& site) {
+    const int T = sh.T, H = L.c.heads, G = L.c.kv_heads;
+    const bool f32 = m->f32;
+    TlmJob j = dense_job(L.in, m->h, m->h_ks, T);
+    j.epi = TLM_EPI_QKV;
+    j.out = m->q;
+    j.out_ld = L.k_ks;
+    j.qkv = TlmQkv{r.kc, r.vc, m->meta + sh.m.crow, H * L.dim_p / 16, G * L.dim_p / 16, L.dim_p / 16, L.nd, H, G};
+    first.j[first.n++] = j;
+    P.site(site + "in");
+    add_jobs(m, P, p, first, L.in.bytes());
+
+    TlmGqaArgs t;
+    memset(&t, 0, sizeof(t));
+    t.q = m->q;
+    t.kc = r.kc;
+    t.vc = r.vc;
+    t.out = m->o;
+    t.out_ks = L.out.KS;
+    t.heads = H;
+    t.kv_heads = G;
+    t.rep = H / G;
+    t.q_ks = L.k_ks;
+    t.nd = L.nd;
+    t.mask = TlmMask{L.c.window, L.c.window > 0 ? L.c.keep_first : 0, L.c.scale * 1.44269504088896340736f};
+    t.sink = L.c.sink;
+    t.n_entries = sh.n_entries;
+    const int bound = gqa_bound(L, m->kstep);
+    const bool wide = !(f32 && bound == 256);            // columns per workgroup of k_tlm_gqa_tile (TlmGqaTile::QT)
+    const bool tiled = sh.groups[L.geo][wide] * G >= ATTN_TILE_GROUPS;
+    const int kind = tiled ? (wide ? 2 : 1) : 0;         // which of the three prefix arrays
+    t.n_tiles = tiled ? sh.groups[L.geo][kind - 1] : sh.tiles[L.geo];
+    t.nsplit = tiled ? 1 : std::max(1, std::min(sh.nsplit, MAX_PARTIALS / std::max(1, t.n_tiles * G)));
+    t.tile0 = m->meta + sh.m.tile0 + (3 * L.geo + kind) * (sh.n_entries + 1);
+    t.erow0 = m->meta + sh.m.erow0;
+    t.elen = m->meta + sh.m.elen;
+    t.epos0 = m->meta + sh.m.epos0;
+    t.eslot = m->meta + sh.m.eslot;
+    t.pages = TlmPages{m->block_table, table_ld(m), m->keep_pages};
+    t.po = m->po;
+    t.pml = m->pml;
+    P.site(site + "attn");
+    P.add([=](hipStream_t s) { return f32 ? launch_gqa_t<TlmF32>(s, t, bound, tiled) : launch_gqa_t<TlmBf16>(s, t, bound, tiled); });
+    return MixerOut{&L.out, m->o, L.out.KS};
+}
+
+template <class Tr, bool DELTA>
+int launch_state_step(hipStream_t s, const TlmLinArgs& a, int n) {
+    const int cgp = tlm_step_groups(a.vdim_p);
+    int block = 64;
+    while (block < 256 && mmi_cdiv(a.dim_p * cgp, block) > 4) block *= 2;
+    while (mmi_cdiv(a.dim_p, block / cgp) > 16) block *= 2;
+    const int parts = block / cgp;
+    const size_t smem = (size_t)(3 * a.dim_p + a.vdim_p + 2 * parts * a.vdim_p) * sizeof(float);
+    if (mmi_cdiv(a.dim_p, parts) <= 4) MMI_LAUNCH((k_tlm_state_step<Tr, DELTA, 4>), dim3(n, a.heads), block, smem, s, a, cgp);
+    else MMI_LAUNCH((k_tlm_state_step<Tr, DELTA, 16>), dim3(n, a.heads), block, smem, s, a, cgp);
+    MMI_CHECK_LAUNCH();
+    return MMI_OK;
+}
+template <bool DELTA>
+int launch_chunk_scan(hipStream_t s, const TlmLinArgs& a, int n_unit) {
+    const int grid = 8 * mmi_cdiv(n_unit * a.heads, 8) * (a.vdim_p / 16), nd = a.dim_p / 16;
+    if (nd <= 4) MMI_LAUNCH((k_tlm_chunk_scan<DELTA, 1>), grid, 256, 0, s, a, n_unit);
+    else if (nd <= 8) MMI_LAUNCH((k_tlm_chunk_scan<DELTA, 2>), grid, 256, 0, s, a, n_unit);
+    else MMI_LAUNCH((k_tlm_chunk_scan<DELTA, 4>), grid, 256, 0, s, a, n_unit);
+    MMI_CHECK_LAUNCH();
+    return MMI_OK;
+}
+
+// the mixers that carry a matrix per head (tlm_linear.h)
+MixerOut build_linear(mmi_tlm* m, MmiProgram& P, const Shape& sh, const Layer& L, const Run& r, TlmJobs first, const Plan& p, const std::string& site) {
+    const int T = sh.T, H = L.c.heads;
+    const bool f32 = m->f32, delta = L.c.mixer == MMI_TLM_MIX_CHANNEL_DELTA;
+    TlmJob j = dense_job(L.in, m->h, m->h_ks, T);
+    j.epi = TLM_EPI_ACT;
+    j.act = delta ? TLM_ACT_NONE : TLM_ACT_SILU;
+    j.act2 = TLM_ACT_SIGMOID;
+    j.act_nt = L.b0 / 16;
+    j.out = m->lin;
+    j.out_ld = L.in_ld;
+    first.j[first.n++] = j;
+    const int lr_ks = L.lr.NT * 16 / m->kstep;
+    if (delta) {
+        j = dense_job(L.lr, m->h, m->h_ks, T);
+        j.epi = TLM_EPI_PACK;
+        j.out = m->lr;
+        j.out_ld = lr_ks;
+        first.j[first.n++] = j;
+    }
+    P.site(site + "in");
+    add_jobs(m, P, p, first, L.in.bytes() + L.lr.bytes());
+
+    TlmLinArgs a;
+    memset(&a, 0, sizeof(a));
+    a.in = m->lin;
+    a.in_ld = L.in_ld;
+    a.q0 = L.q0;
+    a.k0 = L.k0;
+    a.v0 = L.v0;
+    a.b0 = L.b0;
+    a.heads = H;
+    a.kv_heads = delta ? L.c.kv_heads : H;
+    a.dim = L.c.dim;
+    a.vdim = L.c.vdim;
+    a.dim_p = L.dim_p;
+    a.vdim_p = L.vdim_p;
+    a.q_scale = delta ? (float)(1.0 / sqrt((double)L.c.dim)) : 1.f;
+    a.eps = m->cfg.norm_eps;
+    a.conv_w = L.conv_w;
+    a.conv_state = r.conv;
+    a.conv_c = L.conv_c;
+    a.taps = L.c.conv;
+    a.decay = delta ? m->dec : L.decay;
+    a.gate = delta ? m->lgate : m->lin + L.b0;
+    a.gate_ld = delta ? H * L.vdim_p : L.in_ld;
+    a.nw = L.nw;
+    a.state = r.state;
+    a.small = (const TlmUnit*)(m->meta + sh.m.small);
+    a.unit = (const TlmUnit*)(m->meta + sh.m.unit);
+    a.chunk = (const TlmSeg*)(m->meta + sh.m.chunk);
+    a.qkv = m->qkv;
+    a.w = m->cw;
+    a.qg = m->cq_g;
+    a.kt = m->ckt;
+    a.u0 = m->cu0;
+    a.p = m->cp;
+    a.gend = m->cgend;
+    a.o = m->lo;
+    a.out = m->o;
+    a.out_ks = L.out.KS;
+    if (delta) {
+        TlmJobs Q;
+        memset(&Q, 0, sizeof(Q));
+        TlmJob& ja = Q.j[Q.n++];
+        ja = dense_job(L.a2, m->lr, lr_ks, T);
+        ja.epi = TLM_EPI_ACT;
+        ja.act = TLM_ACT_DECAY;
+        ja.act_nt = L.a2.NT;
+        ja.bias = L.decay;
+        ja.out = m->dec;
+        ja.out_ld = H * L.dim_p;
+        TlmJob& jg = Q.j[Q.n++];
+        jg = dense_job(L.g2, (const u32x4*)m->lr + (long)(L.ra / m->kstep) * 64, lr_ks, T);
+        jg.epi = TLM_EPI_ACT;
+        jg.act = TLM_ACT_SIGMOID;
+        jg.act_nt = L.g2.NT;
+        jg.out = m->lgate;
+        jg.out_ld = H * L.vdim_p;
+        P.site(site + "lowrank");
+        add_jobs(m, P, p, Q, L.a2.bytes() + L.g2.bytes());
+    }
+    const int n_small = sh.n_small, n_unit = sh.n_unit, n_chunk = sh.n_chunk;
+    if (n_small) {
+        P.site(site + "step");
+        P.add([=](hipStream_t s) {
+            if (f32) return delta ? launch_state_step<TlmF32, true>(s, a, n_small) : launch_state_step<TlmF32, false>(s, a, n_small);
+            return delta ? launch_state_step<TlmBf16, true>(s, a, n_small) : launch_state_step<TlmBf16, false>(s, a, n_small);
+        });
+    }
+    if (n_chunk) {
+        if (delta) {
+            P.site(site + "conv");
+            P.add([=](hipStream_t s) {
+                MMI_LAUNCH(k_tlm_conv, dim3(n_chunk, 2 * a.kv_heads + a.heads), 256, 0, s, a);
+                MMI_CHECK_LAUNCH();
+                return (int)MMI_OK;
+            });
+        }
+        P.site(site + "chunk");
+        P.add([=](hipStream_t s) {
+            if (delta) {
+                const size_t smem = tlm_chunk_delta_smem();
+                static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(&k_tlm_chunk_delta), hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
+                MMI_HIP_CHECK(attr);
+                MMI_LAUNCH(k_tlm_chunk_delta, dim3(n_chunk, a.heads), 256, smem, s, a);
+            } else {
+                MMI_LAUNCH(k_tlm_chunk_lightning, dim3(n_chunk, a.heads), 256, 0, s, a);
+            }
+            MMI_CHECK_LAUNCH();
+            return (int)MMI_OK;
+        });
+        P.site(site + "scan");
+        P.add([=](hipStream_t s) { return delta ? launch_chunk_scan<true>(s, a, n_unit) : launch_chunk_scan<false>(s, a, n_unit); });
+    }
+    if (!delta || n_chunk) {                             // (the delta rule's norm is per head: single tokens have had theirs)
+        const TlmSeg* chunk = delta ? a.chunk : nullptr;
+        const int rows = delta ? n_chunk * TLM_CHUNK : T;
+        P.site(site + "gate");
+        P.add([=](hipStream_t s) {
+            const size_t smem = (size_t)(a.heads + 4) * sizeof(float);
+            if (f32) MMI_LAUNCH((k_tlm_gated_norm<TlmF32>), rows, 256, smem, s, a, delta ? 1 : 0, chunk);
+            else MMI_LAUNCH((k_tlm_gated_norm<TlmBf16>), rows, 256, smem, s, a, delta ? 1 : 0, chunk);
+            MMI_CHECK_LAUNCH();
+            return (int)MMI_OK;
+        });
+    }
+    return MixerOut{&L.out, m->o, L.out.KS};
+}
+
+const char* mixer_site(int mixer) {
+    switch (mixer) {
+        case MMI_TLM_MIX_MINGRU: return "gru.";
+        case MMI_TLM_MIX_LATENT_ATTENTION: return "mla.";
+        case MMI_TLM_MIX_ATTENTION: return "gqa.";
+        case MMI_TLM_MIX_CHANNEL_DELTA: return "delta.";
+        default: return "light.";
+    }
+}
+
 void build_program(mmi_tlm* m, MmiProgram& P, const Shape& sh) {
     const int T = sh.T;
     const Plan p = plan_rows(T);
@@ -862,6 +1373,13 @@ void build_program(mmi_tlm* m, MmiProgram& P, const Shape& sh) {
     a.updates = m->meta + sh.m.upd;
     a.block_table = m->block_table;
     a.rope = m->rope_dev;
+    a.buckets = m->cfg.bigram_buckets;
+    a.mul_prev = (long)m->cfg.bigram_mul_prev;
+    a.mul_cur = (long)m->cfg.bigram_mul_cur;
+    a.prev = m->meta + sh.m.prev;
+    a.next = m->meta + sh.m.next;
+    a.prev_tok = m->prev_tok;
+    a.brow = m->brow;
     P.site("prepare");
     P.add([=](hipStream_t s) {
         MMI_LAUNCH(k_tlm_prepare, std::min(512, mmi_cdiv(T * 16, 256) + 1), 256, 0, s, a);
@@ -894,36 +1412,80 @@ void build_program(mmi_tlm* m, MmiProgram& P, const Shape& sh) {
     for (size_t i = 0; i < m->runs.size(); ++i) {
         const Run& r = m->runs[i];
         const Layer& L = m->layers[r.layer];
-        const std::string site = (L.c.mixer == MMI_TLM_MIX_MINGRU ? "gru." : "mla.");
+        const std::string site = mixer_site(L.c.mixer);
+        int emb = i == 0 ? TLM_EMB_SET : (r.add_emb ? TLM_EMB_ADD : TLM_EMB_NONE);
+        float* tap = sh.taps && i ? sh.taps + (i - 1) * tap_ld : nullptr;
+        if (r.pass >= 0) {                               // x <- loop.in [x; embedding] + loop.step[pass]
+            P.site("loop.x");
+            Norms raw;
+            raw.raw = m->cat;
+            add_resid(m, P, sh, c, emb, tap, raw, nullptr, T);
+            TlmJobs J;
+            memset(&J, 0, sizeof(J));
+            TlmJob& j = J.j[J.n++];
+            j = dense_job(m->loop_in, m->cat, 2 * m->h_ks, T);
+            j.ksplit = split_for(p, m->loop_in, j.NT);
+            j.epi = TLM_EPI_F32;
+            j.out = m->mix;
+            j.out_ld = m->ld;
+            j.out_ps = (long)T * m->ld;
+            c = Carry();
+            c.mix = m->mix;
+            c.mix_p = j.ksplit;
+            c.replace = true;
+            c.vec = m->loop_step + (size_t)r.pass * m->ld;
+            P.site("loop.in");
+            add_jobs(m, P, p, J, m->loop_in.bytes());
+            emb = TLM_EMB_NONE;
+            tap = nullptr;
+        }
+        const bool moe = L.c.mlp == MMI_TLM_MLP_MOE, dense = L.c.mlp == MMI_TLM_MLP_DENSE;
+        Norms nm;
+        nm.w = L.norm;
+        nm.out = m->h;
+        void* hf = m->h;                                 // what the feed-forward reads
+        if (L.norm2) {
+            nm.w2 = L.norm2;
+            nm.out2 = hf = m->h2;
+        }
         P.site(site + "norm");
-        add_resid(m, P, sh, c, i == 0 ? TLM_EMB_SET : (r.add_emb ? TLM_EMB_ADD : TLM_EMB_NONE), sh.taps && i ? sh.taps + (i - 1) * tap_ld : nullptr, L.norm, m->h,
-                  nullptr, T);
-        const bool moe = L.c.mlp == MMI_TLM_MLP_MOE;
+        add_resid(m, P, sh, c, emb, tap, nm, nullptr, T);
         TlmJobs first;
         memset(&first, 0, sizeof(first));
         if (moe) {
             TlmJob& j = first.j[first.n++];
-            j = routed_job(m, L, L.up, m->h, m->h_ks, L.c.top, T, p);
+            j = routed_job(m, L, L.up, hf, m->h_ks, L.c.top, T, p);
             j.epi = TLM_EPI_PACK;
             j.act = TLM_ACT_RELU2;
             j.out = m->hid;
             j.out_ld = L.down.KS;
+        } else if (dense) {
+            TlmJob& j = first.j[first.n++];
+            j = dense_job(L.up, hf, m->h_ks, T);
+            j.epi = TLM_EPI_GLU;
+            j.scale = L.c.limit;
+            j.out = m->hid;
+            j.out_ld = L.down.KS;
         }
-        const MixerOut mo = L.c.mixer == MMI_TLM_MIX_MINGRU ? build_mingru(m, P, sh, L, r, first, p, site) : build_latent_attention(m, P, sh, L, r, first, p, site);
+        MixerOut mo;
+        if (L.c.mixer == MMI_TLM_MIX_MINGRU) mo = build_mingru(m, P, sh, L, r, first, p, site);
+        else if (L.c.mixer == MMI_TLM_MIX_LATENT_ATTENTION) mo = build_latent_attention(m, P, sh, L, r, first, p, site);
+        else if (L.c.mixer == MMI_TLM_MIX_ATTENTION) mo = build_attention(m, P, sh, L, r, first, p, site);
+        else mo = build_linear(m, P, sh, L, r, first, p, site);
         TlmJobs J;
         memset(&J, 0, sizeof(J));
         c = Carry();
-        if (moe) {
+        if (moe || dense) {
             TlmJob& j = J.j[J.n++];
-            j = routed_job(m, L, L.down, m->hid, L.down.KS, 1, T, p);
-            j.ksplit = split_for(p, L.down, j.NT * j.rblocks);
+            c.top = moe ? L.c.top : 1;
+            j = moe ? routed_job(m, L, L.down, m->hid, L.down.KS, 1, T, p) : dense_job(L.down, m->hid, L.down.KS, T);
+            j.ksplit = split_for(p, L.down, j.NT * (moe ? j.rblocks : 1));
             j.epi = TLM_EPI_F32;
             j.out = m->dn;
             j.out_ld = m->ld;
-            j.out_ps = (long)T * L.c.top * m->ld;
+            j.out_ps = (long)T * c.top * m->ld;
             c.dn = m->dn;
             c.dn_p = j.ksplit;
-            c.top = L.c.top;
             c.ls2 = L.ls2;
         }
         TlmJob& j = J.j[J.n++];
@@ -937,16 +1499,19 @@ void build_program(mmi_tlm* m, MmiProgram& P, const Shape& sh) {
         c.mix_p = j.ksplit;
         c.ls1 = L.ls1;
         P.site(site + "out");
-        add_jobs(m, P, p, J, mo.w->bytes());
+        add_jobs(m, P, p, J, mo.w->bytes() + (dense ? L.down.bytes() : 0));
     }
     if (sh.taps) {
         P.site("taps");
-        add_resid(m, P, sh, c, TLM_EMB_NONE, sh.taps + (m->runs.size() - 1) * tap_ld, nullptr, nullptr, nullptr, T);
+        add_resid(m, P, sh, c, TLM_EMB_NONE, sh.taps + (m->runs.size() - 1) * tap_ld, Norms(), nullptr, T);
         c = Carry();                                                     // (the residual has been written back)
     }
     if (sh.n_want > 0) {
         P.site("final_norm");
-        add_resid(m, P, sh, c, TLM_EMB_NONE, nullptr, m->final_norm, m->h, m->meta + sh.m.want, sh.n_want);
+        Norms nm;
+        nm.w = m->final_norm;
+        nm.out = m->h;
+        add_resid(m, P, sh, c, TLM_EMB_NONE, nullptr, nm, m->meta + sh.m.want, sh.n_want);
         const Plan hp = plan_rows(sh.n_want);
         TlmJobs J;
         memset(&J, 0, sizeof(J));
@@ -975,12 +1540,14 @@ void release_behind_window(mmi_tlm* m, Slot& s) {
     if (!m->has_attn || m->max_window <= 0) return;
     const int64_t first_seen = s.pos - m->max_window + 1;               // the oldest position the next token can see
     while (!s.pages.empty() && (s.first_page + 1) * TLM_PAGE <= first_seen) {
-        m->free_pages.push_back(s.pages.front());
+        if (s.first_page < m->keep_pages) s.kept.push_back(s.pages.front());
+        else m->free_pages.push_back(s.pages.front());
         s.pages.erase(s.pages.begin());
         ++s.first_page;
     }
 }
 void release_slot(mmi_tlm* m, Slot& s) {
+    for (int p : s.kept) m->free_pages.push_back(p);
     for (int p : s.pages) m->free_pages.push_back(p);
     s = Slot();
 }
@@ -1010,29 +1577,60 @@ int create_impl(mmi_tlm* m, const mmi_tensor_desc* weights, int n_weights) {
     Loader ld;
     ld.m = m;
     ld.W = MmiWeights{weights, n_weights};
-    const mmi_tensor_desc* d;
     int rc;
-    if ((rc = ld.find("embed", MMI_BF16, {c.vocab, c.width}, &d))) return rc;
-    MMI_HIP_CHECK(m->wts.alloc(&m->embed, (size_t)c.vocab * c.width));
-    MMI_HIP_CHECK(hipMemcpy(m->embed, d->data, (size_t)c.vocab * c.width * 2, hipMemcpyDeviceToDevice));
-    if ((rc = ld.vec("final.norm", c.width, m->ld, &m->final_norm)) || (rc = ld.linear("head", c.vocab, c.width, &m->head))) return rc;
+    if ((rc = ld.table("embed", c.vocab, c.width, &m->embed)) || (c.bigram_buckets > 0 && (rc = ld.table("bigram", (int64_t)c.bigram_buckets + 1, c.width, &m->bigram))) ||
+        (c.max_positions > 0 && (rc = ld.table("pos", c.max_positions, c.width, &m->pos_emb))) || (rc = ld.vec("final.norm", c.width, m->ld, &m->final_norm)) ||
+        (rc = ld.linear(c.tied_head ? "embed" : "head", c.vocab, c.width, &m->head)))
+        return rc;
+    const bool project = c.loop_inject == MMI_TLM_LOOP_PROJECT && c.loop_stop > c.loop_start;
+    if (project) {
+        const mmi_tensor_desc* d;
+        const int rows = m->ld, half = m->h_ks * m->kstep;      // columns of x, then of the embedding, each padded to whole k-steps
+        std::vector<int> rm(rows, -1), cm(2 * half, -1);
+        for (int i = 0; i < c.width; ++i) {
+            rm[i] = cm[i] = i;
+            cm[half + i] = c.width + i;
+        }
+        if ((rc = ld.find("loop.in", MMI_BF16, {c.width, 2 * (int64_t)c.width}, &d)) || (rc = ld.alloc(&m->loop_in, 1, rows / 16, 2 * m->h_ks)) || (rc = ld.upload(rm, cm)) ||
+            (rc = ld.pack(d, m->loop_in.wp, rows, 2 * half, 2 * c.width, 1)))
+            return rc;
+        std::vector<float> v, vp((size_t)c.loop_times * m->ld, 0.f);
+        if ((rc = ld.host("loop.step", {c.loop_times, c.width}, &v))) return rc;
+        for (int t = 0; t < c.loop_times; ++t)
+            for (int i = 0; i < c.width; ++i) vp[(size_t)t * m->ld + i] = v[(size_t)t * c.width + i];
+        if ((rc = ld.to_device(vp, &m->loop_step))) return rc;
+    }
+    int keep = 0;
     bool unlimited = false;
     for (int i = 0; i < c.n_layers; ++i) {
         m->layers.emplace_back();
         Layer& L = m->layers.back();
         L.c = c.layers[i];
         const std::string p = "l" + std::to_string(i);
-        if ((rc = ld.vec(p + ".norm1", c.width, m->ld, &L.norm)) || (rc = ld.vec(p + ".ls1", c.width, m->ld, &L.ls1))) return rc;
+        if ((rc = ld.vec(p + ".norm1", c.width, m->ld, &L.norm)) || (c.norms == 2 && L.c.mlp != MMI_TLM_MLP_NONE && (rc = ld.vec(p + ".norm2", c.width, m->ld, &L.norm2))) ||
+            (c.layer_scales && (rc = ld.vec(p + ".ls1", c.width, m->ld, &L.ls1))))
+            return rc;
+        auto cached = [&](int columns, int window) {     // a layer with a paged cache, `columns` attention columns per token
+            m->has_attn = true;
+            if (window <= 0) unlimited = true;
+            m->max_window = std::max<int64_t>(m->max_window, window);
+            L.geo = (int)(std::find(m->geo.begin(), m->geo.end(), columns) - m->geo.begin());
+            if (L.geo == (int)m->geo.size()) m->geo.push_back(columns);
+        };
         if (L.c.mixer == MMI_TLM_MIX_MINGRU) {
             m->has_gru = true;
             if ((rc = load_mingru(ld, L, p))) return rc;
+        } else if (L.c.mixer == MMI_TLM_MIX_ATTENTION) {
+            cached(L.c.heads / L.c.kv_heads, L.c.window);
+            if (L.c.window > 0) keep = std::max(keep, L.c.keep_first);
+            if ((rc = load_attention(ld, L, p))) return rc;
+        } else if (L.linear()) {
+            m->has_linear = true;
+            if ((rc = L.c.mixer == MMI_TLM_MIX_CHANNEL_DELTA ? load_channel_delta(ld, L, p) : load_lightning(ld, L, p))) return rc;
         } else {
-            m->has_attn = true;
-            if (L.c.window <= 0) unlimited = true;
-            m->max_window = std::max<int64_t>(m->max_window, L.c.window);
+            m->has_latent = true;
+            cached(L.c.heads, L.c.window);
             if ((rc = load_latent_attention(ld, L, p))) return rc;
-            L.geo = (int)(std::find(m->geo.begin(), m->geo.end(), L.c.heads) - m->geo.begin());
-            if (L.geo == (int)m->geo.size()) m->geo.push_back(L.c.heads);
             if (L.c.rot_dim > 0) {
                 const std::pair<double, int> key(L.c.rot_base, L.c.rot_dim);
                 L.rope = (int)(std::find(m->ropes.begin(), m->ropes.end(), key) - m->ropes.begin());
@@ -1048,23 +1646,27 @@ int create_impl(mmi_tlm* m, const mmi_tensor_desc* weights, int n_weights) {
                 }
             }
         }
-        if (L.c.mlp == MMI_TLM_MLP_MOE) {
-            if ((rc = ld.vec(p + ".ls2", c.width, m->ld, &L.ls2)) || (rc = load_moe(ld, L, p))) return rc;
+        if (L.c.mlp != MMI_TLM_MLP_NONE) {
+            if ((c.layer_scales && (rc = ld.vec(p + ".ls2", c.width, m->ld, &L.ls2))) ||
+                (rc = L.c.mlp == MMI_TLM_MLP_MOE ? load_moe(ld, L, p) : load_dense_glu(ld, L, p)))
+                return rc;
         }
     }
     if (unlimited) m->max_window = 0;
+    if (m->max_window > 0) m->keep_pages = mmi_cdiv(keep, TLM_PAGE);
     const int times = c.loop_stop > c.loop_start ? c.loop_times : 1;
     const int start = c.loop_stop > c.loop_start ? c.loop_start : c.n_layers, stop = c.loop_stop > c.loop_start ? c.loop_stop : c.n_layers;
-    auto run = [&](int layer, bool add) {
+    auto run = [&](int layer, bool add, int pass) {
         Run r;
         r.layer = layer;
         r.add_emb = add;
+        r.pass = pass;
         m->runs.push_back(r);
     };
-    for (int i = 0; i < start; ++i) run(i, false);
+    for (int i = 0; i < start; ++i) run(i, false, -1);
     for (int t = 0; t < times; ++t)
-        for (int i = start; i < stop; ++i) run(i, t > 0 && i == start);
-    for (int i = stop; i < c.n_layers; ++i) run(i, false);
+        for (int i = start; i < stop; ++i) run(i, !project && t > 0 && i == start, project && i == start ? t : -1);
+    for (int i = stop; i < c.n_layers; ++i) run(i, false, -1);
     m->slots.resize(m->max_slots);
     for (int i = m->max_pages - 1; i >= 0; --i) m->free_pages.push_back(i);
     if ((rc = alloc_state(m)) || (rc = alloc_buffers(m))) return rc;
@@ -1139,7 +1741,7 @@ extern "C" int64_t mmi_tlm_info(const mmi_tlm* m, int32_t which, int32_t slot) {
             return n;
         }
         case MMI_TLM_POSITION: return ok ? m->slots[slot].pos : -1;
-        case MMI_TLM_HELD_PAGES: return ok ? (int64_t)m->slots[slot].pages.size() : -1;
+        case MMI_TLM_HELD_PAGES: return ok ? (int64_t)(m->slots[slot].pages.size() + m->slots[slot].kept.size()) : -1;
         case MMI_TLM_WEIGHT_BYTES: return m->weight_bytes;
         case MMI_TLM_LAYER_RUNS: return (int64_t)m->runs.size();
         case MMI_TLM_GRAPHS: return (int64_t)m->progs.size();
@@ -1173,6 +1775,7 @@ extern "C" int mmi_tlm_step(mmi_tlm* m, int32_t n_entries, const int32_t* slots,
         if (counts[e] < 1) return mmi_fail(MMI_ERR_INVALID, "an entry brings no token");
         T64 += counts[e];
         if (m->slots[slots[e]].pos + counts[e] > (int64_t)1 << 24) return mmi_fail(MMI_ERR_SHAPE, "position above 2^24");
+        if (m->cfg.max_positions > 0 && m->slots[slots[e]].pos + counts[e] > m->cfg.max_positions) return mmi_fail(MMI_ERR_SHAPE, "position past the model's last");
         need += pages_for(m, &m->slots[slots[e]], counts[e]);
     }
     if (T64 > m->max_T) return mmi_fail(MMI_ERR_SHAPE, "the step brings more tokens than max_step_tokens");
@@ -1192,6 +1795,11 @@ extern "C" int mmi_tlm_step(mmi_tlm* m, int32_t n_entries, const int32_t* slots,
         const int n = mmi_cdiv(counts[e], TLM_SEG);
         sh.n_seg += n;
         sh.pairs |= n > 1;
+        if (counts[e] <= TLM_SMALL) ++sh.n_small;
+        else {
+            ++sh.n_unit;
+            sh.n_chunk += mmi_cdiv(counts[e], TLM_CHUNK);
+        }
     }
     Meta& M = sh.m;
     int at = 16;
@@ -1204,6 +1812,8 @@ extern "C" int mmi_tlm_step(mmi_tlm* m, int32_t n_entries, const int32_t* slots,
     M.pos = take(T);
     M.rslot = take(T);
     M.crow = take(T);
+    M.prev = take(T);
+    M.next = take(T);
     M.want = take(n_want);
     M.erow0 = take(n_entries);
     M.elen = take(n_entries);
@@ -1211,6 +1821,9 @@ extern "C" int mmi_tlm_step(mmi_tlm* m, int32_t n_entries, const int32_t* slots,
     M.eslot = take(n_entries);
     M.tile0 = take(3 * (int)m->geo.size() * (n_entries + 1));
     M.seg = take(8 * sh.n_seg);
+    M.small = take(8 * sh.n_small);
+    M.unit = take(8 * sh.n_unit);
+    M.chunk = take(8 * sh.n_chunk);
     M.upd = at;
     M.total = at + 2 * (int)need;
     if ((size_t)M.total > m->meta_cap) return mmi_fail(MMI_ERR_SHAPE, "step metadata above its buffer");
@@ -1221,7 +1834,9 @@ extern "C" int mmi_tlm_step(mmi_tlm* m, int32_t n_entries, const int32_t* slots,
     memset(b, 0, 16 * sizeof(int));
     int upd = 0, row = 0, seg = 0;
     int64_t blocks = 0;
-    TlmSeg* sg = (TlmSeg*)(b + M.seg);
+    TlmSeg *sg = (TlmSeg*)(b + M.seg), *ck = (TlmSeg*)(b + M.chunk);
+    TlmUnit *small = (TlmUnit*)(b + M.small), *unit = (TlmUnit*)(b + M.unit);
+    int n_ck = 0;
     sh.tiles.assign(m->geo.size(), 0);
     sh.groups.assign(m->geo.size(), {0, 0});
     for (int e = 0; e < n_entries; ++e) {
@@ -1229,7 +1844,8 @@ extern "C" int mmi_tlm_step(mmi_tlm* m, int32_t n_entries, const int32_t* slots,
         for (int64_t n = pages_for(m, &S, counts[e]); n > 0; --n) {
             const int page = m->free_pages.back();
             m->free_pages.pop_back();
-            const int64_t idx = (int64_t)slots[e] * m->max_pages + (S.first_page + (int64_t)S.pages.size()) % m->max_pages;
+            const int64_t at_page = S.first_page + (int64_t)S.pages.size();
+            const int64_t idx = (int64_t)slots[e] * table_ld(m) + (at_page < m->keep_pages ? at_page : m->keep_pages + (at_page - m->keep_pages) % std::max(1, m->max_pages));
             S.pages.push_back(page);
             b[M.upd + 2 * upd] = (int)idx;
             b[M.upd + 2 * upd + 1] = page;
@@ -1253,15 +1869,26 @@ extern "C" int mmi_tlm_step(mmi_tlm* m, int32_t n_entries, const int32_t* slots,
             const int n = std::min(TLM_SEG, counts[e] - o);
             sg[seg++] = TlmSeg{row + o, n, slots[e], S.par, k, o + n == counts[e] ? 1 : 0, S.pos == 0 ? 1 : 0, 0};
         }
+        if (counts[e] <= TLM_SMALL) {
+            *small++ = TlmUnit{row, counts[e], slots[e], S.par, S.pos == 0 ? 1 : 0, 0, 0, 0};
+        } else {
+            *unit++ = TlmUnit{row, counts[e], slots[e], S.par, S.pos == 0 ? 1 : 0, n_ck, mmi_cdiv(counts[e], TLM_CHUNK), 0};
+            for (int o = 0, k = 0; o < counts[e]; o += TLM_CHUNK, ++k) {
+                const int n = std::min(TLM_CHUNK, counts[e] - o);
+                ck[n_ck++] = TlmSeg{row + o, n, slots[e], S.par, k, o + n == counts[e] ? 1 : 0, S.pos == 0 ? 1 : 0, 0};
+            }
+        }
         for (int i = 0; i < counts[e]; ++i, ++row) {
             const int64_t pos = S.pos + i;
+            b[M.prev + row] = pos == 0 ? -1 : (i > 0 ? -2 : slots[e] * 2 + S.par);
+            b[M.next + row] = i + 1 == counts[e] ? slots[e] * 2 + (S.par ^ 1) : -1;
             b[M.htok + row] = tokens[row];
             b[M.pos + row] = (int)pos;
             b[M.rslot + row] = slots[e];
-            b[M.crow + row] = m->has_attn ? S.pages[pos / TLM_PAGE - S.first_page] * TLM_PAGE + (int)(pos % TLM_PAGE) : 0;
+            b[M.crow + row] = m->has_attn ? S.page(pos / TLM_PAGE) * TLM_PAGE + (int)(pos % TLM_PAGE) : 0;
         }
         int64_t span = S.pos + counts[e];
-        if (m->max_window > 0) span = std::min<int64_t>(span, m->max_window + counts[e]);
+        if (m->max_window > 0) span = std::min<int64_t>(span, m->max_window + counts[e] + m->keep_pages * TLM_PAGE);
         blocks = std::max(blocks, span / 32 + 1);
         S.pos += counts[e];
         S.par ^= 1;

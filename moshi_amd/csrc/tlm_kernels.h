@@ -28,6 +28,7 @@ struct TlmBf16 {
         u32x2 o = {mmi_pack_bf16x2(v[0], v[1]), mmi_pack_bf16x2(v[2], v[3])};
         *reinterpret_cast<u32x2*>(p) = o;
     }
+    static __device__ __forceinline__ void store2(uint16_t* p, float a, float b) { *reinterpret_cast<uint32_t*>(p) = mmi_pack_bf16x2(a, b); }
 };
 struct TlmF32 {
     typedef float elem;
@@ -40,6 +41,7 @@ struct TlmF32 {
     }
     static __device__ __forceinline__ float cvt(float v) { return v; }
     static __device__ __forceinline__ void store4(float* p, f32x4 v) { *reinterpret_cast<f32x4*>(p) = v; }
+    static __device__ __forceinline__ void store2(float* p, float a, float b) { *reinterpret_cast<f32x2*>(p) = f32x2{a, b}; }
 };
 
 // element (row, k) of a fragment-packed matrix with `ks` k-steps per row tile
@@ -64,14 +66,16 @@ __device__ __forceinline__ float tlm_wave_sum(float x) {
 // ------------------------------------------------------------------------------------------------
 template <class Tr>
 __global__ void k_tlm_pack(const uint16_t* __restrict__ src, long sr, long sc, const int* __restrict__ rowmap, const int* __restrict__ colmap,
-                           typename Tr::elem* __restrict__ dst, int NT, int KS, int tmul, int toff) {
+                           typename Tr::elem* __restrict__ dst, int NT, int KS, int tmul, int toff, int keep) {
     const long idx = (long)blockIdx.x * blockDim.x + threadIdx.x;
     if (idx >= (long)NT * KS * 64 * Tr::V) return;
     const int e = (int)(idx % Tr::V);
     const long f = idx / Tr::V;
     const int lane = (int)(f & 63);
     const int ks = (int)((f >> 6) % KS), nt = (int)((f >> 6) / KS);
-    const int r = rowmap[nt * 16 + (lane & 15)], c = colmap[ks * Tr::KSTEP + (lane >> 4) * Tr::V + e];
+    const int r = rowmap[nt * 16 + (lane & 15)];
+    if (r < 0 && keep) return;                     // (rows another call has filled)
+    const int c = colmap[ks * Tr::KSTEP + (lane >> 4) * Tr::V + e];
     const uint16_t h = (r < 0 || c < 0) ? (uint16_t)0 : src[(long)r * sr + (long)c * sc];
     const long at = (((long)nt * tmul + toff) * KS + ks) * 64 * Tr::V + (long)lane * Tr::V + e;      // tile nt of this call is tile nt * tmul + toff of the matrix
     if constexpr (Tr::V == 8) dst[at] = h;
@@ -98,13 +102,29 @@ struct TlmPrepArgs {
     const int* updates;       // (block-table index, page) pairs
     int* block_table;
     const TlmRope* rope;
+    int buckets; long mul_prev, mul_cur;       // bigram embedding (buckets 0: none)
+    const int* prev;          // per row: -1 first token of its sequence, -2 the row before it, otherwise the index of the token in prev_tok
+    const int* next;          // per row: where in prev_tok its token goes (the last of an entry), or -1
+    int* prev_tok;            // [slots][2]: a step reads one copy and writes the other
+    int* brow;                // out: row of the bigram table
 };
 __global__ void k_tlm_prepare(TlmPrepArgs a) {
     const int i0 = (int)(blockIdx.x * blockDim.x + threadIdx.x), n = (int)(gridDim.x * blockDim.x);
     for (int i = i0; i < *a.n_updates; i += n) a.block_table[a.updates[2 * i]] = a.updates[2 * i + 1];
     for (int i = i0; i < a.T; i += n) {
-        const int t = a.htok[i];
-        a.tok[i] = t >= 0 ? t : a.last_tok[a.rslot[i]];
+        const int t = a.htok[i] >= 0 ? a.htok[i] : a.last_tok[a.rslot[i]];
+        a.tok[i] = t;
+        if (a.buckets > 0) {
+            const int w = a.prev[i];
+            int b = a.buckets;
+            if (w != -1) {
+                const int p = w >= 0 ? a.prev_tok[w] : (a.htok[i - 1] >= 0 ? a.htok[i - 1] : a.last_tok[a.rslot[i]]);
+                b = (int)(((long)p * a.mul_prev + (long)t * a.mul_cur) % a.buckets);
+                if (b < 0) b += a.buckets;
+            }
+            a.brow[i] = b;
+            if (a.next[i] >= 0) a.prev_tok[a.next[i]] = t;
+        }
     }
     for (int r = 0; r < a.n_ropes; ++r) {
         const TlmRope q = a.rope[r];
@@ -170,19 +190,31 @@ __global__ __launch_bounds__(1024) void k_tlm_route(TlmRouteArgs a) {
 
 // ------------------------------------------------------------------------------------------------
 // residual update + grouped RMS norm: one workgroup per row
-//   x <- x + ls1 * sum_p mix[p] + ls2 * (1 / top) * sum_choice sum_p dn[p]   (the split-K partials of the two sublayers' last products)
-//   x <- emb[token] (first layer) or x + emb[token] (start of a repeated pass), then h = norm(x) * w -> packed operand
+//   x <- x + ls1 * sum_p mix[p] + ls2 * (1 / top) * sum_choice sum_p dn[p]   (the split-K partials of the two sublayers' last products;
+//        no ls: factor 1), or x <- sum_p mix[p] (`replace`: the product at the start of a repeated pass)
+//   x <- emb[token] (first layer) or x + emb[token] (start of a repeated pass); x <- x + vec; then h = norm(x) * w -> packed operand, and
+//   a second one with weights of its own; `raw`: x itself as a packed operand
+//   emb[token] = table[token] * scale + bigram[row of (previous, token)] + pos[position]
 // ------------------------------------------------------------------------------------------------
 enum { TLM_EMB_NONE = 0, TLM_EMB_SET = 1, TLM_EMB_ADD = 2 };
+struct TlmEmbArgs {
+    const uint16_t* table; const int* tok; float scale;
+    const uint16_t* bigram; const int* brow;       // or null
+    const uint16_t* pos; const int* at;            // or null
+};
 struct TlmResidArgs {
     float* x;
     int width, ld;                       // ld: row stride of x, mix, dn (width rounded up to 16)
-    const float* mix; int mix_p; long mix_ps; const float* ls1;
+    const float* mix; int mix_p; long mix_ps; const float* ls1; int replace;
     const float* dn; int dn_p; long dn_ps; int top; const float* ls2;
-    const uint16_t* emb; const int* tok; int emb_mode;
+    TlmEmbArgs emb; int emb_mode;
+    const float* vec;
     float* tap;                          // copy of the residual stream before the embedding is added again, or null
     const float* w; int groups; float eps;
     void* out; int KS;                   // packed; null: no norm
+    const float* w2; void* out2;
+    void* raw; int raw_ks;               // packed x, or null
+    void* emb_out; int emb_k0;           // TLM_EMB_SET: packed copy of the embedding from column emb_k0 of rows of raw_ks k-steps, or null
     const int* rows;                     // row list (the residual is then not written back), or null
 };
 template <class Tr>
@@ -194,32 +226,43 @@ __global__ __launch_bounds__(1024) void k_tlm_resid_norm(TlmResidArgs a) {
     for (int k = 4 * tid; k < a.ld; k += 4 * nthr) {
         f32x4 v = {0.f, 0.f, 0.f, 0.f}, ev = v;
         if (a.emb_mode != TLM_EMB_NONE) {
-            const uint16_t* e = a.emb + (long)a.tok[r] * a.width + k;
+            const TlmEmbArgs& E = a.emb;
+            const uint16_t* e = E.table + (long)E.tok[r] * a.width + k;
+            const uint16_t* eb = E.bigram ? E.bigram + (long)E.brow[r] * a.width + k : nullptr;
+            const uint16_t* ep = E.pos ? E.pos + (long)E.at[r] * a.width + k : nullptr;
 #pragma unroll
             for (int q = 0; q < 4; ++q)
-                if (k + q < a.width) ev[q] = mmi_bf16_to_f32(e[q]);
+                if (k + q < a.width) {
+                    ev[q] = mmi_bf16_to_f32(e[q]) * E.scale;
+                    if (eb) ev[q] += mmi_bf16_to_f32(eb[q]);
+                    if (ep) ev[q] += mmi_bf16_to_f32(ep[q]);
+                }
         }
         if (a.emb_mode == TLM_EMB_SET) {
             v = ev;
+            if (a.emb_out) Tr::store4((typename Tr::elem*)a.emb_out + tlm_index<Tr>(blockIdx.x, a.emb_k0 + k, a.raw_ks), ev);
         } else {
-            v = *reinterpret_cast<const f32x4*>(x + k);
+            if (!a.replace) v = *reinterpret_cast<const f32x4*>(x + k);
             f32x4 d = {0.f, 0.f, 0.f, 0.f};
             if (a.mix) {
 #pragma unroll 8
                 for (int p = 0; p < a.mix_p; ++p) d += *reinterpret_cast<const f32x4*>(a.mix + p * a.mix_ps + (long)r * a.ld + k);
-                d *= *reinterpret_cast<const f32x4*>(a.ls1 + k);
+                if (a.ls1) d *= *reinterpret_cast<const f32x4*>(a.ls1 + k);
             }
             if (a.dn) {
                 f32x4 f = {0.f, 0.f, 0.f, 0.f};
                 for (int c = 0; c < a.top; ++c)
 #pragma unroll 8
                     for (int p = 0; p < a.dn_p; ++p) f += *reinterpret_cast<const f32x4*>(a.dn + p * a.dn_ps + ((long)r * a.top + c) * a.ld + k);
-                d += f * (1.0f / (float)a.top) * *reinterpret_cast<const f32x4*>(a.ls2 + k);
+                f *= 1.0f / (float)a.top;
+                d += a.ls2 ? f * *reinterpret_cast<const f32x4*>(a.ls2 + k) : f;
             }
             v += d;
             if (a.tap) *reinterpret_cast<f32x4*>(a.tap + (long)r * a.ld + k) = v;
             if (a.emb_mode == TLM_EMB_ADD) v += ev;
         }
+        if (a.vec) v += *reinterpret_cast<const f32x4*>(a.vec + k);
+        if (a.raw) Tr::store4((typename Tr::elem*)a.raw + tlm_index<Tr>(blockIdx.x, k, a.raw_ks), v);
         if (!a.rows) *reinterpret_cast<f32x4*>(x + k) = v;
         *reinterpret_cast<f32x4*>(row + k) = v;
     }
@@ -250,16 +293,24 @@ __global__ __launch_bounds__(1024) void k_tlm_resid_norm(TlmResidArgs a) {
         f32x4 v = *reinterpret_cast<const f32x4*>(row + k);
         const f32x4 w = *reinterpret_cast<const f32x4*>(a.w + k);
 #pragma unroll
-        for (int q = 0; q < 4; ++q) v[q] = k + q < a.width ? v[q] * inv[(k + q) / gs] * w[q] : 0.f;
-        Tr::store4(out + tlm_index<Tr>(blockIdx.x, k, a.KS), v);
+        for (int q = 0; q < 4; ++q) v[q] = k + q < a.width ? v[q] * inv[(k + q) / gs] : 0.f;
+        Tr::store4(out + tlm_index<Tr>(blockIdx.x, k, a.KS), v * w);
+        if (a.out2) Tr::store4((typename Tr::elem*)a.out2 + tlm_index<Tr>(blockIdx.x, k, a.KS), v * *reinterpret_cast<const f32x4*>(a.w2 + k));
     }
 }
 
 // ------------------------------------------------------------------------------------------------
 // matrix products: up to three of them per launch, each dense, grouped (per head) or routed (per expert)
 // ------------------------------------------------------------------------------------------------
-enum { TLM_EPI_F32 = 0, TLM_EPI_PACK = 1, TLM_EPI_ROPE = 2, TLM_EPI_GRU = 3, TLM_EPI_LOGITS = 4 };
-enum { TLM_ACT_NONE = 0, TLM_ACT_RELU2 = 1 };
+enum { TLM_EPI_F32 = 0, TLM_EPI_PACK = 1, TLM_EPI_ROPE = 2, TLM_EPI_GRU = 3, TLM_EPI_LOGITS = 4, TLM_EPI_ACT = 5, TLM_EPI_GLU = 6, TLM_EPI_QKV = 7 };
+enum { TLM_ACT_NONE = 0, TLM_ACT_RELU2 = 1, TLM_ACT_SILU = 2, TLM_ACT_SIGMOID = 3, TLM_ACT_DECAY = 4 };
+// queries, keys and values of grouped attention: head by head, every head padded to whole tiles; keys and values go to the cache
+struct TlmQkv {
+    void *kc, *vc;
+    const int* crow;                     // cache row of the token: 64 page + offset
+    int q_nt, k_nt, h_nt, v_nt;          // tiles of all query heads, of all key heads, per query / key head, per value head
+    int heads, kv_heads;
+};
 struct TlmJob {
     const u32x4* wp; long wgs;           // packed weights; fragments x 64 per group
     const u32x4* xp; int xks, xkg;       // packed activations, their k-steps per row tile; k-step offset per group
@@ -270,20 +321,33 @@ struct TlmJob {
     const int* tiles;
     const int* n_tiles;
     int in_div;
-    int epi, act;
+    int epi, act, act2, act_nt;          // ACT: act2 from tile act_nt on
     void* out; int out_ld; long out_ps;  // fp32: row stride, stride per K split; packed: k-steps per row tile
     int out_mul, out_gadd, out_k0, out_kg;
-    const float* bias;                   // GRU: [2][width]
+    const float* bias;                   // GRU: [2][width]; DECAY: [2][columns]: summand, then factor of the softplus
+    TlmQkv qkv;
     const float* gate; int gate_ld;      // PACK: factor per (row, group), or null
     const float* rope; int rope_ld;      // ROPE: (cos, sin) per row
     int n_valid;                         // LOGITS: columns
-    float scale;
+    float scale;                         // LOGITS: factor; GLU: limit
     int blocks;
 };
 struct TlmJobs {
     TlmJob j[3];
     int n;
 };
+
+__device__ __forceinline__ float tlm_softplus(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
+
+// cached values of grouped attention: the transposed operand of the value product, [page][kv head][keys / KSTEP][16-wide value blocks]
+// fragments whose reduction order is the one the softmax weights have in the registers after S = K Q^T (bf16: keys 4 kq .. 4 kq + 3 of
+// both 16-key halves)
+template <class Tr>
+MMI_HD long tlm_value_index(int crow, int g, int kv_heads, int d, int nd) {
+    const int o = crow & (TLM_PAGE - 1), ko = o % Tr::KSTEP, half = ko >> 4;
+    const long blk = ((long)(crow / TLM_PAGE) * kv_heads + g) * (TLM_PAGE / Tr::KSTEP) + o / Tr::KSTEP;
+    return ((blk * nd + (d >> 4)) * 64 + ((ko & 15) >> 2) * 16 + (d & 15)) * Tr::V + 4 * half + (ko & 3);
+}
 
 template <class Tr, int EPI>
 __device__ __forceinline__ void tlm_epilogue(const TlmJob& j, int g, int split, int id, int nt, int quad, f32x4 v) {
@@ -320,6 +384,44 @@ __device__ __forceinline__ void tlm_epilogue(const TlmJob& j, int g, int split, 
             for (int e = 0; e < 4; ++e) o[e] = (kind == 1 && v[e] >= 0.f) ? v[e] + 0.5f : tlm_sigmoid(v[e]);
         }
         *reinterpret_cast<f32x4*>((float*)j.out + (orow * 3 + kind) * w + c) = o;
+    } else if constexpr (EPI == TLM_EPI_ACT) {
+        const int act = nt < j.act_nt ? j.act : j.act2;
+        if (act == TLM_ACT_DECAY) {
+            const f32x4 b = *reinterpret_cast<const f32x4*>(j.bias + n0), f = *reinterpret_cast<const f32x4*>(j.bias + j.out_ld + n0);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) v[e] = expf(-f[e] * tlm_softplus(v[e] + b[e]));
+        } else if (act != TLM_ACT_NONE) {
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const float s = tlm_sigmoid(v[e]);
+                v[e] = act == TLM_ACT_SILU ? v[e] * s : s;
+            }
+        }
+        *reinterpret_cast<f32x4*>((float*)j.out + orow * j.out_ld + n0) = v;
+    } else if constexpr (EPI == TLM_EPI_GLU) {
+        // gate and up rows alternate (the weight rows are interleaved at load)
+        float y[2];
+#pragma unroll
+        for (int e = 0; e < 2; ++e) {
+            const float g = fminf(v[2 * e], j.scale), u = fminf(fmaxf(v[2 * e + 1], -j.scale), j.scale);
+            y[e] = g * tlm_sigmoid(1.702f * g) * (u + 1.0f);
+        }
+        Tr::store2((typename Tr::elem*)j.out + tlm_index<Tr>(orow, n0 / 2, j.out_ld), y[0], y[1]);
+    } else if constexpr (EPI == TLM_EPI_QKV) {
+        const TlmQkv& z = j.qkv;
+        if (nt < z.q_nt) {
+            const int h = nt / z.h_nt;
+            Tr::store4((typename Tr::elem*)j.out + tlm_index<Tr>((long)id * z.heads + h, n0 - h * z.h_nt * 16, j.out_ld), v);
+        } else if (nt < z.q_nt + z.k_nt) {
+            const int g = (nt - z.q_nt) / z.h_nt, cr = z.crow[id];
+            const long row = ((long)(cr / TLM_PAGE) * z.kv_heads + g) * TLM_PAGE + (cr & (TLM_PAGE - 1));
+            Tr::store4((typename Tr::elem*)z.kc + tlm_index<Tr>(row, n0 - (z.q_nt + g * z.h_nt) * 16, j.out_ld), v);
+        } else {
+            const int t = nt - z.q_nt - z.k_nt, g = t / z.v_nt, cr = z.crow[id], d = n0 - (z.q_nt + z.k_nt + g * z.v_nt) * 16;
+            typename Tr::elem* o = (typename Tr::elem*)z.vc + tlm_value_index<Tr>(cr, g, z.kv_heads, d, z.v_nt);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) o[e * Tr::V] = Tr::cvt(v[e]);
+        }
     } else {
 #pragma unroll
         for (int e = 0; e < 4; ++e)
@@ -336,6 +438,9 @@ __device__ __forceinline__ void tlm_with_epilogue(int epi, F f) {
     else if (epi == TLM_EPI_PACK) f(TlmEpi<TLM_EPI_PACK>());
     else if (epi == TLM_EPI_ROPE) f(TlmEpi<TLM_EPI_ROPE>());
     else if (epi == TLM_EPI_GRU) f(TlmEpi<TLM_EPI_GRU>());
+    else if (epi == TLM_EPI_ACT) f(TlmEpi<TLM_EPI_ACT>());
+    else if (epi == TLM_EPI_GLU) f(TlmEpi<TLM_EPI_GLU>());
+    else if (epi == TLM_EPI_QKV) f(TlmEpi<TLM_EPI_QKV>());
     else f(TlmEpi<TLM_EPI_LOGITS>());
 }
 
@@ -629,22 +734,28 @@ __global__ __launch_bounds__(256) void k_tlm_latent(TlmLatentArgs a) {
 // through the key projection - and the value is the latent itself, so (token, head) pairs are the columns of one product and a key
 // fragment serves 16 of them.  A column tile never mixes sequences.  Keys are walked in blocks of 32; a column sees key j of its
 // token at position i when 0 <= i - j < window.
+// which keys a position sees, and the factor of the scores (times log2(e)): the last `window` ones (0: all), and the first `keep`
+struct TlmMask { int window, keep; float scale; };
+// pages of a sequence: the block table's first `keep` entries are for the pages that no window releases, the others are a ring
+struct TlmPages { const int* table; int ld, keep; };
+__device__ __forceinline__ int tlm_page(const TlmPages& p, const int* row, int i) { return row[i < p.keep ? i : p.keep + (i - p.keep) % (p.ld - p.keep)]; }
+
 struct TlmAttnArgs {
     const void* q;                       // packed rows token * heads + head
     const void* kc;
     void* out; int out_rows;             // packed rows head * out_rows + token, latent columns (the value projection reads head by head)
     int heads, q_ks, nd, out_ks;
-    int window;                          // 0: every earlier position
-    float scale;                         // times log2(e)
+    TlmMask mask;
     int n_entries, n_tiles, nsplit;
     const int* tile0;                    // [entries + 1] first column tile (k_tlm_attn_tile: column group) of each entry
     const int* erow0; const int* elen; const int* epos0; const int* eslot;
-    const int* block_table; int bt_ld;   // [slot][bt_ld]: page of positions 64 i .. at i % bt_ld
+    TlmPages pages;                      // table [slot][ld]
     float* po;                           // nsplit > 1: [tile][split][nd][64] f32x4 un-normalised sums
     float* pml;                          // [tile][split][2][16]: running maximum, sum of weights
 };
 struct TlmCols { int entry, c0, ncol; };
-__device__ __forceinline__ TlmCols tlm_find_tile(const TlmAttnArgs& a, int tile) {
+template <class Args>
+__device__ __forceinline__ TlmCols tlm_find_tile(const Args& a, int tile) {
     // the last entry whose first tile is <= tile: all prefixes compared at once (a binary search would be a chain of dependent loads)
     unsigned below = 0;
     for (int e = mmi_lane(); e < a.n_entries; e += 64) below += a.tile0[e] <= tile ? 1u : 0u;
@@ -720,15 +831,16 @@ __device__ __forceinline__ int tlm_kstep_of(const TlmAttnArgs& a, int s) {
     return s < LK ? min(s, a.out_ks - 1) : min(a.out_ks + s - LK, a.q_ks - 1);
 }
 // scores of 32 keys -> softmax weights as operand fragments, the running maximum and sum moved on; returns the factor of older sums
+// (the lane's keys are k0 .. k0 + 3 and k0 + 16 .. k0 + 19, its column's position is k0 + d0)
 template <class Tr>
-__device__ __forceinline__ float tlm_softmax_block(const TlmAttnArgs& a, f32x4 s0, f32x4 s1, int d0, float& m, float& l, u32x4 (&pf)[32 / (4 * Tr::V)]) {
+__device__ __forceinline__ float tlm_softmax_block(const TlmMask& a, f32x4 s0, f32x4 s1, int k0, int d0, float& m, float& l, u32x4 (&pf)[32 / (4 * Tr::V)]) {
     constexpr int NB = 32 / (4 * Tr::V);
     float mx = m;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
         const int e0 = d0 - r, e1 = d0 - r - 16;
-        s0[r] = e0 >= 0 && (a.window <= 0 || e0 < a.window) ? s0[r] * a.scale : -INFINITY;
-        s1[r] = e1 >= 0 && (a.window <= 0 || e1 < a.window) ? s1[r] * a.scale : -INFINITY;
+        s0[r] = e0 >= 0 && (a.window <= 0 || e0 < a.window || k0 + r < a.keep) ? s0[r] * a.scale : -INFINITY;
+        s1[r] = e1 >= 0 && (a.window <= 0 || e1 < a.window || k0 + r + 16 < a.keep) ? s1[r] * a.scale : -INFINITY;
         mx = fmaxf(mx, fmaxf(s0[r], s1[r]));
     }
     mx = fmaxf(mx, mmi_shfl_xor(mx, 16));
@@ -762,10 +874,10 @@ struct TlmAttnStream {
     u32x4 pf[QT][NB];
     float m[QT], l[QT];
     f32x4 acc[QT][ND];
-    __device__ __forceinline__ void clear() {
+    __device__ __forceinline__ void clear(float m0 = -1e30f) {
 #pragma unroll
         for (int t = 0; t < QT; ++t) {
-            m[t] = -1e30f;
+            m[t] = m0;
             l[t] = 0.f;
 #pragma unroll
             for (int d = 0; d < ND; ++d) acc[t][d] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -780,7 +892,7 @@ struct TlmAttnStream {
     }
     // q(t, k): query fragment k of column tile t
     template <class Qf>
-    __device__ __forceinline__ void use(const TlmAttnArgs& a, Qf q, int buf, int g, const int (&d0)[QT]) {
+    __device__ __forceinline__ void use(const TlmMask& a, Qf q, int buf, int g, int k0, const int (&d0)[QT]) {
 #pragma unroll
         for (int i = 0; i < G; ++i) {
             const int f = g * G + i;
@@ -788,7 +900,7 @@ struct TlmAttnStream {
             if (f < 2 * NK) {
 #pragma unroll
                 for (int t = 0; t < QT; ++t) s[t][f & 1] = Tr::mfma(fr[buf][i], q(t, f >> 1), f < 2 ? f32x4{0.f, 0.f, 0.f, 0.f} : s[t][f & 1]);
-                if (f == 2 * NK - 1) soften(a, d0);
+                if (f == 2 * NK - 1) soften(a, k0, d0);
             } else {
                 const int d = (f - 2 * NK) / NB;
 #pragma unroll
@@ -797,12 +909,12 @@ struct TlmAttnStream {
         }
     }
     // scores -> softmax weights; the sums so far are rescaled when some column's maximum has moved
-    __device__ __forceinline__ void soften(const TlmAttnArgs& a, const int (&d0)[QT]) {
+    __device__ __forceinline__ void soften(const TlmMask& a, int k0, const int (&d0)[QT]) {
         float al[QT];
         bool moved = false;
 #pragma unroll
         for (int t = 0; t < QT; ++t) {
-            al[t] = tlm_softmax_block<Tr>(a, s[t][0], s[t][1], d0[t], m[t], l[t], pf[t]);
+            al[t] = tlm_softmax_block<Tr>(a, s[t][0], s[t][1], k0, d0[t], m[t], l[t], pf[t]);
             moved = moved || al[t] != 1.f;
         }
         if (mmi_any(moved)) {
@@ -831,14 +943,14 @@ __global__ __launch_bounds__(256, Tr::V == 8 && ND <= 16 ? 2 : 1) void k_tlm_att
     const int pos0 = a.epos0[c.entry];
     const int pc = pos0 + col / a.heads;                           // position of this lane's column
     const int plo = pos0 + c.c0 / a.heads, phi = pos0 + (min(c.c0 + 15, c.ncol - 1)) / a.heads;
-    const int klo = a.window > 0 && plo - a.window + 1 > 0 ? plo - a.window + 1 : 0;
+    const int klo = a.mask.window > 0 && plo - a.mask.window + 1 > 0 ? plo - a.mask.window + 1 : 0;
     int b0 = klo / 32, b1 = phi / 32 + 1;
     if (a.nsplit > 1) {
         const int per = (b1 - b0 + a.nsplit - 1) / a.nsplit;
         b0 = min(b1, b0 + split * per);
         b1 = min(b1, b0 + per);
     }
-    const int* bt = a.block_table + (long)a.eslot[c.entry] * a.bt_ld;
+    const int* bt = a.pages.table + (long)a.eslot[c.entry] * a.pages.ld;
     f32x4 acc[ND];
 #pragma unroll
     for (int d = 0; d < ND; ++d) acc[d] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -859,7 +971,7 @@ __global__ __launch_bounds__(256, Tr::V == 8 && ND <= 16 ? 2 : 1) void k_tlm_att
     u32x4 fr[NK][2];
     const u32x4* kp = (const u32x4*)a.kc;
     auto block = [&](int kb) __attribute__((always_inline)) {
-        const long page = bt[(min(kb, b1 - 1) >> 1) % a.bt_ld];    // (past the end: the last block again)
+        const long page = tlm_page(a.pages, bt, min(kb, b1 - 1) >> 1);    // (past the end: the last block again)
         kp = (const u32x4*)a.kc + (page * 4 + (kb & 1) * 2) * a.q_ks * 64 + lane;
     };
     auto load = [&](int k) __attribute__((always_inline)) {
@@ -885,7 +997,7 @@ __global__ __launch_bounds__(256, Tr::V == 8 && ND <= 16 ? 2 : 1) void k_tlm_att
         for (int k = LK; k < NK; ++k) load(k);
         mmi_sched_barrier();
         u32x4 pf[NB];
-        const float al = tlm_softmax_block<Tr>(a, s0, s1, pc - (kb * 32 + 4 * kq), m, l, pf);
+        const float al = tlm_softmax_block<Tr>(a.mask, s0, s1, kb * 32 + 4 * kq, pc - (kb * 32 + 4 * kq), m, l, pf);
         if (mmi_any(al != 1.f)) {
 #pragma unroll
             for (int d = 0; d < ND; ++d) acc[d] *= al;
@@ -967,9 +1079,9 @@ __global__ __launch_bounds__(256) void k_tlm_attn_tile(TlmAttnArgs a) {
     }
     const int pos0 = a.epos0[c.entry];
     const int plo = pos0 + c.c0 / a.heads, phi = pos0 + min(c.c0 + 64 * QT - 1, c.ncol - 1) / a.heads;
-    const int klo = a.window > 0 && plo - a.window + 1 > 0 ? plo - a.window + 1 : 0;
+    const int klo = a.mask.window > 0 && plo - a.mask.window + 1 > 0 ? plo - a.mask.window + 1 : 0;
     const int b0 = klo / 32, b1 = phi / 32 + 1;
-    const int* bt = a.block_table + (long)a.eslot[c.entry] * a.bt_ld;
+    const int* bt = a.pages.table + (long)a.eslot[c.entry] * a.pages.ld;
     typedef TlmAttnStream<Tr, ND, RK, QT, (ND >= 16 ? 4 : 8)> S;
     Q q[QT];
     S sm;
@@ -986,7 +1098,7 @@ __global__ __launch_bounds__(256) void k_tlm_attn_tile(TlmAttnArgs a) {
     }
     // fragments of a block in LDS: keys 0-15 and 16-31 of each k-step, then the turned values; wave w brings k-steps w, w + 4, ..
     u32x4 st[NI][2];
-    auto page_of = [&](int kb) __attribute__((always_inline)) { return bt[(min(kb, b1 - 1) >> 1) % a.bt_ld]; };
+    auto page_of = [&](int kb) __attribute__((always_inline)) { return tlm_page(a.pages, bt, min(kb, b1 - 1) >> 1); };
     long page = page_of(b0);                                       // of the block fetched next
     auto fetch = [&](int kb) __attribute__((always_inline)) {
         const u32x4* kp = (const u32x4*)a.kc + (page * 4 + (kb & 1) * 2) * a.q_ks * 64 + lane;
@@ -1037,7 +1149,7 @@ __global__ __launch_bounds__(256) void k_tlm_attn_tile(TlmAttnArgs a) {
         for (int g = 0; g < S::NG; ++g) {
             if (g + 1 < S::NG) sm.load((g + 1) & 1, g + 1, at);
             mmi_sched_barrier();
-            sm.use(a, qf, g & 1, g, d0);
+            sm.use(a.mask, qf, g & 1, g, kb * 32 + 4 * kq, d0);
         }
         if constexpr (NBUF == 1) __syncthreads();
         else cur ^= 1;

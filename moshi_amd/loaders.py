@@ -194,21 +194,24 @@ def is_token_lm(path: str | Path) -> bool:
     return cfg.exists() and json.loads(cfg.read_text()).get("architecture") in TOKEN_LM_ARCHITECTURES
 
 
-def token_lm_config_from_dict(raw: dict) -> TokenLMConfig:
+def token_lm_config_from_dict(raw: dict, shapes: Optional[Dict[str, tuple]] = None) -> TokenLMConfig:
+    """`shapes`: tensor name -> shape of the checkpoint, for the sizes config.json leaves to the tensors."""
     name = raw.get("architecture")
     if name not in TOKEN_LM_ARCHITECTURES:
         raise ValueError(f"unknown architecture {name!r} (known: {sorted(TOKEN_LM_ARCHITECTURES)})")
-    return TOKEN_LM_ARCHITECTURES[name](raw)
+    return TOKEN_LM_ARCHITECTURES[name](raw, shapes)
 
 
 def get_token_lm(path: str | Path, device: torch.device | str = "cuda", dtype: torch.dtype = torch.bfloat16, max_slots: int = 32,
                  max_tokens: int = 65536, max_step_tokens: Optional[int] = None, load_weight: bool = True, lib=None) -> TokenLM:
     """A token language model from a directory holding config.json and model.safetensors (load_weight=False: seeded random weights)."""
     path = Path(path)
-    cfg = token_lm_config_from_dict(json.loads((path / "config.json").read_text()))
+    raw = json.loads((path / "config.json").read_text())
     if load_weight:
         state = _load_state(path / MOSHI_NAME)
+        cfg = token_lm_config_from_dict(raw, {k: tuple(v.shape) for k, v in state.items()})
     else:
+        cfg = token_lm_config_from_dict(raw)
         from .weights import random_token_lm_state_dict
         state = random_token_lm_state_dict(cfg, seed=0)
     return TokenLM(state, cfg, device=device, dtype=dtype, max_slots=max_slots, max_tokens=max_tokens, max_step_tokens=max_step_tokens, lib=lib)

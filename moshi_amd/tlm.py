@@ -16,7 +16,8 @@ from typing import Dict, List, Optional, Sequence, Tuple
 import torch
 
 from . import _capi
-from .config import LatentAttentionConfig, MinGRUConfig, TokenLMConfig
+from .config import (ChannelDeltaConfig, DenseGLUConfig, GroupedAttentionConfig, LatentAttentionConfig, LightningConfig, MinGRUConfig, MoEConfig,
+                     TokenLMConfig)
 
 Entry = Tuple[int, Sequence[int], Sequence[int]]          # slot, next tokens, wanted places among them
 
@@ -32,17 +33,40 @@ def _cfg_struct(cfg: TokenLMConfig, dtype: torch.dtype):
             out.scale, out.rot_base = m.scale, m.rot_base
         elif isinstance(m, MinGRUConfig):
             out.mixer, out.width = _capi.TLM_MIX_MINGRU, m.width
+        elif isinstance(m, GroupedAttentionConfig):
+            out.mixer, out.heads, out.kv_heads, out.dim, out.vdim = _capi.TLM_MIX_ATTENTION, m.heads, m.kv_heads, m.dim, m.vdim
+            out.scale, out.window, out.keep_first, out.sink = m.scale, m.window, m.keep_first, int(m.sink)
+        elif isinstance(m, ChannelDeltaConfig):
+            out.mixer, out.heads, out.kv_heads, out.dim, out.vdim = _capi.TLM_MIX_CHANNEL_DELTA, m.heads, m.kv_heads, m.dim, m.vdim
+            out.conv, out.decay_rank, out.gate_rank = m.conv, m.decay_rank, m.gate_rank
+        elif isinstance(m, LightningConfig):
+            out.mixer, out.heads, out.dim, out.vdim = _capi.TLM_MIX_LIGHTNING, m.heads, m.dim, m.vdim
+            if len(m.decay) != m.heads:
+                raise ValueError("lightning: one decay per head")
+            out.decay = (C.c_double * m.heads)(*m.decay)
         else:
             raise ValueError(f"unknown mixer {type(m).__name__}")
-        if layer.mlp is not None:
-            if layer.mlp.activation != "relu2" or layer.mlp.router != "token_table":
+        e = layer.mlp
+        if isinstance(e, DenseGLUConfig):
+            if e.activation != "clamped_swiglu":
+                raise NotImplementedError("dense feed-forward: activation clamped_swiglu is implemented")
+            out.mlp, out.ff, out.act, out.limit = _capi.TLM_MLP_DENSE, e.ff, _capi.TLM_ACT_CLAMPED_SWIGLU, e.limit
+        elif isinstance(e, MoEConfig):
+            if e.activation != "relu2" or e.router != "token_table":
                 raise NotImplementedError("experts: activation relu2 and router token_table are implemented")
-            out.mlp, out.experts, out.top, out.ff = _capi.TLM_MLP_MOE, layer.mlp.experts, layer.mlp.top, layer.mlp.ff
+            out.mlp, out.experts, out.top, out.ff = _capi.TLM_MLP_MOE, e.experts, e.top, e.ff
             out.act, out.router = _capi.TLM_ACT_RELU2, _capi.TLM_ROUTE_TOKEN_TABLE
+        elif e is not None:
+            raise ValueError(f"unknown feed-forward {type(e).__name__}")
     s = _capi.TLMCfg()
     s.vocab, s.width, s.n_layers, s.layers = cfg.vocab, cfg.width, len(cfg.layers), layers
     s.loop_start, s.loop_stop, s.loop_times = cfg.loop_start, cfg.loop_stop, cfg.loop_times
     s.norm_groups, s.norm_eps, s.logit_scale = cfg.norm_groups, cfg.norm_eps, cfg.logit_scale
+    s.loop_inject = {"add": _capi.TLM_LOOP_ADD, "project": _capi.TLM_LOOP_PROJECT}[cfg.loop_inject]
+    s.norms, s.layer_scales, s.tied_head, s.embed_scale = cfg.norms, int(cfg.layer_scales), int(cfg.tied_head), cfg.embed_scale
+    if cfg.bigram is not None:
+        s.bigram_buckets, s.bigram_mul_prev, s.bigram_mul_cur = cfg.bigram.buckets, cfg.bigram.mul_prev, cfg.bigram.mul_cur
+    s.max_positions = cfg.max_positions
     s.dtype = _capi.MMI_F32 if dtype == torch.float32 else _capi.MMI_BF16
     return s, layers
 
@@ -74,6 +98,7 @@ class TokenLM:
         self._lib = lib
         self._handle = C.c_void_p()
         self.vocab, self.max_slots = config.vocab, int(max_slots)
+        self.max_positions = config.max_positions              # longest sequence; 0: the pool alone bounds it
         self.max_step_tokens = int(max_step_tokens or max_tokens)
         cfg, keep_layers = _cfg_struct(config, dtype)
         state = {k: (v if v.dtype == torch.int32 else v.to(torch.bfloat16)).to(self.device) for k, v in state_dict.items()}

@@ -59,6 +59,9 @@ class TokenBatcher:
             raise ValueError("a request needs a prompt and at least one new token")
         if any(t < 0 or t >= self.lm.vocab for t in prompt):
             raise ValueError("token outside the vocabulary")
+        limit = getattr(self.lm, "max_positions", 0)
+        if limit and len(prompt) + max_new_tokens - 1 > limit:
+            raise ValueError(f"the request reaches position {len(prompt) + max_new_tokens - 1}, the model has {limit}")
         need = self.lm.pages_needed(-1, len(prompt) + max_new_tokens - 1)
         if need > self.lm.total_pages:
             raise BufferError(f"the request needs {need} pages, the pool has {self.lm.total_pages}")

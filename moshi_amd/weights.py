@@ -14,7 +14,8 @@ from typing import Dict, List, Tuple
 
 import torch
 
-from .config import LatentAttentionConfig, LMConfig, MimiConfig, TokenLMConfig
+from .config import (ChannelDeltaConfig, DenseGLUConfig, GroupedAttentionConfig, LatentAttentionConfig, LightningConfig, LMConfig, MimiConfig,
+                     MinGRUConfig, TokenLMConfig)
 
 Spec = List[Tuple[str, Tuple[int, ...], str]]  # (name, shape, kind)
 
@@ -138,24 +139,55 @@ def token_lm_state_spec(cfg: TokenLMConfig) -> Spec:
     """Names and shapes of a token LM's tensors (model.safetensors: bf16, tables int32).  Linear weights are [out, in]."""
     d = cfg.width
     spec: Spec = [("embed", (cfg.vocab, d), "emb:1")]
+    if cfg.bigram is not None:
+        spec.append(("bigram", (cfg.bigram.buckets + 1, d), "emb:4"))
+    if cfg.max_positions > 0:
+        spec.append(("pos", (cfg.max_positions, d), "emb:16"))
+    if cfg.loop_inject == "project" and cfg.loop_stop > cfg.loop_start:
+        spec += [("loop.in", (d, 2 * d), f"fan:{2 * d}"), ("loop.step", (cfg.loop_times, d), "emb:16")]
+
+    def linear(name, out, inp):
+        return (name, (out, inp), f"fan:{inp}")
     for i, layer in enumerate(cfg.layers):
-        p, m = f"l{i}", layer.mixer
+        p, m, e = f"l{i}", layer.mixer, layer.mlp
+        x = p + ".mix."
         spec.append((f"{p}.norm1", (d,), "alpha"))
+        if cfg.norms == 2 and e is not None:
+            spec.append((f"{p}.norm2", (d,), "alpha"))
         if isinstance(m, LatentAttentionConfig):
-            spec += [(f"{p}.mix.dq", (m.q_rank, d), f"fan:{d}"), (f"{p}.mix.dq.norm", (m.q_rank,), "alpha"),
-                     (f"{p}.mix.uq", (m.heads * (m.dim + m.rot_dim), m.q_rank), f"fan:{m.q_rank}"),
-                     (f"{p}.mix.dkv", (m.kv_rank + m.rot_dim, d), f"fan:{d}"), (f"{p}.mix.dkv.norm", (m.kv_rank,), "alpha"),
-                     (f"{p}.mix.uk", (m.heads * m.dim, m.kv_rank), f"fan:{m.kv_rank}"), (f"{p}.mix.uv", (m.heads * m.vdim, m.kv_rank), f"fan:{m.kv_rank}"),
-                     (f"{p}.mix.g", (m.heads, d), f"fan:{d}"), (f"{p}.mix.o", (d, m.heads * m.vdim), f"fan:{m.heads * m.vdim}")]
+            spec += [linear(x + "dq", m.q_rank, d), (x + "dq.norm", (m.q_rank,), "alpha"), linear(x + "uq", m.heads * (m.dim + m.rot_dim), m.q_rank),
+                     linear(x + "dkv", m.kv_rank + m.rot_dim, d), (x + "dkv.norm", (m.kv_rank,), "alpha"), linear(x + "uk", m.heads * m.dim, m.kv_rank),
+                     linear(x + "uv", m.heads * m.vdim, m.kv_rank), linear(x + "g", m.heads, d), linear(x + "o", d, m.heads * m.vdim)]
+        elif isinstance(m, MinGRUConfig):
+            spec += [linear(x + "z", m.width, d), (x + "z.b", (m.width,), "norm_b"), linear(x + "x", m.width, d), (x + "x.b", (m.width,), "norm_b"),
+                     linear(x + "g", m.width, d), linear(x + "o", d, m.width)]
+        elif isinstance(m, GroupedAttentionConfig):
+            spec += [linear(x + "q", m.heads * m.dim, d), linear(x + "k", m.kv_heads * m.dim, d), linear(x + "v", m.kv_heads * m.vdim, d),
+                     linear(x + "o", d, m.heads * m.vdim)]
+        elif isinstance(m, ChannelDeltaConfig):
+            for n, c in (("q", m.kv_heads * m.dim), ("k", m.kv_heads * m.dim), ("v", m.heads * m.vdim)):
+                spec += [linear(x + n, c, d), (x + n + ".conv", (c, m.conv), f"fan:{m.conv}")]
+            spec += [linear(x + "b", m.heads, d), (x + "A_log", (m.heads,), "norm_b"), (x + "norm", (m.vdim,), "alpha"), linear(x + "a1", m.decay_rank, d),
+                     linear(x + "a2", m.heads * m.dim, m.decay_rank), (x + "dt_bias", (m.heads * m.dim,), "dt_bias"), linear(x + "g1", m.gate_rank, d),
+                     linear(x + "g2", m.heads * m.vdim, m.gate_rank), linear(x + "o", d, m.heads * m.vdim)]
+        elif isinstance(m, LightningConfig):
+            spec += [linear(x + "q", m.heads * m.dim, d), linear(x + "k", m.heads * m.dim, d), linear(x + "v", m.heads * m.vdim, d),
+                     linear(x + "g", m.heads * m.vdim, d), linear(x + "o", d, m.heads * m.vdim), (x + "norm", (m.heads * m.vdim,), "alpha")]
         else:
-            spec += [(f"{p}.mix.z", (m.width, d), f"fan:{d}"), (f"{p}.mix.z.b", (m.width,), "norm_b"), (f"{p}.mix.x", (m.width, d), f"fan:{d}"),
-                     (f"{p}.mix.x.b", (m.width,), "norm_b"), (f"{p}.mix.g", (m.width, d), f"fan:{d}"), (f"{p}.mix.o", (d, m.width), f"fan:{m.width}")]
-        spec.append((f"{p}.ls1", (d,), "layer_scale"))
-        if layer.mlp is not None:
-            for e in range(layer.mlp.experts):
-                spec += [(f"{p}.mlp.e{e}.up", (layer.mlp.ff, d), f"fan:{d}"), (f"{p}.mlp.e{e}.down", (d, layer.mlp.ff), f"fan:{layer.mlp.ff}")]
-            spec += [(f"{p}.mlp.table", (cfg.vocab, layer.mlp.top), f"table:{layer.mlp.experts}"), (f"{p}.ls2", (d,), "layer_scale")]
-    spec += [("final.norm", (d,), "alpha"), ("head", (cfg.vocab, d), f"fan:{d}")]
+            raise ValueError(f"unknown mixer {type(m).__name__}")
+        if cfg.layer_scales:
+            spec.append((f"{p}.ls1", (d,), "layer_scale"))
+        if isinstance(e, DenseGLUConfig):
+            spec += [linear(f"{p}.mlp.gate", e.ff, d), linear(f"{p}.mlp.up", e.ff, d), linear(f"{p}.mlp.down", d, e.ff)]
+        elif e is not None:
+            for k in range(e.experts):
+                spec += [linear(f"{p}.mlp.e{k}.up", e.ff, d), linear(f"{p}.mlp.e{k}.down", d, e.ff)]
+            spec.append((f"{p}.mlp.table", (cfg.vocab, e.top), f"table:{e.experts}"))
+        if e is not None and cfg.layer_scales:
+            spec.append((f"{p}.ls2", (d,), "layer_scale"))
+    spec.append(("final.norm", (d,), "alpha"))
+    if not cfg.tied_head:
+        spec.append(linear("head", cfg.vocab, d))
     return spec
 
 
@@ -179,6 +211,8 @@ def _draw(shape, kind: str, gen: torch.Generator, device, dtype) -> torch.Tensor
         t = 1.0 + 0.1 * rnd(torch.randn, shape)
     elif kind == "norm_b":
         t = 0.05 * rnd(torch.randn, shape)
+    elif kind == "dt_bias":                            # decays from nearly 1 to a few per cent of it
+        t = -3.0 + 2.0 * rnd(torch.randn, shape)
     elif kind == "layer_scale":
         t = 0.3 + 0.05 * rnd(torch.randn, shape)   # larger than the 0.01 init so the transformer matters in tests
     elif kind == "one":
