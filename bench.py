@@ -61,6 +61,7 @@ def parse():
     ap.add_argument("--no-extras", action="store_true",
                     help="skip the extra figures of the default line: `full_context` (every session 3000 positions deep), `c3` (one session), `c5` (64 sessions, int8 x int8) and `c2` (the codec alone, 8 streams)")
     ap.add_argument("--tlm-size", default="", help="tlm workload: only these sizes (comma separated widths)")
+    ap.add_argument("--tlm-design", default="kesirax", choices=["kesirax", "bibapel"], help="tlm workload: the design that is measured")
     ap.add_argument("--tlm-batches", default="1,16,64", help="tlm workload: decode batches")
     ap.add_argument("--no-pin", action="store_true", help="do not pin the rank's host thread to its own block of cores")
     return ap.parse_args()

@@ -4,7 +4,8 @@ weights), beside the Moshi temporal transformer of the same width stepped by its
 One JSON line.  `value` = decoded tokens/s of the largest size at 64 sequences; `sizes` holds, per size, prompt tokens/s (one prompt of
 2048 tokens per step) and decoded tokens/s (1, 16 and 64 sequences 2048 tokens deep), each with the bytes it must move (weights that the
 step's tokens reach, cache in the windows, recurrent state) or the products it must form, and the fraction of the 8 TB/s / 2.5 PFLOP/s
-that is; `moshi` the temporal transformer's step at equal width, layer count and batch.
+that is; `moshi` the temporal transformer's step at equal width, layer count and batch.  `--tlm-design bibapel`: that design, and beside it
+(`kesirax`) the other one at equal width and layer count.
 """
 from __future__ import annotations
 
@@ -33,10 +34,24 @@ def sizes():
             "4096": model(4096, 5120, 32, 1536, 512, 2048, 8, 2, 5632)}
 
 
+def bibapel_sizes():
+    from moshi_amd.config import (BigramConfig, ChannelDeltaConfig, DenseGLUConfig, GroupedAttentionConfig, LightningConfig, TokenLayerConfig, TokenLMConfig)
+
+    def model(width, ff, window, vocab=32000):
+        n = width // 128
+        delta = ChannelDeltaConfig(heads=n, kv_heads=n, dim=128, vdim=128, conv=4, decay_rank=128, gate_rank=128)
+        att = GroupedAttentionConfig(heads=n, kv_heads=n // 4, dim=128, vdim=128, scale=128 ** -0.5, window=window, keep_first=4, sink=True)
+        light = LightningConfig(heads=n, dim=128, vdim=128, decay=[1 - 2.0 ** (-1 - 8 * i / n) for i in range(n)])
+        return TokenLMConfig("Bibapel", vocab=vocab, width=width, layers=[TokenLayerConfig(k, DenseGLUConfig(ff=ff, limit=7.0)) for k in (delta, att, light, light, delta, att)],
+                             loop_start=0, loop_stop=2, loop_times=2, loop_inject="project", norms=2, layer_scales=False, tied_head=True,
+                             bigram=BigramConfig(buckets=65521, mul_prev=31, mul_cur=7), max_positions=8192)
+    return {"1024": model(1024, 2816, 1024), "2048": model(2048, 5632, 1024), "4096": model(4096, 11264, 2048)}
+
+
 def layer_costs(cfg, B, depth, T_per_seq=1):
     """(bytes, products) of one step of B sequences x T tokens at `depth`: weights once per execution, experts as far as the tokens can
     reach them, keys inside the window, state."""
-    from moshi_amd.config import LatentAttentionConfig
+    from moshi_amd.config import ChannelDeltaConfig, DenseGLUConfig, GroupedAttentionConfig, LatentAttentionConfig, LightningConfig
     D, n = cfg.width, B * T_per_seq
     nbytes, flops = 2 * cfg.vocab * D + n * D * 2, 2 * cfg.vocab * D * B
     for i in cfg.layer_runs:
@@ -47,15 +62,33 @@ def layer_costs(cfg, B, depth, T_per_seq=1):
             keys = min(depth + T_per_seq, m.window) if m.window else depth + T_per_seq
             nbytes += 2 * w + B * 2 * keys * (2 * m.kv_rank + m.rot_dim)
             flops += 2 * w * n + 2 * n * min(keys, depth + T_per_seq / 2) * m.heads * (2 * m.kv_rank + m.rot_dim)
+        elif isinstance(m, GroupedAttentionConfig):
+            w = D * (m.heads * (m.dim + m.vdim) + m.kv_heads * (m.dim + m.vdim))
+            keys = min(depth + T_per_seq, m.window + m.keep_first) if m.window else depth + T_per_seq
+            nbytes += 2 * w + B * 2 * keys * m.kv_heads * (m.dim + m.vdim)
+            flops += 2 * w * n + 2 * n * min(keys, depth + T_per_seq / 2) * m.heads * (m.dim + m.vdim)
+        elif isinstance(m, (ChannelDeltaConfig, LightningConfig)):
+            if isinstance(m, LightningConfig):
+                w = D * m.heads * (2 * m.dim + 3 * m.vdim)
+            else:
+                w = D * (2 * m.kv_heads * m.dim + 2 * m.heads * m.vdim + m.heads + m.decay_rank + m.gate_rank) + m.heads * (m.dim * m.decay_rank + m.vdim * m.gate_rank)
+            nbytes += 2 * w + B * 8 * m.heads * m.dim * m.vdim
+            flops += 2 * w * n + 4 * n * m.heads * m.dim * m.vdim
         else:
             w = 4 * D * m.width
             nbytes += 2 * w + B * 8 * m.width
             flops += 2 * w * n
-        if layer.mlp is not None:
+        if isinstance(layer.mlp, DenseGLUConfig):
+            nbytes += 2 * 3 * D * layer.mlp.ff
+            flops += 2 * 3 * D * layer.mlp.ff * n
+        elif layer.mlp is not None:
             e = layer.mlp
             reached = e.experts * (1 - (1 - e.top / e.experts) ** n)
             nbytes += 2 * 2 * D * e.ff * reached
             flops += 2 * 2 * D * e.ff * e.top * n
+    if cfg.loop_inject == "project":
+        nbytes += cfg.loop_times * 4 * D * D
+        flops += cfg.loop_times * 4 * D * D * n
     return nbytes, flops
 
 
@@ -149,15 +182,18 @@ def bench_moshi(width, layers, dev, steps, warmup, batches, launch_lists=None):
 def main(args, dev):
     res = {}
     batches = tuple(int(b) for b in args.tlm_batches.split(","))
-    for name, cfg in sizes().items():
+    bibapel = args.tlm_design == "bibapel"
+    for name, cfg in (bibapel_sizes() if bibapel else sizes()).items():
         if args.tlm_size and name not in args.tlm_size.split(","):
             continue
-        res[name] = bench_model(cfg, dev, args.steps, args.warmup, batches, launch_lists=args.launch_lists, tag=name)
+        res[name] = bench_model(cfg, dev, args.steps, args.warmup, batches, launch_lists=args.launch_lists, tag=("bibapel_" if bibapel else "") + name)
+        if not args.no_extras and bibapel:
+            res[name]["kesirax"] = bench_model(sizes()[name], dev, args.steps, args.warmup, batches, launch_lists=args.launch_lists, tag=name)
         if not args.no_extras:
             res[name]["moshi"] = bench_moshi(cfg.width, len(cfg.layer_runs), dev, args.steps, args.warmup, batches, args.launch_lists)
     last = list(res)[-1]
     d = res[last]["decode"][str(batches[-1])]
     print(json.dumps({"metric": "decoded tokens/s, token language model", "value": d["tokens_per_s"], "unit": "tokens/s", "n_gpus": 1, "steps": args.steps,
                       "warmup": args.warmup, "ms_per_step": d["ms"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16",
-                      "data": "synthetic", "config": {"model": f"Kesirax, width {last}, random weights", "global_batch": batches[-1], "seq_len": DEPTH,
+                      "data": "synthetic", "config": {"model": f"{cfg.architecture}, width {last}, random weights", "global_batch": batches[-1], "seq_len": DEPTH,
                                                       "parallelism": "dp1"}, "sizes": res}), flush=True)

@@ -299,7 +299,7 @@ class TokenLMConfig:
 
 
 def _known(d: dict, keys, what: str) -> dict:
-    extra = sorted(set(d) - set(keys))
+    extra = sorted(k for k, v in d.items() if k not in keys and v is not None)
     if extra:
         raise ValueError(f"{what}: unknown entries {extra}")
     return d
@@ -371,7 +371,6 @@ def bibapel_config(raw: dict, shapes: Optional[dict] = None) -> TokenLMConfig:
             return LightningConfig(heads=heads, dim=dim, vdim=vdim, decay=[float(d) for d in decay])
         raise ValueError(f"mixer type {kind!r} is not part of this design")
 
-    _known(raw, ("architecture", "embedding", "layers", "loop", "max_positions", "norm", "vocab", "width"), "config")
     emb, loop = raw.get("embedding") or {}, raw.get("loop") or {}
     _known(emb, ("scale", "bigram"), "embedding")
     _known(raw["norm"], ("eps",), "norm")

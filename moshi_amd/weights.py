@@ -166,7 +166,7 @@ def token_lm_state_spec(cfg: TokenLMConfig) -> Spec:
                      linear(x + "o", d, m.heads * m.vdim)]
         elif isinstance(m, ChannelDeltaConfig):
             for n, c in (("q", m.kv_heads * m.dim), ("k", m.kv_heads * m.dim), ("v", m.heads * m.vdim)):
-                spec += [linear(x + n, c, d), (x + n + ".conv", (c, m.conv), f"fan:{m.conv}")]
+                spec += [linear(x + n, c, d), (x + n + ".conv", (c, m.conv), f"taps:{m.conv}")]
             spec += [linear(x + "b", m.heads, d), (x + "A_log", (m.heads,), "norm_b"), (x + "norm", (m.vdim,), "alpha"), linear(x + "a1", m.decay_rank, d),
                      linear(x + "a2", m.heads * m.dim, m.decay_rank), (x + "dt_bias", (m.heads * m.dim,), "dt_bias"), linear(x + "g1", m.gate_rank, d),
                      linear(x + "g2", m.heads * m.vdim, m.gate_rank), linear(x + "o", d, m.heads * m.vdim)]
@@ -201,6 +201,8 @@ def _draw(shape, kind: str, gen: torch.Generator, device, dtype) -> torch.Tensor
     if kind.startswith("fan:"):
         fan = int(kind[4:])
         t = (rnd(torch.rand, shape) * 2 - 1) * math.sqrt(3.0 / fan)   # unit-gain uniform
+    elif kind.startswith("taps:"):                     # large enough that the activation behind it leaves mostly positive queries and keys
+        t = 3.0 * (rnd(torch.rand, shape) * 2 - 1) * math.sqrt(3.0 / int(kind[5:]))
     elif kind.startswith("emb:"):
         t = rnd(torch.randn, shape) / math.sqrt(int(kind[4:]))
     elif kind.startswith("codebook"):

@@ -9,7 +9,8 @@ import pytest
 import torch
 
 from moshi_amd import _capi, loaders
-from moshi_amd.config import LatentAttentionConfig, MinGRUConfig, MoEConfig, TokenLayerConfig, tiny_token_lm_config
+from moshi_amd.config import (BigramConfig, ChannelDeltaConfig, DenseGLUConfig, GroupedAttentionConfig, LatentAttentionConfig, LightningConfig, MinGRUConfig,
+                              MoEConfig, TokenLayerConfig, tiny_bibapel_config, tiny_token_lm_config)
 from moshi_amd.token_batcher import TokenBatcher
 from moshi_amd.weights import random_token_lm_state_dict, token_lm_state_spec
 from oracle.token_lm_oracle import TokenLMOracle
@@ -25,6 +26,15 @@ RAW = {
          "mlp": None},
         {"type": "mingru", "mixer": {"width": 34},
          "mlp": {"kind": "moe", "router": {"experts": 3, "top": 2}, "expert": {"ff": 21}}}]}
+
+BIBAPEL = {
+    "architecture": "Bibapel", "vocab": 59, "width": 44, "norm": {"eps": 1e-4}, "max_positions": 90,
+    "embedding": {"scale": 0.7, "bigram": {"buckets": 23, "mul_prev": 13, "mul_cur": 4}}, "loop": {"start": 1, "stop": 3, "times": 2},
+    "layers": [
+        {"type": "lightning", "mixer": {"heads": 2, "dim": 12, "vdim": 20, "decay": [0.5, 0.99]}, "mlp": None},
+        {"type": "channel_delta", "mixer": {"heads": 4, "kv_heads": 2, "dim": 14, "vdim": 18, "conv": 3}, "mlp": {"kind": "dense", "ff": 30, "limit": 1.5}},
+        {"type": "attention", "mixer": {"heads": 3, "kv_heads": 1, "dim": 22, "vdim": 10, "scale": 0.3, "mask": {"size": 17, "keep_first": 2}},
+         "mlp": {"kind": "dense", "ff": 26, "limit": 0.8}}]}
 
 
 def _header():
@@ -83,11 +93,33 @@ def test_configuration_is_read_not_assumed():
             loaders.token_lm_config_from_dict(bad)
 
 
+def test_bibapel_configuration_is_read_not_assumed():
+    cfg = loaders.token_lm_config_from_dict(BIBAPEL, {"l1.mix.a1": (9, 44), "l1.mix.g1": (11, 44)})
+    assert cfg.layers == [
+        TokenLayerConfig(LightningConfig(heads=2, dim=12, vdim=20, decay=[0.5, 0.99]), None),
+        TokenLayerConfig(ChannelDeltaConfig(heads=4, kv_heads=2, dim=14, vdim=18, conv=3, decay_rank=9, gate_rank=11), DenseGLUConfig(ff=30, limit=1.5)),
+        TokenLayerConfig(GroupedAttentionConfig(heads=3, kv_heads=1, dim=22, vdim=10, scale=0.3, window=17, keep_first=2, sink=True), DenseGLUConfig(ff=26, limit=0.8))]
+    assert (cfg.vocab, cfg.width, cfg.norm_eps, cfg.max_positions, cfg.embed_scale, cfg.bigram) == (59, 44, 1e-4, 90, 0.7, BigramConfig(23, 13, 4))
+    assert cfg.layer_runs == [0, 1, 2, 1, 2] and cfg.tied_head and cfg.norms == 2 and not cfg.layer_scales and cfg.loop_inject == "project"
+    bare = loaders.token_lm_config_from_dict({**BIBAPEL, "embedding": {}, "loop": None, "max_positions": 0,
+                                              "layers": [{**BIBAPEL["layers"][2], "mixer": {**BIBAPEL["layers"][2]["mixer"], "mask": None}}]})
+    assert bare.bigram is None and bare.embed_scale == 1.0 and bare.layer_runs == [0] and bare.layers[0].mixer.window == 0
+    for bad in ({**BIBAPEL, "embedding": {"scale": 1.0, "trigram": {}}}, {**BIBAPEL, "layers": [{**BIBAPEL["layers"][1], "type": "mingru"}]},
+                {**BIBAPEL, "layers": [{**BIBAPEL["layers"][0], "mixer": {"heads": 3, "dim": 4, "vdim": 4, "decay": [0.5, 0.9]}}]},
+                {**BIBAPEL, "layers": [{**BIBAPEL["layers"][1], "mlp": {"kind": "moe", "ff": 3, "limit": 1.0}}]}):
+        with pytest.raises(ValueError):
+            loaders.token_lm_config_from_dict(bad)
+
+
 def test_spec_covers_every_tensor_of_every_layer():
     cfg = tiny_token_lm_config()
     spec = {n: s for n, s, _ in token_lm_state_spec(cfg)}
     assert spec["embed"] == (101, 96) and spec["l1.mix.uq"] == (3 * 36, 40) and spec["l1.mlp.table"] == (101, 2)
     assert "l2.ls2" not in spec and "l2.mlp.table" not in spec and "l2.ls1" in spec
+    cfg2 = tiny_bibapel_config()
+    spec2 = {n: s for n, s, _ in token_lm_state_spec(cfg2)}
+    assert spec2["bigram"] == (38, 80) and spec2["pos"] == (1500, 80) and spec2["loop.in"] == (80, 160) and spec2["loop.step"] == (2, 80)
+    assert spec2["l1.mix.v.conv"] == (96, 3) and spec2["l1.mix.a2"] == (80, 10) and "l3.norm2" not in spec2 and "head" not in spec2 and "l0.ls1" not in spec2
     table = random_token_lm_state_dict(cfg)["l1.mlp.table"]
     assert table.dtype == torch.int32 and all(len(set(row)) == 2 for row in table.tolist())
 
@@ -114,12 +146,26 @@ def test_registry_loads_a_directory(tlm_lib, tmp_path):  # noqa: F811
     assert tc.rel(tc.run_cut(lm, toks, [33, 1, 6]), TokenLMOracle(sd, lm.config).logits(toks)) < tc.TOL[tc.F32]
 
 
-def test_command_line_generates(tlm_lib, tmp_path, monkeypatch):  # noqa: F811
+def test_registry_takes_sizes_from_the_tensors(tlm_lib, tmp_path):  # noqa: F811
+    from safetensors.torch import save_file
+    shapes = {"l1.mix.a1": (9, 44), "l1.mix.g1": (11, 44)}
+    sd = random_token_lm_state_dict(loaders.token_lm_config_from_dict(BIBAPEL, shapes), seed=4)
+    save_file(sd, str(tmp_path / "model.safetensors"))
+    (tmp_path / "config.json").write_text(json.dumps(BIBAPEL))
+    assert loaders.is_token_lm(tmp_path)
+    lm = loaders.get_token_lm(tmp_path, device="cpu", dtype=torch.float32, max_slots=2, max_tokens=128, lib=tlm_lib)
+    assert lm.config.layers[1].mixer.decay_rank == 9 and lm.config.layers[1].mixer.gate_rank == 11
+    toks = tc.tokens_of(lm.config, 40)
+    assert tc.rel(tc.run_cut(lm, toks, [33, 1, 6]), TokenLMOracle(sd, lm.config).logits(toks)) < tc.TOL[tc.F32]
+
+
+@pytest.mark.parametrize("raw", [RAW, BIBAPEL], ids=["kesirax", "bibapel"])
+def test_command_line_generates(tlm_lib, tmp_path, monkeypatch, raw):  # noqa: F811
     from moshi_amd import run_inference
-    sd = _save(tmp_path, RAW)
+    sd = _save(tmp_path, raw)
     load = loaders.get_token_lm
     monkeypatch.setattr(loaders, "get_token_lm", lambda path, **kw: load(path, **{**kw, "device": "cpu", "lib": tlm_lib}))
-    cfg = loaders.token_lm_config_from_dict(RAW)
+    cfg = loaders.token_lm_config_from_dict(raw)
     prompts = [tc.tokens_of(cfg, n, seed=n) for n in (7, 40, 2)]
     (tmp_path / "in.txt").write_text("\n".join(" ".join(map(str, p)) for p in prompts) + "\n")
     run_inference.main(["--checkpoint-dir", str(tmp_path), "--greedy", "--dtype", "float32", "--batch-size", "2", "--step-tokens", "16", "--max-new-tokens", "5",

@@ -25,7 +25,8 @@ def test_mechanism_fp32(tlm_lib, name):
     tc.check_mechanism(name, DEV, tlm_lib)
 
 
-@pytest.mark.parametrize("name", ["mingru_experts", "attention_experts", "wide_latent", "repeated", "mixed"])
+@pytest.mark.parametrize("name", ["mingru_experts", "attention_experts", "wide_latent", "repeated", "mixed", "grouped_attention", "delta", "lightning", "glu",
+                                  "projected_passes", "bibapel"])
 def test_mechanism_bf16(tlm_lib, name):
     tc.check_mechanism(name, DEV, tlm_lib, tc.BF16)
 
@@ -95,10 +96,54 @@ def test_trace_replay(tlm_lib, tmp_path):
     tc.check_replay(DEV, tlm_lib, tmp_path)
 
 
-def test_perturbed_schedules_give_the_same_bits(tlm_lib):
+# ---- the mixers with matrix states, grouped attention, and the network that has them all -------------------------------------------
+def test_portions_of_a_prompt_bibapel(tlm_lib):
+    tc.check_portions(DEV, tlm_lib, n=100, cut_sets=((2,), (3, 2, 61, 7), (65, 1), (5,)), name="bibapel")
+
+
+def test_prompt_then_decode_bibapel(tlm_lib):
+    tc.check_prompt_then_decode(DEV, tlm_lib, n=90, tail=20, name="bibapel")
+
+
+def test_unequal_requests_in_one_batch_bibapel(tlm_lib):
+    tc.check_unequal_batch(DEV, tlm_lib, name="bibapel")
+
+
+def test_batched_decode_bibapel(tlm_lib):
+    tc.check_batched_decode(DEV, tlm_lib, steps=4, name="bibapel")
+
+
+def test_pages_and_slots_are_used_again_bibapel(tlm_lib):
+    tc.check_reuse(DEV, tlm_lib, name="bibapel")
+
+
+def test_decoding_longer_than_the_pool_with_kept_pages(tlm_lib):
+    tc.check_long_decode(DEV, tlm_lib, name="two_kept_windows", n=400, held=4)
+
+
+@pytest.mark.parametrize("window,keep", [(70, 6), (64, 1), (33, 64), (0, 0)])
+def test_single_kept_keys(tlm_lib, window, keep):
+    tc.check_single_kept_keys(DEV, tlm_lib, window, keep, queries=(128, 103) if window else (128,))
+
+
+@pytest.mark.parametrize("case", ["sink", "matrix_state_far", "decay_extremes", "glu_limits", "previous_token", "last_position"])
+def test_single_mechanisms(tlm_lib, case):
+    getattr(tc, f"check_{case}")(DEV, tlm_lib)
+
+
+def test_first_tokens_bibapel(tlm_lib):
+    tc.check_first_tokens(DEV, tlm_lib, name="bibapel")
+
+
+def test_greedy_generation_through_the_scheduler_bibapel(tlm_lib):
+    tc.check_generation(DEV, tlm_lib, name="bibapel")
+
+
+@pytest.mark.parametrize("name", ["mixed", "bibapel"])
+def test_perturbed_schedules_give_the_same_bits(tlm_lib, name):
     """Waves and lanes of a workgroup in other orders (a missing barrier would show); the order of a routed expert's pairs comes from
     atomics and must not matter either."""
-    cfg = tc.MECHANISMS["mixed"]
+    cfg = tc.MECHANISMS[name]
     toks = tc.tokens_of(cfg, 80)
 
     def run(mode, seed):

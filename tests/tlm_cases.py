@@ -7,11 +7,12 @@ from dataclasses import replace
 import numpy as np
 import torch
 
-from moshi_amd.config import LatentAttentionConfig, MinGRUConfig, MoEConfig, TokenLayerConfig, TokenLMConfig, tiny_token_lm_config
+from moshi_amd.config import (BigramConfig, ChannelDeltaConfig, DenseGLUConfig, GroupedAttentionConfig, LatentAttentionConfig, LightningConfig, MinGRUConfig,
+                              MoEConfig, TokenLayerConfig, TokenLMConfig, tiny_bibapel_config, tiny_token_lm_config)
 from moshi_amd.tlm import TokenLM
 from moshi_amd.token_batcher import TokenBatcher
 from moshi_amd.weights import random_token_lm_state_dict
-from oracle.token_lm_oracle import TokenLMOracle, rms_norm, rotate
+from oracle.token_lm_oracle import TokenLMOracle, rms_norm
 
 F32, BF16 = torch.float32, torch.bfloat16
 TOL = {F32: 2e-5, BF16: 4e-2}           # of the logits' RMS (mean removed), worst position
@@ -51,6 +52,47 @@ MECHANISMS = {
     "two_windows": one_layer(None, layers=[TokenLayerConfig(ATT, None), TokenLayerConfig(replace(ATT, window=5, heads=2, rot_base=300.0, rot_dim=8), MOE)]),
     "mixed": tiny_token_lm_config(),
 }
+
+GQA = GroupedAttentionConfig(heads=6, kv_heads=2, dim=24, vdim=20, scale=0.3, window=37, keep_first=5, sink=True)
+DELTA = ChannelDeltaConfig(heads=4, kv_heads=2, dim=20, vdim=24, conv=3, decay_rank=10, gate_rank=14)
+LIGHT = LightningConfig(heads=3, dim=18, vdim=28, decay=[0.7, 0.93, 0.995])
+GLU = DenseGLUConfig(ff=44, limit=1.2)
+
+
+def plain_layer(mixer, mlp=None, **kw):
+    """One layer of the two-norm kind: no layer scales, the head is the embedding table."""
+    base = dict(architecture="Bibapel", vocab=67, width=48, norm_eps=1e-5, layers=[TokenLayerConfig(mixer, mlp)], norms=2, layer_scales=False, tied_head=True,
+                loop_inject="project")
+    base.update(kw)
+    return TokenLMConfig(**base)
+
+
+MECHANISMS.update({
+    "grouped_attention": plain_layer(GQA),
+    "grouped_attention_own_heads": plain_layer(replace(GQA, heads=3, kv_heads=3, keep_first=0, sink=False)),
+    "grouped_attention_one_kv_head": plain_layer(replace(GQA, heads=5, kv_heads=1, vdim=33)),
+    "grouped_attention_one_head": plain_layer(replace(GQA, heads=1, kv_heads=1, window=1, keep_first=1)),
+    "grouped_attention_no_window": plain_layer(replace(GQA, window=0, keep_first=0)),
+    "grouped_attention_keeps_more_than_it_sees": plain_layer(replace(GQA, window=3, keep_first=40)),
+    "grouped_attention_wide": plain_layer(replace(GQA, heads=4, kv_heads=2, dim=100, vdim=72, scale=0.1)),
+    "grouped_attention_widest": plain_layer(replace(GQA, heads=2, kv_heads=1, dim=200, vdim=256, scale=0.07)),
+    "delta": plain_layer(DELTA),
+    "delta_own_heads_no_conv": plain_layer(replace(DELTA, heads=3, kv_heads=3, conv=1, vdim=16, dim=16)),
+    "delta_wide_long_conv": plain_layer(replace(DELTA, heads=2, kv_heads=1, dim=72, vdim=40, conv=7, decay_rank=1, gate_rank=70)),
+    "delta_widest": plain_layer(replace(DELTA, heads=1, kv_heads=1, dim=256, vdim=208, conv=2)),
+    "lightning": plain_layer(LIGHT),
+    "lightning_decay_ends": plain_layer(replace(LIGHT, decay=[0.0, 1.0, 0.5])),
+    "lightning_wide": plain_layer(LightningConfig(heads=2, dim=136, vdim=100, decay=[0.9, 0.97])),
+    "glu": plain_layer(LIGHT, GLU),
+    "glu_odd": plain_layer(replace(LIGHT, heads=1, decay=[0.8]), DenseGLUConfig(ff=37, limit=0.5), width=42),
+    "bigram": plain_layer(LIGHT, None, bigram=BigramConfig(buckets=13, mul_prev=5, mul_cur=3), embed_scale=0.5),
+    "positions": plain_layer(LIGHT, None, max_positions=200, embed_scale=2.0),
+    "projected_passes": plain_layer(None, layers=[TokenLayerConfig(DELTA, GLU), TokenLayerConfig(GQA, None)], loop_start=0, loop_stop=2, loop_times=3),
+    "projected_pass_of_one": plain_layer(None, layers=[TokenLayerConfig(LIGHT, GLU), TokenLayerConfig(GQA, GLU), TokenLayerConfig(DELTA, GLU)], width=40,
+                                         loop_start=1, loop_stop=2, loop_times=1, max_positions=150, bigram=BigramConfig(buckets=29, mul_prev=7, mul_cur=2)),
+    "two_kept_windows": plain_layer(None, layers=[TokenLayerConfig(GQA, None), TokenLayerConfig(replace(GQA, window=9, keep_first=70, heads=4, kv_heads=4), GLU)]),
+    "bibapel": tiny_bibapel_config(),
+})
 
 
 def make(cfg, dev, lib, dtype=F32, seed=5, **kw):
@@ -120,8 +162,8 @@ def check_activation_branches(dev, lib):
 
 
 # ---- how a sequence is fed -----------------------------------------------------------------------------------------------------
-def check_portions(dev, lib, dtype=F32, n=132, cut_sets=((2,), (3, 2, 61, 7), (64,), (65, 1), (127, 2), (33,))):
-    cfg = MECHANISMS["mixed"]
+def check_portions(dev, lib, dtype=F32, n=132, cut_sets=((2,), (3, 2, 61, 7), (64,), (65, 1), (127, 2), (33,)), name="mixed"):
+    cfg = MECHANISMS[name]
     lm, orc = make(cfg, dev, lib, dtype)
     toks = tokens_of(cfg, n, seed=1)
     want = orc.logits(toks)
@@ -131,16 +173,16 @@ def check_portions(dev, lib, dtype=F32, n=132, cut_sets=((2,), (3, 2, 61, 7), (6
         assert rel(run_cut(lm, toks, list(cuts)), want) < TOL[dtype], cuts
 
 
-def check_prompt_then_decode(dev, lib, dtype=F32, n=110, tail=30):
-    cfg = MECHANISMS["mixed"]
+def check_prompt_then_decode(dev, lib, dtype=F32, n=110, tail=30, name="mixed"):
+    cfg = MECHANISMS[name]
     lm, orc = make(cfg, dev, lib, dtype)
     toks = tokens_of(cfg, n, seed=2)
     assert rel(run_cut(lm, toks, [n - tail, 1]), orc.logits(toks)) < TOL[dtype]
 
 
-def check_unequal_batch(dev, lib, dtype=F32):
+def check_unequal_batch(dev, lib, dtype=F32, name="mixed"):
     """Requests of different lengths, portions beside single tokens, requests left out of steps: each as if it were alone."""
-    cfg = MECHANISMS["mixed"]
+    cfg = MECHANISMS[name]
     lm, orc = make(cfg, dev, lib, dtype, max_tokens=2048)
     rng = np.random.default_rng(3)
     seqs = [tokens_of(cfg, n, seed=10 + i) for i, n in enumerate((131, 1, 64, 40, 97, 66))]
@@ -166,9 +208,9 @@ def check_unequal_batch(dev, lib, dtype=F32):
         assert rel(np.concatenate(g), orc.logits(s)) < TOL[dtype]
 
 
-def check_batched_decode(dev, lib, dtype=F32, B=5, steps=12):
+def check_batched_decode(dev, lib, dtype=F32, B=5, steps=12, name="mixed"):
     """Pure decode steps at a fixed batch (captured launches): every replay against the oracle."""
-    cfg = MECHANISMS["mixed"]
+    cfg = MECHANISMS[name]
     lm, orc = make(cfg, dev, lib, dtype, max_tokens=2048)
     seqs = [tokens_of(cfg, 20 + 9 * i + steps, seed=30 + i) for i in range(B)]
     want = [orc.logits(s) for s in seqs]
@@ -181,10 +223,10 @@ def check_batched_decode(dev, lib, dtype=F32, B=5, steps=12):
             assert rel(r[None], w[len(t) - steps + k][None]) < 2 * TOL[dtype]
 
 
-def check_reuse(dev, lib, dtype=F32):
+def check_reuse(dev, lib, dtype=F32, name="mixed"):
     """Pages and slots go from request to request: a pool that holds one request at a time, earlier owners with other tokens, closed in
     the middle of a page; the last request's logits equal a fresh engine's, bit for bit."""
-    cfg = MECHANISMS["mixed"]
+    cfg = MECHANISMS[name]
     lm, orc = make(cfg, dev, lib, dtype, max_slots=2, max_tokens=192)
     fresh, _ = make(cfg, dev, lib, dtype, max_slots=2, max_tokens=192)
     for i, n in enumerate((192, 70, 129)):
@@ -199,15 +241,15 @@ def check_reuse(dev, lib, dtype=F32):
     assert lm.free_pages == lm.total_pages == 3
 
 
-def check_long_decode(dev, lib, dtype=F32, n=330, pool=256):
-    """A sequence longer than the pool: pages behind every window are given back and come round again."""
-    cfg = MECHANISMS["two_windows"]
+def check_long_decode(dev, lib, dtype=F32, n=330, pool=256, name="two_windows", held=2):
+    """A sequence longer than the pool: pages behind every window are given back and come round again (but those with kept positions)."""
+    cfg = MECHANISMS[name]
     lm, orc = make(cfg, dev, lib, dtype, max_slots=2, max_tokens=pool)
     toks = tokens_of(cfg, n, seed=4)
     slot = lm.open()
     got = run_cut(lm, toks, [130, 1], slot)
     assert rel(got, orc.logits(toks)) < TOL[dtype]
-    assert lm.position(slot) == n and lm.info(5, slot) <= 2          # held pages: a window of 37 spans at most two
+    assert lm.position(slot) == n and lm.info(5, slot) <= held          # a window of 37 spans at most two pages
     lm.close(slot)
     assert lm.free_pages == lm.total_pages
 
@@ -218,6 +260,16 @@ WIDE_PROMPTS = {
     "latent_128": one_layer(replace(ATT, heads=26, kv_rank=128, rot_dim=40, window=300)),
     "latent_200": one_layer(replace(ATT, heads=26, kv_rank=200, rot_dim=80, window=0)),
     "latent_500": one_layer(replace(ATT, heads=14, kv_rank=500, rot_dim=64, window=129)),
+}
+
+
+# the same for grouped attention (per head-size bound of its kernels), the delta rule and lightning attention over many chunks
+WIDE_PROMPTS_2 = {
+    "gqa_24": plain_layer(replace(GQA, heads=26, kv_heads=2, window=90)),
+    "gqa_128": plain_layer(replace(GQA, heads=28, kv_heads=4, dim=128, vdim=96, window=300, keep_first=100, scale=0.1)),
+    "gqa_256": plain_layer(replace(GQA, heads=26, kv_heads=13, dim=160, vdim=256, window=0, keep_first=0, scale=0.08)),
+    "delta_128": plain_layer(replace(DELTA, heads=4, kv_heads=2, dim=128, vdim=128, conv=4)),
+    "delta_lightning": plain_layer(None, layers=[TokenLayerConfig(DELTA, GLU), TokenLayerConfig(replace(LIGHT, dim=128, vdim=64), None)]),
 }
 
 
@@ -301,8 +353,8 @@ def check_far_state(dev, lib, dtype=F32):
         assert np.abs(diff - (wa[-1] - wb[-1])).max() < 0.05 * effect, cuts
 
 
-def check_first_tokens(dev, lib, dtype=F32):
-    cfg = MECHANISMS["mixed"]
+def check_first_tokens(dev, lib, dtype=F32, name="mixed"):
+    cfg = MECHANISMS[name]
     lm, orc = make(cfg, dev, lib, dtype)
     for seed in range(3):
         toks = tokens_of(cfg, 5, seed=70 + seed)
@@ -311,11 +363,158 @@ def check_first_tokens(dev, lib, dtype=F32):
             assert rel(run_cut(lm, toks, cuts), want) < TOL[dtype]
 
 
+def _attention_pair(orc, cfg):
+    """(query token, key token, plain token) of grouped attention over bare token embeddings: the pair whose score stands out most in some
+    head, and the token that head cares least for."""
+    w, m, p = orc.w, cfg.layers[0].mixer, "l0.mix."
+    h = rms_norm(w["embed"] * cfg.embed_scale, w["l0.norm1"], cfg.norm_eps)
+    q = (h @ w[p + "q"].T).reshape(cfg.vocab, m.heads, m.dim)
+    k = np.repeat((h @ w[p + "k"].T).reshape(cfg.vocab, m.kv_heads, m.dim), m.heads // m.kv_heads, axis=1)
+    s = np.matmul(q.transpose(1, 0, 2), k.transpose(1, 2, 0)).transpose(1, 2, 0)        # [query, key, head]
+    own = s[np.arange(cfg.vocab), np.arange(cfg.vocab)]
+    gap = s - np.maximum(np.maximum(s.min(axis=1), own), 0.0)[:, None, :]
+    query, key, head = np.unravel_index(np.argmax(gap), gap.shape)
+    return int(query), int(key), int(np.argmin(s[query, :, head]))
+
+
+def check_single_kept_keys(dev, lib, window=70, keep=6, dtype=F32, queries=(200, 128, 191, 97)):
+    """One dominating key at chosen places: around the window's edge, page borders, the last kept position and the one after it.  While it is
+    visible the logits are the oracle's and differ from a prompt without it; otherwise they are bit-identical to that."""
+    cfg = plain_layer(replace(GQA, window=window, keep_first=keep, scale=1.0))
+    sd = random_token_lm_state_dict(cfg, seed=5)
+    lm, orc = TokenLM(sd, cfg, device=dev, dtype=dtype, lib=lib, max_slots=2, max_tokens=512), TokenLMOracle(sd, cfg)
+    query, key, plain = _attention_pair(orc, cfg)
+    assert key not in (query, plain)
+    for at in queries:                                   # the query's position
+        base = [plain] * (at + 1)
+        base[at] = query
+        modes = (("prompt", [at + 1]), ("decoded", [at, 1]), ("two", [at - 1, 2]))
+        without = {mode: run_cut(lm, base, cuts)[at] for mode, cuts in modes}
+        ref0 = orc.logits(base)[at]
+        places = {0, 1, keep - 1, keep, keep + 1, 31, 32, 63, 64, at - 1, at - 2, at - window + 1, at - window, at - window - 1, at - at % 64}
+        for j in sorted(x for x in places if 0 <= x < at):
+            toks = list(base)
+            toks[j] = key
+            ref = orc.logits(toks)[at]
+            shows = window == 0 or at - j < window or j < keep
+            assert (rel(ref[None], ref0[None]) > 0.05) == shows, (at, j)
+            for mode, cuts in modes:
+                got = run_cut(lm, toks, cuts)[at]
+                assert rel(got[None], ref[None]) < TOL[dtype], (at, j, mode)
+                if shows:
+                    assert rel(got[None], without[mode][None]) > 0.05, (at, j, mode)
+                else:
+                    assert np.array_equal(got, without[mode]), (at, j, mode)
+
+
+def check_sink(dev, lib):
+    """Weak scores: the one in the denominator takes a share that leaving it out would show.  Strong negative ones: nearly all of it."""
+    for scale, n in ((0.01, 3), (0.01, 90), (-3.0, 40), (3.0, 40)):
+        cfg = plain_layer(replace(GQA, scale=scale))
+        sd = random_token_lm_state_dict(cfg, seed=7)
+        lm, orc = TokenLM(sd, cfg, device=dev, dtype=F32, lib=lib, max_slots=2, max_tokens=256), TokenLMOracle(sd, cfg)
+        without = TokenLMOracle(sd, plain_layer(replace(GQA, scale=scale, sink=False)))
+        toks = tokens_of(cfg, n)
+        want = orc.logits(toks)
+        assert rel(without.logits(toks)[:3], want[:3]) > 0.02
+        for cuts in ([n], [1], [n - 2, 2]):
+            assert rel(run_cut(lm, toks, cuts), want) < TOL[F32], (scale, n, cuts)
+
+
+def check_matrix_state_far(dev, lib, dtype=F32):
+    """What the matrix states remember: with decays of nearly one the first token still shows 200 tokens later, however it was fed."""
+    for name in ("delta", "lightning"):
+        cfg = plain_layer(DELTA if name == "delta" else replace(LIGHT, decay=[0.9995, 0.999, 0.9999]))
+        sd = random_token_lm_state_dict(cfg, seed=3)
+        if name == "delta":
+            sd["l0.mix.A_log"] = torch.full((DELTA.heads,), -7.0).to(BF16)
+        lm, orc = TokenLM(sd, cfg, device=dev, dtype=dtype, lib=lib, max_slots=2, max_tokens=512), TokenLMOracle(sd, cfg)
+        a = tokens_of(cfg, 200, seed=8)
+        b = [(a[0] + 1) % cfg.vocab] + a[1:]
+        wa, wb = orc.logits(a), orc.logits(b)
+        effect = np.abs(wa[-1] - wb[-1]).max()
+        assert effect > 1e-3, (name, effect)
+        for cuts in ([200], [31, 2, 97, 1], [4]):
+            diff = run_cut(lm, a, cuts)[-1].astype(np.float64) - run_cut(lm, b, cuts)[-1]
+            assert np.abs(diff - (wa[-1] - wb[-1])).max() < 0.05 * effect, (name, cuts)
+
+
+def check_decay_extremes(dev, lib):
+    """Channels that forget everything at one token and nothing at the next, in one chunk: the running products lose no precision.  Keys that
+    repeat with step sizes near one: the triangular system at its stiffest."""
+    cfg = plain_layer(replace(DELTA, heads=2, kv_heads=2, dim=32, vdim=16))
+    for amp, alog in ((40.0, 3.0), (8.0, 0.0)):
+        sd = random_token_lm_state_dict(cfg, seed=4)
+        sd["l0.mix.A_log"] = torch.full((2,), alog).to(BF16)
+        sd["l0.mix.a2"] = (sd["l0.mix.a2"].float() * amp).to(BF16)
+        sd["l0.mix.b"] = (sd["l0.mix.b"].float() * 5).to(BF16)
+        lm, orc = TokenLM(sd, cfg, device=dev, dtype=F32, lib=lib, max_slots=2, max_tokens=512), TokenLMOracle(sd, cfg)
+        toks = tokens_of(cfg, 60, seed=9) + [5] * 50 + [5, 9] * 20
+        want = orc.logits(toks)
+        for cuts in ([150], [1], [70, 3, 77]):
+            assert rel(run_cut(lm, toks, cuts), want) < TOL[F32], (amp, cuts)
+
+
+def check_glu_limits(dev, lib):
+    """Gate above its limit (and far below zero: unlimited), up beyond both of its limits."""
+    cfg = MECHANISMS["glu"]
+    sd = random_token_lm_state_dict(cfg, seed=6)
+    for n in ("gate", "up"):
+        sd[f"l0.mlp.{n}"] = (sd[f"l0.mlp.{n}"].float() * 4).to(BF16)
+    lm, orc = TokenLM(sd, cfg, device=dev, dtype=F32, lib=lib, max_slots=2, max_tokens=256), TokenLMOracle(sd, cfg)
+    toks = tokens_of(cfg, 80)
+    want = orc.logits(toks)
+    for cuts in ([80], [30, 1]):
+        assert rel(run_cut(lm, toks, cuts), want) < TOL[F32]
+
+
+def check_previous_token(dev, lib):
+    """The bigram row needs the token before a portion: cut everywhere, with another sequence in between, on a slot used before."""
+    cfg = MECHANISMS["bigram"]
+    sd = random_token_lm_state_dict(cfg, seed=2)
+    sd["bigram"] = (sd["bigram"].float() * 6).to(BF16)
+    lm, orc = TokenLM(sd, cfg, device=dev, dtype=F32, lib=lib, max_slots=2, max_tokens=256), TokenLMOracle(sd, cfg)
+    for seed in range(2):
+        a, b = tokens_of(cfg, 20, seed=seed), tokens_of(cfg, 20, seed=seed + 40)
+        wa, wb = orc.logits(a), orc.logits(b)
+        sa, sb = lm.open(), lm.open()
+        got, at = [], 0
+        for n in (1, 1, 5, 2, 1, 10):
+            if at % 2:
+                rows = lm.step([(sb, b[at:at + n], list(range(n))), (sa, a[at:at + n], list(range(n)))]).cpu().numpy()
+                assert rel(rows[:n], wb[at:at + n]) < TOL[F32]
+                rows = rows[n:]
+            else:
+                rows = lm.step([(sa, a[at:at + n], list(range(n)))]).cpu().numpy()
+                assert rel(lm.step([(sb, b[at:at + n], list(range(n)))]).cpu().numpy(), wb[at:at + n]) < TOL[F32]
+            got.append(rows.copy())
+            at += n
+        assert rel(np.concatenate(got), wa) < TOL[F32]
+        lm.close(sa)
+        lm.close(sb)
+
+
+def check_last_position(dev, lib):
+    import pytest
+    cfg = plain_layer(LIGHT, None, max_positions=70)
+    lm, orc = make(cfg, dev, lib, max_slots=2, max_tokens=256)
+    toks = tokens_of(cfg, 70)
+    slot = lm.open()
+    assert rel(run_cut(lm, toks, [69, 1], slot), orc.logits(toks)) < TOL[F32]
+    with pytest.raises(AssertionError):
+        lm.step([(slot, [1], [0])])
+    assert lm.position(slot) == 70
+    lm.close(slot)
+    with pytest.raises(ValueError):
+        TokenBatcher(lm).submit(toks, 2)
+    assert TokenBatcher(lm).submit(toks, 1)
+
+
 # ---- entry points --------------------------------------------------------------------------------------------------------------
-def check_generation(dev, lib, dtype=F32):
+def check_generation(dev, lib, dtype=F32, name="mixed"):
     """Greedy generation through the scheduler: more requests than slots, prompts cut by the step budget, a pool they must share;
     each request as the oracle generates it alone."""
-    cfg = MECHANISMS["mixed"]
+    cfg = MECHANISMS[name]
     lm, orc = make(cfg, dev, lib, dtype, max_slots=3, max_tokens=320)
     prompts = [tokens_of(cfg, n, seed=80 + i) for i, n in enumerate((50, 3, 120, 1, 66))]
     batcher = TokenBatcher(lm, step_tokens=48)
