@@ -207,10 +207,14 @@ __device__ __forceinline__ bool mmi_any(bool v) { return __any(v) != 0; }
 // streamed-once weights: non-temporal so they do not evict the activations / KV the other kernels reuse
 __device__ __forceinline__ u32x4 mmi_load_nt(const u32x4* p) { return __builtin_nontemporal_load(p); }
 __device__ __forceinline__ f32x4 mmi_load_nt(const f32x4* p) { return __builtin_nontemporal_load(p); }
+__device__ __forceinline__ void mmi_store_nt(f32x4* p, f32x4 v) { __builtin_nontemporal_store(v, p); }
 
 __device__ __forceinline__ float mmi_rsqrtf(float x) { return 1.0f / sqrtf(x); }  // IEEE, matches torch.rsqrt closely
 // natural log on the hardware's v_log_f32 (log2, ~1 ulp) - for the sampler's own noise only (nothing the reference's arithmetic
 // fixes): the library logf is ~25 dependent instructions on a one-wave-per-SIMD kernel that runs at ~9 cycles per instruction
+// base-2 exponential and logarithm in hardware (v_exp_f32, v_log_f32: ~1 ulp, denormals flushed)
+__device__ __forceinline__ float mmi_fast_exp2f(float x) { return __builtin_amdgcn_exp2f(x); }
+__device__ __forceinline__ float mmi_fast_log2f(float x) { return __builtin_amdgcn_logf(x); }
 __device__ __forceinline__ float mmi_fast_logf(float x) { return __logf(x); }
 __device__ __forceinline__ unsigned mmi_atomic_add(unsigned* p, unsigned v) { return atomicAdd(p, v); }
 

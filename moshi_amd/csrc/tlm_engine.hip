@@ -95,6 +95,7 @@ struct Shape {                     // what a launch list depends on
     int n_small = 0, n_unit = 0, n_chunk = 0;      // sequences stepped token by token, sequences cut into chunks, their chunks
     std::vector<int> tiles;        // attention column tiles per head count
     std::vector<std::array<int, 2>> groups;        // column groups of 4 and of 8 tiles per head count
+    std::vector<std::array<int, 3>> split;         // sequences of up to 64 columns: tiles; the others: groups of 4 and of 8 tiles
     Meta m;
     float* logits = nullptr;
     float* taps = nullptr;
@@ -160,6 +161,7 @@ namespace {
 constexpr int MAX_SPLIT = 8;
 constexpr int ROWS_MAX = 64;       // up to here a step takes the weight-streaming kernel
 constexpr int ATTN_TILE_GROUPS = 128;     // from this many column groups the attention stages keys through LDS
+constexpr int PREFIXES = 6;        // prefix arrays over the sequences per head count: tiles, groups of 4, groups of 8, then those of `split`
 constexpr int MAX_PARTIALS = 512;  // (column tile, split) pairs of the attention
 
 // ------------------------------------------------------------------------------------------------
@@ -714,7 +716,7 @@ int alloc_buffers(mmi_tlm* m) {
     MMI_HIP_CHECK(m->scratch.alloc(&m->samp_zero, 1));
     MMI_HIP_CHECK(hipMemset(m->samp_zero, 0, sizeof(int)));
     // metadata: 6 ints per token + wanted rows, per-entry arrays, tile prefixes, segments, sequences and chunks, block-table updates
-    m->meta_cap = 128 + (size_t)7 * T + 20 * (size_t)m->max_slots + 8 * ((size_t)T / TLM_CHUNK + m->max_slots + 1) + 3 * m->geo.size() * ((size_t)m->max_slots + 1) + 8 * ((size_t)T / TLM_SEG + m->max_slots + 1) +
+    m->meta_cap = 128 + (size_t)7 * T + 20 * (size_t)m->max_slots + 8 * ((size_t)T / TLM_CHUNK + m->max_slots + 1) + PREFIXES * m->geo.size() * ((size_t)m->max_slots + 1) + 8 * ((size_t)T / TLM_SEG + m->max_slots + 1) +
                   2 * ((size_t)T / TLM_PAGE + 2 * (size_t)m->max_slots + 2);
     MMI_HIP_CHECK(m->scratch.alloc(&m->meta, m->meta_cap));
     for (Staging& s : m->staging) {
@@ -1121,7 +1123,7 @@ MixerOut build_latent_attention(mmi_tlm* m, MmiProgram& P, const Shape& sh, cons
     const int kind = tiled ? (wide ? 2 : 1) : 0;       // which of the three prefix arrays
     t.n_tiles = tiled ? sh.groups[L.geo][kind - 1] : sh.tiles[L.geo];
     t.nsplit = tiled ? 1 : std::max(1, std::min(sh.nsplit, (L.nd > 16 ? 256 : MAX_PARTIALS) / std::max(1, t.n_tiles)));     // (a wide latent: one workgroup per CU)
-    t.tile0 = m->meta + sh.m.tile0 + (3 * L.geo + kind) * (sh.n_entries + 1);
+    t.tile0 = m->meta + sh.m.tile0 + (PREFIXES * L.geo + kind) * (sh.n_entries + 1);
     t.erow0 = m->meta + sh.m.erow0;
     t.elen = m->meta + sh.m.elen;
     t.epos0 = m->meta + sh.m.epos0;
@@ -1177,11 +1179,14 @@ MixerOut build_attention(mmi_tlm* m, MmiProgram& P, const Shape& sh, const Layer
     t.n_entries = sh.n_entries;
     const int bound = gqa_bound(L, m->kstep);
     const bool wide = !(f32 && bound == 256);            // columns per workgroup of k_tlm_gqa_tile (TlmGqaTile::QT)
-    const bool tiled = sh.groups[L.geo][wide] * G >= ATTN_TILE_GROUPS;
-    const int kind = tiled ? (wide ? 2 : 1) : 0;         // which of the three prefix arrays
-    t.n_tiles = tiled ? sh.groups[L.geo][kind - 1] : sh.tiles[L.geo];
-    t.nsplit = tiled ? 1 : std::max(1, std::min(sh.nsplit, MAX_PARTIALS / std::max(1, t.n_tiles * G)));
-    t.tile0 = m->meta + sh.m.tile0 + (3 * L.geo + kind) * (sh.n_entries + 1);
+    const std::array<int, 3>& sp = sh.split[L.geo];
+    // long portions through the kernel that stages keys, short ones (single tokens) through the other, if there are enough of the former
+    const bool tiled = sp[1 + wide] * G >= ATTN_TILE_GROUPS / 2;
+    auto part = [&](TlmGqaArgs& x, int kind, int n, bool split) {
+        x.tile0 = m->meta + sh.m.tile0 + (PREFIXES * L.geo + kind) * (sh.n_entries + 1);
+        x.n_tiles = n;
+        x.nsplit = split ? std::max(1, std::min(sh.nsplit, MAX_PARTIALS / std::max(1, n * G))) : 1;
+    };
     t.erow0 = m->meta + sh.m.erow0;
     t.elen = m->meta + sh.m.elen;
     t.epos0 = m->meta + sh.m.epos0;
@@ -1189,21 +1194,35 @@ MixerOut build_attention(mmi_tlm* m, MmiProgram& P, const Shape& sh, const Layer
     t.pages = TlmPages{m->block_table, table_ld(m), m->keep_pages};
     t.po = m->po;
     t.pml = m->pml;
+    auto launch = [&](const TlmGqaArgs& x, bool staged) {
+        P.add([=](hipStream_t s) { return f32 ? launch_gqa_t<TlmF32>(s, x, bound, staged) : launch_gqa_t<TlmBf16>(s, x, bound, staged); });
+    };
     P.site(site + "attn");
-    P.add([=](hipStream_t s) { return f32 ? launch_gqa_t<TlmF32>(s, t, bound, tiled) : launch_gqa_t<TlmBf16>(s, t, bound, tiled); });
+    if (tiled) {
+        TlmGqaArgs u = t;
+        part(u, wide ? 5 : 4, sp[1 + wide], false);
+        launch(u, true);
+        part(t, 3, sp[0], true);
+    } else {
+        part(t, 0, sh.tiles[L.geo], true);
+    }
+    if (t.n_tiles) launch(t, false);
     return MixerOut{&L.out, m->o, L.out.KS};
 }
 
 template <class Tr, bool DELTA>
 int launch_state_step(hipStream_t s, const TlmLinArgs& a, int n) {
     const int cgp = tlm_step_groups(a.vdim_p);
-    int block = 64;
-    while (block < 256 && mmi_cdiv(a.dim_p * cgp, block) > 4) block *= 2;
+    int block = 64;                                      // rows of S per thread: 4, in larger workgroups 8, at the largest sizes 16
+    while (block < 256 && mmi_cdiv(a.dim_p, block / cgp) > 4) block *= 2;
+    while (block < 512 && mmi_cdiv(a.dim_p, block / cgp) > 8) block *= 2;
     while (mmi_cdiv(a.dim_p, block / cgp) > 16) block *= 2;
-    const int parts = block / cgp;
-    const size_t smem = (size_t)(3 * a.dim_p + a.vdim_p + 2 * parts * a.vdim_p) * sizeof(float);
-    if (mmi_cdiv(a.dim_p, parts) <= 4) MMI_LAUNCH((k_tlm_state_step<Tr, DELTA, 4>), dim3(n, a.heads), block, smem, s, a, cgp);
-    else MMI_LAUNCH((k_tlm_state_step<Tr, DELTA, 16>), dim3(n, a.heads), block, smem, s, a, cgp);
+    const int parts = block / cgp, rows = mmi_cdiv(a.dim_p, parts);
+    const int rt = rows <= 4 && block <= 256 ? 4 : (rows <= 8 && block <= 512 ? 8 : 16);
+    const size_t smem = (size_t)(3 * parts * rt + a.vdim_p + 2 * parts * a.vdim_p) * sizeof(float);
+    if (rt == 4) MMI_LAUNCH((k_tlm_state_step<Tr, DELTA, 4, 256>), dim3(n, a.heads), block, smem, s, a, cgp);
+    else if (rt == 8) MMI_LAUNCH((k_tlm_state_step<Tr, DELTA, 8, 512>), dim3(n, a.heads), block, smem, s, a, cgp);
+    else MMI_LAUNCH((k_tlm_state_step<Tr, DELTA, 16, 1024>), dim3(n, a.heads), block, smem, s, a, cgp);
     MMI_CHECK_LAUNCH();
     return MMI_OK;
 }
@@ -1222,9 +1241,7 @@ MixerOut build_linear(mmi_tlm* m, MmiProgram& P, const Shape& sh, const Layer& L
     const int T = sh.T, H = L.c.heads;
     const bool f32 = m->f32, delta = L.c.mixer == MMI_TLM_MIX_CHANNEL_DELTA;
     TlmJob j = dense_job(L.in, m->h, m->h_ks, T);
-    j.epi = TLM_EPI_ACT;
-    j.act = delta ? TLM_ACT_NONE : TLM_ACT_SILU;
-    j.act2 = TLM_ACT_SIGMOID;
+    j.epi = delta ? TLM_EPI_F32 : TLM_EPI_SILU;
     j.act_nt = L.b0 / 16;
     j.out = m->lin;
     j.out_ld = L.in_ld;
@@ -1261,6 +1278,7 @@ MixerOut build_linear(mmi_tlm* m, MmiProgram& P, const Shape& sh, const Layer& L
     a.conv_c = L.conv_c;
     a.taps = L.c.conv;
     a.decay = delta ? m->dec : L.decay;
+    a.decay_c = L.decay;
     a.gate = delta ? m->lgate : m->lin + L.b0;
     a.gate_ld = delta ? H * L.vdim_p : L.in_ld;
     a.nw = L.nw;
@@ -1283,17 +1301,12 @@ MixerOut build_linear(mmi_tlm* m, MmiProgram& P, const Shape& sh, const Layer& L
         memset(&Q, 0, sizeof(Q));
         TlmJob& ja = Q.j[Q.n++];
         ja = dense_job(L.a2, m->lr, lr_ks, T);
-        ja.epi = TLM_EPI_ACT;
-        ja.act = TLM_ACT_DECAY;
-        ja.act_nt = L.a2.NT;
-        ja.bias = L.decay;
+        ja.epi = TLM_EPI_F32;
         ja.out = m->dec;
         ja.out_ld = H * L.dim_p;
         TlmJob& jg = Q.j[Q.n++];
         jg = dense_job(L.g2, (const u32x4*)m->lr + (long)(L.ra / m->kstep) * 64, lr_ks, T);
-        jg.epi = TLM_EPI_ACT;
-        jg.act = TLM_ACT_SIGMOID;
-        jg.act_nt = L.g2.NT;
+        jg.epi = TLM_EPI_F32;
         jg.out = m->lgate;
         jg.out_ld = H * L.vdim_p;
         P.site(site + "lowrank");
@@ -1311,7 +1324,7 @@ MixerOut build_linear(mmi_tlm* m, MmiProgram& P, const Shape& sh, const Layer& L
         if (delta) {
             P.site(site + "conv");
             P.add([=](hipStream_t s) {
-                MMI_LAUNCH(k_tlm_conv, dim3(n_chunk, 2 * a.kv_heads + a.heads), 256, 0, s, a);
+                MMI_LAUNCH(k_tlm_conv, dim3(n_chunk, 2 * a.kv_heads + a.heads), 256, 0, s, a, tlm_step_groups(a.dim_p), tlm_step_groups(a.vdim_p));
                 MMI_CHECK_LAUNCH();
                 return (int)MMI_OK;
             });
@@ -1819,7 +1832,7 @@ extern "C" int mmi_tlm_step(mmi_tlm* m, int32_t n_entries, const int32_t* slots,
     M.elen = take(n_entries);
     M.epos0 = take(n_entries);
     M.eslot = take(n_entries);
-    M.tile0 = take(3 * (int)m->geo.size() * (n_entries + 1));
+    M.tile0 = take(PREFIXES * (int)m->geo.size() * (n_entries + 1));
     M.seg = take(8 * sh.n_seg);
     M.small = take(8 * sh.n_small);
     M.unit = take(8 * sh.n_unit);
@@ -1839,6 +1852,7 @@ extern "C" int mmi_tlm_step(mmi_tlm* m, int32_t n_entries, const int32_t* slots,
     int n_ck = 0;
     sh.tiles.assign(m->geo.size(), 0);
     sh.groups.assign(m->geo.size(), {0, 0});
+    sh.split.assign(m->geo.size(), {0, 0, 0});
     for (int e = 0; e < n_entries; ++e) {
         Slot& S = m->slots[slots[e]];
         for (int64_t n = pages_for(m, &S, counts[e]); n > 0; --n) {
@@ -1856,7 +1870,7 @@ extern "C" int mmi_tlm_step(mmi_tlm* m, int32_t n_entries, const int32_t* slots,
         b[M.epos0 + e] = (int)S.pos;
         b[M.eslot + e] = slots[e];
         for (size_t g = 0; g < m->geo.size(); ++g) {
-            int* t = b + M.tile0 + 3 * (int)g * (n_entries + 1) + e;
+            int* t = b + M.tile0 + PREFIXES * (int)g * (n_entries + 1) + e;
             const int n = mmi_cdiv(counts[e] * m->geo[g], 16);
             t[0] = sh.tiles[g];
             t[n_entries + 1] = sh.groups[g][0];
@@ -1864,6 +1878,13 @@ extern "C" int mmi_tlm_step(mmi_tlm* m, int32_t n_entries, const int32_t* slots,
             sh.tiles[g] += n;
             sh.groups[g][0] += mmi_cdiv(n, 4);
             sh.groups[g][1] += mmi_cdiv(n, 8);
+            std::array<int, 3>& sp = sh.split[g];
+            for (int k = 0; k < 3; ++k) t[(3 + k) * (n_entries + 1)] = sp[k];
+            if (n <= 4) sp[0] += n;
+            else {
+                sp[1] += mmi_cdiv(n, 4);
+                sp[2] += mmi_cdiv(n, 8);
+            }
         }
         for (int o = 0, k = 0; o < counts[e]; o += TLM_SEG, ++k) {
             const int n = std::min(TLM_SEG, counts[e] - o);

@@ -103,7 +103,7 @@ __global__ __launch_bounds__(256, Tr::V == 8 && D <= 128 ? 2 : 1) void k_tlm_gqa
         nb = w.block(min(i, i1 - 1));
         pg = (long)tlm_page(a.pages, bt, nb >> 1) * a.kv_heads + g;
     };
-    auto load = [&](int f) __attribute__((always_inline)) { fr[f] = P::at(a, pg, nb, f)[lane]; };
+    auto load = [&](int f) __attribute__((always_inline)) { fr[f] = mmi_load_nt(P::at(a, pg, nb, f) + lane); };
     if (i0 + wave < i1) {
         aim(i0 + wave);
 #pragma unroll
@@ -207,7 +207,7 @@ struct TlmGqaTile {
     static constexpr size_t smem() { return (size_t)2 * NF * 1024; }
 };
 template <class Tr, int D>
-__global__ __launch_bounds__(256) void k_tlm_gqa_tile(TlmGqaArgs a) {
+__global__ __launch_bounds__(256, Tr::V == 8 && D <= 128 ? 2 : 1) void k_tlm_gqa_tile(TlmGqaArgs a) {
     typedef TlmGqa<Tr, D> P;
     constexpr int NK = P::NK, ND = P::ND, QT = TlmGqaTile<Tr, D>::QT, NF = P::F, NI = NF / 4;
     typedef TlmAttnStream<Tr, ND, 0, QT, (ND >= 16 ? 4 : 8)> S;
@@ -215,7 +215,7 @@ __global__ __launch_bounds__(256) void k_tlm_gqa_tile(TlmGqaArgs a) {
     MMI_DYN_SHARED(u32x4, lds);
     const int lane = (int)threadIdx.x & 63, wave = mmi_uniform((int)threadIdx.x >> 6), bl = lane & 15, kq = lane >> 4;
     const int g = (int)blockIdx.y;
-    TlmCols c = P::find(a, (int)blockIdx.x);                       // (tile0 counts groups of 64 QT columns here)
+    TlmCols c = P::find(a, (int)gridDim.x - 1 - (int)blockIdx.x);  // (tile0 counts groups of 64 QT columns here; the last see most keys: they start first)
     c.c0 *= 4 * QT;
     const int pos0 = a.epos0[c.entry];
     const TlmWalk w(a.mask, pos0 + c.c0 / a.rep, pos0 + min(c.c0 + 64 * QT - 1, c.ncol - 1) / a.rep);
@@ -233,25 +233,23 @@ __global__ __launch_bounds__(256) void k_tlm_gqa_tile(TlmGqaArgs a) {
 #pragma unroll
         for (int s = 0; s < NK; ++s) q[t][s] = P::query(a, c, g, col, kq, s);
     }
-    u32x4 st[NI];                                                  // wave w brings fragments w, w + 4, ..
-    auto fetch = [&](int i) __attribute__((always_inline)) {       // (past the end: the last block again)
+    u32x4 st[2][NI];                                               // wave w brings fragments w, w + 4, ..; two blocks ahead of their use
+    long pg = (long)tlm_page(a.pages, bt, w.block(0) >> 1) * a.kv_heads + g;      // page of the block fetched next
+    auto fetch = [&](int set, int i) __attribute__((always_inline)) {      // (past the end: the last block again)
         const int kb = w.block(min(i, n - 1));
-        const long pg = (long)tlm_page(a.pages, bt, kb >> 1) * a.kv_heads + g;
 #pragma unroll
-        for (int f = 0; f < NI; ++f) st[f] = P::at(a, pg, kb, wave + 4 * f)[lane];
+        for (int f = 0; f < NI; ++f) st[set][f] = P::at(a, pg, kb, wave + 4 * f)[lane];
+        pg = (long)tlm_page(a.pages, bt, w.block(min(i + 1, n - 1)) >> 1) * a.kv_heads + g;
     };
     auto stage = [&](int buf) __attribute__((always_inline)) {
 #pragma unroll
-        for (int f = 0; f < NI; ++f) lds[(buf * NF + wave + 4 * f) * 64 + lane] = st[f];
+        for (int f = 0; f < NI; ++f) lds[(buf * NF + wave + 4 * f) * 64 + lane] = st[buf][f];
     };
-    fetch(0);
-    stage(0);
-    __syncthreads();
-    for (int i = 0; i < n; ++i) {
-        fetch(i + 1);
+    auto block = [&](int i, int buf) __attribute__((always_inline)) {      // block i in LDS buffer `buf`; i + 1 in register set buf ^ 1
+        fetch(buf, i + 2);
         mmi_sched_barrier();
-        const int kb = w.block(i);
-        const u32x4* base = lds + (i & 1) * NF * 64 + lane;
+        const int kb = w.block(min(i, n - 1));
+        const u32x4* base = lds + buf * NF * 64 + lane;
         auto at = [&](int f) __attribute__((always_inline)) -> const u32x4* { return base + f * 64; };
         auto qf = [&](int t, int k) __attribute__((always_inline)) { return q[t][k]; };
         int d0[QT];
@@ -264,8 +262,16 @@ __global__ __launch_bounds__(256) void k_tlm_gqa_tile(TlmGqaArgs a) {
             mmi_sched_barrier();
             sm.use(a.mask, qf, s & 1, s, kb * 32 + 4 * kq, d0);
         }
-        stage((i + 1) & 1);
+        stage(buf ^ 1);
         __syncthreads();
+    };
+    fetch(0, 0);
+    fetch(1, 1);
+    stage(0);
+    __syncthreads();
+    for (int i = 0; i < n; i += 2) {
+        block(i, 0);
+        if (i + 1 < n) block(i + 1, 1);
     }
 #pragma unroll
     for (int t = 0; t < QT; ++t) {

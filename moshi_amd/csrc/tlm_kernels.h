@@ -302,8 +302,8 @@ __global__ __launch_bounds__(1024) void k_tlm_resid_norm(TlmResidArgs a) {
 // ------------------------------------------------------------------------------------------------
 // matrix products: up to three of them per launch, each dense, grouped (per head) or routed (per expert)
 // ------------------------------------------------------------------------------------------------
-enum { TLM_EPI_F32 = 0, TLM_EPI_PACK = 1, TLM_EPI_ROPE = 2, TLM_EPI_GRU = 3, TLM_EPI_LOGITS = 4, TLM_EPI_ACT = 5, TLM_EPI_GLU = 6, TLM_EPI_QKV = 7 };
-enum { TLM_ACT_NONE = 0, TLM_ACT_RELU2 = 1, TLM_ACT_SILU = 2, TLM_ACT_SIGMOID = 3, TLM_ACT_DECAY = 4 };
+enum { TLM_EPI_F32 = 0, TLM_EPI_PACK = 1, TLM_EPI_ROPE = 2, TLM_EPI_GRU = 3, TLM_EPI_LOGITS = 4, TLM_EPI_SILU = 5, TLM_EPI_GLU = 6, TLM_EPI_QKV = 7 };
+enum { TLM_ACT_NONE = 0, TLM_ACT_RELU2 = 1 };
 // queries, keys and values of grouped attention: head by head, every head padded to whole tiles; keys and values go to the cache
 struct TlmQkv {
     void *kc, *vc;
@@ -321,10 +321,10 @@ struct TlmJob {
     const int* tiles;
     const int* n_tiles;
     int in_div;
-    int epi, act, act2, act_nt;          // ACT: act2 from tile act_nt on
+    int epi, act, act_nt;                // SILU: the first act_nt tiles
     void* out; int out_ld; long out_ps;  // fp32: row stride, stride per K split; packed: k-steps per row tile
     int out_mul, out_gadd, out_k0, out_kg;
-    const float* bias;                   // GRU: [2][width]; DECAY: [2][columns]: summand, then factor of the softplus
+    const float* bias;                   // GRU: [2][width]
     TlmQkv qkv;
     const float* gate; int gate_ld;      // PACK: factor per (row, group), or null
     const float* rope; int rope_ld;      // ROPE: (cos, sin) per row
@@ -336,8 +336,6 @@ struct TlmJobs {
     TlmJob j[3];
     int n;
 };
-
-__device__ __forceinline__ float tlm_softplus(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
 
 // cached values of grouped attention: the transposed operand of the value product, [page][kv head][keys / KSTEP][16-wide value blocks]
 // fragments whose reduction order is the one the softmax weights have in the registers after S = K Q^T (bf16: keys 4 kq .. 4 kq + 3 of
@@ -384,18 +382,10 @@ __device__ __forceinline__ void tlm_epilogue(const TlmJob& j, int g, int split, 
             for (int e = 0; e < 4; ++e) o[e] = (kind == 1 && v[e] >= 0.f) ? v[e] + 0.5f : tlm_sigmoid(v[e]);
         }
         *reinterpret_cast<f32x4*>((float*)j.out + (orow * 3 + kind) * w + c) = o;
-    } else if constexpr (EPI == TLM_EPI_ACT) {
-        const int act = nt < j.act_nt ? j.act : j.act2;
-        if (act == TLM_ACT_DECAY) {
-            const f32x4 b = *reinterpret_cast<const f32x4*>(j.bias + n0), f = *reinterpret_cast<const f32x4*>(j.bias + j.out_ld + n0);
+    } else if constexpr (EPI == TLM_EPI_SILU) {
+        if (nt < j.act_nt) {
 #pragma unroll
-            for (int e = 0; e < 4; ++e) v[e] = expf(-f[e] * tlm_softplus(v[e] + b[e]));
-        } else if (act != TLM_ACT_NONE) {
-#pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                const float s = tlm_sigmoid(v[e]);
-                v[e] = act == TLM_ACT_SILU ? v[e] * s : s;
-            }
+            for (int e = 0; e < 4; ++e) v[e] *= tlm_sigmoid(v[e]);
         }
         *reinterpret_cast<f32x4*>((float*)j.out + orow * j.out_ld + n0) = v;
     } else if constexpr (EPI == TLM_EPI_GLU) {
@@ -438,7 +428,7 @@ __device__ __forceinline__ void tlm_with_epilogue(int epi, F f) {
     else if (epi == TLM_EPI_PACK) f(TlmEpi<TLM_EPI_PACK>());
     else if (epi == TLM_EPI_ROPE) f(TlmEpi<TLM_EPI_ROPE>());
     else if (epi == TLM_EPI_GRU) f(TlmEpi<TLM_EPI_GRU>());
-    else if (epi == TLM_EPI_ACT) f(TlmEpi<TLM_EPI_ACT>());
+    else if (epi == TLM_EPI_SILU) f(TlmEpi<TLM_EPI_SILU>());
     else if (epi == TLM_EPI_GLU) f(TlmEpi<TLM_EPI_GLU>());
     else if (epi == TLM_EPI_QKV) f(TlmEpi<TLM_EPI_QKV>());
     else f(TlmEpi<TLM_EPI_LOGITS>());
@@ -466,13 +456,12 @@ __global__ __launch_bounds__(WAVES * 64, WAVES == 4 ? 2 : 1) void k_tlm_gemm_row
     } else {
         n = j.rows - r0 < 16 * MT ? j.rows - r0 : 16 * MT;
     }
-    int id[MT];                                               // rows past n repeat the last one, and are dropped at the end
-    const u32x4* xq[MT];
+    const u32x4* xq[MT];                                      // rows past n repeat the last one, and are dropped at the end
 #pragma unroll
     for (int m = 0; m < MT; ++m) {
         const int i = m * 16 + bl < n ? m * 16 + bl : n - 1;
-        id[m] = j.list ? j.list[r0 + i] : r0 + i;
-        const long in = j.list ? id[m] / j.in_div : (long)id[m] * j.in_mul + (long)g * j.in_gadd;
+        const int id = j.list ? j.list[r0 + i] : r0 + i;
+        const long in = j.list ? id / j.in_div : (long)id * j.in_mul + (long)g * j.in_gadd;
         xq[m] = j.xp + ((in >> 4) * j.xks + (long)g * j.xkg) * 64 + (in & 15) + (lane >> 4) * 16;
     }
     // K range of this split, then of this wave
@@ -544,16 +533,15 @@ __global__ __launch_bounds__(WAVES * 64, WAVES == 4 ? 2 : 1) void k_tlm_gemm_row
         for (int m = 0; m < MT; ++m) red[((wave * NTW + t) * MT + m) * 64 + lane] = acc[t][m];
     __syncthreads();
     tlm_with_epilogue(j.epi, [&](auto epi) __attribute__((always_inline)) {
+#pragma unroll 1
+        for (int q = wave; q < NTW * MT; q += WAVES) {
+            const int t = q / MT, i = (q - t * MT) * 16 + bl;
+            if (i >= n || nt0 + t >= j.NT) continue;
+            f32x4 v = red[q * 64 + lane];
 #pragma unroll
-        for (int t = 0; t < NTW; ++t)
-#pragma unroll
-            for (int m = 0; m < MT; ++m) {
-                if ((t * MT + m) % WAVES != wave || m * 16 + bl >= n || nt0 + t >= j.NT) continue;
-                f32x4 v = red[(t * MT + m) * 64 + lane];
-#pragma unroll
-                for (int w = 1; w < WAVES; ++w) v += red[((w * NTW + t) * MT + m) * 64 + lane];
-                tlm_epilogue<Tr, decltype(epi)::value>(j, g, split, id[m], nt0 + t, lane >> 4, v);
-            }
+            for (int w = 1; w < WAVES; ++w) v += red[(w * NTW * MT + q) * 64 + lane];
+            tlm_epilogue<Tr, decltype(epi)::value>(j, g, split, j.list ? j.list[r0 + i] : r0 + i, nt0 + t, lane >> 4, v);
+        }
     });
 }
 
@@ -656,11 +644,13 @@ __global__ __launch_bounds__(256, 2) void k_tlm_gemm_tile(TlmJobs jobs) {
             const int m = (wm * FM + y) * 16 + bl;
             if (m >= n) continue;
             const int id = j.list ? j.list[r0 + m] : r0 + m;
+            // through LDS (a lane reads what it wrote), so that the epilogue's code is there once per y and not once per tile
+            f32x4* buf = reinterpret_cast<f32x4*>(lds) + wave * FN * 64 + lane;
 #pragma unroll
-            for (int x = 0; x < FN; ++x) {
-                const int nt = nt0 + wn * FN + x;
-                if (nt < j.NT) tlm_epilogue<Tr, decltype(epi)::value>(j, g, 0, id, nt, lane >> 4, acc[x][y]);
-            }
+            for (int x = 0; x < FN; ++x) buf[x * 64] = acc[x][y];
+            const int nx = min(FN, j.NT - nt0 - wn * FN);
+#pragma unroll 1
+            for (int x = 0; x < nx; ++x) tlm_epilogue<Tr, decltype(epi)::value>(j, g, 0, id, nt0 + wn * FN + x, lane >> 4, buf[x * 64]);
         }
     });
 }

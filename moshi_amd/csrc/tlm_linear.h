@@ -31,40 +31,59 @@ struct TlmLinArgs {
     int heads, kv_heads, dim, vdim, dim_p, vdim_p;
     float q_scale, eps;
     const float* conv_w; float* conv_state; int conv_c, taps;      // delta: [taps][channels]; [slot][2][taps - 1][channels], read one copy and write the other
-    const float* decay;                  // delta: [row][heads][dim_p]; lightning: powers 0 .. TLM_CHUNK of every head's constant
-    const float* gate; int gate_ld;      // factor of the normalised output
+    const float* decay;                  // delta: projection [row][heads][dim_p] (tlm_decay); lightning: powers 0 .. TLM_CHUNK of every head's constant
+    const float* decay_c;                // delta: [2][heads][dim_p] summand, factor
+    const float* gate; int gate_ld;      // the normalised output's factor, before its sigmoid
     const float* nw;                     // its weight (delta: per head column, lightning: per column)
     float* state;                        // [slot][heads][dim_p][vdim_p]
     const TlmUnit* small; const TlmUnit* unit; const TlmSeg* chunk;
     float* qkv;                          // delta: convolved and normalised [row][conv_c], same columns as `in`
-    float *w, *qg, *kt, *u0, *p, *gend;  // per (chunk, head): [64][dim_p], [64][dim_p], [dim_p][64], [64][vdim_p], [64][64], [dim_p]
+    // per (chunk, head), in fragments of 16 x 16 (a lane's four elements together, so that the walk's loads are contiguous): w and qg
+    // [64][dim_p], kt [dim_p][64], p [64][64] by tlm_tile; u0 [64][vdim_p] in the layout of the matrix core's sums; gend [dim_p]
+    float *w, *qg, *kt, *u0, *p, *gend;
     float* o;                            // [row][heads][vdim_p] before the norm
     void* out; int out_ks;               // packed operand of the output projection
 };
 
+// decay of channel d of a head: exp(-factor softplus(z)), z = projection + summand, as 2^(-factor log2(1 + e^z)).  With u = e^z rounded
+// and w = 1 + u rounded, log2(w) u / (w - 1) is log2(1 + u) to the last bits however small u is.
+__device__ __forceinline__ float tlm_decay(const TlmLinArgs& a, long row, int h, int d) {
+    constexpr float LOG2E = 1.44269504088896340736f;
+    const int c = h * a.dim_p + d;
+    const float z = a.decay[row * a.heads * a.dim_p + c] + a.decay_c[c];
+    const float u = mmi_fast_exp2f(fminf(z, 30.f) * LOG2E), w = 1.0f + u;
+    float l = w > 1.0f ? mmi_fast_log2f(w) * u / (w - 1.0f) : u * LOG2E;
+    if (z > 20.f) l = z * LOG2E;
+    return mmi_fast_exp2f(-a.decay_c[a.heads * a.dim_p + c] * l);
+}
 __device__ __forceinline__ float tlm_silu(float x) { return x * tlm_sigmoid(x); }
 
-// channel c of the convolution at token t of a sequence whose rows start at row0 of the projection
-__device__ __forceinline__ float tlm_conv(const TlmLinArgs& a, const float* old, int fresh, int row0, int t, int c) {
-    float s = 0.f;
-    for (int j = 0; j < a.taps; ++j) {
-        const int at = t - (a.taps - 1) + j;
-        float x = 0.f;
-        if (at >= 0) x = a.in[(long)(row0 + at) * a.in_ld + c];
-        else if (!fresh) x = old[(long)(a.taps - 1 + at) * a.conv_c + c];
-        s = mmi_fma(a.conv_w[(long)j * a.conv_c + c], x, s);
+// element (row, k) of an operand with `ks` 16-wide blocks per 16 rows
+MMI_HD long tlm_tile(int row, int k, int ks) { return (((long)(row >> 4) * ks + (k >> 4)) * 64 + ((k & 15) >> 2) * 16 + (row & 15)) * 4 + (k & 3); }
+
+// channel(s) from c of the convolution at token t of a sequence whose rows start at row0 of the projection; four taps are requested at a
+// time (a tap before the sequence's start reads some valid address and counts as zero).  `now`: where the taps - 1 inputs that the next
+// step's first token needs stay, or null
+template <class T>
+__device__ __forceinline__ T tlm_conv(const TlmLinArgs& a, const float* old, int fresh, int row0, int t, int c, float* now) {
+    T s = T{};
+    for (int j0 = 0; j0 < a.taps; j0 += 4) {
+        T x[4], w[4];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const int tap = min(j0 + j, a.taps - 1), at = t - (a.taps - 1) + tap;
+            x[j] = *reinterpret_cast<const T*>(at >= 0 || fresh ? a.in + (long)(row0 + max(at, 0)) * a.in_ld + c : old + (long)(a.taps - 1 + at) * a.conv_c + c);
+            w[j] = *reinterpret_cast<const T*>(a.conv_w + (long)tap * a.conv_c + c);
+            if (j0 + j >= a.taps || (at < 0 && fresh)) x[j] = T{};
+        }
+#pragma unroll
+        for (int j = 0; j < 4; ++j) s += w[j] * x[j];
+        if (now)
+#pragma unroll
+            for (int j = 0; j < 4; ++j)
+                if (j0 + j >= 1 && j0 + j < a.taps) *reinterpret_cast<T*>(now + (long)(j0 + j - 1) * a.conv_c + c) = x[j];
     }
     return s;
-}
-// the last taps - 1 inputs of channel c after n tokens
-__device__ __forceinline__ void tlm_conv_keep(const TlmLinArgs& a, const float* old, float* now, int fresh, int row0, int n, int c) {
-    for (int s = 0; s < a.taps - 1; ++s) {
-        const int at = n - (a.taps - 1) + s;
-        float x = 0.f;
-        if (at >= 0) x = a.in[(long)(row0 + at) * a.in_ld + c];
-        else if (!fresh) x = old[(long)(n + s) * a.conv_c + c];
-        now[(long)s * a.conv_c + c] = x;
-    }
 }
 
 // ------------------------------------------------------------------------------------------------
@@ -75,23 +94,23 @@ inline int tlm_step_groups(int vdim_p) {                  // column groups of 4,
     while (4 * g < vdim_p) g *= 2;
     return g;
 }
-template <class Tr, bool DELTA, int RT>
-__global__ __launch_bounds__(1024) void k_tlm_state_step(TlmLinArgs a, int cgp) {
-    MMI_DYN_SHARED(float, sh);                             // q, k, g [dim_p], v [vdim_p], red [2][parts][vdim_p]
+template <class Tr, bool DELTA, int RT, int MAXB>
+__global__ __launch_bounds__(MAXB, MAXB == 512 && !DELTA ? 5 : 4) void k_tlm_state_step(TlmLinArgs a, int cgp) {
+    MMI_DYN_SHARED(float, sh);                             // q, k, g [parts * RT] (zeros from dim_p on), v [vdim_p], red [2][parts][vdim_p]
     const int tid = (int)threadIdx.x, nthr = (int)blockDim.x, lane = tid & 63;
     const int parts = nthr / cgp, cg = tid & (cgp - 1), part = tid / cgp, col = 4 * cg;
     const TlmUnit un = a.small[blockIdx.x];
     const int h = (int)blockIdx.y, rep = a.heads / a.kv_heads, kh = h / rep, D = a.dim_p, V = a.vdim_p;
-    float *q = sh, *k = q + D, *g = k + D, *v = g + D, *red = v + V;
+    float *q = sh, *k = q + parts * RT, *g = k + parts * RT, *v = g + parts * RT, *red = v + V;
+    for (int i = D + tid; i < parts * RT; i += nthr) q[i] = k[i] = g[i] = 0.f;
     const bool mine = col < V;
     float* S = a.state + ((long)un.slot * a.heads + h) * D * V;
     f32x4 s[RT];
 #pragma unroll
-    for (int i = 0; i < RT; ++i) {
-        const int d = part + parts * i;
-        s[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-        if (!un.fresh && mine && d < D) s[i] = *reinterpret_cast<const f32x4*>(S + (long)d * V + col);
-    }
+    for (int i = 0; i < RT; ++i) s[i] = mmi_load_nt(reinterpret_cast<const f32x4*>(S + (long)min(part + parts * i, D - 1) * V + min(col, V - 4)));
+#pragma unroll
+    for (int i = 0; i < RT; ++i)
+        if (un.fresh || !mine || part + parts * i >= D) s[i] = f32x4{0.f, 0.f, 0.f, 0.f};
     const float* old = nullptr;
     float* now = nullptr;
     if constexpr (DELTA) {
@@ -101,18 +120,22 @@ __global__ __launch_bounds__(1024) void k_tlm_state_step(TlmLinArgs a, int cgp) 
     for (int t = 0; t < un.n; ++t) {
         const long row = un.row0 + t;
         const float* in = a.in + row * a.in_ld;
+#pragma unroll 1
         for (int i = tid; i < 2 * D + V; i += nthr) {
             const int c = i < D ? a.q0 + kh * D + i : (i < 2 * D ? a.k0 + kh * D + i - D : a.v0 + h * V + i - 2 * D);
             float x;
-            if constexpr (DELTA) x = tlm_silu(tlm_conv(a, old, un.fresh, un.row0, t, c));
+            if constexpr (DELTA) x = tlm_silu(tlm_conv<float>(a, old, un.fresh, un.row0, t, c, t + 1 == un.n && (i >= 2 * D || h % rep == 0) ? now : nullptr));      // (the heads of a group share query and key channels)
             else x = in[c];
-            if (i < 2 * D) q[i] = x;
+            if (i < D) q[i] = x;
+            else if (i < 2 * D) k[i - D] = x;
             else v[i - 2 * D] = x;
         }
         if constexpr (DELTA)
-            for (int i = tid; i < D; i += nthr) g[i] = a.decay[(row * a.heads + h) * D + i];
+#pragma unroll 1
+            for (int i = tid; i < D; i += nthr) g[i] = tlm_decay(a, row, h, i);
         __syncthreads();
         float qq = 0.f, kk = 0.f, kq = 0.f;                // every wave sums for itself
+#pragma unroll 1
         for (int i = lane; i < D; i += 64) {
             qq = mmi_fma(q[i], q[i], qq);
             kk = mmi_fma(k[i], k[i], kk);
@@ -124,7 +147,7 @@ __global__ __launch_bounds__(1024) void k_tlm_state_step(TlmLinArgs a, int cgp) 
             iq = a.q_scale / sqrtf(tlm_wave_sum(qq) + 1e-6f);
             ik = 1.0f / sqrtf(tlm_wave_sum(kk) + 1e-6f);
             kq *= iq * ik;
-            beta = in[a.b0 + h];
+            beta = tlm_sigmoid(in[a.b0 + h]);
         } else {
             dec = a.decay[h * (TLM_CHUNK + 1) + 1];
         }
@@ -132,7 +155,6 @@ __global__ __launch_bounds__(1024) void k_tlm_state_step(TlmLinArgs a, int cgp) 
 #pragma unroll
         for (int i = 0; i < RT; ++i) {
             const int d = part + parts * i;
-            if (d >= D) continue;
             s[i] *= DELTA ? g[d] : dec;
             if constexpr (DELTA) ak += (k[d] * ik) * s[i];
             aq += (q[d] * iq) * s[i];
@@ -144,6 +166,7 @@ __global__ __launch_bounds__(1024) void k_tlm_state_step(TlmLinArgs a, int cgp) 
         __syncthreads();
         f32x4 u = {0.f, 0.f, 0.f, 0.f}, o = u;
         if (mine) {
+#pragma unroll 4
             for (int p = 0; p < parts; ++p) {
                 o += *reinterpret_cast<const f32x4*>(red + (long)p * V + col);
                 if constexpr (DELTA) u += *reinterpret_cast<const f32x4*>(red + (long)(parts + p) * V + col);
@@ -155,14 +178,17 @@ __global__ __launch_bounds__(1024) void k_tlm_state_step(TlmLinArgs a, int cgp) 
 #pragma unroll
         for (int i = 0; i < RT; ++i) {
             const int d = part + parts * i;
-            if (d < D) s[i] += (k[d] * ik) * u;
+            s[i] += (k[d] * ik) * u;
         }
         if constexpr (DELTA) {
             float ss = o[0] * o[0] + o[1] * o[1] + o[2] * o[2] + o[3] * o[3];
             for (int x = 1; x < cgp; x *= 2) ss += mmi_shfl_xor(ss, x);      // (the groups of one row part are neighbours in a wave)
             const float inv = 1.0f / sqrtf(ss / (float)a.vdim + a.eps);
             if (part == 0 && mine) {
-                const f32x4 w = *reinterpret_cast<const f32x4*>(a.nw + col), gt = *reinterpret_cast<const f32x4*>(a.gate + row * a.gate_ld + h * V + col);
+                const f32x4 w = *reinterpret_cast<const f32x4*>(a.nw + col);
+                f32x4 gt = *reinterpret_cast<const f32x4*>(a.gate + row * a.gate_ld + h * V + col);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) gt[e] = tlm_sigmoid(gt[e]);
                 Tr::store4((typename Tr::elem*)a.out + tlm_index<Tr>(row, h * V + col, a.out_ks), o * inv * w * gt);
             }
         } else if (part == 0 && mine) {
@@ -173,106 +199,109 @@ __global__ __launch_bounds__(1024) void k_tlm_state_step(TlmLinArgs a, int cgp) 
 #pragma unroll
     for (int i = 0; i < RT; ++i) {
         const int d = part + parts * i;
-        if (mine && d < D) *reinterpret_cast<f32x4*>(S + (long)d * V + col) = s[i];
+        if (mine && d < D) mmi_store_nt(reinterpret_cast<f32x4*>(S + (long)d * V + col), s[i]);
     }
-    if constexpr (DELTA)
-        for (int i = tid; i < 2 * D + V; i += nthr) {
-            if (i < 2 * D && h % rep) continue;            // query and key channels are shared by the heads of a group
-            tlm_conv_keep(a, old, now, un.fresh, un.row0, un.n, i < D ? a.q0 + kh * D + i : (i < 2 * D ? a.k0 + kh * D + i - D : a.v0 + h * V + i - 2 * D));
-        }
 }
 
 // ------------------------------------------------------------------------------------------------
-// chunks: convolutions and unit norms (delta).  grid: chunks, 2 kv_heads + heads; a wave takes 16 tokens, its lanes the channels of a head
+// chunks: convolutions and unit norms (delta).  grid: chunks, 2 kv_heads + heads; a lane takes 4 channels, a power of two of lanes a token
 // ------------------------------------------------------------------------------------------------
-inline __global__ __launch_bounds__(256) void k_tlm_conv(TlmLinArgs a) {
-    const int lane = (int)threadIdx.x & 63, wave = (int)threadIdx.x >> 6, y = (int)blockIdx.y;
+inline __global__ __launch_bounds__(256) void k_tlm_conv(TlmLinArgs a, int kgroups, int vgroups) {
+    const int y = (int)blockIdx.y;
     const TlmSeg ck = a.chunk[blockIdx.x];
     const int kind = y < a.kv_heads ? 0 : (y < 2 * a.kv_heads ? 1 : 2);
-    const int width = kind == 2 ? a.vdim_p : a.dim_p;
+    const int width = kind == 2 ? a.vdim_p : a.dim_p, groups = kind == 2 ? vgroups : kgroups;
     const int c0 = kind == 0 ? a.q0 + y * a.dim_p : (kind == 1 ? a.k0 + (y - a.kv_heads) * a.dim_p : a.v0 + (y - 2 * a.kv_heads) * a.vdim_p);
     const float* old = a.conv_state + ((long)ck.slot * 2 + ck.par) * (a.taps - 1) * a.conv_c;
+    float* now = a.conv_state + ((long)ck.slot * 2 + (ck.par ^ 1)) * (a.taps - 1) * a.conv_c;
     const int first = ck.row0 - ck.index * TLM_CHUNK;      // the sequence's first row of this step
-    for (int t = wave; t < ck.n; t += 4) {
-        float x[4], ss = 0.f;
+    const int c = 4 * ((int)threadIdx.x & (groups - 1)), step = 256 / groups;
+    for (int t0 = 0; t0 < ck.n; t0 += step) {              // (every lane of a wave goes round as often)
+        const int t = t0 + (int)threadIdx.x / groups;
+        f32x4 x = {0.f, 0.f, 0.f, 0.f};
+        if (t < ck.n && c < width) {
+            x = tlm_conv<f32x4>(a, old, ck.fresh, first, ck.index * TLM_CHUNK + t, c0 + c, ck.last && t + 1 == ck.n ? now : nullptr);
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            const int c = lane + 64 * i;
-            x[i] = c < width ? tlm_silu(tlm_conv(a, old, ck.fresh, first, ck.index * TLM_CHUNK + t, c0 + c)) : 0.f;
-            ss = mmi_fma(x[i], x[i], ss);
+            for (int e = 0; e < 4; ++e) x[e] = tlm_silu(x[e]);
         }
-        float f = 1.f;
-        if (kind != 2) f = (kind == 0 ? a.q_scale : 1.0f) / sqrtf(tlm_wave_sum(ss) + 1e-6f);
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            const int c = lane + 64 * i;
-            if (c < width) a.qkv[(long)(ck.row0 + t) * a.conv_c + c0 + c] = x[i] * f;
+        if (kind != 2) {
+            float ss = x[0] * x[0] + x[1] * x[1] + x[2] * x[2] + x[3] * x[3];
+            for (int m = 1; m < groups; m *= 2) ss += mmi_shfl_xor(ss, m);
+            x *= (kind == 0 ? a.q_scale : 1.0f) / sqrtf(ss + 1e-6f);
         }
-    }
-    if (ck.last) {
-        float* now = a.conv_state + ((long)ck.slot * 2 + (ck.par ^ 1)) * (a.taps - 1) * a.conv_c;
-        for (int c = (int)threadIdx.x; c < width; c += 256) tlm_conv_keep(a, old, now, ck.fresh, first, ck.index * TLM_CHUNK + ck.n, c0 + c);
+        if (t < ck.n && c < width) *reinterpret_cast<f32x4*>(a.qkv + (long)(ck.row0 + t) * a.conv_c + c0 + c) = x;
     }
 }
 
 // ------------------------------------------------------------------------------------------------
 // chunks, lightning: P, the decayed queries, the decayed transposed keys.  grid: chunks, heads
 // ------------------------------------------------------------------------------------------------
-inline __global__ __launch_bounds__(256) void k_tlm_chunk_lightning(TlmLinArgs a) {
-    const int lane = (int)threadIdx.x & 63, wave = (int)threadIdx.x >> 6, bl = lane & 15, kq = lane >> 4, h = (int)blockIdx.y;
+inline __global__ __launch_bounds__(256, 4) void k_tlm_chunk_lightning(TlmLinArgs a) {
+    const int tid = (int)threadIdx.x, lane = tid & 63, wave = mmi_uniform(tid >> 6), bl = lane & 15, kq = lane >> 4, h = (int)blockIdx.y;
     const TlmSeg ck = a.chunk[blockIdx.x];
     const int D = a.dim_p;
     const long id = (long)blockIdx.x * a.heads + h;
-    MMI_SHARED float pw[TLM_CHUNK + 1];
-    for (int i = (int)threadIdx.x; i <= TLM_CHUNK; i += 256) pw[i] = a.decay[h * (TLM_CHUNK + 1) + i];
-    __syncthreads();
+    MMI_SHARED __attribute__((aligned(16))) float Q[TLM_CHUNK * TLM_PST], K[TLM_CHUNK * TLM_PST], pw[TLM_CHUNK + 1];
+    for (int i = tid; i <= TLM_CHUNK; i += 256) pw[i] = a.decay[h * (TLM_CHUNK + 1) + i];
     const float* qp = a.in + (long)ck.row0 * a.in_ld + a.q0 + h * D;
     const float* kp = a.in + (long)ck.row0 * a.in_ld + a.k0 + h * D;
-    auto fetch = [&](const float* base, int t, int d) __attribute__((always_inline)) {
-        const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
-        return t < ck.n ? *reinterpret_cast<const f32x4*>(base + (long)t * a.in_ld + d) : zero;
-    };
+    float *Qg = a.qg + id * TLM_CHUNK * D, *Kt = a.kt + id * TLM_CHUNK * D, *P = a.p + id * (TLM_CHUNK * TLM_CHUNK);
     f32x4 acc[4];
 #pragma unroll
     for (int j = 0; j < 4; ++j) acc[j] = f32x4{0.f, 0.f, 0.f, 0.f};
-    for (int d = 0; d < D; d += 16) {
-        const f32x4 qv = fetch(qp, 16 * wave + bl, d + 4 * kq);
-        f32x4 kv[4];
+    for (int c0 = 0; c0 < D; c0 += 64) {                   // panels of 64 channels (a multiple of 16 in the last one)
+        const int cn = min(64, D - c0);
+        f32x4 qv[4], kv[4];
 #pragma unroll
-        for (int j = 0; j < 4; ++j) kv[j] = fetch(kp, 16 * j + bl, d + 4 * kq);
+        for (int i = 0; i < 4; ++i) {                      // (rows and columns past the end: a valid address, as zeros)
+            const int t = (tid >> 4) + 16 * i, c = min(4 * (tid & 15), cn - 4);
+            qv[i] = *reinterpret_cast<const f32x4*>(qp + (long)min(t, ck.n - 1) * a.in_ld + c0 + c);
+            kv[i] = *reinterpret_cast<const f32x4*>(kp + (long)min(t, ck.n - 1) * a.in_ld + c0 + c);
+        }
+        __syncthreads();
 #pragma unroll
-        for (int j = 0; j < 4; ++j)
-            if (j <= wave) acc[j] = TlmF32::mfma(__builtin_bit_cast(u32x4, qv), __builtin_bit_cast(u32x4, kv[j]), acc[j]);
+        for (int i = 0; i < 4; ++i) {
+            const int t = (tid >> 4) + 16 * i, c = 4 * (tid & 15);
+            if (t >= ck.n || c >= cn) qv[i] = kv[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+            *reinterpret_cast<f32x4*>(Q + t * TLM_PST + c) = qv[i];
+            *reinterpret_cast<f32x4*>(K + t * TLM_PST + c) = kv[i];
+            if (c < cn) *reinterpret_cast<f32x4*>(Qg + tlm_tile(t, c0 + c, D / 16)) = qv[i] * pw[t + 1];
+        }
+        __syncthreads();
+        for (int c = 4 * kq; c < cn; c += 16) {
+            const u32x4 q = *reinterpret_cast<const u32x4*>(Q + (16 * wave + bl) * TLM_PST + c);
+#pragma unroll
+            for (int j = 0; j < 4; ++j)
+                if (j <= wave) acc[j] = TlmF32::mfma(q, *reinterpret_cast<const u32x4*>(K + (16 * j + bl) * TLM_PST + c), acc[j]);
+        }
+        for (int i = wave; i < cn / 4; i += 4) {           // transposed fragments: 16 channels x 16 tokens
+            const int c = 16 * (i >> 2) + bl, t = 16 * (i & 3) + 4 * kq;
+            f32x4 v;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) v[e] = t + e < ck.n ? K[(t + e) * TLM_PST + c] * pw[ck.n - 1 - t - e] : 0.f;
+            *reinterpret_cast<f32x4*>(Kt + tlm_tile(c0 + c, t, 4)) = v;
+        }
     }
-    float* P = a.p + id * (TLM_CHUNK * TLM_CHUNK);
 #pragma unroll
     for (int j = 0; j < 4; ++j)
         if (j <= wave)
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int t = 16 * wave + 4 * kq + r, s = 16 * j + bl;
-                P[t * TLM_CHUNK + s] = s <= t ? acc[j][r] * pw[t - s] : 0.f;
+                P[tlm_tile(t, s, 4)] = s <= t ? acc[j][r] * pw[t - s] : 0.f;
             }
-    float* Q = a.qg + id * TLM_CHUNK * D;
-    float* K = a.kt + id * TLM_CHUNK * D;
-    const float ke = lane < ck.n ? pw[ck.n - 1 - lane] : 0.f;
-    for (int d = 4 * wave; d < D; d += 16) {               // lane: token
-        *reinterpret_cast<f32x4*>(Q + (long)lane * D + d) = fetch(qp, lane, d) * pw[lane + 1];
-        const f32x4 kv = fetch(kp, lane, d);
-#pragma unroll
-        for (int e = 0; e < 4; ++e) K[(long)(d + e) * TLM_CHUNK + lane] = kv[e] * ke;
-    }
-    for (int d = (int)threadIdx.x; d < D; d += 256) a.gend[id * D + d] = pw[ck.n];
+    for (int d = tid; d < D; d += 256) a.gend[id * D + d] = pw[ck.n];
 }
 
 // ------------------------------------------------------------------------------------------------
 // chunks, delta: P, W, U0, the decayed queries and transposed keys.  grid: chunks, heads; wave w owns tokens 16 w .. 16 w + 15
 // ------------------------------------------------------------------------------------------------
-inline size_t tlm_chunk_delta_smem() { return (size_t)(4 * TLM_CHUNK * TLM_PST + 4 * 64 + 4 * 16 * 20 + TLM_CHUNK) * sizeof(float); }
-inline __global__ __launch_bounds__(256) void k_tlm_chunk_delta(TlmLinArgs a) {
+inline size_t tlm_chunk_delta_smem() { return (size_t)(3 * TLM_CHUNK * TLM_PST + 4 * 64 + TLM_CHUNK) * sizeof(float); }
+inline __global__ __launch_bounds__(256, 2) void k_tlm_chunk_delta(TlmLinArgs a) {
     MMI_DYN_SHARED(float, sh);
-    float *K = sh, *Q = K + TLM_CHUNK * TLM_PST, *G = Q + TLM_CHUNK * TLM_PST, *A = G + TLM_CHUNK * TLM_PST;      // [64][TLM_PST] each
-    float *tot = A + TLM_CHUNK * TLM_PST, *ti = tot + 4 * 64, *beta = ti + 4 * 16 * 20;                            // [4][64], [4][16][20], [64]
+    float *K = sh, *Q = K + TLM_CHUNK * TLM_PST, *G = Q + TLM_CHUNK * TLM_PST;      // [64][TLM_PST] each
+    float *tot = G + TLM_CHUNK * TLM_PST, *beta = tot + 4 * 64;                     // [4][64], [64]
+    float *A = K, *ti = Q;                                                          // once the panels are done: [64][TLM_PST], [4][16][20]
     const int tid = (int)threadIdx.x, lane = tid & 63, wave = mmi_uniform(tid >> 6), bl = lane & 15, kq = lane >> 4, h = (int)blockIdx.y;
     const TlmSeg ck = a.chunk[blockIdx.x];
     const int D = a.dim_p, V = a.vdim_p, kh = h / (a.heads / a.kv_heads);
@@ -280,7 +309,7 @@ inline __global__ __launch_bounds__(256) void k_tlm_chunk_delta(TlmLinArgs a) {
     const float* qkv = a.qkv + (long)ck.row0 * a.conv_c;
     float *Wg = a.w + id * TLM_CHUNK * D, *Qg = a.qg + id * TLM_CHUNK * D, *Kt = a.kt + id * TLM_CHUNK * D, *Ug = a.u0 + id * TLM_CHUNK * V;
     float* P = a.p + id * (TLM_CHUNK * TLM_CHUNK);
-    if (tid < TLM_CHUNK) beta[tid] = tid < ck.n ? a.in[(long)(ck.row0 + tid) * a.in_ld + a.b0 + h] : 0.f;
+    if (tid < TLM_CHUNK) beta[tid] = tid < ck.n ? tlm_sigmoid(a.in[(long)(ck.row0 + tid) * a.in_ld + a.b0 + h]) : 0.f;
     float dA[16], dP[16];                                  // pairs (16 w + bl, 16 w + s) of this lane's quarter of the channels
 #pragma unroll
     for (int s = 0; s < 16; ++s) dA[s] = dP[s] = 0.f;
@@ -299,7 +328,8 @@ inline __global__ __launch_bounds__(256) void k_tlm_chunk_delta(TlmLinArgs a) {
             if (t < ck.n && c < cn) {
                 qv = *reinterpret_cast<const f32x4*>(qkv + (long)t * a.conv_c + a.q0 + kh * D + c0 + c);
                 kv = *reinterpret_cast<const f32x4*>(qkv + (long)t * a.conv_c + a.k0 + kh * D + c0 + c);
-                gv = *reinterpret_cast<const f32x4*>(a.decay + ((long)(ck.row0 + t) * a.heads + h) * D + c0 + c);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) gv[e] = tlm_decay(a, ck.row0 + t, h, c0 + c + e);
             }
             *reinterpret_cast<f32x4*>(Q + t * TLM_PST + c) = qv;
             *reinterpret_cast<f32x4*>(K + t * TLM_PST + c) = kv;
@@ -361,16 +391,21 @@ inline __global__ __launch_bounds__(256) void k_tlm_chunk_delta(TlmLinArgs a) {
             if (c >= cn) continue;
             f32x4 f = {1.f, 1.f, 1.f, 1.f};
             for (int m = 0; m < t >> 4; ++m) f *= *reinterpret_cast<const f32x4*>(tot + m * 64 + c);
-            *reinterpret_cast<f32x4*>(Qg + (long)t * D + c0 + c) = *reinterpret_cast<const f32x4*>(Q + t * TLM_PST + c) * f;
-            *reinterpret_cast<f32x4*>(Wg + (long)t * D + c0 + c) = *reinterpret_cast<const f32x4*>(K + t * TLM_PST + c) * f * beta[t];
+            *reinterpret_cast<f32x4*>(Qg + tlm_tile(t, c0 + c, D / 16)) = *reinterpret_cast<const f32x4*>(Q + t * TLM_PST + c) * f;
+            *reinterpret_cast<f32x4*>(Wg + tlm_tile(t, c0 + c, D / 16)) = *reinterpret_cast<const f32x4*>(K + t * TLM_PST + c) * f * beta[t];
         }
-        for (int c = wave; c < cn; c += 4) {               // lane: token
+        for (int i = wave; i < cn / 4; i += 4) {           // transposed fragments: 16 channels x 16 tokens
+            const int c = 16 * (i >> 2) + bl, t = 16 * (i & 3) + 4 * kq;
             float f = 1.f;
-            for (int m = (lane >> 4) + 1; m < 4; ++m) f *= tot[m * 64 + c];
-            Kt[(long)(c0 + c) * TLM_CHUNK + lane] = G[lane * TLM_PST + c] * f;
+            for (int m = (i & 3) + 1; m < 4; ++m) f *= tot[m * 64 + c];
+            f32x4 v;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) v[e] = G[(t + e) * TLM_PST + c] * f;
+            *reinterpret_cast<f32x4*>(Kt + tlm_tile(c0 + c, t, 4)) = v;
         }
         if (tid < cn) a.gend[id * D + c0 + tid] = tot[tid] * tot[64 + tid] * tot[128 + tid] * tot[192 + tid];
     }
+    __syncthreads();
     // - A: the strictly lower triangle (columns right of it inside the diagonal blocks: zero), P
 #pragma unroll
     for (int s = 0; s < 16; ++s) {
@@ -382,7 +417,7 @@ inline __global__ __launch_bounds__(256) void k_tlm_chunk_delta(TlmLinArgs a) {
         const int t = 16 * wave + bl, at = 16 * wave + s;
         if (kq == 0) {
             A[t * TLM_PST + at] = s < bl ? -beta[t] * x : 0.f;
-            P[t * TLM_CHUNK + at] = s <= bl ? y : 0.f;
+            P[tlm_tile(t, at, 4)] = s <= bl ? y : 0.f;
         }
     }
 #pragma unroll
@@ -392,7 +427,7 @@ inline __global__ __launch_bounds__(256) void k_tlm_chunk_delta(TlmLinArgs a) {
             for (int r = 0; r < 4; ++r) {
                 const int t = 16 * bi[b] + 4 * kq + r, s = 16 * bj[b] + bl;
                 A[t * TLM_PST + s] = -beta[t] * oA[b][r];
-                P[t * TLM_CHUNK + s] = oP[b][r];
+                P[tlm_tile(t, s, 4)] = oP[b][r];
             }
     __syncthreads();
     {                                                      // (I + A_ww)^-1, one column per lane
@@ -407,43 +442,66 @@ inline __global__ __launch_bounds__(256) void k_tlm_chunk_delta(TlmLinArgs a) {
         }
     }
     __syncthreads();
-    // forward substitution by blocks of 16, one 16-column strip of [W | U0] at a time
+    // forward substitution by blocks of 16; a wave takes four 16-column strips of [W | U0] at a time
     const int nd = D / 16, ns = nd + V / 16;
-    for (int st = wave; st < ns; st += 4) {
-        float* dst = st < nd ? Wg + 16 * st + bl : Ug + 16 * (st - nd) + bl;
-        const int ld = st < nd ? D : V;
-        f32x4 x[4];
+    for (int s0 = wave; s0 < ns; s0 += 16) {
+        f32x4 x[4][4];
 #pragma unroll
-        for (int i = 0; i < 4; ++i)
+        for (int k = 0; k < 4; ++k) {
+            const int st = min(s0 + 4 * k, ns - 1);        // (past the end: the last strip again, not stored)
+            const float* src = st < nd ? Wg : qkv + a.v0 + h * V + 16 * (st - nd) + bl;
 #pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const int t = 16 * i + 4 * kq + r;
-                if (st < nd) x[i][r] = dst[(long)t * ld];
-                else x[i][r] = t < ck.n ? beta[t] * qkv[(long)t * a.conv_c + a.v0 + h * V + 16 * (st - nd) + bl] : 0.f;
-            }
+            for (int i = 0; i < 4; ++i)
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            f32x4 b = x[i];
+                for (int r = 0; r < 4; ++r) {
+                    const int t = 16 * i + 4 * kq + r;
+                    x[k][i][r] = src[st < nd ? tlm_tile(t, 16 * st + bl, nd) : (long)min(t, ck.n - 1) * a.conv_c];
+                }
 #pragma unroll
-            for (int j = 0; j < i; ++j)
-                b = TlmF32::mfma(*reinterpret_cast<const u32x4*>(A + (16 * i + bl) * TLM_PST + 16 * j + 4 * kq), __builtin_bit_cast(u32x4, x[j]), b);
-            x[i] = TlmF32::mfma(*reinterpret_cast<const u32x4*>(ti + (i * 16 + bl) * 20 + 4 * kq), __builtin_bit_cast(u32x4, b), f32x4{0.f, 0.f, 0.f, 0.f});
+            for (int i = 0; i < 4; ++i)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    const int t = 16 * i + 4 * kq + r;
+                    x[k][i][r] = t < ck.n ? x[k][i][r] * (st < nd ? 1.f : beta[t]) : 0.f;
+                }
         }
 #pragma unroll
-        for (int i = 0; i < 4; ++i)
+        for (int i = 0; i < 4; ++i) {
 #pragma unroll
-            for (int r = 0; r < 4; ++r) dst[(long)(16 * i + 4 * kq + r) * ld] = x[i][r];
+            for (int j = 0; j < i; ++j) {
+                const u32x4 av = *reinterpret_cast<const u32x4*>(A + (16 * i + bl) * TLM_PST + 16 * j + 4 * kq);
+#pragma unroll
+                for (int k = 0; k < 4; ++k) x[k][i] = TlmF32::mfma(av, __builtin_bit_cast(u32x4, x[k][j]), x[k][i]);
+            }
+            const u32x4 tv = *reinterpret_cast<const u32x4*>(ti + (i * 16 + bl) * 20 + 4 * kq);
+#pragma unroll
+            for (int k = 0; k < 4; ++k) x[k][i] = TlmF32::mfma(tv, __builtin_bit_cast(u32x4, x[k][i]), f32x4{0.f, 0.f, 0.f, 0.f});
+        }
+#pragma unroll
+        for (int k = 0; k < 4; ++k)
+            if (s0 + 4 * k < ns)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    const int st = s0 + 4 * k;
+                    if (st >= nd) *reinterpret_cast<f32x4*>(Ug + (((long)i * (V / 16) + st - nd) * 64 + lane) * 4) = x[k][i];
+                    else
+#pragma unroll
+                        for (int r = 0; r < 4; ++r) Wg[tlm_tile(16 * i + 4 * kq + r, 16 * st + bl, nd)] = x[k][i][r];
+                }
     }
 }
 
 // ------------------------------------------------------------------------------------------------
-// chunks: the walk over a sequence's chunks.  One workgroup per (sequence, head, 16 columns of S); wave w holds rows of S in the layout the
-// matrix core leaves them in, which is also the layout it takes them as an operand; the waves' shares of W S and Qg S meet in LDS.
+// chunks: the walk over a sequence's chunks.  One workgroup per (sequence, head, 16 columns of S).  Wave w owns token block w of every chunk
+// and a quarter of the rows of S, in the layout the matrix core leaves them in, which is also the layout it takes them as an operand; S and
+// U go round through LDS.
 // grid: 8 x ceil(sequences x heads / 8) x vdim_p / 16, the column blocks of one head on one XCD (they read the same W, Qg, Kt, P)
 // ------------------------------------------------------------------------------------------------
+__device__ __forceinline__ float tlm_f(unsigned v) { return __builtin_bit_cast(float, v); }
 template <bool DELTA, int NDW>
 __global__ __launch_bounds__(256, 1) void k_tlm_chunk_scan(TlmLinArgs a, int n_units) {
-    MMI_SHARED __attribute__((aligned(16))) f32x4 red[2][DELTA ? 2 : 1][4][4][64];      // [parity][Qg S, W S][wave][token block][lane]
+    constexpr int ND = 4 * NDW;                            // 16-row blocks of S; past the model's: zeros
+    MMI_SHARED __attribute__((aligned(16))) f32x4 Sl[ND][64], Ul[4][64];
     const int lane = (int)threadIdx.x & 63, wave = mmi_uniform((int)threadIdx.x >> 6), bl = lane & 15, kq = lane >> 4;
     const int ncb = a.vdim_p / 16, j0 = (int)blockIdx.x >> 3;
     const int uh = ((int)blockIdx.x & 7) + 8 * (j0 / ncb), cb = j0 % ncb;
@@ -459,83 +517,121 @@ __global__ __launch_bounds__(256, 1) void k_tlm_chunk_scan(TlmLinArgs a, int n_u
         if (!un.fresh && d < nd)
 #pragma unroll
             for (int r = 0; r < 4; ++r) s[i][r] = S[(long)(16 * d + 4 * kq + r) * V];
+        Sl[d][lane] = s[i];
     }
+    __syncthreads();
     struct Frags {
-        u32x4 w[DELTA ? 4 : 1][NDW], q[4][NDW], k[NDW][4], p[4];
-        f32x4 u[4], g[NDW];
+        u32x4 w[DELTA ? ND : 1], q[ND], k[NDW][4], p[4];
+        f32x4 u, g[NDW];
     };
-    auto load = [&](Frags& f, int c) __attribute__((always_inline)) {
+    auto load = [&](Frags& f, int c) __attribute__((always_inline)) {      // (blocks past the end: a valid address, against rows of S that stay zero)
         const long id = (long)(un.chunk0 + c) * a.heads + h;
         const int n = min(TLM_CHUNK, un.n - c * TLM_CHUNK);
 #pragma unroll
-        for (int i = 0; i < NDW; ++i) {
-            const int d = min(wave * NDW + i, nd - 1);     // (past the end: a valid address, against rows of S that stay zero)
+        for (int d = 0; d < ND; ++d) {
+            const long at = id * TLM_CHUNK * D + (((long)wave * nd + min(d, nd - 1)) * 64 + lane) * 4;
+            if constexpr (DELTA) f.w[d] = *reinterpret_cast<const u32x4*>(a.w + at);
+            f.q[d] = *reinterpret_cast<const u32x4*>(a.qg + at);
+        }
 #pragma unroll
-            for (int t = 0; t < 4; ++t) {
-                const long at = id * TLM_CHUNK * D + (long)(16 * t + bl) * D + 16 * d + 4 * kq;
-                if constexpr (DELTA) f.w[t][i] = *reinterpret_cast<const u32x4*>(a.w + at);
-                f.q[t][i] = *reinterpret_cast<const u32x4*>(a.qg + at);
-                f.k[i][t] = *reinterpret_cast<const u32x4*>(a.kt + id * TLM_CHUNK * D + (long)(16 * d + bl) * TLM_CHUNK + 16 * t + 4 * kq);
-            }
+        for (int i = 0; i < NDW; ++i) {
+            const int d = min(wave * NDW + i, nd - 1);
+#pragma unroll
+            for (int t = 0; t < 4; ++t) f.k[i][t] = *reinterpret_cast<const u32x4*>(a.kt + id * TLM_CHUNK * D + (((long)d * 4 + t) * 64 + lane) * 4);
             f.g[i] = *reinterpret_cast<const f32x4*>(a.gend + id * D + 16 * d + 4 * kq);
         }
 #pragma unroll
-        for (int t = 0; t < 4; ++t) {
-            f.p[t] = *reinterpret_cast<const u32x4*>(a.p + id * (TLM_CHUNK * TLM_CHUNK) + (16 * wave + bl) * TLM_CHUNK + 16 * min(t, wave) + 4 * kq);
+        for (int t = 0; t < 4; ++t)
+            f.p[t] = *reinterpret_cast<const u32x4*>(a.p + id * (TLM_CHUNK * TLM_CHUNK) + ((wave * 4 + min(t, wave)) * 64 + lane) * 4);
+        if constexpr (DELTA) {
+            f.u = *reinterpret_cast<const f32x4*>(a.u0 + id * TLM_CHUNK * V + (((long)wave * ncb + cb) * 64 + lane) * 4);
+        } else {
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
-                const int tok = 16 * t + 4 * kq + r;
-                if constexpr (DELTA) f.u[t][r] = a.u0[(id * TLM_CHUNK + tok) * V + 16 * cb + bl];
-                else f.u[t][r] = tok < n ? a.in[(long)(un.row0 + c * TLM_CHUNK + tok) * a.in_ld + a.v0 + h * V + 16 * cb + bl] : 0.f;
+                const int tok = 16 * wave + 4 * kq + r;
+                const float v = a.in[(long)(un.row0 + c * TLM_CHUNK + min(tok, n - 1)) * a.in_ld + a.v0 + h * V + 16 * cb + bl];
+                f.u[r] = tok < n ? v : 0.f;
             }
         }
     };
-    Frags f;
-    load(f, 0);
-    for (int c = 0; c < un.n_chunks; ++c) {
+    auto chunk = [&](const Frags& f, int c) __attribute__((always_inline)) {
         const int n = min(TLM_CHUNK, un.n - c * TLM_CHUNK);
-        f32x4 x[4], y[4];
+        // four independent sums go round, one step of four each: a matrix instruction never waits for the one before it
+        const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+        f32x4 x0 = zero, x1 = zero, o0 = zero, o1 = zero;
+        if constexpr (!DELTA) Ul[wave][lane] = f.u;
 #pragma unroll
-        for (int t = 0; t < 4; ++t) {
-            x[t] = y[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int d = 0; d < ND; d += 2) {
+            const f32x4 sa = Sl[d][lane], sb = Sl[d + 1][lane];
 #pragma unroll
-            for (int i = 0; i < NDW; ++i) {
-                if constexpr (DELTA) x[t] = TlmF32::mfma(f.w[t][i], __builtin_bit_cast(u32x4, s[i]), x[t]);
-                y[t] = TlmF32::mfma(f.q[t][i], __builtin_bit_cast(u32x4, s[i]), y[t]);
+            for (int e = 0; e < 4; ++e) {
+                if constexpr (DELTA) {
+                    x0 = mmi_mfma_f32_16x16x4(tlm_f(f.w[d][e]), sa[e], x0);
+                    x1 = mmi_mfma_f32_16x16x4(tlm_f(f.w[d + 1][e]), sb[e], x1);
+                }
+                o0 = mmi_mfma_f32_16x16x4(tlm_f(f.q[d][e]), sa[e], o0);
+                o1 = mmi_mfma_f32_16x16x4(tlm_f(f.q[d + 1][e]), sb[e], o1);
             }
-            if constexpr (DELTA) red[c & 1][DELTA][wave][t][lane] = x[t];
-            red[c & 1][0][wave][t][lane] = y[t];
         }
-        Frags nx;                                          // (the last chunk asks for itself again)
-        load(nx, min(c + 1, un.n_chunks - 1));
-        mmi_sched_barrier();
+        if constexpr (DELTA) Ul[wave][lane] = f.u - (x0 + x1);
         __syncthreads();
-        f32x4 u[4], o = {0.f, 0.f, 0.f, 0.f};
+        f32x4 u[4], sh[NDW];
 #pragma unroll
-        for (int t = 0; t < 4; ++t) {
-            u[t] = f.u[t];
-            if constexpr (DELTA)
+        for (int t = 0; t < 4; ++t) u[t] = Ul[t][lane];
 #pragma unroll
-                for (int v = 0; v < 4; ++v) u[t] -= red[c & 1][DELTA][v][t][lane];
+        for (int i = 0; i < NDW; ++i) {
+            s[i] *= f.g[i];
+            sh[i] = zero;
         }
 #pragma unroll
-        for (int v = 0; v < 4; ++v) o += red[c & 1][0][v][wave][lane];
+        for (int t = 0; t < 4; t += 2)
 #pragma unroll
-        for (int t = 0; t < 4; ++t)
-            if (t <= wave) o = TlmF32::mfma(f.p[t], __builtin_bit_cast(u32x4, u[t]), o);
+            for (int e = 0; e < 4; ++e)
+#pragma unroll
+                for (int i = 0; i < NDW; ++i) {
+                    s[i] = mmi_mfma_f32_16x16x4(tlm_f(f.k[i][t][e]), u[t][e], s[i]);
+                    sh[i] = mmi_mfma_f32_16x16x4(tlm_f(f.k[i][t + 1][e]), u[t + 1][e], sh[i]);
+                }
+#pragma unroll
+        for (int i = 0; i < NDW; ++i) {
+            s[i] += sh[i];
+            if (wave * NDW + i >= nd) s[i] = zero;
+            Sl[wave * NDW + i][lane] = s[i];
+        }
+#pragma unroll
+        for (int t = 0; t < 4; t += 2)                     // (blocks right of the diagonal: zeros instead)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                o0 = mmi_mfma_f32_16x16x4(t <= wave ? tlm_f(f.p[t][e]) : 0.f, u[t][e], o0);
+                o1 = mmi_mfma_f32_16x16x4(t + 1 <= wave ? tlm_f(f.p[t + 1][e]) : 0.f, u[t + 1][e], o1);
+            }
+        const f32x4 o = o0 + o1;
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
             const int tok = 16 * wave + 4 * kq + r;
             if (tok < n) a.o[((long)(un.row0 + c * TLM_CHUNK + tok) * a.heads + h) * V + 16 * cb + bl] = o[r];
         }
-#pragma unroll
-        for (int i = 0; i < NDW; ++i) {
-            s[i] *= f.g[i];
-#pragma unroll
-            for (int t = 0; t < 4; ++t) s[i] = TlmF32::mfma(f.k[i][t], __builtin_bit_cast(u32x4, u[t]), s[i]);
-            if (wave * NDW + i >= nd) s[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+        __syncthreads();
+    };
+    if constexpr (NDW <= 2) {
+        // the next chunk's operands are on their way while a chunk is computed (the last one asks for itself again)
+        Frags fa, fb;
+        load(fa, 0);
+        for (int c = 0; c < un.n_chunks; c += 2) {
+            load(fb, min(c + 1, un.n_chunks - 1));
+            mmi_sched_barrier();
+            chunk(fa, c);
+            if (c + 1 == un.n_chunks) break;
+            load(fa, min(c + 2, un.n_chunks - 1));
+            mmi_sched_barrier();
+            chunk(fb, c + 1);
         }
-        f = nx;
+    } else {
+        Frags f;
+        for (int c = 0; c < un.n_chunks; ++c) {
+            load(f, c);
+            chunk(f, c);
+        }
     }
 #pragma unroll
     for (int i = 0; i < NDW; ++i) {
@@ -584,7 +680,10 @@ __global__ __launch_bounds__(256) void k_tlm_gated_norm(TlmLinArgs a, int per_he
     __syncthreads();
     for (int c = 4 * tid; c < ld; c += 1024) {
         const int h = c / V;
-        const f32x4 w = *reinterpret_cast<const f32x4*>(a.nw + (per_head ? c - h * V : c)), g = *reinterpret_cast<const f32x4*>(a.gate + row * a.gate_ld + c);
+        const f32x4 w = *reinterpret_cast<const f32x4*>(a.nw + (per_head ? c - h * V : c));
+        f32x4 g = *reinterpret_cast<const f32x4*>(a.gate + row * a.gate_ld + c);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) g[e] = tlm_sigmoid(g[e]);
         Tr::store4((typename Tr::elem*)a.out + tlm_index<Tr>(row, c, a.out_ks), *reinterpret_cast<const f32x4*>(o + c) * inv[h] * w * g);
     }
 }

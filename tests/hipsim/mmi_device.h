@@ -349,7 +349,10 @@ inline int mmi_uniform(int v) { return v; }
 inline bool mmi_any(bool v) { unsigned x = v ? 1u : 0u; for (int m = 1; m < 64; m <<= 1) { const unsigned o = mmi_shfl_xor(x, m); x = o > x ? o : x; } return x != 0; }
 inline u32x4 mmi_load_nt(const u32x4* p) { return *p; }
 inline f32x4 mmi_load_nt(const f32x4* p) { return *p; }
+inline void mmi_store_nt(f32x4* p, f32x4 v) { *p = v; }
 inline float mmi_rsqrtf(float x) { return 1.0f / sqrtf(x); }
+inline float mmi_fast_exp2f(float x) { return exp2f(x); }
+inline float mmi_fast_log2f(float x) { return log2f(x); }
 inline float mmi_fast_logf(float x) { return logf(x); }
 inline unsigned mmi_wave_sum_u32(unsigned x) { for (int m = 1; m < 64; m <<= 1) x += mmi_shfl_xor(x, m); return x; }
 inline unsigned mmi_wave_max_u32(unsigned x) { for (int m = 1; m < 64; m <<= 1) { const unsigned o = mmi_shfl_xor(x, m); x = o > x ? o : x; } return x; }
