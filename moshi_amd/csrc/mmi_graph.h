@@ -40,20 +40,6 @@ struct MmiProgram {
 
     void site(const std::string& label) { site_ = label; }
     void add(std::function<int(hipStream_t)> f, long bytes = 0) {
-        // MMI_SKIP_SITES="enc.tr,dec.res" (timing experiments ONLY - the outputs are then garbage): ops whose site label starts with
-        // one of the prefixes are left out of the list.  How round 6 found which part of the codec stretches the depth-transformer
-        // phase under the duplex pipeline (profiles/r06_logs/pipeline_skip_sites.txt)
-        if (const char* e = getenv("MMI_SKIP_SITES")) {
-            std::string all(e);
-            size_t i = 0;
-            while (i <= all.size()) {
-                const size_t j = all.find(',', i);
-                const std::string pre = all.substr(i, j == std::string::npos ? std::string::npos : j - i);
-                if (!pre.empty() && site_.compare(0, pre.size(), pre) == 0) return;
-                if (j == std::string::npos) break;
-                i = j + 1;
-            }
-        }
         ops.push_back(std::move(f)); sites.push_back(site_); op_bytes.push_back(bytes);
     }
     bool logged() const { return logged_[variant]; }

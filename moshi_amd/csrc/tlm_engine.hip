@@ -162,6 +162,7 @@ constexpr int MAX_SPLIT = 8;
 constexpr int ROWS_MAX = 64;       // up to here a step takes the weight-streaming kernel
 constexpr int ATTN_TILE_GROUPS = 128;     // from this many column groups the attention stages keys through LDS
 constexpr int PREFIXES = 6;        // prefix arrays over the sequences per head count: tiles, groups of 4, groups of 8, then those of `split`
+constexpr int MAX_KEY_SPLIT = 16;
 constexpr int MAX_PARTIALS = 512;  // (column tile, split) pairs of the attention
 
 // ------------------------------------------------------------------------------------------------
@@ -903,7 +904,7 @@ int launch_gqa_d(hipStream_t s, const TlmGqaArgs& a, bool tiled) {
         MMI_LAUNCH((k_tlm_gqa_tile<Tr, D>), dim3(a.n_tiles, a.kv_heads), 256, smem, s, a);
     } else {
         MMI_LAUNCH((k_tlm_gqa<Tr, D>), dim3(a.n_tiles, a.kv_heads, a.nsplit), 256, 0, s, a);
-        if (a.nsplit > 1) MMI_LAUNCH((k_tlm_gqa_combine<Tr>), dim3(a.n_tiles, a.kv_heads), 256, 0, s, a);
+        if (a.nsplit > 1) MMI_LAUNCH((k_tlm_gqa_combine<Tr>), dim3(a.n_tiles, a.kv_heads, mmi_cdiv(a.nd, 4)), 256, 0, s, a);
     }
     MMI_CHECK_LAUNCH();
     return MMI_OK;
@@ -1919,7 +1920,7 @@ extern "C" int mmi_tlm_step(mmi_tlm* m, int32_t n_entries, const int32_t* slots,
     // few column tiles and long contexts: split the keys over workgroups, at least 4 blocks of 32 keys each
     int tiles_max = 1;
     for (int t : sh.tiles) tiles_max = std::max(tiles_max, t);
-    while (sh.nsplit < 16 && tiles_max * sh.nsplit * 2 <= MAX_PARTIALS && blocks / (sh.nsplit * 2) >= 4) sh.nsplit *= 2;
+    while (sh.nsplit < MAX_KEY_SPLIT && tiles_max * sh.nsplit * 2 <= MAX_PARTIALS && blocks / (sh.nsplit * 2) >= 4) sh.nsplit *= 2;
     MMI_HIP_CHECK(hipMemcpyAsync(m->meta, b, (size_t)M.total * sizeof(int), hipMemcpyHostToDevice, s));
     MMI_HIP_CHECK(hipEventRecord(st.ev, s));
     st.used = true;

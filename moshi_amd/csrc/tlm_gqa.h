@@ -175,28 +175,37 @@ __global__ __launch_bounds__(256, Tr::V == 8 && D <= 128 ? 2 : 1) void k_tlm_gqa
     }
 }
 
-// the splits of one column tile -> output.  grid: column tiles, kv heads
+// the splits (at most 16) of one column tile -> output; a wave takes one 16-wide block of values, all its loads in flight together.
+// grid: column tiles, kv heads, blocks / 4
 template <class Tr>
 __global__ __launch_bounds__(256) void k_tlm_gqa_combine(TlmGqaArgs a) {
     typedef TlmGqa<Tr, 64> P;                                      // (nothing below depends on the bound)
+    constexpr int MAXS = 16;
     const int lane = (int)threadIdx.x & 63, wave = mmi_uniform((int)threadIdx.x >> 6), bl = lane & 15, kq = lane >> 4;
-    const int tile = (int)blockIdx.x, g = (int)blockIdx.y;
-    const TlmCols c = P::find(a, tile);
+    const int tile = (int)blockIdx.x, g = (int)blockIdx.y, d = wave + 4 * (int)blockIdx.z;
+    if (d >= a.nd) return;
     const long part = ((long)tile * a.kv_heads + g) * a.nsplit;
-    const float* q = a.pml + part * 32;
-    float M = -1e30f, L = 0.f;
-#pragma unroll 4
-    for (int s = 0; s < a.nsplit; ++s) M = fmaxf(M, q[s * 32 + bl]);
-#pragma unroll 4
-    for (int s = 0; s < a.nsplit; ++s) L += q[s * 32 + 16 + bl] * exp2f(q[s * 32 + bl] - M);
-    const float inv = 1.0f / (a.sink ? L + exp2f(-M) : L);
-    for (int d = wave; d < a.nd; d += 4) {
-        f32x4 v = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-        for (int s = 0; s < a.nsplit; ++s)
-            v += *reinterpret_cast<const f32x4*>(a.po + (((part + s) * a.nd + d) * 64 + lane) * 4) * exp2f(q[s * 32 + bl] - M);
-        P::store(a, c, g, bl, kq, d, v * inv);
+    float m[MAXS], l[MAXS];
+    f32x4 v[MAXS];
+#pragma unroll
+    for (int s = 0; s < MAXS; ++s) {                               // (past the end: the last split again, with weight zero)
+        const long p = part + min(s, a.nsplit - 1);
+        m[s] = a.pml[p * 32 + bl];
+        l[s] = a.pml[p * 32 + 16 + bl];
+        v[s] = *reinterpret_cast<const f32x4*>(a.po + ((p * a.nd + d) * 64 + lane) * 4);
     }
+    const TlmCols c = P::find(a, tile);
+    float M = m[0], L = 0.f;
+#pragma unroll
+    for (int s = 1; s < MAXS; ++s) M = fmaxf(M, m[s]);
+    f32x4 o = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int s = 0; s < MAXS; ++s) {
+        const float f = s < a.nsplit ? exp2f(m[s] - M) : 0.f;
+        L = mmi_fma(l[s], f, L);
+        o += v[s] * f;
+    }
+    P::store(a, c, g, bl, kq, d, o * (1.0f / (a.sink ? L + exp2f(-M) : L)));
 }
 
 // Many columns (prompts): four waves x QT column tiles of one sequence and kv head walk the same keys; a block's fragments are staged

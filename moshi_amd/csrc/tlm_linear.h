@@ -120,8 +120,20 @@ __global__ __launch_bounds__(MAXB, MAXB == 512 && !DELTA ? 5 : 4) void k_tlm_sta
     for (int t = 0; t < un.n; ++t) {
         const long row = un.row0 + t;
         const float* in = a.in + row * a.in_ld;
+        // everything the token needs is requested before anything is used: q, k, v and (delta) the decays, one value per thread and round
+        f32x4 gt = {0.f, 0.f, 0.f, 0.f}, nw = gt;
+        float beta = 0.f;
+        if constexpr (DELTA) {
+            beta = in[a.b0 + h];
+            gt = *reinterpret_cast<const f32x4*>(a.gate + row * a.gate_ld + h * V + min(col, V - 4));
+            nw = *reinterpret_cast<const f32x4*>(a.nw + min(col, V - 4));
+        }
 #pragma unroll 1
-        for (int i = tid; i < 2 * D + V; i += nthr) {
+        for (int i = tid; i < (DELTA ? 3 : 2) * D + V; i += nthr) {
+            if (DELTA && i >= 2 * D + V) {
+                g[i - 2 * D - V] = tlm_decay(a, row, h, i - 2 * D - V);
+                continue;
+            }
             const int c = i < D ? a.q0 + kh * D + i : (i < 2 * D ? a.k0 + kh * D + i - D : a.v0 + h * V + i - 2 * D);
             float x;
             if constexpr (DELTA) x = tlm_silu(tlm_conv<float>(a, old, un.fresh, un.row0, t, c, t + 1 == un.n && (i >= 2 * D || h % rep == 0) ? now : nullptr));      // (the heads of a group share query and key channels)
@@ -130,9 +142,6 @@ __global__ __launch_bounds__(MAXB, MAXB == 512 && !DELTA ? 5 : 4) void k_tlm_sta
             else if (i < 2 * D) k[i - D] = x;
             else v[i - 2 * D] = x;
         }
-        if constexpr (DELTA)
-#pragma unroll 1
-            for (int i = tid; i < D; i += nthr) g[i] = tlm_decay(a, row, h, i);
         __syncthreads();
         float qq = 0.f, kk = 0.f, kq = 0.f;                // every wave sums for itself
 #pragma unroll 1
@@ -142,12 +151,12 @@ __global__ __launch_bounds__(MAXB, MAXB == 512 && !DELTA ? 5 : 4) void k_tlm_sta
             kq = mmi_fma(k[i], q[i], kq);
         }
         kq = tlm_wave_sum(kq);
-        float iq = 1.f, ik = 1.f, beta = 1.f, dec = 1.f;
+        float iq = 1.f, ik = 1.f, dec = 1.f;
         if constexpr (DELTA) {
             iq = a.q_scale / sqrtf(tlm_wave_sum(qq) + 1e-6f);
             ik = 1.0f / sqrtf(tlm_wave_sum(kk) + 1e-6f);
             kq *= iq * ik;
-            beta = tlm_sigmoid(in[a.b0 + h]);
+            beta = tlm_sigmoid(beta);
         } else {
             dec = a.decay[h * (TLM_CHUNK + 1) + 1];
         }
@@ -185,11 +194,9 @@ __global__ __launch_bounds__(MAXB, MAXB == 512 && !DELTA ? 5 : 4) void k_tlm_sta
             for (int x = 1; x < cgp; x *= 2) ss += mmi_shfl_xor(ss, x);      // (the groups of one row part are neighbours in a wave)
             const float inv = 1.0f / sqrtf(ss / (float)a.vdim + a.eps);
             if (part == 0 && mine) {
-                const f32x4 w = *reinterpret_cast<const f32x4*>(a.nw + col);
-                f32x4 gt = *reinterpret_cast<const f32x4*>(a.gate + row * a.gate_ld + h * V + col);
 #pragma unroll
                 for (int e = 0; e < 4; ++e) gt[e] = tlm_sigmoid(gt[e]);
-                Tr::store4((typename Tr::elem*)a.out + tlm_index<Tr>(row, h * V + col, a.out_ks), o * inv * w * gt);
+                Tr::store4((typename Tr::elem*)a.out + tlm_index<Tr>(row, h * V + col, a.out_ks), o * inv * nw * gt);
             }
         } else if (part == 0 && mine) {
             *reinterpret_cast<f32x4*>(a.o + (row * a.heads + h) * V + col) = o;

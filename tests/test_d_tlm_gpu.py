@@ -54,6 +54,12 @@ def test_long_prompt_per_head_size(lib, name, dtype):
     tc.check_long_prompt(DEV, lib, dtype, n=800, cfg=tc.WIDE_PROMPTS_2[name])
 
 
+@pytest.mark.parametrize("dtype", [tc.F32, tc.BF16], ids=["fp32", "bf16"])
+@pytest.mark.parametrize("name", sorted(tc.BESIDE))
+def test_long_prompt_beside_decoding(lib, name, dtype):
+    tc.check_long_prompt_beside_decoding(DEV, lib, dtype, n=900, name=name)
+
+
 @pytest.mark.parametrize("window,keep", [(70, 6), (64, 1), (33, 64), (0, 0)])
 def test_single_kept_keys(lib, window, keep):
     tc.check_single_kept_keys(DEV, lib, window, keep)

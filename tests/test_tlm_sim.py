@@ -109,6 +109,10 @@ def test_unequal_requests_in_one_batch_bibapel(tlm_lib):
     tc.check_unequal_batch(DEV, tlm_lib, name="bibapel")
 
 
+def test_long_prompt_beside_decoding(tlm_lib):
+    tc.check_long_prompt_beside_decoding(DEV, tlm_lib, name="all")
+
+
 def test_batched_decode_bibapel(tlm_lib):
     tc.check_batched_decode(DEV, tlm_lib, steps=4, name="bibapel")
 

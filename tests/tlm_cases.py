@@ -288,6 +288,46 @@ def check_long_prompt(dev, lib, dtype=F32, n=1300, cfg=None):
     lm.close(slot)
 
 
+def check_long_prompt_beside_decoding(dev, lib, dtype=F32, n=340, name="many_kv_heads"):
+    """A long portion beside single tokens and short portions of other sequences in one step: the two forms of the attention kernel and of
+    the recurrences share a step, and leave each other's rows alone."""
+    cfg = BESIDE[name]
+    lm, orc = make(cfg, dev, lib, dtype, max_tokens=2048)
+    lens = (90, 33, 70, 12)
+    seqs = [tokens_of(cfg, k + 7, seed=20 + i) for i, k in enumerate(lens)]
+    long = tokens_of(cfg, n, seed=30)
+    slots = [lm.open() for _ in seqs]
+    for s, t, k in zip(slots, seqs, lens):
+        lm.step([(s, t[:k], [])])
+    ls = lm.open()
+    want = [orc.logits(t) for t in seqs]
+    wl = orc.logits(long)
+    pick = [0, 63, 64, n // 2, n - 6]
+    counts = (1, 4, 1, 5)
+    entries = [(s, t[k:k + c], list(range(c))) for s, t, k, c in zip(slots, seqs, lens, counts)]
+    entries.insert(2, (ls, long[:n - 5], pick))
+    rows = lm.step(entries).cpu().numpy()
+    at = 0
+    for i in (0, 1, None, 2, 3):
+        m = len(pick) if i is None else counts[i]
+        ref = wl[pick] if i is None else want[i][lens[i]:lens[i] + m]
+        assert rel(rows[at:at + m], ref) < TOL[dtype], i
+        at += m
+    entries = [(s, t[k + c:k + c + 2], [0, 1]) for s, t, k, c in zip(slots, seqs, lens, counts)] + [(ls, long[n - 5:], list(range(5)))]
+    rows = lm.step(entries).cpu().numpy()
+    ref = np.concatenate([w[k + c:k + c + 2] for w, k, c in zip(want, lens, counts)] + [wl[n - 5:]])
+    assert rel(rows, ref) < TOL[dtype]
+    for s in slots + [ls]:
+        lm.close(s)
+
+
+BESIDE = {
+    "many_kv_heads": plain_layer(replace(GQA, heads=26, kv_heads=13, window=150)),
+    "all": plain_layer(None, layers=[TokenLayerConfig(DELTA, GLU), TokenLayerConfig(replace(GQA, heads=26, kv_heads=13, window=100), GLU), TokenLayerConfig(LIGHT, None)],
+                       bigram=BigramConfig(buckets=29, mul_prev=7, mul_cur=2), max_positions=2000, loop_start=1, loop_stop=3, loop_times=2),
+}
+
+
 # ---- single keys ---------------------------------------------------------------------------------------------------------------
 def _pair_that_stands_out(orc, cfg):
     """(query token, key token, plain token): of all pairs the one whose un-rotated score beats the plain token's by most."""
