@@ -44,7 +44,7 @@ def bibapel_sizes():
         light = LightningConfig(heads=n, dim=128, vdim=128, decay=[1 - 2.0 ** (-1 - 8 * i / n) for i in range(n)])
         return TokenLMConfig("Bibapel", vocab=vocab, width=width, layers=[TokenLayerConfig(k, DenseGLUConfig(ff=ff, limit=7.0)) for k in (delta, att, light, light, delta, att)],
                              loop_start=0, loop_stop=2, loop_times=2, loop_inject="project", norms=2, layer_scales=False, tied_head=True,
-                             bigram=BigramConfig(buckets=65521, mul_prev=31, mul_cur=7), max_positions=8192)
+                             bigram=BigramConfig(buckets=65521, mul_prev=40503, mul_cur=9176), max_positions=8192)
     return {"1024": model(1024, 2816, 1024), "2048": model(2048, 5632, 1024), "4096": model(4096, 11264, 2048)}
 
 

@@ -60,7 +60,7 @@ def test_long_prompt_beside_decoding(lib, name, dtype):
     tc.check_long_prompt_beside_decoding(DEV, lib, dtype, n=900, name=name)
 
 
-@pytest.mark.parametrize("window,keep", [(70, 6), (64, 1), (33, 64), (0, 0)])
+@pytest.mark.parametrize("window,keep", [(70, 7), (64, 1), (33, 64), (0, 0)])
 def test_single_kept_keys(lib, window, keep):
     tc.check_single_kept_keys(DEV, lib, window, keep)
 

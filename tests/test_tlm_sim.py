@@ -125,7 +125,7 @@ def test_decoding_longer_than_the_pool_with_kept_pages(tlm_lib):
     tc.check_long_decode(DEV, tlm_lib, name="two_kept_windows", n=400, held=4)
 
 
-@pytest.mark.parametrize("window,keep", [(70, 6), (64, 1), (33, 64), (0, 0)])
+@pytest.mark.parametrize("window,keep", [(70, 7), (64, 1), (33, 64), (0, 0)])
 def test_single_kept_keys(tlm_lib, window, keep):
     tc.check_single_kept_keys(DEV, tlm_lib, window, keep, queries=(128, 103) if window else (128,))
 

@@ -417,7 +417,7 @@ def _attention_pair(orc, cfg):
     return int(query), int(key), int(np.argmin(s[query, :, head]))
 
 
-def check_single_kept_keys(dev, lib, window=70, keep=6, dtype=F32, queries=(200, 128, 191, 97)):
+def check_single_kept_keys(dev, lib, window=70, keep=7, dtype=F32, queries=(200, 128, 191, 97)):
     """One dominating key at chosen places: around the window's edge, page borders, the last kept position and the one after it.  While it is
     visible the logits are the oracle's and differ from a prompt without it; otherwise they are bit-identical to that."""
     cfg = plain_layer(replace(GQA, window=window, keep_first=keep, scale=1.0))
